@@ -4,5 +4,7 @@ from .manirax import ManiraxConfig
 from .risonex import RisonexConfig
 from .dupolorn import DupolornConfig
 from .favizen import FavizenConfig
+from .dopivik import DopivikConfig
 
-__all__ = ["PartSpec", "SubLayerSpec", "LayerSpec", "ScheduleEntry", "ModelSpec", "ConfigError", "LlamaConfig", "ManiraxConfig", "RisonexConfig", "DupolornConfig", "FavizenConfig"]
+__all__ = ["PartSpec", "SubLayerSpec", "LayerSpec", "ScheduleEntry", "ModelSpec", "ConfigError", "LlamaConfig", "ManiraxConfig", "RisonexConfig",
+           "DupolornConfig", "FavizenConfig", "DopivikConfig"]

@@ -44,13 +44,15 @@ struct CachePtrs {
 // `block` b: a token at position p reads no key before p - p % b; `sink` [H]: every head's sum of weights also counts
 // exp(sink[h]), a score with no key and no value that is not scaled; `slopes` [H]: the score of the key at position j
 // loses slopes[h] * (p - j); `gate`: head h's output is multiplied by sigmoid(gate[token][gate_col + h]) (float32 rows of
-// gate_stride numbers).
+// gate_stride numbers), with `gate_elem` its element d by sigmoid(gate[token][gate_col + h * HD + d]); `softcap` c: a
+// scaled score s becomes c tanh(s / c) before anything else.
 struct AttnExtras {
     int block;
     const float* sink;
     const float* slopes;
     const float* gate;
-    int gate_stride, gate_col;
+    int gate_stride, gate_col, gate_elem;
+    float softcap;
 };
 
 template <class T>
@@ -90,15 +92,22 @@ struct WaveAttn {
 
     // Scores of the page's keys (starting at key t0) against this wave's rows, mask, running
     // maximum and sum; leaves the probabilities in s.  This lane's row sees keys lo..hi.
-    // `per` (not 0): every score loses per for every position between the row (at position hi) and its key.
+    // `per` (not 0): every score loses per for every position between the row (at position hi) and its key; `cap` (not 0):
+    // the soft cap of the unscaled scores (soft_cap).
     __device__ __forceinline__ void scores(const v8 (&kf)[2 * KS], f32x16 (&s)[2], int t0, int lo, int hi,
-                                           float scale2, bool masked = true, float per = 0.f) {
+                                           float scale2, bool masked = true, float per = 0.f, float cap = 0.f, float cap_per = 0.f) {
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
 #pragma unroll
             for (int r = 0; r < 16; ++r) s[b][r] = 0.f;
 #pragma unroll
             for (int ks = 0; ks < KS; ++ks) s[b] = mfma32(kf[b * KS + ks], q[ks], s[b]);
+        }
+        if (cap != 0.f) {
+#pragma unroll
+            for (int b = 0; b < 2; ++b)
+#pragma unroll
+                for (int r = 0; r < 16; ++r) s[b][r] = soft_cap(s[b][r], cap, cap_per);
         }
         if (per != 0.f) {
             const int lane = threadIdx.x & 63;
@@ -306,6 +315,14 @@ struct PrefillWave {
             }
     }
 
+    // The soft cap of the unscaled scores.
+    __device__ __forceinline__ void cap(f32x16 (&n)[2], float c, float a) const {
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) n[b][r] = soft_cap(n[b][r], c, a);
+    }
+
     // The running maximum takes in a page's largest score mx; alpha is what the sums so far are
     // to be multiplied by before that page is added.
     __device__ __forceinline__ void take_max(float mx, float scale2) {
@@ -399,6 +416,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
     const int lo = live ? first_key(pos) : 0;
     // scores are kept unscaled until the exponential: the bias by distance in their units
     const float per = ex.slopes ? ex.slopes[h] / scale : 0.f;
+    const float cap = ex.softcap / scale, cap_per = ex.softcap > 0.f ? 2.f * LOG2E / ex.softcap * scale : 0.f;
     int lo_max = lo, hi_min = pos;
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) {
@@ -457,6 +475,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
         for (; p < own_lo - 1; ++p) step(p);
         step(p);                                                 // p = own_lo - 1: the first page's scores
         a.template scores<false>(kaddr(p + 1), sa, sa, pf, scale2);
+        if (cap != 0.f) a.cap(sa, cap, cap_per);
         if (per != 0.f) a.bias(sa, (p + 1) * PAGE, pos, per);
         if (is_masked(p + 1)) a.mask(sa, (p + 1) * PAGE, lo, pos);
         {
@@ -469,6 +488,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
         auto both = [&](f32x16 (&cur)[2], f32x16 (&nxt)[2]) {    // page p from cur, the scores of p+1 into nxt
             step(p);
             a.template scores<true>(kaddr(p + 1), nxt, cur, pf, scale2);
+            if (cap != 0.f) a.cap(nxt, cap, cap_per);
             if (per != 0.f) a.bias(nxt, (p + 1) * PAGE, pos, per);
             if (is_masked(p + 1)) a.mask(nxt, (p + 1) * PAGE, lo, pos);
             a.rescale();
@@ -504,7 +524,8 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
         inv = f / (a.total() * f + __builtin_amdgcn_exp2f(s2 - big));
     } else inv = 1.f / a.total();
     if (!live) return;
-    if (ex.gate) inv *= 1.f / (1.f + expf(-ex.gate[tok * ex.gate_stride + ex.gate_col + h]));
+    const float* grow = ex.gate ? ex.gate + tok * ex.gate_stride + ex.gate_col : nullptr;
+    if (grow && !ex.gate_elem) inv *= 1.f / (1.f + expf(-grow[h]));
     T* orow = out + (tok * H + h) * HD;
 #pragma unroll
     for (int b = 0; b < DB; ++b)
@@ -512,8 +533,13 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
         for (int g = 0; g < 4; ++g) {
             const int d = 32 * b + 8 * g + 4 * (lane >> 5);
             if (d < HD) {
-                typename Vec<T>::v4 v = {from_f32<T>(a.o[b][4 * g] * inv), from_f32<T>(a.o[b][4 * g + 1] * inv),
-                                         from_f32<T>(a.o[b][4 * g + 2] * inv), from_f32<T>(a.o[b][4 * g + 3] * inv)};
+                float f[4] = {inv, inv, inv, inv};
+                if (grow && ex.gate_elem) {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) f[i] *= 1.f / (1.f + expf(-grow[h * HD + d + i]));
+                }
+                typename Vec<T>::v4 v = {from_f32<T>(a.o[b][4 * g] * f[0]), from_f32<T>(a.o[b][4 * g + 1] * f[1]),
+                                         from_f32<T>(a.o[b][4 * g + 2] * f[2]), from_f32<T>(a.o[b][4 * g + 3] * f[3])};
                 *(typename Vec<T>::v4*)(orow + d) = v;
             }
         }
@@ -547,6 +573,7 @@ __global__ __launch_bounds__(64 * W) void attn_decode_kernel(
     int lo = window > 0 ? max(0, pos - window + 1) : 0;
     if (ex.block > 0) lo = max(lo, pos - pos % ex.block);
     const float bias_per = (ex.slopes && live) ? ex.slopes[h] / scale : 0.f;    // in the units of the unscaled scores
+    const float cap = ex.softcap / scale, cap_per = ex.softcap > 0.f ? 2.f * LOG2E / ex.softcap * scale : 0.f;
     const int p_first = lo / PAGE, p_end = pos / PAGE + 1;
     const int per = (p_end - p_first + S - 1) / S;
     const int p0 = p_first + split * per, p1 = min(p_end, p0 + per);
@@ -561,7 +588,8 @@ __global__ __launch_bounds__(64 * W) void attn_decode_kernel(
     if (p0 < p1) a.load_k(kbase + (int64_t)table[p0] * c.page_stride, kf);
     for (int p = p0; p < p1; ++p) {
         a.load_v(vbase + (int64_t)table[p] * c.page_stride, vf);
-        a.scores(kf, s, p * PAGE, lo, live ? pos : -1, scale2, p * PAGE < lo || p * PAGE + PAGE - 1 > pos, bias_per);
+        a.scores(kf, s, p * PAGE, lo, live ? pos : -1, scale2, p * PAGE < lo || p * PAGE + PAGE - 1 > pos, bias_per, cap,
+                 cap_per);
         if (p + 1 < p1) a.load_k(kbase + (int64_t)table[p + 1] * c.page_stride, kf);
         a.mix(vf, s);
     }
@@ -619,7 +647,8 @@ __global__ __launch_bounds__(64 * W) void attn_decode_kernel(
             const float f = (a.m == -INFINITY) ? 0.f : exp2f(a.m - big);
             inv = f / (total * f + exp2f(s2 - big));
         } else inv = 1.f / total;
-        if (ex.gate) inv *= 1.f / (1.f + expf(-ex.gate[(int64_t)b * ex.gate_stride + ex.gate_col + h]));
+        const float* grow = ex.gate ? ex.gate + (int64_t)b * ex.gate_stride + ex.gate_col : nullptr;
+        if (grow && !ex.gate_elem) inv *= 1.f / (1.f + expf(-grow[h]));
         T* orow = out + ((int64_t)b * H + h) * HD;
 #pragma unroll
         for (int blk = 0; blk < DB; ++blk)
@@ -628,7 +657,10 @@ __global__ __launch_bounds__(64 * W) void attn_decode_kernel(
                 const int d = 32 * blk + 8 * g + 4 * (lane >> 5);
                 if (d < HD) {
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) orow[d + i] = from_f32<T>(a.o[blk][4 * g + i] * inv);
+                    for (int i = 0; i < 4; ++i) {
+                        const float ge = grow && ex.gate_elem ? 1.f / (1.f + expf(-grow[h * HD + d + i])) : 1.f;
+                        orow[d + i] = from_f32<T>(a.o[blk][4 * g + i] * inv * ge);
+                    }
                 }
             }
         return;
@@ -665,12 +697,14 @@ __global__ void attn_merge_kernel(const float* __restrict__ part_o, const float*
     float L = block_sum(tid < S ? ml[2 * tid + 1] * w : 0.f, scratch);
     if (ex.sink) L += exp2f(s2 - M);
     float inv = 1.f / L;
-    if (ex.gate) inv *= 1.f / (1.f + expf(-ex.gate[(row / H) * ex.gate_stride + ex.gate_col + h]));
+    const float* grow = ex.gate ? ex.gate + (row / H) * ex.gate_stride + ex.gate_col : nullptr;
+    if (grow && !ex.gate_elem) inv *= 1.f / (1.f + expf(-grow[h]));
     if (tid < 64) wgt[tid] = w;
     __syncthreads();
     for (int d = tid; d < HD; d += blockDim.x) {
         float acc = 0.f;
         for (int s = 0; s < S; ++s) acc += part_o[(row * S + s) * HD + d] * wgt[s];
+        if (grow && ex.gate_elem) acc *= 1.f / (1.f + expf(-grow[h * HD + d]));
         out[row * HD + d] = from_f32<T>(acc * inv);
     }
 }
@@ -740,12 +774,15 @@ extern "C" int li_attn_prefill(const void* q, void* out, int dt, const void* k, 
                                const int* page_table, int max_pages, const int* tile_seq, const int* tile_q0,
                                int n_tiles, const int* seq_slot, const int* seq_qstart, const int* seq_qlen,
                                const int* seq_ctx, int H, int K, float scale, int window, int key_block, const float* sink,
-                               const float* slopes, const float* gate, int gate_stride, int gate_col, hipStream_t stream) {
+                               const float* slopes, const float* gate, int gate_stride, int gate_col, int gate_elem, float softcap,
+                               hipStream_t stream) {
     if (check_heads(H, K)) return LI_BAD_ARG;
-    if (key_block < 0 || !(scale > 0.f) || (gate && (gate_col < 0 || gate_col + H > gate_stride))) return LI_BAD_ARG;
+    if (key_block < 0 || !(scale > 0.f) || !(softcap >= 0.f) ||
+        (gate && (gate_col < 0 || gate_col + (gate_elem ? H * HD : H) > gate_stride)))
+        return LI_BAD_ARG;
     if (n_tiles <= 0) return LI_OK;
     CachePtrs c{k, v, page_stride, page_table, max_pages};
-    const AttnExtras ex{key_block, sink, slopes, gate, gate_stride, gate_col};
+    const AttnExtras ex{key_block, sink, slopes, gate, gate_stride, gate_col, gate_elem, softcap};
     const int G = H / K;
     const int gw = G % 4 == 0 ? 4 : (G % 2 == 0 ? 2 : 1);        // query heads of a KV head per workgroup
     dim3 grid(n_tiles * gw, K * (G / gw)), block(256);
@@ -799,10 +836,12 @@ extern "C" int li_attn_decode(const void* q, void* out, int dt, const void* k, c
                               const int* page_table, int max_pages, const int* seq_slot, const int* seq_ctx,
                               int n_seqs, int H, int K, float scale, int window, int splits, float* part_o,
                               float* part_ml, int key_block, const float* sink, const float* slopes, const float* gate,
-                              int gate_stride, int gate_col, hipStream_t stream) {
+                              int gate_stride, int gate_col, int gate_elem, float softcap, hipStream_t stream) {
     if (check_heads(H, K) || splits < 1 || splits > 64) return LI_BAD_ARG;
-    if (key_block < 0 || !(scale > 0.f) || (gate && (gate_col < 0 || gate_col + H > gate_stride))) return LI_BAD_ARG;
-    const AttnExtras ex{key_block, sink, slopes, gate, gate_stride, gate_col};
+    if (key_block < 0 || !(scale > 0.f) || !(softcap >= 0.f) ||
+        (gate && (gate_col < 0 || gate_col + (gate_elem ? H * HD : H) > gate_stride)))
+        return LI_BAD_ARG;
+    const AttnExtras ex{key_block, sink, slopes, gate, gate_stride, gate_col, gate_elem, softcap};
     const int w = waves_per_group(splits), parts = splits / w;
     if (parts > 64 || (parts > 1 && (!part_o || !part_ml))) return LI_BAD_ARG;
     if (dt != DT_F16 && dt != DT_BF16) return LI_BAD_ARG;

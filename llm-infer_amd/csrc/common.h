@@ -96,6 +96,12 @@ __device__ __forceinline__ float gate_activation(float g, bool gelu) {
     return g / (1.f + expf(-g));
 }
 
+// A score's soft cap, c tanh(x / c), with a = 2 log2(e) / c beside c: tanh z = 1 - 2 / (e^(2z) + 1) by the hardware's
+// 2^x and reciprocal (an error of some 1e-7 c; for large |x| the exponential becomes infinite or 0 and the result +-c).
+__device__ __forceinline__ float soft_cap(float x, float c, float a) {
+    return c - 2.f * c * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x * a) + 1.f);
+}
+
 // ---------------------------------------------------------------------------
 // Layout of a cache page.  A page holds PAGE (64) tokens of one layer for all
 // KV heads.  Keys and values are stored in the order in which a wave's lanes

@@ -13,7 +13,9 @@
 // divided by its root mean square over the value size and multiplied by out_scale.  `sink` not null: every map's sum
 // of weights also counts exp(sink[head]), a score with no key and no value that is not scaled.  `slopes` not null:
 // the score of the key at position j loses slopes[head] * (p - j), the sink nothing.  `gate` not null: a head's output
-// is multiplied by the sigmoid of gate[token][gate_col + head] (float32 rows of gate_stride numbers).
+// is multiplied by the sigmoid of gate[token][gate_col + head] (float32 rows of gate_stride numbers), with `gate_elem`
+// every element of it by the sigmoid of gate[token][gate_col + head * dv + element].  softcap c > 0: a scaled score s
+// becomes c tanh(s / c) before anything else.
 #include "common.h"
 
 #ifndef MAP_DIM
@@ -41,7 +43,7 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
     const int* __restrict__ tok_slot, const int* __restrict__ tile_t0, const int* __restrict__ tile_n, int H, int G,
     int dv, float scale, int block, int window, float lambda, float out_eps, float out_scale, int split,
     const float* __restrict__ sink, float* __restrict__ shares_out, const float* __restrict__ slopes,
-    const float* __restrict__ gate, int gate_stride, int gate_col) {
+    const float* __restrict__ gate, int gate_stride, int gate_col, int gate_elem, float softcap) {
     typedef typename Vec<T>::v8 v8;
     constexpr int D16 = MAP_DIM / 16, KW = MAPS * MAP_DIM, DVB = VALUE_DIM / 32;
     extern __shared__ float lds[];
@@ -145,6 +147,11 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
             }
             // scores in units of log 2, so that a weight is one hardware 2^x; 32 keys that every query of a whole tile
             // sees need no mask
+            if (softcap > 0.f) {
+                const float back = 1.f / scale, per = 2.f * 1.4426950408889634f / softcap * scale;
+#pragma unroll
+                for (int r = 0; r < 16; ++r) acc[r] = soft_cap(acc[r], softcap * back, per);
+            }
             float tmax = -INFINITY;
             if (whole_tile && kt * 32 >= lo_last && kt * 32 + 31 <= p0) {
                 if (slopes) {
@@ -294,8 +301,9 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
         }
     ss += __shfl_xor(ss, 32, WAVE);
     float rr = out_eps >= 0.f ? out_scale / sqrtf(ss / (float)dv + out_eps) : out_scale;
-    if (gate && has_query)             // one number a (token, head)
-        rr *= 1.f / (1.f + expf(-gate[(int64_t)(t0 + (HC ? 0 : col)) * gate_stride + gate_col + hq]));
+    const float* grow = gate ? gate + (int64_t)(t0 + (HC || !has_query ? 0 : col)) * gate_stride + gate_col : nullptr;
+    if (gate && !gate_elem && has_query)             // one number a (token, head)
+        rr *= 1.f / (1.f + expf(-grow[hq]));
     if (has_query) {
         T* orow = out + ((int64_t)(t0 + (HC ? 0 : col)) * H + hq) * dv;
 #pragma unroll
@@ -303,7 +311,7 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 const int dim = b * 32 + 8 * (r >> 2) + 4 * half + (r & 3);
-                if (dim < dv) orow[dim] = from_f32<T>(o[0][b][r] * rr);
+                if (dim < dv) orow[dim] = from_f32<T>(o[0][b][r] * rr * (gate_elem ? 1.f / (1.f + expf(-grow[hq * dv + dim])) : 1.f));
             }
     }
     }      // the item's tiles
@@ -316,7 +324,7 @@ template <class T, int MAPS>
 __global__ __launch_bounds__(64) void diff_attn_merge_kernel(const float* __restrict__ part, T* __restrict__ out, int H,
                                                              int S, int dv, float lambda, float out_eps, float out_scale,
                                                              const float* __restrict__ sink, const float* __restrict__ gate,
-                                                             int gate_stride, int gate_col) {
+                                                             int gate_stride, int gate_col, int gate_elem) {
     constexpr int W = 2 + VALUE_DIM, NV = (VALUE_DIM + 63) / 64;
     const int64_t unit = blockIdx.x;
     const int h = (int)(unit % H), lane = threadIdx.x;
@@ -353,9 +361,12 @@ __global__ __launch_bounds__(64) void diff_attn_merge_kernel(const float* __rest
     }
     ss = wave_sum(ss);
     float rr = out_eps >= 0.f ? out_scale / sqrtf(ss / (float)dv + out_eps) : out_scale;
-    if (gate) rr *= 1.f / (1.f + expf(-gate[(unit / H) * gate_stride + gate_col + h]));
+    const float* grow = gate ? gate + (unit / H) * gate_stride + gate_col : nullptr;
+    if (gate && !gate_elem) rr *= 1.f / (1.f + expf(-grow[h]));
 #pragma unroll
-    for (int v = 0; v < NV; ++v) if (v * 64 + lane < dv) out[unit * dv + v * 64 + lane] = from_f32<T>(res[v] * rr);
+    for (int v = 0; v < NV; ++v)
+        if (v * 64 + lane < dv)
+            out[unit * dv + v * 64 + lane] = from_f32<T>(res[v] * rr * (gate_elem ? 1.f / (1.f + expf(-grow[h * dv + v * 64 + lane])) : 1.f));
 }
 
 extern "C" int li_diffattn_map_dim() { return MAP_DIM; }
@@ -368,9 +379,12 @@ extern "C" int li_diffattn(const void* q, void* out, int dt, const void* k_pages
                            const int* page_table, int max_pages, const int* pos, const int* tok_slot, const int* tile_t0,
                            const int* tile_n, int n_tiles, int H, int G, int maps, int dv, float scale, int block, int window,
                            float lambda, float out_eps, float out_scale, const float* sink, int key_shares, float* part,
-                           const float* slopes, const float* gate, int gate_stride, int gate_col, hipStream_t stream) {
+                           const float* slopes, const float* gate, int gate_stride, int gate_col, int gate_elem, float softcap,
+                           hipStream_t stream) {
     if (n_tiles <= 0) return LI_OK;
-    if (gate && (gate_col < 0 || gate_col + H > gate_stride)) return LI_BAD_ARG;
+    if (gate && (gate_col < 0 || gate_col + (gate_elem ? H * dv : H) > gate_stride)) return LI_BAD_ARG;
+    if (!gate) gate_elem = 0;
+    if (softcap < 0.f || (softcap > 0.f && !(scale > 0.f))) return LI_BAD_ARG;
     if (H <= 0 || G <= 0 || H % G || dv <= 0 || dv > VALUE_DIM || block < 0 || window < 0) return LI_BAD_ARG;
     if (maps < 1 || maps > 2 || (dt != DT_F16 && dt != DT_BF16)) return LI_UNSUPPORTED;
     if ((tile_t0 == nullptr) != (tile_n == nullptr)) return LI_BAD_ARG;
@@ -395,10 +409,11 @@ extern "C" int li_diffattn(const void* q, void* out, int dt, const void* k_pages
             hipFuncSetAttribute((const void*)kfn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)              \
             return LI_HIP_ERROR;                                                                                                     \
         kfn<<<grid, threads, lds, stream>>>((const T*)q, (T*)out, pg, pos, tok_slot, tile_t0, tile_n, H, G, dv, scale, block, window, \
-                                            lambda, out_eps, out_scale, split, sink, part, slopes, gate, gate_stride, gate_col);     \
+                                            lambda, out_eps, out_scale, split, sink, part, slopes, gate, gate_stride, gate_col,      \
+                                            gate_elem, softcap);                                                                     \
         if (shares > 1)                                                                                                              \
             diff_attn_merge_kernel<T, M><<<n_tiles * H, 64, 0, stream>>>(part, (T*)out, H, shares, dv, lambda, out_eps, out_scale, sink, \
-                                                                      gate, gate_stride, gate_col);                                  \
+                                                                      gate, gate_stride, gate_col, gate_elem);                       \
     } while (0)
 #define GO(T, M) do { if (hc) GO1(T, M, false, true); else if (split) GO1(T, M, false, false); else GO1(T, M, true, false); } while (0)
     if (dt == DT_F16) { if (maps == 1) GO(f16, 1); else GO(f16, 2); }

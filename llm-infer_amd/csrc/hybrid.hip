@@ -73,7 +73,7 @@ extern "C" int li_concat_cast(const float* a, const float* b, void* out, int dt,
 }
 
 // ---------------------------------------------------------------------------
-// out = act(in), float32 in, type T out.  act: 0 gelu (erf), 1 gelu (tanh), 2 silu, 3 the square of relu.
+// out = act(in), float32 in, type T out.  act: 0 gelu (erf), 1 gelu (tanh), 2 silu, 3 the square of relu, 4 tanh.
 // ---------------------------------------------------------------------------
 template <class T>
 __global__ void activation_kernel(const float* __restrict__ in, T* __restrict__ out, int64_t n, int act) {
@@ -81,12 +81,12 @@ __global__ void activation_kernel(const float* __restrict__ in, T* __restrict__ 
     if (i >= n) return;
     const float z = in[i];
     const float r = fmaxf(z, 0.f);
-    out[i] = from_f32<T>(act == 0 ? gelu_erff_(z) : (act == 1 ? gate_activation(z, true) : (act == 2 ? siluf_(z) : r * r)));
+    out[i] = from_f32<T>(act == 0 ? gelu_erff_(z) : (act == 1 ? gate_activation(z, true) : (act == 2 ? siluf_(z) : (act == 3 ? r * r : tanhf(z)))));
 }
 
 extern "C" int li_activation(const float* in, void* out, int dt, int64_t n, int act, hipStream_t stream) {
     if (n <= 0) return LI_OK;
-    if (act < 0 || act > 3) return LI_BAD_ARG;
+    if (act < 0 || act > 4) return LI_BAD_ARG;
     DISPATCH_T(dt, (activation_kernel<T><<<(unsigned)((n + 255) / 256), 256, 0, stream>>>(in, (T*)out, n, act)));
     LI_CHECK_LAUNCH();
     return LI_OK;
@@ -167,7 +167,9 @@ extern "C" int li_qk_norm_store(const float* qkv, int stride, int col0, const fl
 // divided by its root mean square over dv and multiplied by out_scale.  `sink` not null: every map's sum of weights
 // also counts exp(sink[head]), a score with no key and no value that is not scaled.  `slopes` not null: the score of
 // the key at position j loses slopes[head] * (p - j) (the sink loses nothing).  `gate` not null: the head's output is
-// multiplied by the sigmoid of gate[t][gate_col + head] (float32 rows of gate_stride numbers).  Scores, weights, sums: float32.
+// multiplied by the sigmoid of gate[t][gate_col + head] (float32 rows of gate_stride numbers), with `gate_elem` every
+// element of it by the sigmoid of gate[t][gate_col + head * dv + element].  softcap c > 0: a scaled score s becomes
+// c tanh(s / c) before anything else.  Scores, weights, sums: float32.
 // The waves of the workgroup take the tiles of 64 keys in turn, a lane a key; each keeps a running maximum and
 // sum per map (online softmax) and its share of the output, and the shares are merged through LDS in wave order.
 // ---------------------------------------------------------------------------
@@ -179,7 +181,7 @@ __global__ __launch_bounds__(64 * DA_WAVES) void diff_attn_kernel(
     const T* __restrict__ q, T* __restrict__ out, MapPages pg, const int* __restrict__ pos,
     const int* __restrict__ tok_slot, int H, int G, int d, int dv, float scale, int block, int window, float lambda,
     float out_eps, float out_scale, const float* __restrict__ sink, const float* __restrict__ slopes,
-    const float* __restrict__ gate, int gate_stride, int gate_col) {
+    const float* __restrict__ gate, int gate_stride, int gate_col, int gate_elem, float softcap) {
     extern __shared__ float lds[];
     const int DP = round_up(d, 16), KW = MAPS * DP;
     float* sq = lds;                                   // [KW]
@@ -212,7 +214,9 @@ __global__ __launch_bounds__(64 * DA_WAVES) void diff_attn_kernel(
         for (int a = 0; a < MAPS; ++a) {
             float acc = 0.f;
             if (kh) for (int i = 0; i < d; ++i) acc += sq[a * DP + i] * to_f32(kh[k_offset(j % PAGE, a * DP + i, KW)]);
-            s[a] = kh ? acc * scale - slope * (float)(p - j) : -INFINITY;
+            float sc = acc * scale;
+            if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+            s[a] = kh ? sc - slope * (float)(p - j) : -INFINITY;
         }
         float pw[MAPS];
 #pragma unroll
@@ -285,12 +289,15 @@ __global__ __launch_bounds__(64 * DA_WAVES) void diff_attn_kernel(
     }
     float r = out_scale;
     if (out_eps >= 0.f) r = out_scale / sqrtf(block_sum(ss, scratch) / (float)dv + out_eps);   // waves 1.. add 0
-    if (gate) r *= sigmoidf_(gate[(int64_t)t * gate_stride + gate_col + h]);                   // one number a head
+    if (gate && !gate_elem) r *= sigmoidf_(gate[(int64_t)t * gate_stride + gate_col + h]);     // one number a head
     if (wave == 0) {
 #pragma unroll
         for (int c = 0; c < DA_MAXV; ++c) {
             const int i = lane + 64 * c;
-            if (i < dv) out[((int64_t)t * H + h) * dv + i] = from_f32<T>(res[c] * r);
+            if (i < dv) {
+                const float ge = gate && gate_elem ? sigmoidf_(gate[(int64_t)t * gate_stride + gate_col + h * dv + i]) : 1.f;
+                out[((int64_t)t * H + h) * dv + i] = from_f32<T>(res[c] * r * ge);
+            }
         }
     }
 }
@@ -299,10 +306,10 @@ extern "C" int li_diff_attn(const void* q, void* out, int dt, void* k_pages, voi
                             const int* page_table, int max_pages, const int* pos, const int* tok_slot, int n, int H, int G,
                             int maps, int d, int dv, float scale, int block, int window, float lambda, float out_eps,
                             float out_scale, const float* sink, const float* slopes, const float* gate, int gate_stride,
-                            int gate_col, hipStream_t stream) {
+                            int gate_col, int gate_elem, float softcap, hipStream_t stream) {
     if (n <= 0) return LI_OK;
-    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || block < 0 || window < 0) return LI_BAD_ARG;
-    if (gate && (gate_col < 0 || gate_col + H > gate_stride)) return LI_BAD_ARG;
+    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || block < 0 || window < 0 || softcap < 0.f) return LI_BAD_ARG;
+    if (gate && (gate_col < 0 || gate_col + (gate_elem ? H * dv : H) > gate_stride)) return LI_BAD_ARG;
     if (maps < 1 || maps > 2 || dv > 64 * DA_MAXV) return LI_UNSUPPORTED;
     MapPages pg{k_pages, v_pages, page_stride, page_table, max_pages};
     dim3 grid(n, H), blk(64 * DA_WAVES);
@@ -310,7 +317,7 @@ extern "C" int li_diff_attn(const void* q, void* out, int dt, void* k_pages, voi
     if (lds > 60000) return LI_UNSUPPORTED;
 #define GO(M) diff_attn_kernel<T, M><<<grid, blk, lds, stream>>>((const T*)q, (T*)out, pg, pos, tok_slot, H, G, d, dv, scale, \
                                                                  block, window, lambda, out_eps, out_scale, sink, slopes, gate, \
-                                                                 gate_stride, gate_col)
+                                                                 gate_stride, gate_col, gate_elem, softcap)
     DISPATCH_T(dt, { if (maps == 1) GO(1); else GO(2); });
 #undef GO
     LI_CHECK_LAUNCH();
@@ -367,12 +374,13 @@ __global__ void conv_history_kernel(const float* __restrict__ in, int stride, in
 
 extern "C" int li_conv_silu(const float* in, int stride, int col0, const float* w, const float* b, float* hist,
                             const int* pos, const int* tok_slot, const int* seq_slot, const int* seq_qstart,
-                            const int* seq_qlen, float* out, int n_tokens, int n_seqs, int channels, int taps,
+                            const int* seq_qlen, void* out, int dt, int n_tokens, int n_seqs, int channels, int taps,
                             hipStream_t stream) {
     if (n_tokens <= 0) return LI_OK;
     if (channels <= 0 || taps < 1 || taps > CONV_MAX_TAPS) return LI_BAD_ARG;
     dim3 cgrid(n_tokens, (channels + 255) / 256);
-    conv_silu_kernel<float, true, false><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, out, channels, taps);
+    DISPATCH_T(dt, (conv_silu_kernel<T, true, false><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, (T*)out,
+                                                                                channels, taps)));
     if (taps > 1) {
         dim3 grid(n_seqs, (channels + 255) / 256);
         conv_history_kernel<<<grid, 256, 0, stream>>>(in, stride, col0, hist, seq_slot, seq_qstart, seq_qlen, channels, taps);

@@ -610,12 +610,14 @@ extern "C" int li_mlstm_scan(const float* proj, int stride, int q_col, int k_col
 // ---------------------------------------------------------------------------
 // out[t][h][j] = y[t][h][j] / sqrt(mean over j of y[t][h]^2 + eps) * w[h * dv + j] * sigmoid(gate[t][h * dv + j]):
 // every head's part of a row divided by its own root mean square, then a weight over all heads and a gate
-// (float32 rows `gate_stride` apart; null: none).  One wave per (token, head).
+// (float32 rows `gate_stride` apart; null: none).  `w_shared`: w has dv numbers, the same for all heads; `gate_silu`: the
+// gate's silu instead of its sigmoid.  One wave per (token, head).
 // ---------------------------------------------------------------------------
 template <class T>
 __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __restrict__ y, const float* __restrict__ w,
                                                               const float* __restrict__ gate, int64_t gate_stride,
-                                                              T* __restrict__ out, int n_units, int H, int dv, float eps) {
+                                                              T* __restrict__ out, int n_units, int H, int dv, float eps,
+                                                              int w_shared, int gate_silu) {
     const int unit = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (unit >= n_units) return;
     const int t = unit / H, h = unit - t * H;
@@ -624,18 +626,22 @@ __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __res
     for (int i = lane; i < dv; i += 64) ss += yr[i] * yr[i];
     const float r = 1.f / sqrtf(wave_sum(ss) / (float)dv + eps);
     for (int i = lane; i < dv; i += 64) {
-        float v = yr[i] * r * (w ? w[h * dv + i] : 1.f);
-        if (gate) v *= lt_sigmoid(gate[(int64_t)t * gate_stride + h * dv + i]);
+        float v = yr[i] * r * (w ? w[w_shared ? i : h * dv + i] : 1.f);
+        if (gate) {
+            const float z = gate[(int64_t)t * gate_stride + h * dv + i];
+            v *= gate_silu ? z * lt_sigmoid(z) : lt_sigmoid(z);
+        }
         out[(int64_t)unit * dv + i] = from_f32<T>(v);
     }
 }
 
 extern "C" int li_gated_head_norm(const float* y, const float* w, const float* gate, int64_t gate_stride, void* out, int dt,
-                                  int n_rows, int H, int dv, float eps, hipStream_t stream) {
+                                  int n_rows, int H, int dv, float eps, int w_shared, int gate_silu, hipStream_t stream) {
     if (n_rows <= 0) return LI_OK;
     if (H <= 0 || dv <= 0) return LI_BAD_ARG;
     const int units = n_rows * H;
-    DISPATCH_T(dt, (gated_head_norm_kernel<T><<<(units + 3) / 4, 256, 0, stream>>>(y, w, gate, gate_stride, (T*)out, units, H, dv, eps)));
+    DISPATCH_T(dt, (gated_head_norm_kernel<T><<<(units + 3) / 4, 256, 0, stream>>>(y, w, gate, gate_stride, (T*)out, units, H, dv, eps,
+                                                                             w_shared, gate_silu)));
     LI_CHECK_LAUNCH();
     return LI_OK;
 }

@@ -1,5 +1,5 @@
-// Kernels of the mixers and arrangements beside the softmax decoder's: layer norm (alone, and fused with
-// the scaled residual sum of a post-norm layer), token shift with its per-sequence state, rotation in the
+// Kernels of the mixers and arrangements beside the softmax decoder's: layer norm (alone, fused with the scaled
+// residual sum of a post-norm layer, and on a sub-layer's output with the sum and the norm that comes next), token shift with its per-sequence state, rotation in the
 // half layout followed by a unit-RMS norm of q and k with the write into the paged cache, attention whose
 // weights are sigmoids of the scores, linear attention with a constant decay per head and a float32 state
 // per sequence, the gated RMS norm behind it, and the PolyNorm activation.  Every size is a run-time value.
@@ -19,11 +19,11 @@ __device__ __forceinline__ float sigmoidf(float z) { return 1.f / (1.f + expf(-z
 __device__ __forceinline__ float siluf(float z) { return z / (1.f + expf(-z)); }
 
 // ---------------------------------------------------------------------------
-// Layer norm with a weight and no bias: out = (x - mean) / sqrt(var + eps) * w, var the mean of the
+// Layer norm with a weight and a bias (null: none): out = (x - mean) / sqrt(var + eps) * w + b, var the mean of the
 // squared deviations.  `rows` (may be null) picks rows.
 // ---------------------------------------------------------------------------
 template <class TO>
-__global__ void layernorm_kernel(const float* __restrict__ x, const float* __restrict__ w,
+__global__ void layernorm_kernel(const float* __restrict__ x, const float* __restrict__ w, const float* __restrict__ b,
                                  const int* __restrict__ rows, TO* __restrict__ out, int d, float eps) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
@@ -35,17 +35,17 @@ __global__ void layernorm_kernel(const float* __restrict__ x, const float* __res
     float ss = 0.f;
     for (int i = threadIdx.x; i < d; i += blockDim.x) { const float v = xr[i] - mean; ss += v * v; }
     const float sd = sqrtf(block_sum(ss, scratch) / (float)d + eps);
-    for (int i = threadIdx.x; i < d; i += blockDim.x) o[i] = from_f32<TO>((xr[i] - mean) / sd * w[i]);
+    for (int i = threadIdx.x; i < d; i += blockDim.x) o[i] = from_f32<TO>((xr[i] - mean) / sd * w[i] + (b ? b[i] : 0.f));
 }
 
-extern "C" int li_layernorm(const float* x, const float* w, const int* rows, void* out, int out_dt, int n_rows,
+extern "C" int li_layernorm(const float* x, const float* w, const float* b, const int* rows, void* out, int out_dt, int n_rows,
                             int d, float eps, hipStream_t stream) {
     if (n_rows <= 0) return LI_OK;
     if (d <= 0) return LI_BAD_ARG;
     dim3 grid(n_rows), block(d >= 2048 ? 512 : (d >= 256 ? 256 : 64));
-    if (out_dt == DT_F32) layernorm_kernel<float><<<grid, block, 0, stream>>>(x, w, rows, (float*)out, d, eps);
-    else if (out_dt == DT_F16) layernorm_kernel<f16><<<grid, block, 0, stream>>>(x, w, rows, (f16*)out, d, eps);
-    else if (out_dt == DT_BF16) layernorm_kernel<bf16><<<grid, block, 0, stream>>>(x, w, rows, (bf16*)out, d, eps);
+    if (out_dt == DT_F32) layernorm_kernel<float><<<grid, block, 0, stream>>>(x, w, b, rows, (float*)out, d, eps);
+    else if (out_dt == DT_F16) layernorm_kernel<f16><<<grid, block, 0, stream>>>(x, w, b, rows, (f16*)out, d, eps);
+    else if (out_dt == DT_BF16) layernorm_kernel<bf16><<<grid, block, 0, stream>>>(x, w, b, rows, (bf16*)out, d, eps);
     else return LI_BAD_ARG;
     LI_CHECK_LAUNCH();
     return LI_OK;
@@ -229,6 +229,171 @@ extern "C" int li_add_layernorm(float* x, float alpha, const float* y1, float s1
     return LI_OK;
 }
 
+// ---------------------------------------------------------------------------
+// A sub-layer between two layer norms, everything behind its last product in one pass over the row:
+//   y <- a, or (a2 not null) y <- pair_scale (N(a) w1 + N(a2) w2),  N(v) = v / sqrt(mean(v^2) + pair_eps): two results
+//        side by side, each with an RMS norm of its own;
+//   x <- x + LN(y) w + b;   next <- LN(x) nw + nb in type TN (nw null: left out), the norm that reads the row next.
+// w null: y alone is wanted and goes to x (which is then only written).
+// One workgroup a row; the row stays in registers up to 4 * KEEP * THREADS elements (a multiple of 4), else it is read again.
+// ---------------------------------------------------------------------------
+struct LnAdd {
+    float* x;
+    const float* a;
+    const float* a2;
+    const float *w1, *w2;
+    float pair_eps, pair_scale;
+    const float *w, *b;
+    float eps;
+    const float *nw, *nb;
+    float next_eps;
+    void* next;
+};
+
+template <class TN, int THREADS, int KEEP>
+__global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int width) {
+    struct alignas(4 * sizeof(TN)) Out4 { TN v[4]; };
+    __shared__ float scratch[16];
+    const int64_t at = (int64_t)blockIdx.x * width;
+    const float *ar = p.a + at, *a2r = p.a2 ? p.a2 + at : nullptr;
+    float* xr = p.x + at;
+    TN* nr = (TN*)p.next + at;
+    const int tid = threadIdx.x;
+    const float inv_n = 1.f / (float)width;
+    if ((width & 3) == 0 && width <= 4 * KEEP * THREADS) {
+        const int quads = width >> 2;
+        f32x4 y[KEEP], xs[KEEP];
+        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+        float s0 = 0.f, s1 = 0.f;
+#pragma unroll
+        for (int c = 0; c < KEEP; ++c) {
+            const int i = tid + c * THREADS;
+            y[c] = xs[c] = zero;
+            if (i < quads) {
+                y[c] = *(const f32x4*)(ar + 4 * i);
+                if (p.w) xs[c] = *(const f32x4*)(xr + 4 * i);
+            }
+        }
+        if (a2r) {
+            f32x4 z[KEEP];
+#pragma unroll
+            for (int c = 0; c < KEEP; ++c) {
+                const int i = tid + c * THREADS;
+                z[c] = i < quads ? *(const f32x4*)(a2r + 4 * i) : zero;
+#pragma unroll
+                for (int k = 0; k < 4; ++k) { s0 += y[c][k] * y[c][k]; s1 += z[c][k] * z[c][k]; }
+            }
+            const float r1 = p.pair_scale / sqrtf(block_sum(s0, scratch) * inv_n + p.pair_eps);
+            const float r2 = p.pair_scale / sqrtf(block_sum(s1, scratch) * inv_n + p.pair_eps);
+#pragma unroll
+            for (int c = 0; c < KEEP; ++c) {
+                const int i = tid + c * THREADS;
+                if (i < quads) {
+                    const f32x4 u1 = *(const f32x4*)(p.w1 + 4 * i), u2 = *(const f32x4*)(p.w2 + 4 * i);
+#pragma unroll
+                    for (int k = 0; k < 4; ++k) y[c][k] = y[c][k] * r1 * u1[k] + z[c][k] * r2 * u2[k];
+                }
+            }
+        }
+        if (!p.w) {
+#pragma unroll
+            for (int c = 0; c < KEEP; ++c) { const int i = tid + c * THREADS; if (i < quads) *(f32x4*)(xr + 4 * i) = y[c]; }
+            return;
+        }
+        // (what lies beyond the row is zero and stays out of the sums of squared deviations)
+        auto normed = [&](f32x4 (&v)[KEEP], float eps) {
+            float s = 0.f;
+#pragma unroll
+            for (int c = 0; c < KEEP; ++c) s += (v[c][0] + v[c][1]) + (v[c][2] + v[c][3]);
+            const float mean = block_sum(s, scratch) * inv_n;
+            s = 0.f;
+#pragma unroll
+            for (int c = 0; c < KEEP; ++c) {
+                if (tid + c * THREADS < quads) {
+#pragma unroll
+                    for (int k = 0; k < 4; ++k) { v[c][k] -= mean; s += v[c][k] * v[c][k]; }
+                }
+            }
+            return 1.f / sqrtf(block_sum(s, scratch) * inv_n + eps);
+        };
+        const float r = normed(y, p.eps);
+#pragma unroll
+        for (int c = 0; c < KEEP; ++c) {
+            const int i = tid + c * THREADS;
+            if (i < quads) {
+                const f32x4 w = *(const f32x4*)(p.w + 4 * i), b = p.b ? *(const f32x4*)(p.b + 4 * i) : zero;
+#pragma unroll
+                for (int k = 0; k < 4; ++k) xs[c][k] += y[c][k] * r * w[k] + b[k];
+                *(f32x4*)(xr + 4 * i) = xs[c];
+            }
+        }
+        if (!p.nw) return;
+        const float rn = normed(xs, p.next_eps);
+#pragma unroll
+        for (int c = 0; c < KEEP; ++c) {
+            const int i = tid + c * THREADS;
+            if (i < quads) {
+                const f32x4 w = *(const f32x4*)(p.nw + 4 * i), b = p.nb ? *(const f32x4*)(p.nb + 4 * i) : zero;
+                Out4 o;
+#pragma unroll
+                for (int k = 0; k < 4; ++k) o.v[k] = from_f32<TN>(xs[c][k] * rn * w[k] + b[k]);
+                *(Out4*)(nr + 4 * i) = o;
+            }
+        }
+        return;
+    }
+    float r1 = 1.f, r2 = 0.f;
+    if (a2r) {
+        float s0 = 0.f, s1 = 0.f;
+        for (int i = tid; i < width; i += THREADS) { s0 += ar[i] * ar[i]; s1 += a2r[i] * a2r[i]; }
+        r1 = p.pair_scale / sqrtf(block_sum(s0, scratch) * inv_n + p.pair_eps);
+        r2 = p.pair_scale / sqrtf(block_sum(s1, scratch) * inv_n + p.pair_eps);
+    }
+    auto y = [&](int i) { return a2r ? ar[i] * r1 * p.w1[i] + a2r[i] * r2 * p.w2[i] : ar[i]; };
+    if (!p.w) {
+        for (int i = tid; i < width; i += THREADS) xr[i] = y(i);
+        return;
+    }
+    float s = 0.f;
+    for (int i = tid; i < width; i += THREADS) s += y(i);
+    float mean = block_sum(s, scratch) * inv_n;
+    s = 0.f;
+    for (int i = tid; i < width; i += THREADS) { const float v = y(i) - mean; s += v * v; }
+    float r = 1.f / sqrtf(block_sum(s, scratch) * inv_n + p.eps);
+    s = 0.f;
+    for (int i = tid; i < width; i += THREADS) {
+        const float v = xr[i] + (y(i) - mean) * r * p.w[i] + (p.b ? p.b[i] : 0.f);
+        xr[i] = v;                                     // read back by the same thread below
+        s += v;
+    }
+    if (!p.nw) return;
+    mean = block_sum(s, scratch) * inv_n;
+    s = 0.f;
+    for (int i = tid; i < width; i += THREADS) { const float v = xr[i] - mean; s += v * v; }
+    r = 1.f / sqrtf(block_sum(s, scratch) * inv_n + p.next_eps);
+    for (int i = tid; i < width; i += THREADS) nr[i] = from_f32<TN>((xr[i] - mean) * r * p.nw[i] + (p.nb ? p.nb[i] : 0.f));
+}
+
+extern "C" int li_layernorm_add(float* x, const float* a, const float* a2, const float* w1, const float* w2, float pair_eps,
+                                float pair_scale, const float* w, const float* b, float eps, const float* nw, const float* nb,
+                                float next_eps, void* next, int next_dt, int n_rows, int width, hipStream_t stream) {
+    if (n_rows <= 0) return LI_OK;
+    if (width <= 0 || !x || !a || (a2 && (!w1 || !w2)) || (nw && (!next || !w))) return LI_BAD_ARG;
+    if ((uintptr_t)x % 16 || (uintptr_t)a % 16 || (uintptr_t)a2 % 16 || (uintptr_t)w1 % 16 || (uintptr_t)w2 % 16 || (uintptr_t)w % 16 ||
+        (uintptr_t)b % 16 || (uintptr_t)nw % 16 || (uintptr_t)nb % 16 || (uintptr_t)next % 16)
+        return LI_BAD_ARG;
+    if (!nw) next_dt = DT_F32;
+    const LnAdd p{x, a, a2, w1, w2, pair_eps, pair_scale, w, b, eps, nw, nb, next_eps, next};
+    // few rows (a decode step): as many threads a row as there are pieces of four, so that a row waits for memory once
+#define GO1(TN, TH, K) layernorm_add_kernel<TN, TH, K><<<n_rows, TH, 0, stream>>>(p, width)
+#define GO(TN) do { if (width <= 1024) GO1(TN, 256, 1); else if (n_rows <= 256 || width > 8192) GO1(TN, 1024, 4); else GO1(TN, 256, 8); } while (0)
+    if (next_dt == DT_F32) GO(float); else if (next_dt == DT_F16) GO(f16); else if (next_dt == DT_BF16) GO(bf16); else return LI_BAD_ARG;
+#undef GO
+#undef GO1
+    LI_CHECK_LAUNCH();
+    return LI_OK;
+}
+
 // out = y1 * s1 (+ y2 * s2) added into x: the same sum for an arrangement without the norm behind it.
 __global__ void add_scaled_kernel(float* __restrict__ x, const float* __restrict__ y1, float s1,
                                   const float* __restrict__ y2, float s2, int64_t n) {
@@ -264,19 +429,40 @@ extern "C" int li_cast(const float* x, void* out, int out_dt, int64_t n, hipStre
     return LI_OK;
 }
 
+// out[t][i] = rows[t][col0 + i] in another type: some columns of float32 rows as rows of their own.
+template <class TO>
+__global__ void cast_columns_kernel(const float* __restrict__ rows, int stride, int col0, TO* __restrict__ out, int64_t total, int n) {
+    const int64_t e = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (e < total) out[e] = from_f32<TO>(rows[e / n * stride + col0 + e % n]);
+}
+
+extern "C" int li_cast_columns(const float* rows, int stride, int col0, void* out, int out_dt, int n_rows, int n, hipStream_t stream) {
+    if (n_rows <= 0 || n <= 0) return LI_OK;
+    if (col0 < 0 || col0 + n > stride) return LI_BAD_ARG;
+    const int64_t total = (int64_t)n_rows * n;
+    dim3 grid((unsigned)((total + 255) / 256)), block(256);
+    if (out_dt == DT_F32) cast_columns_kernel<float><<<grid, block, 0, stream>>>(rows, stride, col0, (float*)out, total, n);
+    else if (out_dt == DT_F16) cast_columns_kernel<f16><<<grid, block, 0, stream>>>(rows, stride, col0, (f16*)out, total, n);
+    else if (out_dt == DT_BF16) cast_columns_kernel<bf16><<<grid, block, 0, stream>>>(rows, stride, col0, (bf16*)out, total, n);
+    else return LI_BAD_ARG;
+    LI_CHECK_LAUNCH();
+    return LI_OK;
+}
+
 // ---------------------------------------------------------------------------
 // Token shift: out_t = x_t + (x_{t-1} - x_t) * mu, channel by channel, where x_{t-1} is the row of the
 // token before in the same sequence: the row above in this step, or, for the first token that a sequence
 // brings to this step, the row that the step before left in `state[slot]`; zeros at position 0.  A second
 // kernel then leaves each sequence's last row of this step in its state.  The rows of one sequence are
-// consecutive and no two sequences share a slot, so a change of tok_slot marks a sequence's edge.
+// consecutive and no two sequences share a slot, so a change of tok_slot marks a sequence's edge.  `n_mix` mixing
+// vectors, mu [n_mix, d], give as many results of the same two rows, out [n_mix, T, d].
 // ---------------------------------------------------------------------------
 // `single`: every sequence brings one row (decoding), so each row is its sequence's first and last; the thread
 // that has read an element of the state then writes the row's own element there, and no second kernel runs.
 template <class TO>
 __global__ void token_shift_kernel(const float* __restrict__ x, const float* __restrict__ mu,
                                    float* __restrict__ state, const int* __restrict__ pos,
-                                   const int* __restrict__ tok_slot, TO* __restrict__ out, int d, int single) {
+                                   const int* __restrict__ tok_slot, TO* __restrict__ out, int d, int single, int n_mix) {
     const int t = blockIdx.x;
     const int slot = tok_slot[t];
     const bool first = single || t == 0 || tok_slot[t - 1] != slot;
@@ -284,9 +470,10 @@ __global__ void token_shift_kernel(const float* __restrict__ x, const float* __r
     const float* prev = pos[t] == 0 ? nullptr : (first ? st : x + (int64_t)(t - 1) * d);
     const float* xr = x + (int64_t)t * d;
     TO* o = out + (int64_t)t * d;
+    const int64_t apart = (int64_t)gridDim.x * d;
     for (int i = threadIdx.x; i < d; i += blockDim.x) {
         const float h = xr[i], p = prev ? prev[i] : 0.f;
-        o[i] = from_f32<TO>(h + (p - h) * mu[i]);
+        for (int m = 0; m < n_mix; ++m) o[m * apart + i] = from_f32<TO>(h + (p - h) * mu[(int64_t)m * d + i]);
         if (single) st[i] = h;
     }
 }
@@ -302,15 +489,15 @@ __global__ void token_shift_save_kernel(const float* __restrict__ x, float* __re
 }
 
 extern "C" int li_token_shift(const float* x, const float* mu, float* state, const int* pos, const int* tok_slot,
-                              void* out, int out_dt, int n_tokens, int d, int single, hipStream_t stream) {
+                              void* out, int out_dt, int n_tokens, int d, int single, int n_mix, hipStream_t stream) {
     if (n_tokens <= 0) return LI_OK;
-    if (d <= 0) return LI_BAD_ARG;
+    if (d <= 0 || n_mix < 1) return LI_BAD_ARG;
     // a few rows (a decode step): as many threads a row as it has elements to four, so that a thread's loads are few
     const int wide = min(1024, (d / 4 + 63) / 64 * 64);
     dim3 grid(n_tokens), block(n_tokens < 256 && wide > 64 ? wide : (d >= 1024 ? 256 : 64));
-    if (out_dt == DT_F32) token_shift_kernel<float><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (float*)out, d, single);
-    else if (out_dt == DT_F16) token_shift_kernel<f16><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (f16*)out, d, single);
-    else if (out_dt == DT_BF16) token_shift_kernel<bf16><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (bf16*)out, d, single);
+    if (out_dt == DT_F32) token_shift_kernel<float><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (float*)out, d, single, n_mix);
+    else if (out_dt == DT_F16) token_shift_kernel<f16><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (f16*)out, d, single, n_mix);
+    else if (out_dt == DT_BF16) token_shift_kernel<bf16><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (bf16*)out, d, single, n_mix);
     else return LI_BAD_ARG;
     LI_CHECK_LAUNCH();
     if (single) return LI_OK;

@@ -204,6 +204,15 @@ def hybrid_library(force=False):
     return _load("libli_hybrid.so", HYBRID_SOURCES, (), force)
 
 
+RECURRENT_SOURCES = ("recurrent.hip",)
+
+
+def recurrent_library(force=False):
+    """The recurrent mixers' kernels (csrc/recurrent.hip: the gated delta rule, the selective scan with a decay for every
+    channel and state, time mixing with a decay for every key channel): a library of its own, as the mixers' is."""
+    return _load("libli_recurrent.so", RECURRENT_SOURCES, (), force)
+
+
 DIFF_ATTN_SOURCE = "diff_attention.hip"
 
 
@@ -245,6 +254,7 @@ def build_all(head_dims=(16, 32, 48, 64, 128), force=True, sigmoid_head_dims=((4
     core_library(force=force)
     mixers_library(force=force)
     hybrid_library(force=force)
+    recurrent_library(force=force)
     with ThreadPoolExecutor(max_workers=4) as pool:
         list(pool.map(lambda p: _build_library(*_sigmoid_attention_args(*p), force), sigmoid_head_dims))
         list(pool.map(lambda p: _build_library(*_diff_attention_args(*p), force), diff_head_dims))

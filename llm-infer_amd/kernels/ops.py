@@ -177,6 +177,10 @@ def prepared_rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype):
     return normed
 
 
+# (the weight tensor says which norm it is: a layer norm that a pass has taken along is found in the same way)
+prepared_norm = prepared_rmsnorm
+
+
 def lazy_rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype):
     """A ``LazyNorm`` of ``x`` if the product that last added into ``x`` prepared this very norm (same
     weight tensor, same 16-bit type) and nothing has written to ``x`` since (torch counts its own
@@ -681,19 +685,22 @@ def prefill_meta(ctx) -> dict:
 
 
 def attention_prefill(q, kv, meta, n_heads, n_kv_heads, head_dim, scale, window, block=None, sink=None, slopes=None,
-                      gate=None, gate_col: int = 0) -> torch.Tensor:
+                      gate=None, gate_col: int = 0, softcap: float | None = None, gate_elem: bool = False) -> torch.Tensor:
     """16-bit attention for a step with whole prompts.  ``kv``: (k_pages, v_pages, page_stride,
     page_table); ``meta``: dict of int32 device arrays tile_seq, tile_q0, seq_slot, seq_qstart,
     seq_qlen, seq_ctx and the int n_tiles.  ``block`` b: a token at position p reads no key before p - p % b;
     ``sink`` (float32 [H]): every head's sum of weights also counts exp(sink[h]); ``slopes`` (float32 [H]): the
     score of the key at position j loses slopes[h] * (p - j); ``gate`` (float32 rows [T, >= gate_col + H]): head
-    h's output is multiplied by sigmoid(gate[t][gate_col + h])."""
+    h's output is multiplied by sigmoid(gate[t][gate_col + h]), with ``gate_elem`` its element d by
+    sigmoid(gate[t][gate_col + h * hd + d]); ``softcap`` c: a scaled score s becomes c tanh(s / c) before anything else."""
     k_pages, v_pages, page_stride, page_table = kv
     _dev(q, k_pages, v_pages, page_table, sink, slopes, gate)
     for name, vec in (("sink", sink), ("slopes", slopes)):
         _need(vec is None or (vec.dtype == torch.float32 and vec.numel() == n_heads and vec.is_contiguous()), f"{name}: float32 [H]")
     _need(gate is None or (gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == q.shape[0] and gate.stride(1) == 1
-                           and 0 <= gate_col and gate_col + n_heads <= gate.shape[1]), "gate: float32 rows with a column for every head")
+                           and 0 <= gate_col and gate_col + n_heads * (head_dim if gate_elem else 1) <= gate.shape[1]),
+          "gate: float32 rows with a column for every head (or every element of every head)")
+    _need(softcap is None or softcap > 0, "softcap: positive")
     _need(q.dtype in (torch.float16, torch.bfloat16) and q.shape[1:] == (n_heads, head_dim), "q: 16-bit [T, H, hd]")
     _check_pages(k_pages, v_pages, page_table, n_kv_heads, head_dim, q.dtype)
     out = torch.empty_like(q)
@@ -702,20 +709,23 @@ def attention_prefill(q, kv, meta, n_heads, n_kv_heads, head_dim, scale, window,
         page_table.shape[1], _ptr(meta["tile_seq"]), _ptr(meta["tile_q0"]), meta["n_tiles"], _ptr(meta["seq_slot"]),
         _ptr(meta["seq_qstart"]), _ptr(meta["seq_qlen"]), _ptr(meta["seq_ctx"]), n_heads, n_kv_heads,
         c_float(scale), int(window or 0), int(block or 0), _ptr(sink), _ptr(slopes), _ptr(gate),
-        gate.stride(0) if gate is not None else 0, int(gate_col), _stream()), "attn_prefill")
+        gate.stride(0) if gate is not None else 0, int(gate_col), int(bool(gate_elem and gate is not None)),
+        c_float(softcap or 0.0), _stream()), "attn_prefill")
     return out
 
 
 def attention_decode(q, kv, seq_slot, seq_ctx, n_seqs, n_heads, n_kv_heads, head_dim, scale, window,
-                     splits: int = 1, block=None, sink=None, slopes=None, gate=None, gate_col: int = 0) -> torch.Tensor:
-    """16-bit attention for one new token per sequence; q [B, H, hd].  ``block``, ``sink``, ``slopes``, ``gate``: as
-    for ``attention_prefill``."""
+                     splits: int = 1, block=None, sink=None, slopes=None, gate=None, gate_col: int = 0, softcap: float | None = None, gate_elem: bool = False) -> torch.Tensor:
+    """16-bit attention for one new token per sequence; q [B, H, hd].  ``block``, ``sink``, ``slopes``, ``gate``,
+    ``gate_elem``, ``softcap``: as for ``attention_prefill``."""
     k_pages, v_pages, page_stride, page_table = kv
     _dev(q, k_pages, v_pages, page_table, seq_slot, seq_ctx, sink, slopes, gate)
     for name, vec in (("sink", sink), ("slopes", slopes)):
         _need(vec is None or (vec.dtype == torch.float32 and vec.numel() == n_heads and vec.is_contiguous()), f"{name}: float32 [H]")
     _need(gate is None or (gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] >= n_seqs and gate.stride(1) == 1
-                           and 0 <= gate_col and gate_col + n_heads <= gate.shape[1]), "gate: float32 rows with a column for every head")
+                           and 0 <= gate_col and gate_col + n_heads * (head_dim if gate_elem else 1) <= gate.shape[1]),
+          "gate: float32 rows with a column for every head (or every element of every head)")
+    _need(softcap is None or softcap > 0, "softcap: positive")
     _need(q.dtype in (torch.float16, torch.bfloat16) and q.shape == (n_seqs, n_heads, head_dim), "q: 16-bit [B, H, hd]")
     _check_pages(k_pages, v_pages, page_table, n_kv_heads, head_dim, q.dtype)
     _need(seq_slot.numel() >= n_seqs and seq_ctx.numel() >= n_seqs, "per-sequence arrays too short")
@@ -732,7 +742,8 @@ def attention_decode(q, kv, seq_slot, seq_ctx, n_seqs, n_heads, n_kv_heads, head
         _ptr(q), _ptr(out), DT[q.dtype], _ptr(k_pages), _ptr(v_pages), c_int64(page_stride), _ptr(page_table),
         page_table.shape[1], _ptr(seq_slot), _ptr(seq_ctx), n_seqs, n_heads, n_kv_heads, c_float(scale),
         int(window or 0), splits, _ptr(part_o), _ptr(part_ml), int(block or 0), _ptr(sink), _ptr(slopes), _ptr(gate),
-        gate.stride(0) if gate is not None else 0, int(gate_col), _stream()), "attn_decode")
+        gate.stride(0) if gate is not None else 0, int(gate_col), int(bool(gate_elem and gate is not None)),
+        c_float(softcap or 0.0), _stream()), "attn_decode")
     return out
 
 
@@ -861,16 +872,17 @@ def _f32_rows(x, what):
     _need(x.dtype == torch.float32 and x.dim() == 2, f"{what}: float32 [T, n]")
 
 
-def layernorm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype, rows: torch.Tensor | None = None) -> torch.Tensor:
-    """out[r] = (x[rows[r]] - mean) / sqrt(var + eps) * w, float32 inside; no bias."""
-    _dev(x, w, rows)
+def layernorm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype, rows: torch.Tensor | None = None, bias=None) -> torch.Tensor:
+    """out[r] = (x[rows[r]] - mean) / sqrt(var + eps) * w (+ bias), float32 inside."""
+    _dev(x, w, rows, bias)
+    _need(bias is None or (bias.dtype == torch.float32 and bias.shape == w.shape), "norm bias: float32 [d]")
     _f32_rows(x, "layernorm x")
     _need(w.dtype == torch.float32 and w.shape == (x.shape[1],), "norm weight: float32 [d]")
     if rows is not None:
         _need(rows.dtype == torch.int32, "rows: int32")
     n = x.shape[0] if rows is None else rows.numel()
     out = torch.empty((n, x.shape[1]), dtype=out_dtype, device=x.device)
-    _check(mixers().li_layernorm(_ptr(x), _ptr(w), _ptr(rows), _ptr(out), DT[out_dtype], n, x.shape[1], c_float(eps),
+    _check(mixers().li_layernorm(_ptr(x), _ptr(w), _ptr(bias), _ptr(rows), _ptr(out), DT[out_dtype], n, x.shape[1], c_float(eps),
                                  _stream()), "layernorm")
     return out
 
@@ -896,6 +908,55 @@ def add_layernorm(x, alpha: float, addends, w, eps: float, copy_dtype=None):
     return copy
 
 
+class NormedPair:
+    """Two results side by side, each with an RMS norm of its own: scale * (N(a) w1 + N(b) w2), N(v) = v / sqrt(mean(v^2) +
+    eps), for float32 rows a, b and float32 weights; ``rows()`` makes the sum, ``layernorm_add`` takes it as it is."""
+
+    def __init__(self, a, w1, b, w2, eps: float, scale: float):
+        self.a, self.w1, self.b, self.w2, self.eps, self.scale = a, w1, b, w2, float(eps), float(scale)
+        self.shape, self.device = a.shape, a.device
+
+    def rows(self) -> torch.Tensor:
+        out = torch.empty_like(self.a)
+        _layernorm_add(out, self, None, None, 0.0, None, None, 0.0, None)
+        return out
+
+
+def _layernorm_add(x, y, w, b, eps, nw, nb, n_eps, normed):
+    pair = y if isinstance(y, NormedPair) else None
+    a = pair.a if pair else y
+    width = a.shape[1]
+    _dev(x, a, w, b, nw, nb)
+    _f32_rows(a, "layernorm_add y")
+    _need(x.dtype == torch.float32 and x.shape == a.shape, "layernorm_add: float32 rows of one shape")
+    for v in (w, b, nw, nb) + ((pair.w1, pair.w2) if pair else ()):
+        _need(v is None or (v.dtype == torch.float32 and v.shape == (width,) and v.is_cuda and v.is_contiguous()), "layernorm_add: float32 [width] vectors")
+    if pair:
+        _dev(pair.b)
+        _need(pair.b.dtype == torch.float32 and pair.b.shape == a.shape, "layernorm_add: two results of one shape")
+    _check(mixers().li_layernorm_add(
+        _ptr(x), _ptr(a), _ptr(pair.b if pair else None), _ptr(pair.w1 if pair else None), _ptr(pair.w2 if pair else None),
+        c_float(pair.eps if pair else 0.0), c_float(pair.scale if pair else 1.0), _ptr(w), _ptr(b), c_float(eps), _ptr(nw),
+        _ptr(nb), c_float(n_eps), _ptr(normed), DT[normed.dtype] if normed is not None else 0, a.shape[0], width, _stream()),
+        "layernorm_add")
+
+
+def layernorm_add(x, y, weight, bias, eps: float, next_norm=None) -> torch.Tensor:
+    """x += LN(y) * weight + bias, row by row, in place on the float32 rows of ``x``; ``y``: float32 rows or a
+    ``NormedPair``.  ``next_norm`` (weight, bias or None, eps, dtype): the layer norm that reads the finished rows next is
+    taken in the same pass and left for it (``prepared_norm`` finds it as long as nothing else writes into ``x``)."""
+    _drop_row_stats(x)
+    nw = nb = normed = None
+    n_eps = 0.0
+    if next_norm is not None:
+        nw, nb, n_eps, n_dt = next_norm
+        normed = torch.empty(x.shape, dtype=n_dt, device=x.device)
+    _layernorm_add(x, y, weight, bias, eps, nw, nb, n_eps, normed)
+    if normed is not None:
+        x._li_normed = (normed, nw, float(n_eps), x._version)
+    return x
+
+
 def add_scaled(x, addends) -> None:
     """x += sum of scale_i * y_i (one or two addends, float32 of x's shape)."""
     _need(1 <= len(addends) <= 2, "add_scaled: one or two addends")
@@ -919,20 +980,31 @@ def cast(x: torch.Tensor, dtype) -> torch.Tensor:
     return out
 
 
+def cast_columns(rows, col0: int, n: int, dtype) -> torch.Tensor:
+    """Columns col0 .. col0 + n of float32 rows as rows of their own in ``dtype``."""
+    _dev(rows)
+    _f32_rows(rows, "cast_columns rows")
+    _need(dtype in DT and n >= 1 and 0 <= col0 and col0 + n <= rows.shape[1], "cast_columns: columns within the rows")
+    out = torch.empty((rows.shape[0], n), dtype=dtype, device=rows.device)
+    _check(mixers().li_cast_columns(_ptr(rows), rows.shape[1], col0, _ptr(out), DT[dtype], rows.shape[0], n, _stream()), "cast_columns")
+    return out
+
+
 def token_shift(x, mu, state, pos, tok_slot, out_dtype, single: bool = False) -> torch.Tensor:
     """out_t = x_t + (x_{t-1} - x_t) * mu with the row before from this step or from ``state[slot]`` (zeros at
     position 0); afterwards ``state[slot]`` holds each sequence's last row of this step.  ``single``: every
-    sequence brings exactly one row (a decode step), which one kernel then serves."""
+    sequence brings exactly one row (a decode step), which one kernel then serves.  ``mu`` [n, d]: n results of the same
+    two rows, one for each mixing vector, returned as [n, T, d]."""
     _dev(x, mu, state, pos, tok_slot)
     _f32_rows(x, "token_shift x")
     t, d = x.shape
-    _need(mu.dtype == torch.float32 and mu.shape == (d,), "token_shift: float32 [d] mixing weights")
+    _need(mu.dtype == torch.float32 and mu.dim() in (1, 2) and mu.shape[-1] == d, "token_shift: float32 [d] or [n, d] mixing weights")
     _need(state.dtype == torch.float32 and state.dim() == 2 and state.shape[1] == d, "token_shift: state float32 [slots, d]")
     _need(pos.dtype == torch.int32 and tok_slot.dtype == torch.int32 and pos.numel() >= t and tok_slot.numel() >= t,
           "token_shift: int32 positions and slots for every token")
-    out = torch.empty((t, d), dtype=out_dtype, device=x.device)
+    out = torch.empty(tuple(mu.shape[:-1]) + (t, d), dtype=out_dtype, device=x.device)
     _check(mixers().li_token_shift(_ptr(x), _ptr(mu), _ptr(state), _ptr(pos), _ptr(tok_slot), _ptr(out), DT[out_dtype],
-                                   t, d, int(bool(single)), _stream()), "token_shift")
+                                   t, d, int(bool(single)), mu.shape[0] if mu.dim() == 2 else 1, _stream()), "token_shift")
     return out
 
 
@@ -1152,7 +1224,7 @@ def polynorm(z, coef, eps, out_dtype) -> torch.Tensor:
 # routed experts, a scaled embedding with sinusoidal positions
 # ---------------------------------------------------------------------------
 _hybrid = None
-ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu2": 3}
+ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu2": 3, "tanh": 4}      # (tanh: not an expert's)
 
 
 def hybrid():
@@ -1192,7 +1264,7 @@ def concat_cast(a, b, dtype) -> torch.Tensor:
 
 
 def activation(z, kind: str, out_dtype) -> torch.Tensor:
-    """act(z) for float32 z in ``out_dtype``; kind: gelu (erf), gelu_tanh, silu, relu2 (the square of relu)."""
+    """act(z) for float32 z in ``out_dtype``; kind: gelu (erf), gelu_tanh, silu, relu2 (the square of relu), tanh."""
     _dev(z)
     _need(z.dtype == torch.float32 and kind in ACTIVATIONS and out_dtype in DT, f"activation {kind!r}: float32 in, one of {', '.join(ACTIVATIONS)}")
     out = torch.empty(z.shape, dtype=out_dtype, device=z.device)
@@ -1292,7 +1364,8 @@ def diff_tiles(ctx, block=None, window=None):
 
 
 def diff_attention(q, kv, pos, tok_slot, n_heads, n_kv_heads, maps, d, dv, scale, block, window, lam, out_eps, out_scale,
-                   out_dtype, tiles=None, sink=None, key_shares: int = 1, slopes=None, gate=None, gate_col: int = 0) -> torch.Tensor:
+                   out_dtype, tiles=None, sink=None, key_shares: int = 1, slopes=None, gate=None, gate_col: int = 0,
+                   softcap: float | None = None, gate_elem: bool = False) -> torch.Tensor:
     """Attention of ``maps`` softmax maps (1 or 2) over the same values: o = a_1 - lam a_2, then (``out_eps`` not
     None) o divided by its root mean square over dv, times ``out_scale``.  A token at position p sees the keys
     from p - p % block on (``block`` 0: from 0; ``window`` w: at most the last w).  q [T, H, maps * DP] as
@@ -1303,13 +1376,18 @@ def diff_attention(q, kv, pos, tok_slot, n_heads, n_kv_heads, maps, d, dv, scale
     ``key_shares`` (a decode step on the matrix cores with four or more query heads on a key/value head): that many
     workgroups share a token's keys, and a second kernel adds up their states in order.
     ``slopes`` (float32 [H]): the score of the key at position j loses slopes[head] * (p - j); the sink loses nothing.
-    ``gate`` (float32 rows [T, >= gate_col + H]): head h's output is multiplied by sigmoid(gate[t][gate_col + h])."""
+    ``gate`` (float32 rows [T, >= gate_col + H]): head h's output is multiplied by sigmoid(gate[t][gate_col + h]),
+    with ``gate_elem`` its element i by sigmoid(gate[t][gate_col + h * dv + i]).  ``softcap`` c: a scaled score s becomes
+    c tanh(s / c) before anything else."""
     _dev(q, pos, tok_slot, sink, slopes, gate)
     _need(sink is None or (sink.dtype == torch.float32 and sink.numel() == n_heads), "sink: float32 [H]")
     _need(slopes is None or (slopes.dtype == torch.float32 and slopes.numel() == n_heads and slopes.is_contiguous()), "slopes: float32 [H]")
     _need(gate is None or (gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == q.shape[0] and gate.stride(1) == 1
-                           and 0 <= gate_col and gate_col + n_heads <= gate.shape[1]), "gate: float32 rows with a column for every head")
-    extra = (_ptr(slopes), _ptr(gate), gate.stride(0) if gate is not None else 0, int(gate_col))
+                           and 0 <= gate_col and gate_col + n_heads * (dv if gate_elem else 1) <= gate.shape[1]),
+          "gate: float32 rows with a column for every head (or every element of every head)")
+    _need(softcap is None or softcap > 0, "softcap: positive")
+    extra = (_ptr(slopes), _ptr(gate), gate.stride(0) if gate is not None else 0, int(gate_col),
+             int(bool(gate_elem and gate is not None)), c_float(softcap or 0.0))
     t = q.shape[0]
     dp = padded_map_dim(d)
     _need(maps in (1, 2) and dv <= 512 and n_heads % n_kv_heads == 0, "diff_attention: one or two maps, values up to 512 wide")
@@ -1359,10 +1437,11 @@ def small_logits(h, w) -> torch.Tensor:
     return out
 
 
-def conv_silu(rows, col0, channels, weight, bias, history, ctx) -> torch.Tensor:
+def conv_silu(rows, col0, channels, weight, bias, history, ctx, out_dtype=torch.float32) -> torch.Tensor:
     """silu of a causal convolution per channel over ``channels`` columns of the float32 ``rows`` from ``col0`` on;
     weight float32 [channels, taps] (last column: the current token), bias [channels] or None; ``history``
-    float32 [slots, taps - 1, channels] holds every sequence's last inputs and is brought up to date."""
+    float32 [slots, taps - 1, channels] holds every sequence's last inputs and is brought up to date.  The result has
+    the type ``out_dtype``."""
     _dev(rows, weight, bias, history)
     _f32_rows(rows, "conv rows")
     t, taps = rows.shape[0], weight.shape[1]
@@ -1376,10 +1455,10 @@ def conv_silu(rows, col0, channels, weight, bias, history, ctx) -> torch.Tensor:
     _i32(ctx.seq_slot, ctx.n_seqs, "sequence slots")
     qstart, qlen = getattr(ctx, "seq_qstart", None), getattr(ctx, "seq_qlen", None)
     _need((qstart is None) == (qlen is None) and (qstart is not None or t == ctx.n_seqs), "conv: per-sequence starts and lengths")
-    out = torch.empty((t, channels), dtype=torch.float32, device=rows.device)
+    out = torch.empty((t, channels), dtype=out_dtype, device=rows.device)
     _check(hybrid().li_conv_silu(_ptr(rows), rows.shape[1], col0, _ptr(weight), _ptr(bias), _ptr(history), _ptr(ctx.pos),
-                                 _ptr(ctx.tok_slot), _ptr(ctx.seq_slot), _ptr(qstart), _ptr(qlen), _ptr(out), t, ctx.n_seqs,
-                                 channels, taps, _stream()), "conv_silu")
+                                 _ptr(ctx.tok_slot), _ptr(ctx.seq_slot), _ptr(qstart), _ptr(qlen), _ptr(out), DT[out_dtype],
+                                 t, ctx.n_seqs, channels, taps, _stream()), "conv_silu")
     return out
 
 
@@ -1715,14 +1794,16 @@ def mlstm_scan(proj, q_col, k_col, v_col, i_col, f_col, i_bias, f_bias, cap, q_s
     return y
 
 
-def gated_head_norm(y, weight, gate_rows, gate_col, heads, eps, out_dtype) -> torch.Tensor:
+def gated_head_norm(y, weight, gate_rows, gate_col, heads, eps, out_dtype, gate_silu: bool = False) -> torch.Tensor:
     """Every head's part of a float32 row [heads * dv] divided by its own root mean square, then times ``weight``
-    [heads * dv] (None: none) and sigmoid of columns gate_col .. of the float32 ``gate_rows`` (None: no gate)."""
+    [heads * dv] (or [dv]: the same for all heads; None: none) and the sigmoid (``gate_silu``: silu) of columns gate_col ..
+    of the float32 ``gate_rows`` (None: no gate)."""
     _dev(y, weight, gate_rows)
     _f32_rows(y, "head norm rows")
     t, n = y.shape
     _need(heads >= 1 and n % heads == 0, "head norm: equal heads")
-    _need(weight is None or (weight.dtype == torch.float32 and weight.shape == (n,)), "head norm weight: float32 [heads * dv]")
+    _need(weight is None or (weight.dtype == torch.float32 and weight.dim() == 1 and weight.numel() in (n, n // heads)),
+          "head norm weight: float32 [heads * dv] or [dv]")
     if gate_rows is not None:
         _f32_rows(gate_rows, "head norm gate")
         _need(gate_rows.shape[0] == t and gate_col >= 0 and gate_col + n <= gate_rows.shape[1], "head norm: gate columns beyond the rows")
@@ -1730,7 +1811,8 @@ def gated_head_norm(y, weight, gate_rows, gate_col, heads, eps, out_dtype) -> to
     _check(hybrid().li_gated_head_norm(_ptr(y), _ptr(weight),
                                        c_void_p(gate_rows.data_ptr() + 4 * gate_col) if gate_rows is not None else None,
                                        c_int64(gate_rows.shape[1] if gate_rows is not None else 0), _ptr(out), DT[out_dtype], t,
-                                       heads, n // heads, c_float(eps), _stream()), "gated_head_norm")
+                                       heads, n // heads, c_float(eps), int(weight is not None and heads > 1 and weight.numel() == n // heads),
+                                       int(bool(gate_silu)), _stream()), "gated_head_norm")
     return out
 
 
@@ -1743,7 +1825,7 @@ def expert_act(z, weights, n_blocks, ff, tail, kind: str, on_input: bool, out_dt
     _dev(z, weights, idx)
     _f32_rows(z, "expert rows")
     rows = z.shape[0]
-    _need(kind in ACTIVATIONS and z.shape[1] == n_blocks * ff + tail, "expert_act: [rows, blocks * ff + tail], a known activation")
+    _need(kind in ACTIVATIONS and kind != "tanh" and z.shape[1] == n_blocks * ff + tail, "expert_act: [rows, blocks * ff + tail], a known activation")
     wcols = 0
     if weights is not None:
         _need(weights.dtype == torch.float32 and weights.dim() == 2, "expert_act: float32 weights [tokens, columns]")
@@ -1884,3 +1966,129 @@ def table_route(token_ids, table, n_experts: int, gate_logits=None, has_gate: in
     _check(hybrid().li_table_route(_ptr(token_ids), _ptr(table), table.shape[1], n_experts, _ptr(gate_logits), int(has_gate),
                                    _ptr(w), t, _stream()), "table_route")
     return w
+
+
+# ---------------------------------------------------------------------------
+# recurrent mixers: the gated delta rule, the selective scan with a decay for every channel and state, time mixing with a
+# decay for every key channel (csrc/recurrent.hip)
+# ---------------------------------------------------------------------------
+_recurrent = None
+
+
+def recurrent():
+    global _recurrent
+    if _recurrent is None:
+        _recurrent = build.recurrent_library()
+    return _recurrent
+
+
+def _segment_args(segments, ctx, qstart, what):
+    """The segment lists as the C interface takes them; None: no segments."""
+    if segments is None:
+        return (None, None, None, None, None, 0)
+    _need(qstart is not None, f"{what} in segments: per-sequence starts and lengths")
+    k = segments["n"]
+    for name, n in (("seg_seq", k), ("seg_t0", k), ("seg_n", k), ("seq_seg0", ctx.n_seqs), ("seq_nseg", ctx.n_seqs)):
+        _i32(segments[name], n, f"{what} {name}")
+    return tuple(_ptr(segments[name]) for name in ("seg_seq", "seg_t0", "seg_n", "seq_seg0", "seq_nseg")) + (k,)
+
+
+def delta_prepare(proj, col0, b_col, a_col, conv_w, history, a_log, dt_bias, ctx, heads, kv_heads, d, dv):
+    """What the gated delta rule reads of a step's tokens, from the float32 rows ``proj``: the columns q [kv_heads, d],
+    k [kv_heads, d], v [heads, dv] from ``col0`` on behind a causal convolution (``conv_w`` float32 [channels, taps],
+    ``history`` float32 [slots, taps - 1, channels], brought up to date) and silu, q and k as unit vectors and q times
+    d^(-1/2); the decays' logarithms -exp(a_log) softplus(proj[a_col + h] + dt_bias) and beta = sigmoid(proj[b_col + h]).
+    Returns float32 (rows [T, channels], gates [T, heads, 2], k . q [T, kv_heads])."""
+    _dev(proj, conv_w, history, a_log, dt_bias)
+    _f32_rows(proj, "delta projections")
+    t, channels, taps = proj.shape[0], 2 * kv_heads * d + heads * dv, conv_w.shape[1]
+    _need(heads % kv_heads == 0 and 1 <= d <= 256, "delta rule: heads a multiple of key heads, keys up to 256 wide")
+    _need(min(col0, b_col, a_col) >= 0 and max(col0 + channels, b_col + heads, a_col + heads) <= proj.shape[1], "delta rule: columns beyond the rows")
+    _need(conv_w.dtype == torch.float32 and conv_w.shape == (channels, taps) and 1 <= taps <= 16, "conv weight: float32 [channels, taps <= 16]")
+    _need(history.dtype == torch.float32 and history.dim() == 3 and tuple(history.shape[1:]) == (max(taps - 1, 1), channels),
+          "conv history: float32 [slots, taps - 1, channels]")
+    for v in (a_log, dt_bias):
+        _need(v.dtype == torch.float32 and v.shape == (heads,), "delta rule: float32 [heads] vectors")
+    _i32(ctx.pos, t, "positions")
+    _i32(ctx.tok_slot, t, "slots")
+    dev = proj.device
+    qkv = torch.empty((t, channels), dtype=torch.float32, device=dev)
+    gates = torch.empty((t, heads, 2), dtype=torch.float32, device=dev)
+    kq = torch.empty((t, kv_heads), dtype=torch.float32, device=dev)
+    _check(recurrent().li_delta_prep(_ptr(proj), proj.shape[1], col0, b_col, a_col, _ptr(conv_w), taps, _ptr(history), _ptr(ctx.pos),
+                                     _ptr(ctx.tok_slot), _ptr(a_log), _ptr(dt_bias), _ptr(qkv), _ptr(gates), _ptr(kq), t, heads,
+                                     kv_heads, d, dv, _stream()), "delta_prep")
+    if taps > 1:
+        conv_history(proj, col0, channels, taps, history, ctx)
+    return qkv, gates, kq
+
+
+def delta_scan(qkv, gates, kq, state, ctx, heads, kv_heads, d, dv) -> torch.Tensor:
+    """The gated delta rule token by token, S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, on what
+    ``delta_prepare`` left; ``state`` float32 [slots, heads, d, dv] is read and left up to date.  Returns float32 [T, heads * dv]."""
+    _dev(qkv, gates, kq, state)
+    t = qkv.shape[0]
+    _need(qkv.dtype == torch.float32 and qkv.shape == (t, 2 * kv_heads * d + heads * dv) and gates.shape == (t, heads, 2)
+          and kq.shape == (t, kv_heads), "delta rule: what delta_prepare returns")
+    _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, d, dv), "delta state: float32 [slots, heads, d, dv]")
+    seq_slot, qstart, qlen = _seq_arrays(ctx, t)
+    y = torch.empty((t, heads * dv), dtype=torch.float32, device=qkv.device)
+    _check(recurrent().li_delta_scan(_ptr(qkv), _ptr(gates), _ptr(kq), _ptr(state), _ptr(seq_slot), _ptr(qstart), _ptr(qlen),
+                                     _ptr(y), ctx.n_seqs, heads, kv_heads, d, dv, _stream()), "delta_scan")
+    return y
+
+
+def selective_scan(x, raw, dt_bias, bc, b_col, c_col, z_rows, z_col, a2, d_skip, state, ctx, segments=None) -> torch.Tensor:
+    """The selective scan with a decay for every channel and state: dt = softplus(raw + dt_bias), S[c, i] <- exp(dt A[c,
+    i]) S[c, i] + dt x_c B_i, y_c = S[c] . C + D_c x_c, and y silu(z).  ``x`` [T, channels] (its type is the result's), ``raw``
+    float32 [T, channels]; B and C are columns of the float32 rows ``bc``, z columns of ``z_rows``; ``a2`` float32 [n,
+    channels] holds A log2(e); ``state`` float32 [slots, n, channels] is read and left up to date.  ``segments``
+    (``ssm_segments``): the tokens run in segments side by side, each twice; None: every sequence in order."""
+    _dev(x, raw, dt_bias, bc, z_rows, a2, d_skip, state)
+    t, channels = x.shape
+    n = a2.shape[0]
+    _need(x.dtype in DT and raw.dtype == torch.float32 and raw.shape == x.shape, "selective scan: rows of one shape")
+    _f32_rows(bc, "selective scan B and C")
+    _f32_rows(z_rows, "selective scan z")
+    _need(bc.shape[0] == t and z_rows.shape[0] == t and min(b_col, c_col, z_col) >= 0 and max(b_col, c_col) + n <= bc.shape[1]
+          and z_col + channels <= z_rows.shape[1], "selective scan: columns beyond the rows")
+    _need(a2.dtype == torch.float32 and a2.shape == (n, channels) and 1 <= n <= 256, "selective scan: A float32 [n <= 256, channels]")
+    for v in (dt_bias, d_skip):
+        _need(v.dtype == torch.float32 and v.shape == (channels,), "selective scan: float32 [channels] vectors")
+    _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (n, channels), "selective scan state: float32 [slots, n, channels]")
+    seq_slot, qstart, qlen = _seq_arrays(ctx, t)
+    seg = _segment_args(segments, ctx, qstart, "selective scan")
+    seg_state = seg_dt = None
+    if segments is not None:
+        seg_state = torch.empty((seg[-1], n, channels), dtype=torch.float32, device=x.device)
+        seg_dt = torch.empty((seg[-1], channels), dtype=torch.float32, device=x.device)
+    out = torch.empty_like(x)
+    _check(recurrent().li_sel_scan(_ptr(x), DT[x.dtype], _ptr(raw), _ptr(dt_bias), _ptr(bc), bc.shape[1], b_col, c_col, _ptr(z_rows),
+                                   z_rows.shape[1], z_col, _ptr(a2), _ptr(d_skip), _ptr(state), _ptr(seq_slot), _ptr(qstart),
+                                   _ptr(qlen), _ptr(out), ctx.n_seqs, channels, n, *seg, _ptr(seg_state), _ptr(seg_dt), _stream()),
+           "sel_scan")
+    return out
+
+
+def wkv_scan(r, k, v, raw, bonus, state, ctx, heads, d, segments=None) -> torch.Tensor:
+    """Time mixing with a decay for every key channel: w = exp(-exp(raw)), o = (S + diag(bonus) k v^T)^T r,
+    S <- diag(w) S + k v^T per head.  r, k, v [T, heads * d] of one type, ``raw`` float32 of that shape, ``bonus`` float32
+    [heads, d]; ``state`` float32 [slots, heads, d, d] is read and left up to date.  ``segments``: as for
+    ``selective_scan``.  Returns float32 [T, heads * d]."""
+    _dev(r, k, v, raw, bonus, state)
+    t = r.shape[0]
+    for x in (r, k, v, raw):
+        _need(x.shape == (t, heads * d) and x.dtype == (torch.float32 if x is raw else r.dtype), "wkv: rows [T, heads * d] of one type, float32 decays")
+    _need(r.dtype in DT and 1 <= d <= 256 and bonus.dtype == torch.float32 and bonus.shape == (heads, d), "wkv: heads up to 256 wide, float32 bonus [heads, d]")
+    _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, d, d), "wkv state: float32 [slots, heads, d, d]")
+    seq_slot, qstart, qlen = _seq_arrays(ctx, t)
+    seg = _segment_args(segments, ctx, qstart, "wkv")
+    seg_state = seg_lw = None
+    if segments is not None:
+        seg_state = torch.empty((seg[-1], heads, d, d), dtype=torch.float32, device=r.device)
+        seg_lw = torch.empty((seg[-1], heads, d), dtype=torch.float32, device=r.device)
+    y = torch.empty((t, heads * d), dtype=torch.float32, device=r.device)
+    _check(recurrent().li_wkv_scan(_ptr(r), _ptr(k), _ptr(v), DT[r.dtype], _ptr(raw), _ptr(bonus), _ptr(state), _ptr(seq_slot),
+                                   _ptr(qstart), _ptr(qlen), _ptr(y), ctx.n_seqs, heads, d, *seg, _ptr(seg_state), _ptr(seg_lw),
+                                   _stream()), "wkv_scan")
+    return y

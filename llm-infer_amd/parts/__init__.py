@@ -16,9 +16,11 @@ from .short_conv import ConvMixer
 from .latent_attention import LatentAttention
 from .mlstm import MatrixLSTM
 from .gated_attention import GatedAttention
+from .recurrent import GatedDelta, SelectiveScan, TimeMixing
 
 __all__ = ["Part", "collect_params", "RMSNorm", "RotaryPosition", "NoPosition", "Attention", "GatedMLP",
            "Embedding", "LMHead", "Block", "PreNormBlock", "SubLayer", "LayerNorm", "PolyNormMLP", "ShiftedMixer",
            "ParallelMixers", "SigmoidAttention", "DecayLinearAttention", "PostNormBlock", "DifferentialAttention",
            "SelectiveStateSpace", "Reinject", "DenseMLP", "RoutedExperts", "DepthAverage", "BigramEmbedding", "ParallelBlock",
-           "ConvMixer", "LatentAttention", "MatrixLSTM", "GatedAttention", "SandwichBlock", "HalfRotaryPosition"]
+           "ConvMixer", "LatentAttention", "MatrixLSTM", "GatedAttention", "SandwichBlock", "HalfRotaryPosition",
+           "GatedDelta", "SelectiveScan", "TimeMixing"]

@@ -120,9 +120,11 @@ class PolyNormMLP(Part):
 @register_feed_forward("dense_mlp")
 class DenseMLP(Part):
     """down(act(up(x))) added into the residual stream: no gate.  ``activation``: "gelu" (the exact form with
-    erf), "gelu_tanh" or "silu", computed in float32 on the product's sums.  ``names``: local tensor names."""
+    erf), "gelu_tanh", "silu" or "relu2" (the square of relu), computed in float32 on the product's sums.  ``names``:
+    local tensor names."""
 
     takes_lazy_norm = True
+    writes_rows = True          # forward_into overwrites the rows it is handed
 
     def __init__(self, *, hidden_size, intermediate_size, activation="gelu", names=None, prefix, dtype, device):
         if activation not in ops.ACTIVATIONS:
@@ -140,9 +142,16 @@ class DenseMLP(Part):
         n = self.names
         self.w_up, self.w_down = ops.prepare_weight(tensors[n["up"]]), ops.prepare_weight(tensors[n["down"]])
 
+    def _hidden(self, h):
+        return ops.activation(ops.linear(h, self.w_up, out_dtype=torch.float32), self.activation, self.dtype)
+
     def forward(self, h, residual):
-        z = ops.linear(h, self.w_up, out_dtype=torch.float32)
-        ops.linear(ops.activation(z, self.activation, self.dtype), self.w_down, ops.EPI_ADD, out=residual)
+        ops.linear(self._hidden(h), self.w_down, ops.EPI_ADD, out=residual)
+
+    def forward_into(self, h, out, ctx=None, view=None, owns_cache=True):
+        """The result written over the float32 rows ``out``."""
+        ops.linear(self._hidden(h), self.w_down, out=out)
+        return None
 
 
 @register_feed_forward("routed_experts")

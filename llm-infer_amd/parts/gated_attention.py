@@ -26,6 +26,8 @@ class GatedAttention(Part):
     ``window`` w only i - j < w, with ``block`` b only the j of i's own block of b positions (counted from position 0).
     ``sink`` / ``gate`` False leave those out.  Variants, all parameters:
 
+    * ``gate`` "elements": a gate for every element of every head's output instead of one a head, W_g [H dv, hidden].
+    * ``softcap`` c: a score becomes c tanh(s / c) before anything is subtracted from it.
     * ``values`` "keys": there is no value projection; a token's values are its keys as projected, before any rotation.
     * the layer's position part (``rope_half``): q and k are turned in their first ``rotary_dim`` dimensions, i paired
       with i + rotary_dim / 2; values never are.
@@ -39,7 +41,8 @@ class GatedAttention(Part):
     * ``keep_window`` / ``keep_block``: what the cache may give back (default: what this layer's own mask lets go of;
       a layer whose cache another layer reads with another mask keeps what both need).
 
-    The input products are one product against [W_q; W_k; W_v; W_g].  The cache keeps keys (after rotation or
+    The input products are one product against [W_q; W_k; W_v; W_g] (``ParallelMixers`` may share it with a mixer beside
+    this one: ``in_rows``, ``proj``).  The cache keeps keys (after rotation or
     convolution) and values in the matrix cores' operand order (one map of keys: the layout that the softmax decoder's
     kernels read too).  A 16-bit model whose keys and values have one size that is a multiple of 16 runs prompts
     through the softmax decoder's prompt kernel (``ops.attention_prefill``, which takes the sink, the slopes, the
@@ -51,7 +54,7 @@ class GatedAttention(Part):
     writes_rows = True          # forward_into overwrites the rows it is handed
 
     def __init__(self, *, hidden_size, n_heads, n_kv_heads, head_dim, v_head_dim=None, scale, window=None, block=None,
-                 sink=True, gate=True, values="own", bias=False, conv_taps=0, slope_exponent=None, reads_kv=False,
+                 sink=True, gate=True, softcap=None, values="own", bias=False, conv_taps=0, slope_exponent=None, reads_kv=False,
                  keep_window="own", keep_block="own", names=None, position=None, prefix, dtype, device):
         if n_heads % n_kv_heads != 0:
             raise ValueError("n_heads must be a multiple of n_kv_heads")
@@ -73,7 +76,13 @@ class GatedAttention(Part):
         self.block = None if block is None else int(block)
         self.keep_window = self.window if keep_window == "own" else (None if keep_window is None else int(keep_window))
         self.keep_block = self.block if keep_block == "own" else (None if keep_block is None else int(keep_block))
+        if gate not in (True, False, "elements"):
+            raise ValueError("gated attention: gate True (one number a head), 'elements' or False")
+        if softcap is not None and not float(softcap) > 0:
+            raise ValueError("gated attention: a positive soft cap")
         self.sink, self.gate, self.values_are_keys, self.bias = bool(sink), bool(gate), values == "keys", bool(bias)
+        self.gate_elem, self.softcap = gate == "elements", None if softcap is None else float(softcap)
+        self.gate_rows = (n_heads * v_head_dim if self.gate_elem else n_heads) if self.gate else 0
         self.conv_taps, self.reads_kv = int(conv_taps), bool(reads_kv)
         self.slope_exponent = None if slope_exponent is None else float(slope_exponent)
         self.position = position
@@ -108,7 +117,7 @@ class GatedAttention(Part):
         if self.sink:
             out[n["sink"]] = ParamSpec((H,), "vector", "small")
         if self.gate:
-            out[n["g"]] = ParamSpec((H, w))
+            out[n["g"]] = ParamSpec((self.gate_rows, w))
         return out
 
     def bind(self, tensors):
@@ -120,7 +129,7 @@ class GatedAttention(Part):
         if self.bias:
             # a bias for every column of the one input product: those of q, k and v, none for the gate's
             b = torch.cat([plain(tensors[n[k + "_bias"]]).float() for k in keys])
-            pad = torch.zeros(self.n_heads if self.gate else 0, dtype=torch.float32, device=b.device)
+            pad = torch.zeros(self.gate_rows, dtype=torch.float32, device=b.device)
             self.b_in = ops.glu_params(torch.cat([b, pad]).contiguous())
         if self.conv_taps:
             self.conv = torch.cat([plain(tensors[n[k + "_conv"]]).float() for k in keys], 0).contiguous()
@@ -135,6 +144,14 @@ class GatedAttention(Part):
         if self.conv_taps:
             return [StateSpec((max(self.conv_taps - 1, 1), self.channels), "float32"), kv]
         return [kv]
+
+    def in_rows(self) -> int:
+        return self.channels + self.gate_rows
+
+    @property
+    def shares_product(self) -> bool:
+        """True if the input product may be shared (a bias is added in this mixer's own)."""
+        return not self.bias
 
     def _key_shares(self, ctx) -> int:
         """Workgroups that share a token's keys in a decode step of a 16-bit model (a mask bounds what a token sees)."""
@@ -157,19 +174,23 @@ class GatedAttention(Part):
                 splits = min(splits, max(1, span // 128))
         return 1 << (splits.bit_length() - 1)
 
-    def attend(self, h, ctx, views, owns_cache):
-        """The heads' gated outputs side by side, [T, H * dv] in the model's type."""
+    def attend(self, h, ctx, views, owns_cache, proj=None, col0=0):
+        """The heads' gated outputs side by side, [T, H * dv] in the model's type.  ``proj`` (float32 [T, n]) with this
+        mixer's columns from ``col0`` on: the product is not run here."""
         if owns_cache == self.reads_kv:
             raise ValueError("gated attention: a layer without key and value tensors reads another run's cache, and only such a layer")
         H, G, d, dv = self.n_heads, self.n_kv_heads, self.head_dim, self.v_head_dim
-        kv = views[-1].as_tuple()
-        if self.bias:
+        kv = (views[-1] if isinstance(views, (list, tuple)) else views).as_tuple()
+        if proj is not None:
+            if self.conv_taps and col0:
+                raise ValueError("gated attention: a convolution covers the first columns of its own product")
+        elif self.bias:
             proj = ops.linear(h, self.w_in, ops.EPI_BIAS, out_dtype=torch.float32, params=self.b_in)
         else:
             proj = ops.linear(h, self.w_in, out_dtype=torch.float32)
         # the convolution rides in the kernel that turns and stores; the history is brought up to date behind it
         conv = (self.conv, views[0].state) if self.conv_taps else None
-        q = ops.rot_store(proj, self.q_col, self.k_col, self.v_col, getattr(self.position, "inv_freq", None) if self.rot else None,
+        q = ops.rot_store(proj, col0 + self.q_col, col0 + self.k_col, col0 + self.v_col, getattr(self.position, "inv_freq", None) if self.rot else None,
                           self.rot, ctx.pos, ctx.tok_slot, kv, H, 0 if self.reads_kv else G, d, dv, kv[0].dtype, conv)
         if self.conv_taps > 1:
             ops.conv_history(proj, 0, self.channels, self.conv_taps, views[0].state, ctx)
@@ -177,19 +198,20 @@ class GatedAttention(Part):
             # a 16-bit model whose keys and values have one size the kernels take as it is: the softmax decoder's own
             # kernels (prompts: pages through LDS, scores of the next page under the weights of this one; decode steps:
             # a wave per (sequence, key/value head, split of the keys that the mask leaves))
-            gate = proj if self.gate else None
+            gate, gate_col = proj if self.gate else None, col0 + self.gate_col
             if ctx.is_decode:
                 a = ops.attention_decode(q, kv, ctx.seq_slot, ctx.seq_ctx, ctx.n_seqs, H, G, d, self.scale, self.window,
-                                         self._splits(ctx), self.block, self.sinks, self.slopes, gate, self.gate_col)
+                                         self._splits(ctx), self.block, self.sinks, self.slopes, gate, gate_col, self.softcap, self.gate_elem)
             else:
                 a = ops.attention_prefill(q, kv, ops.prefill_meta(ctx), H, G, d, self.scale, self.window, self.block, self.sinks,
-                                          self.slopes, gate, self.gate_col)
+                                          self.slopes, gate, gate_col, self.softcap, self.gate_elem)
             return a.view(a.shape[0], H * dv)
         sixteen = self.dtype != torch.float32 and ops.diff_attention_fits(d, dv)
         return ops.diff_attention(q, kv, ctx.pos, ctx.tok_slot, H, G, 1, d, dv, self.scale, self.block, self.window, 0.0, None, 1.0,
                                   self.dtype, ops.diff_tiles(ctx, self.block, self.window) if sixteen else None, sink=self.sinks,
                                   key_shares=self._key_shares(ctx) if sixteen else 1, slopes=self.slopes,
-                                  gate=proj if self.gate else None, gate_col=self.gate_col)
+                                  gate=proj if self.gate else None, gate_col=col0 + self.gate_col, softcap=self.softcap,
+                                  gate_elem=self.gate_elem)
 
     def forward(self, h, ctx, views, residual, owns_cache=True):
         ops.linear(self.attend(h, ctx, views, owns_cache), self.wo, ops.EPI_ADD, out=residual)
@@ -198,3 +220,10 @@ class GatedAttention(Part):
         """The mixer's result written over the float32 rows ``out`` (nothing is added to what they held)."""
         ops.linear(self.attend(h, ctx, views, owns_cache), self.wo, out=out)
         return None
+
+    def rows(self, h, ctx, views, owns_cache=True, proj=None, col0=0):
+        """The mixer's result as float32 rows."""
+        return ops.linear(self.attend(h, ctx, views, owns_cache, proj, col0), self.wo, out_dtype=torch.float32)
+
+    def addends(self, h, ctx, views, owns_cache=True, proj=None, col0=0):
+        return [(self.rows(h, ctx, views, owns_cache, proj, col0), 1.0)]

@@ -50,22 +50,51 @@ class RMSNorm(Part):
                 return ready
         return ops.rmsnorm(x, self.weight, self.eps, self.dtype, rows)
 
+    def add_into(self, x, y, bias=None, next_norm=None) -> None:
+        """x += this norm of (y + bias), in one pass that also takes the norm that reads ``x`` next where that is one of
+        this kind."""
+        nxt = None
+        if isinstance(next_norm, RMSNorm) and next_norm.weight is not None:
+            nxt = (next_norm.weight, next_norm.eps, next_norm.dtype)
+        ops.rmsnorm_add(x, y.rows() if isinstance(y, ops.NormedPair) else y, self.weight, self.eps, bias, nxt)
+
 
 @register_norm("layernorm")
 class LayerNorm(Part):
-    """out = (x - mean) / sqrt(var + eps) * weight in float32, var the mean of the squared deviations; a weight
-    and no bias.  ``name`` is the local name of the weight's tensor."""
+    """out = (x - mean) / sqrt(var + eps) * weight (+ bias) in float32, var the mean of the squared deviations.  ``name``
+    is the local name of the weight's tensor, ``bias`` that of the bias (None: there is none)."""
 
-    def __init__(self, *, size: int, eps: float, name: str = "weight", prefix: str, dtype, device):
-        self.size, self.eps, self.name = size, float(eps), name
+    def __init__(self, *, size: int, eps: float, name: str = "weight", bias: str | None = None, prefix: str, dtype, device):
+        self.size, self.eps, self.name, self.bias_name = size, float(eps), name, bias
         self.prefix, self.dtype, self.device = prefix, dtype, device
-        self.weight = None
+        self.weight = self.bias = None
 
     def params(self):
-        return {self.name: ParamSpec((self.size,), "vector", "ones")}
+        out = {self.name: ParamSpec((self.size,), "vector", "ones")}
+        if self.bias_name is not None:
+            out[self.bias_name] = ParamSpec((self.size,), "vector", "small")
+        return out
 
     def bind(self, tensors):
         self.weight = tensors[self.name]
+        self.bias = tensors[self.bias_name] if self.bias_name is not None else None
 
-    def forward(self, x: torch.Tensor, rows: torch.Tensor | None = None):
-        return ops.layernorm(x, self.weight, self.eps, self.dtype, rows)
+    def forward(self, x: torch.Tensor, rows: torch.Tensor | None = None, lazy: bool = False, out_dtype=None):
+        """The normed rows in the compute dtype, or in ``out_dtype``."""
+        dtype = out_dtype or self.dtype
+        if rows is None:
+            ready = ops.prepared_norm(x, self.weight, self.eps, dtype)        # taken by the pass before
+            if ready is not None:
+                return ready
+        return ops.layernorm(x, self.weight, self.eps, dtype, rows, self.bias)
+
+    def add_into(self, x, y, bias=None, next_norm=None) -> None:
+        """x += this norm of (y + bias), in one pass that also takes the norm that reads ``x`` next where that is one of
+        this kind; ``y`` may be an ``ops.NormedPair``."""
+        if bias is not None:
+            y = y.rows() if isinstance(y, ops.NormedPair) else y
+            ops.add_bias(y, 0, bias)
+        nxt = None
+        if isinstance(next_norm, LayerNorm) and next_norm.weight is not None:
+            nxt = (next_norm.weight, next_norm.bias, next_norm.eps, next_norm.dtype)
+        ops.layernorm_add(x, y, self.weight, self.bias, self.eps, nxt)

@@ -31,6 +31,7 @@ class ParamSpec:
     shape: tuple
     kind: str = "matrix"        # "matrix" | "vector" | "int"
     init: str = "normal"        # random-weights mode: "normal" N(0, 0.02) | "ones" 1 + N(0, 0.01) | "small" | "half" | "wide" | "mean"
+    free: tuple = ()            # axes whose size the checkpoint sets (``shape`` holds what random weights take there)
 
 
 class Checkpoint:
@@ -111,7 +112,7 @@ def check_tensors(needed: dict, found, ignorable=()) -> None:
     for n, spec in needed.items():
         if n in have:
             dtype, shape = found.info(n)
-            if tuple(shape) != tuple(spec.shape):
+            if len(shape) != len(spec.shape) or any(a != b for i, (a, b) in enumerate(zip(shape, spec.shape)) if i not in spec.free):
                 wrong.append(f"{n}: expected {list(spec.shape)}, got {list(shape)}")
             elif spec.kind == "int" and dtype.is_floating_point:
                 wrong.append(f"{n}: expected an integer table, got {dtype}")
