@@ -62,7 +62,7 @@ def main() -> int:
                     help="leave out the long contexts, batch 128 and the generation run that the default run adds to points")
     ap.add_argument("--generate", type=int, default=0,
                     help="also generate for this many 128-token prompts with budgets drawn from 16..512 tokens")
-    ap.add_argument("--compare", default="", choices=["", "manirax", "risonex", "dupolorn", "favizen"],
+    ap.add_argument("--compare", default="", choices=["", "manirax", "risonex", "dupolorn", "favizen", "dopivik"],
                     help="instead of the default workload: prefill and decode throughput of this design at a few "
                          "layer sizes beside the Llama decoder at equal sizes (random weights, a few layers each)")
     ap.add_argument("--sizes", default="", help="with --compare: the layer sizes to run, comma separated (default: all)")
@@ -201,6 +201,20 @@ def compare_configs(design: str, size: dict, layers: int, context: int) -> dict:
                 mixer["kv_from"] = i - 1
             stack.append({"type": kind, "mixer": mixer, "mlp": dense if i % 2 == 0 else routed})
         other = {"architecture": "Favizen", "embedding": {"scale": 1.0}, "layers": stack, "logit_scale": 1.0, "norm": {"eps": 1e-5},
+                 "vocab": size["vocab"], "width": w, "max_positions": context}
+        return {"llama": llama, design: other}
+    if design == "dopivik":
+        # parallel layers (the Llama decoder's attention heads with scores softly capped, chunks of 1,024 positions and a gate
+        # for every element, beside a delta rule of as many value heads on half as many key heads, states of hd x hd) in the
+        # first and fourth of four layers; a selective scan of twice the width inside with 16 states a channel; time mixing
+        # with heads of 64; feed-forwards of the Llama decoder's width without a gate
+        left = {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "softcap": 50.0, "mask": {"size": 1024},
+                "rot": {"base": 500000.0, "dims": hd}}
+        right = {"heads": H, "kv_heads": H // 2, "dim": hd, "vdim": hd, "conv": 4}
+        kinds = [("parallel", {"left": left, "right": right}), ("mamba1", {"inner": 2 * w, "state": 16, "dt_rank": w // 16, "conv": 4}),
+                 ("wkv", {"heads": w // 64, "dim": 64}), ("parallel", {"left": left, "right": right})]
+        stack = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": size["ff"]}} for i in range(layers)]
+        other = {"architecture": "Dopivik", "embedding": {"scale": 1.0}, "layers": stack, "norm": {"eps": 1e-5},
                  "vocab": size["vocab"], "width": w, "max_positions": context}
         return {"llama": llama, design: other}
     assert design == "manirax"

@@ -5,7 +5,8 @@
 
 enum { EPI_STORE = 0, EPI_ADD = 1, EPI_SWIGLU = 2, EPI_ROPE = 3, EPI_GEGLU = 4, EPI_BIAS = 5, EPI_CLAMPGLU = 6 };
 
-// What EPI_BIAS and EPI_CLAMPGLU need (handed over where EPI_ROPE's RopeStore is).  EPI_BIAS: C = sums + bias[n].
+// What EPI_BIAS and EPI_CLAMPGLU need (handed over where EPI_ROPE's RopeStore is).  EPI_BIAS: C = act(sums + bias[n]),
+// act 0: none, 1: the square of relu, 2: tanh (with an activation the bias may be null).
 // EPI_CLAMPGLU: columns 2j (gate) and 2j + 1 (up), each plus its bias (null: none), give
 //   h[m, j] = g sigmoid(alpha g) (u + shift),  g = min(gate, limit),  u = clamp(up, -limit, limit);
 // the outputs from tail_col on (an expert of another kind behind the others) take tail_limit.
@@ -13,6 +14,7 @@ struct GluParams {
     const float* bias;          // [N] float32, or null
     float limit, tail_limit, alpha, shift;
     int tail_col;               // first output column that takes tail_limit (>= N / 2: none)
+    int act;                    // EPI_BIAS: the activation
 };
 
 __device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float shift) {
@@ -128,9 +130,18 @@ __device__ __forceinline__ void epilogue_extra4(const Epilogue& e, int m, int n,
         }
         return;
     }
+    float o[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-        if (n + j < e.N) store_one(e.C, e.out_dt, (int64_t)m * e.N + n + j, v[j] + e.gp.bias[n + j]);
+    for (int j = 0; j < 4; ++j) {
+        o[j] = v[j] + (e.gp.bias && n + j < e.N ? e.gp.bias[n + j] : 0.f);
+        if (e.gp.act == 1) { const float r = fmaxf(o[j], 0.f); o[j] = r * r; }
+        else if (e.gp.act == 2) o[j] = tanhf(o[j]);
+    }
+    if ((e.N & 3) == 0) store_four(e.C, e.out_dt, (int64_t)m * e.N + n, o);
+    else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) if (n + j < e.N) store_one(e.C, e.out_dt, (int64_t)m * e.N + n + j, o[j]);
+    }
 }
 
 // The other epilogues.  v[0..3] are the results for row m and columns n..n+3 (n a multiple of 4).
@@ -372,7 +383,7 @@ static int make_epilogue(Epilogue& e, void* C, int mode, int out_dt, int M, int 
     e.gp = GluParams{};
     if (mode == EPI_BIAS || mode == EPI_CLAMPGLU) {
         const GluParams* gp = (const GluParams*)rs;            // these modes' own parameters come in the same place
-        if (!gp || (mode == EPI_BIAS && !gp->bias) || (mode == EPI_CLAMPGLU && !(gp->limit > 0.f && gp->tail_limit > 0.f)))
+        if (!gp || (mode == EPI_BIAS && ((!gp->bias && !gp->act) || gp->act < 0 || gp->act > 2)) || (mode == EPI_CLAMPGLU && !(gp->limit > 0.f && gp->tail_limit > 0.f)))
             return LI_BAD_ARG;
         e.gp = *gp;
         return LI_OK;

@@ -9,6 +9,7 @@
 // Whatever a norm, a score, an attention weight, a decay, a step size or a recurrent state is made of is float32
 // here, whatever the type of the matrices.
 #include "common.h"
+#include "conv.h"
 
 __device__ __forceinline__ float sigmoidf_(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float siluf_(float z) { return z / (1.f + expf(-z)); }
@@ -73,7 +74,7 @@ extern "C" int li_concat_cast(const float* a, const float* b, void* out, int dt,
 }
 
 // ---------------------------------------------------------------------------
-// out = act(in), float32 in, type T out.  act: 0 gelu (erf), 1 gelu (tanh), 2 silu, 3 the square of relu, 4 tanh.
+// out = act(in), float32 in, type T out.  act: 0 gelu (erf), 1 gelu (tanh), 2 silu, 3 the square of relu.
 // ---------------------------------------------------------------------------
 template <class T>
 __global__ void activation_kernel(const float* __restrict__ in, T* __restrict__ out, int64_t n, int act) {
@@ -81,12 +82,12 @@ __global__ void activation_kernel(const float* __restrict__ in, T* __restrict__ 
     if (i >= n) return;
     const float z = in[i];
     const float r = fmaxf(z, 0.f);
-    out[i] = from_f32<T>(act == 0 ? gelu_erff_(z) : (act == 1 ? gate_activation(z, true) : (act == 2 ? siluf_(z) : (act == 3 ? r * r : tanhf(z)))));
+    out[i] = from_f32<T>(act == 0 ? gelu_erff_(z) : (act == 1 ? gate_activation(z, true) : (act == 2 ? siluf_(z) : r * r)));
 }
 
 extern "C" int li_activation(const float* in, void* out, int dt, int64_t n, int act, hipStream_t stream) {
     if (n <= 0) return LI_OK;
-    if (act < 0 || act > 4) return LI_BAD_ARG;
+    if (act < 0 || act > 3) return LI_BAD_ARG;
     DISPATCH_T(dt, (activation_kernel<T><<<(unsigned)((n + 255) / 256), 256, 0, stream>>>(in, (T*)out, n, act)));
     LI_CHECK_LAUNCH();
     return LI_OK;
@@ -332,29 +333,51 @@ extern "C" int li_diff_attn(const void* q, void* out, int dt, void* k_pages, voi
 // of the steps before, oldest first); before position 0 they are zero.  conv_history_kernel then leaves every
 // sequence's last taps - 1 inputs there.
 // ---------------------------------------------------------------------------
-#define CONV_MAX_TAPS 16
-
-template <class T, bool SILU, bool ADD>
+// TAPS 4: a thread walks `tile` consecutive tokens of the step with a channel's last inputs in registers; TAPS 0: any number of
+// taps, a token at a time.
+template <class T, bool SILU, bool ADD, int TAPS>
 __global__ void conv_silu_kernel(const float* __restrict__ in, int stride, int col0, const float* __restrict__ w,
                                  const float* __restrict__ b, const float* __restrict__ hist, const int* __restrict__ pos,
-                                 const int* __restrict__ tok_slot, T* __restrict__ out, int channels, int taps) {
-    const int t = blockIdx.x, p = pos[t], slot = tok_slot[t];
-    // how many tokens before this one its sequence has in this step (at most taps - 1 matter)
-    int inside = 0;
-    while (inside < taps - 1 && t - inside - 1 >= 0 && tok_slot[t - inside - 1] == slot) ++inside;
-    const float* h = hist + (int64_t)slot * (taps - 1) * channels;
+                                 const int* __restrict__ tok_slot, T* __restrict__ out, int channels, int taps, int n_tokens, int tile) {
+    const int t0 = blockIdx.x * tile, t1 = min(n_tokens, t0 + tile);
     for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < channels; c += gridDim.y * blockDim.x) {
-        float acc = b ? b[c] : 0.f;
-        for (int back = 0; back < taps; ++back) {                  // back = taps - 1 - j
-            float u = 0.f;
-            if (back <= inside) u = in[(int64_t)(t - back) * stride + col0 + c];
-            else if (p - back >= 0) u = h[(int64_t)(taps - 1 - (back - inside)) * channels + c];
-            acc += w[(int64_t)c * taps + (taps - 1 - back)] * u;
+        constexpr int K = TAPS ? TAPS : 1;
+        ConvWindow<K> win;
+        float wc[K];
+        const float bias = b ? b[c] : 0.f;
+        if (TAPS) {
+#pragma unroll
+            for (int j = 0; j < K; ++j) wc[j] = w[(int64_t)c * K + j];
         }
-        if (ADD) acc += in[(int64_t)t * stride + col0 + c];        // the input itself beside its convolution
-        out[(int64_t)t * channels + c] = from_f32<T>(SILU ? siluf_(acc) : acc);
+        int last = -1;
+        for (int t = t0; t < t1; ++t) {
+            const int slot = tok_slot[t];
+            const float* at = in + (int64_t)t * stride + col0 + c;
+            const float* h = hist + (int64_t)slot * (taps - 1) * channels;
+            float acc;
+            if (TAPS) {
+                if (slot != last) win.start(at, stride, conv_inside(tok_slot, t, slot, taps), pos[t], h, channels, c);
+                else win.next(*at);
+                last = slot;
+                acc = win.sum(wc, bias);
+            } else acc = conv_at(at, stride, conv_inside(tok_slot, t, slot, taps), pos[t], h, channels, c, w, taps, bias);
+            if (ADD) acc += *at;                               // the input itself beside its convolution
+            out[(int64_t)t * channels + c] = from_f32<T>(SILU ? siluf_(acc) : acc);
+        }
     }
 }
+
+#define CONV_GO(T, SILU, ADD)                                                                                                       \
+    do {                                                                                                                            \
+        const int tile = n_tokens >= 256 && taps == 4 ? 8 : 1;                                                                      \
+        dim3 cgrid((n_tokens + tile - 1) / tile, (channels + 255) / 256);                                                           \
+        if (taps == 4)                                                                                                              \
+            conv_silu_kernel<T, SILU, ADD, 4><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, (T*)out, channels, \
+                                                                         taps, n_tokens, tile);                                     \
+        else                                                                                                                        \
+            conv_silu_kernel<T, SILU, ADD, 0><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, (T*)out, channels, \
+                                                                         taps, n_tokens, tile);                                     \
+    } while (0)
 
 __global__ void conv_history_kernel(const float* __restrict__ in, int stride, int col0, float* __restrict__ hist,
                                     const int* __restrict__ seq_slot, const int* __restrict__ seq_qstart,
@@ -378,9 +401,7 @@ extern "C" int li_conv_silu(const float* in, int stride, int col0, const float* 
                             hipStream_t stream) {
     if (n_tokens <= 0) return LI_OK;
     if (channels <= 0 || taps < 1 || taps > CONV_MAX_TAPS) return LI_BAD_ARG;
-    dim3 cgrid(n_tokens, (channels + 255) / 256);
-    DISPATCH_T(dt, (conv_silu_kernel<T, true, false><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, (T*)out,
-                                                                                channels, taps)));
+    DISPATCH_T(dt, CONV_GO(T, true, false));
     if (taps > 1) {
         dim3 grid(n_seqs, (channels + 255) / 256);
         conv_history_kernel<<<grid, 256, 0, stream>>>(in, stride, col0, hist, seq_slot, seq_qstart, seq_qlen, channels, taps);
@@ -397,9 +418,7 @@ extern "C" int li_conv_add(const float* in, int stride, int col0, const float* w
                            hipStream_t stream) {
     if (n_tokens <= 0) return LI_OK;
     if (channels <= 0 || taps < 1 || taps > CONV_MAX_TAPS) return LI_BAD_ARG;
-    dim3 cgrid(n_tokens, (channels + 255) / 256);
-    DISPATCH_T(dt, (conv_silu_kernel<T, false, true><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, (T*)out,
-                                                                                channels, taps)));
+    DISPATCH_T(dt, CONV_GO(T, false, true));
     if (taps > 1) {
         dim3 grid(n_seqs, (channels + 255) / 256);
         conv_history_kernel<<<grid, 256, 0, stream>>>(in, stride, col0, hist, seq_slot, seq_qstart, seq_qlen, channels, taps);

@@ -613,6 +613,35 @@ extern "C" int li_mlstm_scan(const float* proj, int stride, int q_col, int k_col
 // (float32 rows `gate_stride` apart; null: none).  `w_shared`: w has dv numbers, the same for all heads; `gate_silu`: the
 // gate's silu instead of its sigmoid.  One wave per (token, head).
 // ---------------------------------------------------------------------------
+// Heads of 4 LANES elements: LANES lanes a head, four elements each, 64 / LANES heads a wave.
+template <class T, int LANES>
+__global__ __launch_bounds__(256) void gated_head_norm_vec_kernel(const float* __restrict__ y, const float* __restrict__ w,
+                                                                  const float* __restrict__ gate, int64_t gate_stride,
+                                                                  T* __restrict__ out, int n_units, int H, float eps, int w_shared,
+                                                                  int gate_silu) {
+    struct alignas(4 * sizeof(T)) Out4 { T v[4]; };
+    constexpr int dv = 4 * LANES;
+    const int unit = (blockIdx.x * 256 + threadIdx.x) / LANES, i = 4 * (threadIdx.x & (LANES - 1));
+    const bool live = unit < n_units;
+    const int u = live ? unit : n_units - 1, t = u / H, h = u - t * H;
+    const f32x4 v = *(const f32x4*)(y + (int64_t)u * dv + i);
+    f32x4 g = {0.f, 0.f, 0.f, 0.f}, wv = {1.f, 1.f, 1.f, 1.f};
+    if (gate) g = *(const f32x4*)(gate + (int64_t)t * gate_stride + h * dv + i);
+    if (w) wv = *(const f32x4*)(w + (w_shared ? i : h * dv + i));
+    float ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+#pragma unroll
+    for (int o = LANES / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);
+    const float r = 1.f / sqrtf(ss / (float)dv + eps);
+    Out4 o;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+        float x = v[k] * r * wv[k];
+        if (gate) x *= gate_silu ? g[k] * lt_sigmoid(g[k]) : lt_sigmoid(g[k]);
+        o.v[k] = from_f32<T>(x);
+    }
+    if (live) *(Out4*)(out + (int64_t)u * dv + i) = o;
+}
+
 template <class T>
 __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __restrict__ y, const float* __restrict__ w,
                                                               const float* __restrict__ gate, int64_t gate_stride,
@@ -640,6 +669,15 @@ extern "C" int li_gated_head_norm(const float* y, const float* w, const float* g
     if (n_rows <= 0) return LI_OK;
     if (H <= 0 || dv <= 0) return LI_BAD_ARG;
     const int units = n_rows * H;
+    if ((dv == 32 || dv == 64 || dv == 128 || dv == 256) && gate_stride % 4 == 0 &&
+        !(((uintptr_t)y | (uintptr_t)w | (uintptr_t)gate | (uintptr_t)out) & 15)) {
+#define GO(L) gated_head_norm_vec_kernel<T, L><<<(int)(((int64_t)units * L + 255) / 256), 256, 0, stream>>>(y, w, gate, gate_stride, (T*)out, \
+                                                                                                       units, H, eps, w_shared, gate_silu)
+        DISPATCH_T(dt, { if (dv == 32) GO(8); else if (dv == 64) GO(16); else if (dv == 128) GO(32); else GO(64); });
+#undef GO
+        LI_CHECK_LAUNCH();
+        return LI_OK;
+    }
     DISPATCH_T(dt, (gated_head_norm_kernel<T><<<(units + 3) / 4, 256, 0, stream>>>(y, w, gate, gate_stride, (T*)out, units, H, dv, eps,
                                                                              w_shared, gate_silu)));
     LI_CHECK_LAUNCH();

@@ -253,7 +253,18 @@ struct LnAdd {
 template <class TN, int THREADS, int KEEP>
 __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int width) {
     struct alignas(4 * sizeof(TN)) Out4 { TN v[4]; };
-    __shared__ float scratch[16];
+    __shared__ float scratch[6][16];                   // a row of it for every sum: one barrier each
+    int sums = 0;
+    auto block_total = [&](float v) {
+        float* mine = scratch[sums++];
+        v = wave_sum(v);
+        if ((threadIdx.x & 63) == 0) mine[threadIdx.x >> 6] = v;
+        __syncthreads();
+        float t = 0.f;
+#pragma unroll
+        for (int i = 0; i < THREADS / 64; ++i) t += mine[i];
+        return t;
+    };
     const int64_t at = (int64_t)blockIdx.x * width;
     const float *ar = p.a + at, *a2r = p.a2 ? p.a2 + at : nullptr;
     float* xr = p.x + at;
@@ -283,8 +294,8 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
 #pragma unroll
                 for (int k = 0; k < 4; ++k) { s0 += y[c][k] * y[c][k]; s1 += z[c][k] * z[c][k]; }
             }
-            const float r1 = p.pair_scale / sqrtf(block_sum(s0, scratch) * inv_n + p.pair_eps);
-            const float r2 = p.pair_scale / sqrtf(block_sum(s1, scratch) * inv_n + p.pair_eps);
+            const float r1 = p.pair_scale / sqrtf(block_total(s0) * inv_n + p.pair_eps);
+            const float r2 = p.pair_scale / sqrtf(block_total(s1) * inv_n + p.pair_eps);
 #pragma unroll
             for (int c = 0; c < KEEP; ++c) {
                 const int i = tid + c * THREADS;
@@ -305,7 +316,7 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
             float s = 0.f;
 #pragma unroll
             for (int c = 0; c < KEEP; ++c) s += (v[c][0] + v[c][1]) + (v[c][2] + v[c][3]);
-            const float mean = block_sum(s, scratch) * inv_n;
+            const float mean = block_total(s) * inv_n;
             s = 0.f;
 #pragma unroll
             for (int c = 0; c < KEEP; ++c) {
@@ -314,7 +325,7 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
                     for (int k = 0; k < 4; ++k) { v[c][k] -= mean; s += v[c][k] * v[c][k]; }
                 }
             }
-            return 1.f / sqrtf(block_sum(s, scratch) * inv_n + eps);
+            return 1.f / sqrtf(block_total(s) * inv_n + eps);
         };
         const float r = normed(y, p.eps);
 #pragma unroll
@@ -346,8 +357,8 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
     if (a2r) {
         float s0 = 0.f, s1 = 0.f;
         for (int i = tid; i < width; i += THREADS) { s0 += ar[i] * ar[i]; s1 += a2r[i] * a2r[i]; }
-        r1 = p.pair_scale / sqrtf(block_sum(s0, scratch) * inv_n + p.pair_eps);
-        r2 = p.pair_scale / sqrtf(block_sum(s1, scratch) * inv_n + p.pair_eps);
+        r1 = p.pair_scale / sqrtf(block_total(s0) * inv_n + p.pair_eps);
+        r2 = p.pair_scale / sqrtf(block_total(s1) * inv_n + p.pair_eps);
     }
     auto y = [&](int i) { return a2r ? ar[i] * r1 * p.w1[i] + a2r[i] * r2 * p.w2[i] : ar[i]; };
     if (!p.w) {
@@ -356,10 +367,10 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
     }
     float s = 0.f;
     for (int i = tid; i < width; i += THREADS) s += y(i);
-    float mean = block_sum(s, scratch) * inv_n;
+    float mean = block_total(s) * inv_n;
     s = 0.f;
     for (int i = tid; i < width; i += THREADS) { const float v = y(i) - mean; s += v * v; }
-    float r = 1.f / sqrtf(block_sum(s, scratch) * inv_n + p.eps);
+    float r = 1.f / sqrtf(block_total(s) * inv_n + p.eps);
     s = 0.f;
     for (int i = tid; i < width; i += THREADS) {
         const float v = xr[i] + (y(i) - mean) * r * p.w[i] + (p.b ? p.b[i] : 0.f);
@@ -367,10 +378,10 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
         s += v;
     }
     if (!p.nw) return;
-    mean = block_sum(s, scratch) * inv_n;
+    mean = block_total(s) * inv_n;
     s = 0.f;
     for (int i = tid; i < width; i += THREADS) { const float v = xr[i] - mean; s += v * v; }
-    r = 1.f / sqrtf(block_sum(s, scratch) * inv_n + p.next_eps);
+    r = 1.f / sqrtf(block_total(s) * inv_n + p.next_eps);
     for (int i = tid; i < width; i += THREADS) nr[i] = from_f32<TN>((xr[i] - mean) * r * p.nw[i] + (p.nb ? p.nb[i] : 0.f));
 }
 
@@ -386,7 +397,11 @@ extern "C" int li_layernorm_add(float* x, const float* a, const float* a2, const
     const LnAdd p{x, a, a2, w1, w2, pair_eps, pair_scale, w, b, eps, nw, nb, next_eps, next};
     // few rows (a decode step): as many threads a row as there are pieces of four, so that a row waits for memory once
 #define GO1(TN, TH, K) layernorm_add_kernel<TN, TH, K><<<n_rows, TH, 0, stream>>>(p, width)
-#define GO(TN) do { if (width <= 1024) GO1(TN, 256, 1); else if (n_rows <= 256 || width > 8192) GO1(TN, 1024, 4); else GO1(TN, 256, 8); } while (0)
+#define GO(TN)                                                                                                   \
+    do {                                                                                                         \
+        if (width <= 1024) GO1(TN, 256, 1); else if (width <= 2048) GO1(TN, 512, 1);                             \
+        else if (width <= 4096) GO1(TN, 1024, 1); else GO1(TN, 1024, 4);                                         \
+    } while (0)
     if (next_dt == DT_F32) GO(float); else if (next_dt == DT_F16) GO(f16); else if (next_dt == DT_BF16) GO(bf16); else return LI_BAD_ARG;
 #undef GO
 #undef GO1
@@ -471,6 +486,22 @@ __global__ void token_shift_kernel(const float* __restrict__ x, const float* __r
     const float* xr = x + (int64_t)t * d;
     TO* o = out + (int64_t)t * d;
     const int64_t apart = (int64_t)gridDim.x * d;
+    if ((d & 3) == 0) {                                  // four channels a thread at a time
+        struct alignas(4 * sizeof(TO)) Out4 { TO v[4]; };
+        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+        for (int i = 4 * threadIdx.x; i < d; i += 4 * blockDim.x) {
+            const f32x4 h = *(const f32x4*)(xr + i), p = prev ? *(const f32x4*)(prev + i) : zero;
+            for (int m = 0; m < n_mix; ++m) {
+                const f32x4 w = *(const f32x4*)(mu + (int64_t)m * d + i);
+                Out4 r;
+#pragma unroll
+                for (int k = 0; k < 4; ++k) r.v[k] = from_f32<TO>(h[k] + (p[k] - h[k]) * w[k]);
+                *(Out4*)(o + m * apart + i) = r;
+            }
+            if (single) *(f32x4*)(st + i) = h;
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < d; i += blockDim.x) {
         const float h = xr[i], p = prev ? prev[i] : 0.f;
         for (int m = 0; m < n_mix; ++m) o[m * apart + i] = from_f32<TO>(h + (p - h) * mu[(int64_t)m * d + i]);

@@ -1,13 +1,20 @@
 // Recurrent mixers with a float32 state per sequence: the gated delta rule, the selective scan with a decay for every
 // channel and state, and the time mixing with a decay for every key channel and a bonus for the current token.  Each
-// has a kernel that walks a sequence's tokens in order (decode steps, float32 models), and a form for the prompts of a
-// 16-bit model that works on many tokens at a time.  Every size is a run-time value.  Unit norms, decays and their
+// has a kernel that walks a sequence's tokens in order (decode steps, float32 models); for the prompts of a 16-bit model
+// the selective scan runs in segments side by side, the other two in recurrent_chunks.hip.  Every size is a run-time value.  Unit norms, decays and their
 // logarithms, step sizes, gates of the recurrences and the states are float32 whatever the type of the matrices.
 #include "common.h"
+#include "conv.h"
 
 __device__ __forceinline__ float rc_sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float rc_silu(float z) { return z / (1.f + expf(-z)); }
-__device__ __forceinline__ float rc_softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+// log(1 + e^z) = max(z, 0) + log(1 + u), u = e^-|z|; with w = 1 + u as rounded, log(1 + u) = log(w) u / (w - 1) to the last
+// bits (the rounding of w cancels), and u itself where w is 1.
+__device__ __forceinline__ float rc_softplus(float z) {
+    const float u = __builtin_amdgcn_exp2f(-fabsf(z) * 1.4426950408889634f), w = 1.f + u, d = w - 1.f;
+    const float l = d == 0.f ? u : __builtin_amdgcn_logf(w) * 0.6931471805599453f * u * __builtin_amdgcn_rcpf(d);
+    return fmaxf(z, 0.f) + l;
+}
 
 #define DISPATCH_T(dt, CALL)                                     \
     do {                                                         \
@@ -37,89 +44,149 @@ struct Segments {
     const int* seq_nseg;
 };
 
-// One column of float32 rows through a causal convolution over time (weights [channels, taps], the last tap the
-// token's own), then silu: inputs before the first token that a sequence brings to the step come from `hist` [slots,
-// taps - 1, channels] (oldest first), before position 0 they are zero.  `inside`: how many tokens before this one its
-// sequence has in this step (at most taps - 1 of them matter).
-struct Conv {
-    const float* w;
-    const float* b;          // [channels] or null
-    const float* hist;
-    int taps, channels;
-};
-__device__ __forceinline__ int tokens_inside(const int* tok_slot, int t, int slot, int taps) {
-    int inside = 0;
-    while (inside < taps - 1 && t - inside - 1 >= 0 && tok_slot[t - inside - 1] == slot) ++inside;
-    return inside;
-}
-__device__ __forceinline__ float conv_silu_at(const float* row, int64_t stride, int c, const Conv& cv, int inside, int p, int slot) {
-    float acc = cv.b ? cv.b[c] : 0.f;
-    const float* h = cv.hist + (int64_t)slot * (cv.taps - 1) * cv.channels;
-    for (int back = 0; back < cv.taps; ++back) {
-        float u = 0.f;
-        if (back <= inside) u = row[c - back * stride];
-        else if (p - back >= 0) u = h[(int64_t)(cv.taps - 1 - (back - inside)) * cv.channels + c];
-        acc += cv.w[(int64_t)c * cv.taps + (cv.taps - 1 - back)] * u;
-    }
-    return rc_silu(acc);
-}
-
 // ---------------------------------------------------------------------------
 // The gated delta rule.  Per sequence and head h with key head e = h / (H / G), S [d, dv] float32:
 //   S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q
 // q, k, v: columns of the rows `proj` (from col0 on: q [G, d], k [G, d], v [H, dv]) behind a convolution and silu; q
 // and k then unit vectors, x / sqrt(sum x^2 + 1e-6), q times d^(-1/2); beta = sigmoid(proj[b_col + h]),
 // g = exp(-exp(A_log[h]) softplus(proj[a_col + h] + dt_bias[h])).
-// delta_prep_kernel: a wave a (token, key head), (token, 64 values) or (token) for the gates.  `qkv` [T, 2 G d + H dv]
-// float32 receives q and k as unit vectors and v; `gates` [T, H, 2] log g and beta; `kq` [T, G] k . q.
+// delta_prep_kernel: a wave a key head, 64 values or the gates, for `tile` consecutive tokens of the step; the gates go to
+// `gates` [T, H, 2], log g (no less than LOG_DECAY_MIN, whose exponential is 0 next to anything) and beta.  For the kernel
+// that walks token by token: q and k as unit vectors and v to `rows` [T, 2 G d + H dv] float32, k . q to `aux` [T, G].  For
+// the chunked kernels (HALF): q, k and v behind silu to `rows` in bfloat16, d^(-1/2) / |q| and 1 / |k| of what was written to
+// `aux` [T, G, 2].
 // ---------------------------------------------------------------------------
 #define DELTA_UNIT_EPS 1e-6f
 #define DELTA_MAXV 4             // keys up to 64 * DELTA_MAXV wide
+#define LOG_DECAY_MIN -88.f
 
-__global__ __launch_bounds__(256) void delta_prep_kernel(const float* __restrict__ proj, int stride, int col0, int b_col,
-                                                         int a_col, Conv cv, Steps st, const float* __restrict__ A_log,
-                                                         const float* __restrict__ dt_bias, float* __restrict__ qkv,
-                                                         float* __restrict__ gates, float* __restrict__ kq, int H, int G,
-                                                         int d, int dv) {
-    const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const int p = st.pos[t], slot = st.tok_slot[t], inside = tokens_inside(st.tok_slot, t, slot, cv.taps);
-    const float* row = proj + (int64_t)t * stride + col0;
-    float* out = qkv + (int64_t)t * cv.channels;
-    const int nv = (H * dv + 63) / 64, units = G + nv + 1;
-    const float qs = 1.f / sqrtf((float)d);
-    for (int u = blockIdx.y * 4 + wave; u < units; u += gridDim.y * 4) {
-        if (u < G) {
-            float q[DELTA_MAXV], k[DELTA_MAXV], sq = 0.f, sk = 0.f, dot = 0.f;
+struct DeltaPrep {
+    const float* proj;
+    int stride, col0, b_col, a_col;
+    const float* w;              // [channels, taps]
+    const float* hist;           // [slots, taps - 1, channels]
+    const int* pos;
+    const int* tok_slot;
+    const float* A_log;
+    const float* dt_bias;
+    void* rows;
+    float* gates;
+    float* aux;
+    int n, taps, H, G, d, dv, tile;
+};
+
+// Up to NV channels a lane, c0 + 64 v + lane, from token to token.
+template <int TAPS, int NV>
+struct ConvLanes {
+    static constexpr int K = TAPS ? TAPS : 1;
+    ConvWindow<K> win[NV];
+    float w[NV][K];
+    __device__ __forceinline__ void weights(const DeltaPrep& p, int c0, int lane, int count) {
+        if (TAPS) {
 #pragma unroll
-            for (int v = 0; v < DELTA_MAXV; ++v) {
-                const int i = v * 64 + lane;
-                q[v] = k[v] = 0.f;
-                if (i < d) {
-                    q[v] = conv_silu_at(row, stride, u * d + i, cv, inside, p, slot);
-                    k[v] = conv_silu_at(row, stride, (G + u) * d + i, cv, inside, p, slot);
+            for (int v = 0; v < NV; ++v)
+                if (v * 64 + lane < count) {
+#pragma unroll
+                    for (int j = 0; j < K; ++j) w[v][j] = p.w[(int64_t)(c0 + v * 64 + lane) * K + j];
                 }
+        }
+    }
+    // silu of the convolution at token t, 0 beyond `count`
+    __device__ __forceinline__ void at(const DeltaPrep& p, int channels, int c0, int lane, int count, int t, int slot, bool fresh, int inside,
+                                       float (&out)[NV]) {
+        const float* h = p.hist + (int64_t)slot * (p.taps - 1) * channels;
+#pragma unroll
+        for (int v = 0; v < NV; ++v) {
+            out[v] = 0.f;
+            if (v * 64 + lane < count) {
+                const int c = c0 + v * 64 + lane;
+                const float* x = p.proj + (int64_t)t * p.stride + p.col0 + c;
+                float acc;
+                if (TAPS) {
+                    if (fresh) win[v].start(x, p.stride, inside, p.pos[t], h, channels, c);
+                    else win[v].next(*x);
+                    acc = win[v].sum(w[v], 0.f);
+                } else acc = conv_at(x, p.stride, inside, p.pos[t], h, channels, c, p.w, p.taps, 0.f);
+                out[v] = rc_silu(acc);
+            }
+        }
+    }
+};
+
+template <int TAPS, bool HALF, int NV>
+__global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrep p) {
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), H = p.H, G = p.G, d = p.d;
+    const int t0 = blockIdx.x * p.tile, t1 = min(p.n, t0 + p.tile), channels = 2 * G * d + H * p.dv;
+    const int nv = (H * p.dv + 63) / 64, units = G + nv + 1, u = blockIdx.y * 4 + wave;
+    if (u >= units) return;
+    const float qs = 1.f / sqrtf((float)d);
+    int last = -1;
+    if (u < G) {
+        ConvLanes<TAPS, NV> cq, ck;
+        cq.weights(p, u * d, lane, d);
+        ck.weights(p, (G + u) * d, lane, d);
+        for (int t = t0; t < t1; ++t) {
+            const int slot = p.tok_slot[t];
+            const bool fresh = slot != last;
+            const int inside = fresh || !TAPS ? conv_inside(p.tok_slot, t, slot, p.taps) : 0;
+            last = slot;
+            float q[NV], k[NV], sq = 0.f, sk = 0.f;
+            cq.at(p, channels, u * d, lane, d, t, slot, fresh, inside, q);
+            ck.at(p, channels, (G + u) * d, lane, d, t, slot, fresh, inside, k);
+#pragma unroll
+            for (int v = 0; v < NV; ++v) {
+                if (HALF) { q[v] = (float)(bf16)q[v]; k[v] = (float)(bf16)k[v]; }
                 sq += q[v] * q[v];
                 sk += k[v] * k[v];
             }
             const float rq = qs / sqrtf(wave_sum(sq) + DELTA_UNIT_EPS), rk = 1.f / sqrtf(wave_sum(sk) + DELTA_UNIT_EPS);
+            if (HALF) {
+                bf16* out = (bf16*)p.rows + (int64_t)t * channels;
 #pragma unroll
-            for (int v = 0; v < DELTA_MAXV; ++v) {
-                const int i = v * 64 + lane;
-                q[v] *= rq;
-                k[v] *= rk;
-                dot += q[v] * k[v];
-                if (i < d) { out[u * d + i] = q[v]; out[(G + u) * d + i] = k[v]; }
+                for (int v = 0; v < NV; ++v) {
+                    const int i = v * 64 + lane;
+                    if (i < d) { out[u * d + i] = (bf16)q[v]; out[(G + u) * d + i] = (bf16)k[v]; }
+                }
+                if (lane == 0) { p.aux[((int64_t)t * G + u) * 2] = rq; p.aux[((int64_t)t * G + u) * 2 + 1] = rk; }
+            } else {
+                float* out = (float*)p.rows + (int64_t)t * channels;
+                float dot = 0.f;
+#pragma unroll
+                for (int v = 0; v < NV; ++v) {
+                    const int i = v * 64 + lane;
+                    q[v] *= rq;
+                    k[v] *= rk;
+                    dot += q[v] * k[v];
+                    if (i < d) { out[u * d + i] = q[v]; out[(G + u) * d + i] = k[v]; }
+                }
+                dot = wave_sum(dot);
+                if (lane == 0) p.aux[(int64_t)t * G + u] = dot;
             }
-            dot = wave_sum(dot);
-            if (lane == 0) kq[(int64_t)t * G + u] = dot;
-        } else if (u < G + nv) {
-            const int c = 2 * G * d + (u - G) * 64 + lane;
-            if (c < cv.channels) out[c] = conv_silu_at(row, stride, c, cv, inside, p, slot);
-        } else {
-            const float* r = proj + (int64_t)t * stride;
+        }
+    } else if (u < G + nv) {
+        const int c0 = 2 * G * d + (u - G) * 64, count = min(64, channels - c0);
+        ConvLanes<TAPS, 1> cv;
+        cv.weights(p, c0, lane, count);
+        for (int t = t0; t < t1; ++t) {
+            const int slot = p.tok_slot[t];
+            const bool fresh = slot != last;
+            const int inside = fresh || !TAPS ? conv_inside(p.tok_slot, t, slot, p.taps) : 0;
+            last = slot;
+            float v[1];
+            cv.at(p, channels, c0, lane, count, t, slot, fresh, inside, v);
+            if (lane < count) {
+                const int64_t at = (int64_t)t * channels + c0 + lane;
+                if (HALF) ((bf16*)p.rows)[at] = (bf16)v[0];
+                else ((float*)p.rows)[at] = v[0];
+            }
+        }
+    } else {
+        for (int t = t0; t < t1; ++t) {
+            const float* r = p.proj + (int64_t)t * p.stride;
             for (int h = lane; h < H; h += 64) {
-                gates[((int64_t)t * H + h) * 2] = -expf(A_log[h]) * rc_softplus(r[a_col + h] + dt_bias[h]);
-                gates[((int64_t)t * H + h) * 2 + 1] = rc_sigmoid(r[b_col + h]);
+                float* g = p.gates + ((int64_t)t * H + h) * 2;
+                g[0] = fmaxf(-expf(p.A_log[h]) * rc_softplus(r[p.a_col + h] + p.dt_bias[h]), LOG_DECAY_MIN);
+                g[1] = rc_sigmoid(r[p.b_col + h]);
             }
         }
     }
@@ -181,19 +248,25 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void delta_scan_kernel(const float
     }
 }
 
+// half 0: rows float32, aux [T, G]; half 1: rows bfloat16, aux [T, G, 2] (see delta_prep_kernel).
 extern "C" int li_delta_prep(const float* proj, int stride, int col0, int b_col, int a_col, const float* conv_w, int taps,
                              const float* hist, const int* pos, const int* tok_slot, const float* A_log, const float* dt_bias,
-                             float* qkv, float* gates, float* kq, int n, int H, int G, int d, int dv, hipStream_t stream) {
+                             void* rows, float* gates, float* aux, int half, int n, int H, int G, int d, int dv, hipStream_t stream) {
     if (n <= 0) return LI_OK;
-    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || taps < 1 || taps > 16 || !hist) return LI_BAD_ARG;
+    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || taps < 1 || taps > CONV_MAX_TAPS || !hist) return LI_BAD_ARG;
     if (d > 64 * DELTA_MAXV) return LI_UNSUPPORTED;
     const int channels = 2 * G * d + H * dv;
     if (col0 < 0 || col0 + channels > stride || b_col < 0 || b_col + H > stride || a_col < 0 || a_col + H > stride) return LI_BAD_ARG;
-    Conv cv{conv_w, nullptr, hist, taps, channels};
-    Steps st{pos, tok_slot, nullptr, nullptr, nullptr};
+    const DeltaPrep p{proj, stride, col0, b_col, a_col, conv_w, hist, pos, tok_slot, A_log, dt_bias, rows, gates, aux, n, taps, H, G, d, dv,
+                      n >= 256 && taps == 4 ? 8 : 1};
     const int units = G + (H * dv + 63) / 64 + 1;
-    delta_prep_kernel<<<dim3(n, (units + 3) / 4), 256, 0, stream>>>(proj, stride, col0, b_col, a_col, cv, st, A_log, dt_bias, qkv,
-                                                                    gates, kq, H, G, d, dv);
+    dim3 grid((n + p.tile - 1) / p.tile, (units + 3) / 4);
+#define GO1(TAPS, HALF) do { if (d <= 64) delta_prep_kernel<TAPS, HALF, 1><<<grid, 256, 0, stream>>>(p); \
+        else if (d <= 128) delta_prep_kernel<TAPS, HALF, 2><<<grid, 256, 0, stream>>>(p); else delta_prep_kernel<TAPS, HALF, 4><<<grid, 256, 0, stream>>>(p); } while (0)
+#define GO(TAPS) do { if (half) GO1(TAPS, true); else GO1(TAPS, false); } while (0)
+    if (taps == 4) GO(4); else GO(0);
+#undef GO
+#undef GO1
     LI_CHECK_LAUNCH();
     return LI_OK;
 }
@@ -380,55 +453,39 @@ extern "C" int li_sel_scan(const void* x, int dt, const float* raw, const float*
 // float32 (rows: key channels), w = exp(-exp(raw)) per key channel:
 //   o = (S + diag(u) k v^T)^T r;   S <- diag(w) S + k v^T
 // r, k, v [T, H d] in type T, raw [T, H d] float32 (its bias included), u [H, d].
-// A workgroup of 4 waves per (sequence or segment, head, 64 columns); a lane keeps its column's NR rows of its wave's share
-// in registers, the waves' shares of o meet in LDS.  PASS 0, 1 and 3 as above (a segment's decay: exp of the sum of
-// its logarithms, one a key channel).
+// A workgroup of 4 waves per (sequence, head, 64 columns); a lane keeps its column's NR rows of its wave's share in
+// registers, the waves' shares of o meet in LDS.
 // ---------------------------------------------------------------------------
-template <class T, int NR, int PASS>
+template <class T, int NR>
 __global__ __launch_bounds__(64 * SCAN_WAVES) void wkv_scan_kernel(const T* __restrict__ r_, const T* __restrict__ k_,
                                                                    const T* __restrict__ v_, const float* __restrict__ raw,
                                                                    const float* __restrict__ bonus, float* __restrict__ state,
-                                                                   Steps st, Segments sg, float* __restrict__ seg_state,
-                                                                   float* __restrict__ seg_lw, float* __restrict__ y, int H, int d) {
+                                                                   Steps st, float* __restrict__ y, int H, int d) {
     constexpr int DP = NR * SCAN_WAVES;
     __shared__ __attribute__((aligned(16))) float sr[3][DP], sk[3][DP], sw[3][DP];
     __shared__ float part[2][SCAN_WAVES][64], ruk[3][SCAN_WAVES];
-    const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = blockIdx.z * 64 + lane, r0 = wave * NR;
-    int q0, n;
-    float* S;
-    if (PASS == 0) {
-        const int seq = blockIdx.x;
-        q0 = st.seq_qstart ? st.seq_qstart[seq] : seq;
-        n = st.seq_qlen ? st.seq_qlen[seq] : 1;
-        S = state + (((int64_t)st.seq_slot[seq] * H + h) * d) * d + col;
-    } else {
-        const int seg = blockIdx.x;
-        q0 = st.seq_qstart[sg.seg_seq[seg]] + sg.seg_t0[seg];
-        n = sg.seg_n[seg];
-        S = seg_state + (((int64_t)seg * H + h) * d) * d + col;
-    }
+    const int seq = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int col = blockIdx.z * 64 + lane, r0 = wave * NR;
+    const int q0 = st.seq_qstart ? st.seq_qstart[seq] : seq, n = st.seq_qlen ? st.seq_qlen[seq] : 1;
     if (n <= 0) return;
     const bool live = col < d;
+    float* S = state + (((int64_t)st.seq_slot[seq] * H + h) * d) * d + col;
     float s[NR];
 #pragma unroll
-    for (int r = 0; r < NR; ++r) s[r] = (PASS != 1 && live && r0 + r < d) ? S[(int64_t)(r0 + r) * d] : 0.f;
-    float lw_sum = 0.f;
+    for (int r = 0; r < NR; ++r) s[r] = (live && r0 + r < d) ? S[(int64_t)(r0 + r) * d] : 0.f;
     static_assert(DP <= 64 * SCAN_WAVES, "a thread a key channel");
     const float ub = tid < d ? bonus[h * d + tid] : 0.f;
     auto stage = [&](int t) {
         const int64_t at = (int64_t)(q0 + t) * H * d + h * d;
-        float rr = 0.f, kk = 0.f, lw = 0.f;
+        float rr = 0.f, kk = 0.f, w = 0.f;
         if (tid < d) {
+            rr = to_f32(r_[at + tid]);
             kk = to_f32(k_[at + tid]);
-            lw = -expf(raw[at + tid]);
-            if (PASS != 1) rr = to_f32(r_[at + tid]);
+            w = expf(-expf(raw[at + tid]));
         }
-        if (tid < DP) { sr[t % 3][tid] = rr; sk[t % 3][tid] = kk; sw[t % 3][tid] = expf(lw); }
-        lw_sum += lw;
-        if (PASS != 1) {
-            const float b = wave_sum(rr * ub * kk);
-            if (lane == 0) ruk[t % 3][wave] = b;
-        }
+        if (tid < DP) { sr[t % 3][tid] = rr; sk[t % 3][tid] = kk; sw[t % 3][tid] = w; }
+        const float b = wave_sum(rr * ub * kk);
+        if (lane == 0) ruk[t % 3][wave] = b;
     };
     stage(0);
     __syncthreads();
@@ -439,67 +496,36 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void wkv_scan_kernel(const T* __re
         float a = 0.f;
 #pragma unroll
         for (int r = 0; r < NR; ++r) {
-            if (PASS != 1) a += s[r] * rr[r];
+            a += s[r] * rr[r];
             s[r] = w[r] * s[r] + k[r] * v;
         }
-        if (PASS != 1) part[t & 1][wave][lane] = a;
+        part[t & 1][wave][lane] = a;
         if (t + 1 < n) stage(t + 1);
         __syncthreads();
-        if (PASS != 1 && wave == 0 && live) {
+        if (wave == 0 && live) {
             float o = 0.f, b = 0.f;
 #pragma unroll
             for (int i = 0; i < SCAN_WAVES; ++i) { o += part[t & 1][i][lane]; b += ruk[t % 3][i]; }
             y[tok * H * d + h * d + col] = o + b * v;
         }
     }
-    if (PASS != 3 && live) {
+    if (live) {
 #pragma unroll
         for (int r = 0; r < NR; ++r) if (r0 + r < d) S[(int64_t)(r0 + r) * d] = s[r];
     }
-    if (PASS == 1 && blockIdx.z == 0 && tid < d) seg_lw[((int64_t)blockIdx.x * H + h) * d + tid] = lw_sum;
-}
-
-// One thread per element of a head's state: walks a sequence's segments in order, a decay a key channel.
-__global__ void wkv_combine_kernel(float* __restrict__ state, const int* __restrict__ seq_slot, Segments sg,
-                                   float* __restrict__ seg_state, const float* __restrict__ seg_lw, int H, int d) {
-    const int seq = blockIdx.x, h = blockIdx.y, e = blockIdx.z * blockDim.x + threadIdx.x, per = d * d;
-    if (e >= per) return;
-    const int g0 = sg.seq_seg0[seq], ng = sg.seq_nseg[seq], row = e / d;
-    float* S = state + ((int64_t)seq_slot[seq] * H + h) * per + e;
-    float s = *S;
-    for (int g = g0; g < g0 + ng; ++g) {
-        float* L = seg_state + ((int64_t)g * H + h) * per + e;
-        const float own = *L;
-        *L = s;
-        s = expf(seg_lw[((int64_t)g * H + h) * d + row]) * s + own;
-    }
-    *S = s;
 }
 
 extern "C" int li_wkv_scan(const void* r, const void* k, const void* v, int dt, const float* raw, const float* bonus, float* state,
                            const int* seq_slot, const int* seq_qstart, const int* seq_qlen, float* y, int n_seqs, int H, int d,
-                           const int* seg_seq, const int* seg_t0, const int* seg_n, const int* seq_seg0, const int* seq_nseg,
-                           int n_segs, float* seg_state, float* seg_lw, hipStream_t stream) {
+                           hipStream_t stream) {
     if (n_seqs <= 0) return LI_OK;
     if (H <= 0 || d <= 0) return LI_BAD_ARG;
     if (d > 256) return LI_UNSUPPORTED;
     Steps st{nullptr, nullptr, seq_slot, seq_qstart, seq_qlen};
-    Segments sg{seg_seq, seg_t0, seg_n, seq_seg0, seq_nseg};
-#define GO1(NR, PASS, ITEMS) wkv_scan_kernel<T, NR, PASS><<<dim3(ITEMS, H, (d + 63) / 64), 64 * SCAN_WAVES, 0, stream>>>((const T*)r, \
-        (const T*)k, (const T*)v, raw, bonus, state, st, sg, seg_state, seg_lw, y, H, d)
-#define GO(PASS, ITEMS)                                                                                               \
-    do {                                                                                                              \
-        if (d <= 16) GO1(4, PASS, ITEMS); else if (d <= 32) GO1(8, PASS, ITEMS); else if (d <= 64) GO1(16, PASS, ITEMS); \
-        else if (d <= 128) GO1(32, PASS, ITEMS); else GO1(64, PASS, ITEMS);                                            \
-    } while (0)
-    if (n_segs <= 0) {
-        DISPATCH_T(dt, GO(0, n_seqs));
-    } else {
-        if (!seq_qstart || !seq_qlen || !seg_seq || !seg_t0 || !seg_n || !seq_seg0 || !seq_nseg || !seg_state || !seg_lw) return LI_BAD_ARG;
-        DISPATCH_T(dt, GO(1, n_segs));
-        wkv_combine_kernel<<<dim3(n_seqs, H, (d * d + 255) / 256), 256, 0, stream>>>(state, seq_slot, sg, seg_state, seg_lw, H, d);
-        DISPATCH_T(dt, GO(3, n_segs));
-    }
+#define GO1(T, NR) wkv_scan_kernel<T, NR><<<dim3(n_seqs, H, (d + 63) / 64), 64 * SCAN_WAVES, 0, stream>>>((const T*)r, (const T*)k, \
+        (const T*)v, raw, bonus, state, st, y, H, d)
+#define GO(T) do { if (d <= 16) GO1(T, 4); else if (d <= 32) GO1(T, 8); else if (d <= 64) GO1(T, 16); else if (d <= 128) GO1(T, 32); else GO1(T, 64); } while (0)
+    if (dt == DT_F32) GO(float); else if (dt == DT_BF16) GO(bf16); else return LI_BAD_ARG;
 #undef GO
 #undef GO1
     LI_CHECK_LAUNCH();

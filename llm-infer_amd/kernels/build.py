@@ -27,7 +27,8 @@ CORE_SOURCES = ("elementwise.hip", "gemm.hip", "gemm_prefill.hip", "sampling.hip
 ATTN_SOURCE = "attention.hip"
 MIXER_SOURCES = ("mixers.hip",)
 # the headers a library's sources include (its stamp covers them)
-HEADERS = {"libli_core.so": ("common.h", "gemm_common.h", "no_alloc.h")}
+HEADERS = {"libli_core.so": ("common.h", "gemm_common.h", "no_alloc.h"), "libli_hybrid.so": ("common.h", "conv.h"),
+           "libli_recurrent.so": ("common.h", "conv.h")}
 DEFAULT_HEADERS = ("common.h",)
 FLAGS = ["--offload-arch=" + ARCH, "-O3", "-std=c++17", "-fPIC",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unused-command-line-argument"]
@@ -204,11 +205,11 @@ def hybrid_library(force=False):
     return _load("libli_hybrid.so", HYBRID_SOURCES, (), force)
 
 
-RECURRENT_SOURCES = ("recurrent.hip",)
+RECURRENT_SOURCES = ("recurrent.hip", "recurrent_chunks.hip")
 
 
 def recurrent_library(force=False):
-    """The recurrent mixers' kernels (csrc/recurrent.hip: the gated delta rule, the selective scan with a decay for every
+    """The recurrent mixers' kernels (csrc/recurrent.hip, and csrc/recurrent_chunks.hip for prompts: the gated delta rule, the selective scan with a decay for every
     channel and state, time mixing with a decay for every key channel): a library of its own, as the mixers' is."""
     return _load("libli_recurrent.so", RECURRENT_SOURCES, (), force)
 

@@ -16,6 +16,7 @@ from ..tensor import Tensor
 PAGE = 64
 DT = {torch.float32: 0, torch.float16: 1, torch.bfloat16: 2}
 EPI_STORE, EPI_ADD, EPI_SWIGLU, EPI_ROPE, EPI_GEGLU, EPI_BIAS, EPI_CLAMPGLU = 0, 1, 2, 3, 4, 5, 6
+EPI_ACTS = {None: 0, "relu2": 1, "tanh": 2}       # activations that EPI_BIAS can apply
 GATED = (EPI_SWIGLU, EPI_GEGLU, EPI_CLAMPGLU)   # gate and up rows interleaved in W, act(gate) * up written
 _STATUS = {1: "bad argument", 2: "unsupported size or alignment", 3: "HIP launch error"}
 
@@ -197,18 +198,19 @@ def lazy_rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype):
 
 class _GluParams(ctypes.Structure):
     _fields_ = [("bias", c_void_p), ("limit", c_float), ("tail_limit", c_float), ("alpha", c_float), ("shift", c_float),
-                ("tail_col", c_int)]
+                ("tail_col", c_int), ("act", c_int)]
 
 
 def glu_params(bias=None, limit: float = 1.0, tail_limit: float | None = None, alpha: float = 1.702, shift: float = 1.0,
-               tail_col: int | None = None):
-    """What ``linear`` needs for EPI_BIAS (``bias`` float32 [N]) and EPI_CLAMPGLU (gate and up columns interleaved; a bias
+               tail_col: int | None = None, act: str | None = None):
+    """What ``linear`` needs for EPI_BIAS (``bias`` float32 [N]; ``act`` "relu2", the square of relu, or "tanh" of the sums and
+    the bias, which may then be None) and EPI_CLAMPGLU (gate and up columns interleaved; a bias
     for every column or None; g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + shift); the
     outputs from ``tail_col`` on take ``tail_limit``).  Keeps the bias alive as long as it lives itself."""
     _need(bias is None or (bias.dtype == torch.float32 and bias.dim() == 1 and bias.is_contiguous() and bias.is_cuda),
           "a float32 bias on the device")
     p = _GluParams(bias.data_ptr() if bias is not None else None, limit, limit if tail_limit is None else tail_limit, alpha, shift,
-                   (1 << 30) if tail_col is None else tail_col)
+                   (1 << 30) if tail_col is None else tail_col, EPI_ACTS[act])
     p._bias = bias
     return p
 
@@ -292,7 +294,7 @@ def linear(x: torch.Tensor, w, mode: int = EPI_STORE, out: torch.Tensor | None =
         _need(out is not None and out.dtype == torch.float32, "add epilogue needs a float32 output")
     rs = ctypes.byref(_rope) if _rope is not None else None
     if mode in (EPI_BIAS, EPI_CLAMPGLU):
-        _need(isinstance(params, _GluParams) and (mode != EPI_BIAS or (params._bias is not None and params._bias.numel() == n)) and
+        _need(isinstance(params, _GluParams) and (mode != EPI_BIAS or params._bias is not None or params.act) and
               (params._bias is None or params._bias.numel() == n), "this epilogue needs its parameters (glu_params), a bias for every column")
         rs = ctypes.byref(params)
     if mode == EPI_ROPE:
@@ -1224,7 +1226,7 @@ def polynorm(z, coef, eps, out_dtype) -> torch.Tensor:
 # routed experts, a scaled embedding with sinusoidal positions
 # ---------------------------------------------------------------------------
 _hybrid = None
-ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu2": 3, "tanh": 4}      # (tanh: not an expert's)
+ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu2": 3}
 
 
 def hybrid():
@@ -1264,7 +1266,7 @@ def concat_cast(a, b, dtype) -> torch.Tensor:
 
 
 def activation(z, kind: str, out_dtype) -> torch.Tensor:
-    """act(z) for float32 z in ``out_dtype``; kind: gelu (erf), gelu_tanh, silu, relu2 (the square of relu), tanh."""
+    """act(z) for float32 z in ``out_dtype``; kind: gelu (erf), gelu_tanh, silu, relu2 (the square of relu)."""
     _dev(z)
     _need(z.dtype == torch.float32 and kind in ACTIVATIONS and out_dtype in DT, f"activation {kind!r}: float32 in, one of {', '.join(ACTIVATIONS)}")
     out = torch.empty(z.shape, dtype=out_dtype, device=z.device)
@@ -1825,7 +1827,7 @@ def expert_act(z, weights, n_blocks, ff, tail, kind: str, on_input: bool, out_dt
     _dev(z, weights, idx)
     _f32_rows(z, "expert rows")
     rows = z.shape[0]
-    _need(kind in ACTIVATIONS and kind != "tanh" and z.shape[1] == n_blocks * ff + tail, "expert_act: [rows, blocks * ff + tail], a known activation")
+    _need(kind in ACTIVATIONS and z.shape[1] == n_blocks * ff + tail, "expert_act: [rows, blocks * ff + tail], a known activation")
     wcols = 0
     if weights is not None:
         _need(weights.dtype == torch.float32 and weights.dim() == 2, "expert_act: float32 weights [tokens, columns]")
@@ -1993,12 +1995,14 @@ def _segment_args(segments, ctx, qstart, what):
     return tuple(_ptr(segments[name]) for name in ("seg_seq", "seg_t0", "seg_n", "seq_seg0", "seq_nseg")) + (k,)
 
 
-def delta_prepare(proj, col0, b_col, a_col, conv_w, history, a_log, dt_bias, ctx, heads, kv_heads, d, dv):
+def delta_prepare(proj, col0, b_col, a_col, conv_w, history, a_log, dt_bias, ctx, heads, kv_heads, d, dv, chunked: bool = False):
     """What the gated delta rule reads of a step's tokens, from the float32 rows ``proj``: the columns q [kv_heads, d],
     k [kv_heads, d], v [heads, dv] from ``col0`` on behind a causal convolution (``conv_w`` float32 [channels, taps],
     ``history`` float32 [slots, taps - 1, channels], brought up to date) and silu, q and k as unit vectors and q times
     d^(-1/2); the decays' logarithms -exp(a_log) softplus(proj[a_col + h] + dt_bias) and beta = sigmoid(proj[b_col + h]).
-    Returns float32 (rows [T, channels], gates [T, heads, 2], k . q [T, kv_heads])."""
+    Returns float32 (rows [T, channels], gates [T, heads, 2], k . q [T, kv_heads]) for ``delta_scan``; ``chunked``: for
+    ``delta_chunks``, the rows in bfloat16 before the division by the norms, and in the third place d^(-1/2) / |q| and
+    1 / |k| [T, kv_heads, 2]."""
     _dev(proj, conv_w, history, a_log, dt_bias)
     _f32_rows(proj, "delta projections")
     t, channels, taps = proj.shape[0], 2 * kv_heads * d + heads * dv, conv_w.shape[1]
@@ -2012,15 +2016,15 @@ def delta_prepare(proj, col0, b_col, a_col, conv_w, history, a_log, dt_bias, ctx
     _i32(ctx.pos, t, "positions")
     _i32(ctx.tok_slot, t, "slots")
     dev = proj.device
-    qkv = torch.empty((t, channels), dtype=torch.float32, device=dev)
+    qkv = torch.empty((t, channels), dtype=torch.bfloat16 if chunked else torch.float32, device=dev)
     gates = torch.empty((t, heads, 2), dtype=torch.float32, device=dev)
-    kq = torch.empty((t, kv_heads), dtype=torch.float32, device=dev)
+    aux = torch.empty((t, kv_heads, 2) if chunked else (t, kv_heads), dtype=torch.float32, device=dev)
     _check(recurrent().li_delta_prep(_ptr(proj), proj.shape[1], col0, b_col, a_col, _ptr(conv_w), taps, _ptr(history), _ptr(ctx.pos),
-                                     _ptr(ctx.tok_slot), _ptr(a_log), _ptr(dt_bias), _ptr(qkv), _ptr(gates), _ptr(kq), t, heads,
-                                     kv_heads, d, dv, _stream()), "delta_prep")
+                                     _ptr(ctx.tok_slot), _ptr(a_log), _ptr(dt_bias), _ptr(qkv), _ptr(gates), _ptr(aux), int(bool(chunked)),
+                                     t, heads, kv_heads, d, dv, _stream()), "delta_prep")
     if taps > 1:
         conv_history(proj, col0, channels, taps, history, ctx)
-    return qkv, gates, kq
+    return qkv, gates, aux
 
 
 def delta_scan(qkv, gates, kq, state, ctx, heads, kv_heads, d, dv) -> torch.Tensor:
@@ -2035,6 +2039,32 @@ def delta_scan(qkv, gates, kq, state, ctx, heads, kv_heads, d, dv) -> torch.Tens
     y = torch.empty((t, heads * dv), dtype=torch.float32, device=qkv.device)
     _check(recurrent().li_delta_scan(_ptr(qkv), _ptr(gates), _ptr(kq), _ptr(state), _ptr(seq_slot), _ptr(qstart), _ptr(qlen),
                                      _ptr(y), ctx.n_seqs, heads, kv_heads, d, dv, _stream()), "delta_scan")
+    return y
+
+
+def _scratch(n_elems: int, dtype, device):
+    return torch.empty((n_elems,), dtype=dtype, device=device)
+
+
+def delta_chunks(rows, gates, norms, state, ctx, heads, kv_heads, d, dv) -> torch.Tensor:
+    """What ``delta_scan`` computes, for the prompts of a 16-bit model: 32 tokens at a time on the matrix cores, on what
+    ``delta_prepare(chunked=True)`` left.  Returns float32 [T, heads * dv]."""
+    _dev(rows, gates, norms, state)
+    t = rows.shape[0]
+    _need(rows.dtype == torch.bfloat16 and rows.shape == (t, 2 * kv_heads * d + heads * dv) and gates.shape == (t, heads, 2)
+          and norms.shape == (t, kv_heads, 2) and 1 <= d <= 256, "delta rule: what delta_prepare(chunked=True) returns")
+    _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, d, dv), "delta state: float32 [slots, heads, d, dv]")
+    seq_slot, qstart, qlen = _seq_arrays(ctx, t)
+    _need(qstart is not None, "delta rule in chunks: per-sequence starts and lengths")
+    chunks, dev, lib = decay_chunks(ctx), rows.device, recurrent()
+    n = chunks["n_chunks"]
+    mats = _scratch(n * heads * lib.li_delta_chunk_elems(d, 0), torch.bfloat16, dev)
+    packs = _scratch(n * kv_heads * lib.li_delta_chunk_elems(d, 1), torch.bfloat16, dev)
+    coef = torch.empty((n, heads, 4, DECAY_CHUNK), dtype=torch.float32, device=dev)
+    y = torch.empty((t, heads * dv), dtype=torch.float32, device=dev)
+    _check(lib.li_delta_chunks(_ptr(rows), _ptr(norms), _ptr(gates), _ptr(state), _ptr(seq_slot), _ptr(qstart), _ptr(qlen),
+                               _ptr(chunks["chunk_seq"]), _ptr(chunks["chunk_t0"]), _ptr(chunks["seq_chunk0"]), n, _ptr(mats),
+                               _ptr(coef), _ptr(packs), _ptr(y), ctx.n_seqs, heads, kv_heads, d, dv, _stream()), "delta_chunks")
     return y
 
 
@@ -2070,25 +2100,43 @@ def selective_scan(x, raw, dt_bias, bc, b_col, c_col, z_rows, z_col, a2, d_skip,
     return out
 
 
-def wkv_scan(r, k, v, raw, bonus, state, ctx, heads, d, segments=None) -> torch.Tensor:
-    """Time mixing with a decay for every key channel: w = exp(-exp(raw)), o = (S + diag(bonus) k v^T)^T r,
-    S <- diag(w) S + k v^T per head.  r, k, v [T, heads * d] of one type, ``raw`` float32 of that shape, ``bonus`` float32
-    [heads, d]; ``state`` float32 [slots, heads, d, d] is read and left up to date.  ``segments``: as for
-    ``selective_scan``.  Returns float32 [T, heads * d]."""
+def _wkv_check(r, k, v, raw, bonus, state, heads, d):
     _dev(r, k, v, raw, bonus, state)
     t = r.shape[0]
     for x in (r, k, v, raw):
         _need(x.shape == (t, heads * d) and x.dtype == (torch.float32 if x is raw else r.dtype), "wkv: rows [T, heads * d] of one type, float32 decays")
-    _need(r.dtype in DT and 1 <= d <= 256 and bonus.dtype == torch.float32 and bonus.shape == (heads, d), "wkv: heads up to 256 wide, float32 bonus [heads, d]")
+    _need(1 <= d <= 256 and bonus.dtype == torch.float32 and bonus.shape == (heads, d), "wkv: heads up to 256 wide, float32 bonus [heads, d]")
     _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, d, d), "wkv state: float32 [slots, heads, d, d]")
+    return t
+
+
+def wkv_scan(r, k, v, raw, bonus, state, ctx, heads, d) -> torch.Tensor:
+    """Time mixing with a decay for every key channel, token by token: w = exp(-exp(raw)), o = (S + diag(bonus) k v^T)^T r,
+    S <- diag(w) S + k v^T per head.  r, k, v [T, heads * d] of one type (float32 or bfloat16), ``raw`` float32 of that
+    shape, ``bonus`` float32 [heads, d]; ``state`` float32 [slots, heads, d, d] is read and left up to date.  Returns float32
+    [T, heads * d]."""
+    t = _wkv_check(r, k, v, raw, bonus, state, heads, d)
+    _need(r.dtype in (torch.float32, torch.bfloat16), "wkv: float32 or bfloat16 rows")
     seq_slot, qstart, qlen = _seq_arrays(ctx, t)
-    seg = _segment_args(segments, ctx, qstart, "wkv")
-    seg_state = seg_lw = None
-    if segments is not None:
-        seg_state = torch.empty((seg[-1], heads, d, d), dtype=torch.float32, device=r.device)
-        seg_lw = torch.empty((seg[-1], heads, d), dtype=torch.float32, device=r.device)
     y = torch.empty((t, heads * d), dtype=torch.float32, device=r.device)
     _check(recurrent().li_wkv_scan(_ptr(r), _ptr(k), _ptr(v), DT[r.dtype], _ptr(raw), _ptr(bonus), _ptr(state), _ptr(seq_slot),
-                                   _ptr(qstart), _ptr(qlen), _ptr(y), ctx.n_seqs, heads, d, *seg, _ptr(seg_state), _ptr(seg_lw),
-                                   _stream()), "wkv_scan")
+                                   _ptr(qstart), _ptr(qlen), _ptr(y), ctx.n_seqs, heads, d, _stream()), "wkv_scan")
+    return y
+
+
+def wkv_chunks(r, k, v, raw, bonus, state, ctx, heads, d) -> torch.Tensor:
+    """What ``wkv_scan`` computes, for the prompts of a 16-bit model: bfloat16 rows, 32 tokens at a time on the matrix
+    cores."""
+    t = _wkv_check(r, k, v, raw, bonus, state, heads, d)
+    _need(r.dtype == torch.bfloat16, "wkv in chunks: bfloat16 rows")
+    seq_slot, qstart, qlen = _seq_arrays(ctx, t)
+    _need(qstart is not None, "wkv in chunks: per-sequence starts and lengths")
+    chunks, dev, lib = decay_chunks(ctx), r.device, recurrent()
+    n = chunks["n_chunks"]
+    mats, packs = (_scratch(n * heads * lib.li_wkv_chunk_elems(d, i), torch.bfloat16, dev) for i in (0, 1))
+    coef = _scratch(n * heads * lib.li_wkv_chunk_elems(d, 2), torch.float32, dev)
+    y = torch.empty((t, heads * d), dtype=torch.float32, device=dev)
+    _check(lib.li_wkv_chunks(_ptr(r), _ptr(k), _ptr(v), _ptr(raw), _ptr(bonus), _ptr(state), _ptr(seq_slot), _ptr(qstart), _ptr(qlen),
+                             _ptr(chunks["chunk_seq"]), _ptr(chunks["chunk_t0"]), _ptr(chunks["seq_chunk0"]), n, _ptr(mats),
+                             _ptr(coef), _ptr(packs), _ptr(y), ctx.n_seqs, heads, d, _stream()), "wkv_chunks")
     return y

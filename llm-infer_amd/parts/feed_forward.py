@@ -143,6 +143,8 @@ class DenseMLP(Part):
         self.w_up, self.w_down = ops.prepare_weight(tensors[n["up"]]), ops.prepare_weight(tensors[n["down"]])
 
     def _hidden(self, h):
+        if self.activation in ops.EPI_ACTS:          # on the product's float32 sums, in its epilogue
+            return ops.linear(h, self.w_up, ops.EPI_BIAS, out_dtype=self.dtype, params=ops.glu_params(act=self.activation))
         return ops.activation(ops.linear(h, self.w_up, out_dtype=torch.float32), self.activation, self.dtype)
 
     def forward(self, h, residual):

@@ -21,6 +21,12 @@ def _segments(part, ctx, waves_a_token: int):
     return ops.ssm_segments(ctx, length) if max(ctx.host_qlens) > length else None
 
 
+def _in_chunks(part, ctx) -> bool:
+    """True where a recurrence runs a chunk of tokens at a time: the prompts of a 16-bit model.  (A float32 model and every
+    decode step go token by token, which gives the same bits however a prompt is cut.)"""
+    return part.dtype != torch.float32 and not ctx.is_decode and bool(getattr(ctx, "host_qlens", None))
+
+
 def _own_state(owns_cache, what):
     if not owns_cache:
         raise ValueError(f"{what} keeps a state of its own in every run")
@@ -37,7 +43,8 @@ class GatedDelta(Part):
 
     Every head's o is divided by its root mean square (``norm_eps``), multiplied by a weight [dv] that the heads share and
     by silu(W_g x), and projected.  S (float32 [n_heads, d, dv]) and the convolution's last taps - 1 inputs are state of
-    every sequence.  Unit norms, gates, decays and the recurrence are float32 whatever the matrices' type.  The input
+    every sequence.  Unit norms, gates, decays and the recurrence are float32 whatever the matrices' type.  The prompts of a
+    16-bit model run 32 tokens at a time on the matrix cores, with q, k and v in bfloat16 behind the convolution.  The input
     products are one product against [W_q; W_k; W_v; W_g; W_b; W_a], which ``ParallelMixers`` may share with the mixer
     beside this one.  ``names``: local tensor names."""
 
@@ -92,9 +99,10 @@ class GatedDelta(Part):
         H, G, d, dv = self.n_heads, self.n_kv_heads, self.head_dim, self.v_head_dim
         if proj is None:
             proj, col0 = ops.linear(h, self.w_in, out_dtype=torch.float32), 0
-        qkv, gates, kq = ops.delta_prepare(proj, col0, col0 + self.b_col, col0 + self.a_col, self.conv, views[1].state, self.a_log,
-                                           self.dt_bias, ctx, H, G, d, dv)
-        o = ops.delta_scan(qkv, gates, kq, views[0].state, ctx, H, G, d, dv)
+        chunked = _in_chunks(self, ctx)
+        rows = ops.delta_prepare(proj, col0, col0 + self.b_col, col0 + self.a_col, self.conv, views[1].state, self.a_log,
+                                 self.dt_bias, ctx, H, G, d, dv, chunked)
+        o = (ops.delta_chunks if chunked else ops.delta_scan)(*rows, views[0].state, ctx, H, G, d, dv)
         return ops.gated_head_norm(o, self.norm, proj, col0 + self.g_col, H, self.norm_eps, self.dtype, gate_silu=True)
 
     def addends(self, h, ctx, views, owns_cache=True, proj=None, col0=0):
@@ -185,7 +193,8 @@ class TimeMixing(Part):
     Every head's o is divided by its root mean square (``norm_eps``); the heads side by side are multiplied by a weight
     [n_heads d] and by silu(W_g mix_g), and projected.  S (float32 [n_heads, d, d]) and the previous token's input are
     state of every sequence.  The part reads its rows in float32 (``reads_float32``); decays and the recurrence are float32
-    whatever the matrices' type.  ``names``: local tensor names."""
+    whatever the matrices' type.  The prompts of a 16-bit model run 32 tokens at a time on the matrix cores, with r, k and v in
+    bfloat16.  ``names``: local tensor names."""
 
     NAMES = {"mu": "mu_{}", "r": "r_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "g": "g_proj.weight", "w1": "w1", "w2": "w2",
              "w0": "w0", "u": "u", "norm": "norm.weight", "o": "o_proj.weight"}
@@ -230,12 +239,14 @@ class TimeMixing(Part):
             raise ValueError("time mixing reads float32 rows")
         mix = dict(zip(self.MIXES, ops.token_shift(h, self.mu, views[1].state, ctx.pos, ctx.tok_slot, self.dtype,
                                                    single=ctx.n_tokens == ctx.n_seqs)))
-        r, k, v = (ops.linear(mix[s], self.w[s], out_dtype=self.dtype) for s in "rkv")
+        # (bfloat16 whichever 16-bit type the matrices have: the recurrence's chunks take it as it is)
+        kept = torch.float32 if self.dtype == torch.float32 else torch.bfloat16
+        r, k, v = (ops.linear(mix[s], self.w[s], out_dtype=kept) for s in "rkv")
         gate = ops.linear(mix["g"], self.w["g"], out_dtype=torch.float32)
-        low = ops.activation(ops.linear(mix["w"], self.w["w1"], out_dtype=torch.float32), "tanh", self.dtype)
+        low = ops.linear(mix["w"], self.w["w1"], ops.EPI_BIAS, out_dtype=self.dtype, params=ops.glu_params(act="tanh"))
         raw = ops.linear(low, self.w["w2"], ops.EPI_BIAS, out_dtype=torch.float32, params=self.w0)
-        o = ops.wkv_scan(r, k, v, raw, self.bonus, views[0].state, ctx, self.n_heads, self.head_dim,
-                         _segments(self, ctx, self.n_heads * 4 * ((self.head_dim + 63) // 64)))
+        o = (ops.wkv_chunks if _in_chunks(self, ctx) else ops.wkv_scan)(r, k, v, raw, self.bonus, views[0].state, ctx, self.n_heads,
+                                                                        self.head_dim)
         return ops.gated_head_norm(o, self.norm, gate, 0, self.n_heads, self.norm_eps, self.dtype, gate_silu=True)
 
     def forward_into(self, h, out, ctx, views, owns_cache=True):
