@@ -28,6 +28,11 @@ struct ConvWindow {
         for (int b = TAPS - 1; b > 0; --b) u[b] = u[b - 1];
         u[0] = v;
     }
+    // the history as the next token will find it (only where no other thread still reads this column's)
+    __device__ __forceinline__ void keep(float* hist, int channels, int c) const {
+#pragma unroll
+        for (int r = 0; r < TAPS - 1; ++r) hist[(int64_t)r * channels + c] = u[TAPS - 2 - r];
+    }
     __device__ __forceinline__ float sum(const float* w, float acc) const {        // w [TAPS], the last one the token's own
 #pragma unroll
         for (int b = 0; b < TAPS; ++b) acc += w[TAPS - 1 - b] * u[b];
@@ -45,4 +50,8 @@ __device__ __forceinline__ float conv_at(const float* at, int64_t stride, int in
         acc += w[(int64_t)c * taps + (taps - 1 - b)] * u;
     }
     return acc;
+}
+__device__ __forceinline__ void conv_keep(float v, float* hist, int channels, int c, int taps) {
+    for (int r = 0; r + 2 < taps; ++r) hist[(int64_t)r * channels + c] = hist[(int64_t)(r + 1) * channels + c];
+    if (taps > 1) hist[(int64_t)(taps - 2) * channels + c] = v;
 }

@@ -290,9 +290,17 @@ __global__ void tile_weight_kernel(const T* __restrict__ W, T* __restrict__ out,
     *(v8*)(out + i * 8) = n < N ? *(const v8*)(W + (int64_t)n * K + k) : z;
 }
 
+// Several products of one M and K as one launch, their weights stacked: the rows of W from row g * rows on (the last group: all
+// that are left) read the rows of X that begin at X + g * stride.  rows 0: one X for all.
+struct XGroups {
+    int rows, n;
+    int64_t stride;
+};
+
 template <class T, int NT, int MT, int KW>
 __global__ __launch_bounds__(64 * KW) void gemv_tiled_kernel(const T* __restrict__ X, const T* __restrict__ Wt,
-                                                             int K, Epilogue e, RowsOut ro, RowScale rsc) {
+                                                             int K, Epilogue e, RowsOut ro, RowScale rsc, XGroups xg) {
+    if (xg.rows) X += min((int)blockIdx.x * NT * 16 / xg.rows, xg.n - 1) * xg.stride;
     // NT tiles of 16 rows of W and MT tiles of 16 rows of X per wave; W comes from HBM once, the
     // rows of X from the caches (they are few)
     typedef typename Vec<T>::v8 v8;
@@ -766,9 +774,8 @@ extern "C" int li_gemv_tiled_blocks(int M, int N, int K, int nt, int kw) {
     return blocks;
 }
 
-extern "C" int li_gemv_tiled(const void* X, const void* Wt, int dt, void* C, int out_dt, int mode,
-                             int M, int N, int K, int nt, int kw, const RopeStore* rs, const RowsOut* ro,
-                             const RowScale* rsc, hipStream_t stream) {
+static int gemv_tiled(const void* X, const void* Wt, int dt, void* C, int out_dt, int mode, int M, int N, int K, int nt, int kw,
+                      const RopeStore* rs, const RowsOut* ro, const RowScale* rsc, XGroups xg, hipStream_t stream) {
     int rc = check_common(X, Wt, C, M, N, K, mode, out_dt);
     if (rc) return rc;
     if (dt != DT_F16 && dt != DT_BF16) return LI_BAD_ARG;
@@ -790,7 +797,7 @@ extern "C" int li_gemv_tiled(const void* X, const void* Wt, int dt, void* C, int
     const RowScale no_scale{};
 #define LAUNCH(T, NT, MT, KW) \
     gemv_tiled_kernel<T, NT, MT, KW><<<blocks, 64 * KW, 0, stream>>>((const T*)X, (const T*)Wt, K, e, \
-                                                                     ro ? *ro : no_out, rsc ? *rsc : no_scale)
+                                                                     ro ? *ro : no_out, rsc ? *rsc : no_scale, xg)
 #define PICK_KW(T, NT, MT)                                \
     do {                                                  \
         if (kw == 4) LAUNCH(T, NT, MT, 4);                \
@@ -819,6 +826,21 @@ extern "C" int li_gemv_tiled(const void* X, const void* Wt, int dt, void* C, int
 // of W a workgroup, kw: 4 or 8 waves that share K (8: up to 64 rows of X) (0: chosen here); ldx: elements from
 // one row of X to the next.  ro (or null; mode EPI_ADD, at most 16 rows, one tile a workgroup): RowsOut, with one
 // partial sum a row for each of the N / 16 workgroups.
+
+extern "C" int li_gemv_tiled(const void* X, const void* Wt, int dt, void* C, int out_dt, int mode,
+                             int M, int N, int K, int nt, int kw, const RopeStore* rs, const RowsOut* ro,
+                             const RowScale* rsc, hipStream_t stream) {
+    return gemv_tiled(X, Wt, dt, C, out_dt, mode, M, N, K, nt, kw, rs, ro, rsc, XGroups{0, 1, 0}, stream);
+}
+
+// X [groups, M, K]: the rows of W from g * group_rows on (a multiple of 32; the last group: all that are left) against X[g].
+extern "C" int li_gemv_tiled_groups(const void* X, const void* Wt, int dt, void* C, int out_dt, int M, int N, int K, int groups,
+                                    int group_rows, hipStream_t stream) {
+    if (groups < 1 || group_rows <= 0 || group_rows % 32 || (int64_t)(groups - 1) * group_rows >= N) return LI_BAD_ARG;
+    return gemv_tiled(X, Wt, dt, C, out_dt, EPI_STORE, M, N, K, 0, 0, nullptr, nullptr, nullptr,
+                      XGroups{group_rows, groups, (int64_t)M * K}, stream);
+}
+
 extern "C" int li_gemm_rows(const void* X, const void* Wt, int dt, void* C, int out_dt, int mode,
                             int M, int N, int K, int ldx, int nt, int kw, const RopeStore* rs, const RowsOut* ro,
                             hipStream_t stream) {

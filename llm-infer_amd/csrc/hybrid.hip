@@ -334,11 +334,12 @@ extern "C" int li_diff_attn(const void* q, void* out, int dt, void* k_pages, voi
 // sequence's last taps - 1 inputs there.
 // ---------------------------------------------------------------------------
 // TAPS 4: a thread walks `tile` consecutive tokens of the step with a channel's last inputs in registers; TAPS 0: any number of
-// taps, a token at a time.
+// taps, a token at a time.  `single` (decode steps): every sequence brings one token; the thread that has read a channel's
+// history then brings it up to date itself.
 template <class T, bool SILU, bool ADD, int TAPS>
 __global__ void conv_silu_kernel(const float* __restrict__ in, int stride, int col0, const float* __restrict__ w,
-                                 const float* __restrict__ b, const float* __restrict__ hist, const int* __restrict__ pos,
-                                 const int* __restrict__ tok_slot, T* __restrict__ out, int channels, int taps, int n_tokens, int tile) {
+                                 const float* __restrict__ b, float* __restrict__ hist, const int* __restrict__ pos,
+                                 const int* __restrict__ tok_slot, T* __restrict__ out, int channels, int taps, int n_tokens, int tile, int single) {
     const int t0 = blockIdx.x * tile, t1 = min(n_tokens, t0 + tile);
     for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < channels; c += gridDim.y * blockDim.x) {
         constexpr int K = TAPS ? TAPS : 1;
@@ -353,14 +354,18 @@ __global__ void conv_silu_kernel(const float* __restrict__ in, int stride, int c
         for (int t = t0; t < t1; ++t) {
             const int slot = tok_slot[t];
             const float* at = in + (int64_t)t * stride + col0 + c;
-            const float* h = hist + (int64_t)slot * (taps - 1) * channels;
+            float* h = hist + (int64_t)slot * (taps - 1) * channels;
             float acc;
             if (TAPS) {
-                if (slot != last) win.start(at, stride, conv_inside(tok_slot, t, slot, taps), pos[t], h, channels, c);
+                if (slot != last) win.start(at, stride, single ? 0 : conv_inside(tok_slot, t, slot, taps), pos[t], h, channels, c);
                 else win.next(*at);
                 last = slot;
                 acc = win.sum(wc, bias);
-            } else acc = conv_at(at, stride, conv_inside(tok_slot, t, slot, taps), pos[t], h, channels, c, w, taps, bias);
+                if (single) win.keep(h, channels, c);
+            } else {
+                acc = conv_at(at, stride, single ? 0 : conv_inside(tok_slot, t, slot, taps), pos[t], h, channels, c, w, taps, bias);
+                if (single) conv_keep(*at, h, channels, c, taps);
+            }
             if (ADD) acc += *at;                               // the input itself beside its convolution
             out[(int64_t)t * channels + c] = from_f32<T>(SILU ? siluf_(acc) : acc);
         }
@@ -369,14 +374,14 @@ __global__ void conv_silu_kernel(const float* __restrict__ in, int stride, int c
 
 #define CONV_GO(T, SILU, ADD)                                                                                                       \
     do {                                                                                                                            \
-        const int tile = n_tokens >= 256 && taps == 4 ? 8 : 1;                                                                      \
+        const int single = n_tokens == n_seqs, tile = !single && n_tokens >= 256 && taps == 4 ? 8 : 1;                               \
         dim3 cgrid((n_tokens + tile - 1) / tile, (channels + 255) / 256);                                                           \
         if (taps == 4)                                                                                                              \
             conv_silu_kernel<T, SILU, ADD, 4><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, (T*)out, channels, \
-                                                                         taps, n_tokens, tile);                                     \
+                                                                         taps, n_tokens, tile, single);                                     \
         else                                                                                                                        \
             conv_silu_kernel<T, SILU, ADD, 0><<<cgrid, 256, 0, stream>>>(in, stride, col0, w, b, hist, pos, tok_slot, (T*)out, channels, \
-                                                                         taps, n_tokens, tile);                                     \
+                                                                         taps, n_tokens, tile, single);                                     \
     } while (0)
 
 __global__ void conv_history_kernel(const float* __restrict__ in, int stride, int col0, float* __restrict__ hist,
@@ -402,7 +407,7 @@ extern "C" int li_conv_silu(const float* in, int stride, int col0, const float* 
     if (n_tokens <= 0) return LI_OK;
     if (channels <= 0 || taps < 1 || taps > CONV_MAX_TAPS) return LI_BAD_ARG;
     DISPATCH_T(dt, CONV_GO(T, true, false));
-    if (taps > 1) {
+    if (taps > 1 && n_tokens != n_seqs) {
         dim3 grid(n_seqs, (channels + 255) / 256);
         conv_history_kernel<<<grid, 256, 0, stream>>>(in, stride, col0, hist, seq_slot, seq_qstart, seq_qlen, channels, taps);
     }
@@ -419,7 +424,7 @@ extern "C" int li_conv_add(const float* in, int stride, int col0, const float* w
     if (n_tokens <= 0) return LI_OK;
     if (channels <= 0 || taps < 1 || taps > CONV_MAX_TAPS) return LI_BAD_ARG;
     DISPATCH_T(dt, CONV_GO(T, false, true));
-    if (taps > 1) {
+    if (taps > 1 && n_tokens != n_seqs) {
         dim3 grid(n_seqs, (channels + 255) / 256);
         conv_history_kernel<<<grid, 256, 0, stream>>>(in, stride, col0, hist, seq_slot, seq_qstart, seq_qlen, channels, taps);
     }

@@ -38,10 +38,15 @@ __global__ void layernorm_kernel(const float* __restrict__ x, const float* __res
     for (int i = threadIdx.x; i < d; i += blockDim.x) o[i] = from_f32<TO>((xr[i] - mean) / sd * w[i] + (b ? b[i] : 0.f));
 }
 
+static int layernorm_in_registers(const float* x, const float* w, const float* b, const int* rows, void* out, int out_dt, int n_rows,
+                                  int d, float eps, hipStream_t stream);
+
 extern "C" int li_layernorm(const float* x, const float* w, const float* b, const int* rows, void* out, int out_dt, int n_rows,
                             int d, float eps, hipStream_t stream) {
     if (n_rows <= 0) return LI_OK;
     if (d <= 0) return LI_BAD_ARG;
+    if (d % 4 == 0 && d <= 16384 && !(((uintptr_t)x | (uintptr_t)w | (uintptr_t)b | (uintptr_t)out) & 15))
+        return layernorm_in_registers(x, w, b, rows, out, out_dt, n_rows, d, eps, stream);
     dim3 grid(n_rows), block(d >= 2048 ? 512 : (d >= 256 ? 256 : 64));
     if (out_dt == DT_F32) layernorm_kernel<float><<<grid, block, 0, stream>>>(x, w, b, rows, (float*)out, d, eps);
     else if (out_dt == DT_F16) layernorm_kernel<f16><<<grid, block, 0, stream>>>(x, w, b, rows, (f16*)out, d, eps);
@@ -234,8 +239,10 @@ extern "C" int li_add_layernorm(float* x, float alpha, const float* y1, float s1
 //   y <- a, or (a2 not null) y <- pair_scale (N(a) w1 + N(a2) w2),  N(v) = v / sqrt(mean(v^2) + pair_eps): two results
 //        side by side, each with an RMS norm of its own;
 //   x <- x + LN(y) w + b;   next <- LN(x) nw + nb in type TN (nw null: left out), the norm that reads the row next.
-// w null: y alone is wanted and goes to x (which is then only written).
+// w null: no sum; with nw, next <- LN(y) nw + nb of the rows `rows` names (null: all) and x is not touched (a layer norm by
+// itself), else y alone is wanted and goes to x (which is then only written).
 // One workgroup a row; the row stays in registers up to 4 * KEEP * THREADS elements (a multiple of 4), else it is read again.
+// With KEEP 1 everything the row needs is asked for at once, so that it waits for memory once and not once a phase.
 // ---------------------------------------------------------------------------
 struct LnAdd {
     float* x;
@@ -248,6 +255,7 @@ struct LnAdd {
     const float *nw, *nb;
     float next_eps;
     void* next;
+    const int* rows;
 };
 
 template <class TN, int THREADS, int KEEP>
@@ -266,15 +274,24 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
         return t;
     };
     const int64_t at = (int64_t)blockIdx.x * width;
-    const float *ar = p.a + at, *a2r = p.a2 ? p.a2 + at : nullptr;
+    const float *ar = p.a + (p.rows ? (int64_t)p.rows[blockIdx.x] * width : at), *a2r = p.a2 ? p.a2 + at : nullptr;
     float* xr = p.x + at;
     TN* nr = (TN*)p.next + at;
     const int tid = threadIdx.x;
     const float inv_n = 1.f / (float)width;
     if ((width & 3) == 0 && width <= 4 * KEEP * THREADS) {
         const int quads = width >> 2;
+        constexpr bool EARLY = KEEP == 1;
         f32x4 y[KEEP], xs[KEEP];
         const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+        f32x4 ew = zero, eb = zero, enw = zero, enb = zero, e1 = zero, e2 = zero;
+        if (EARLY && tid < quads) {
+            if (p.w) ew = *(const f32x4*)(p.w + 4 * tid);
+            if (p.b) eb = *(const f32x4*)(p.b + 4 * tid);
+            if (p.nw) enw = *(const f32x4*)(p.nw + 4 * tid);
+            if (p.nb) enb = *(const f32x4*)(p.nb + 4 * tid);
+            if (a2r) { e1 = *(const f32x4*)(p.w1 + 4 * tid); e2 = *(const f32x4*)(p.w2 + 4 * tid); }
+        }
         float s0 = 0.f, s1 = 0.f;
 #pragma unroll
         for (int c = 0; c < KEEP; ++c) {
@@ -300,13 +317,13 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
             for (int c = 0; c < KEEP; ++c) {
                 const int i = tid + c * THREADS;
                 if (i < quads) {
-                    const f32x4 u1 = *(const f32x4*)(p.w1 + 4 * i), u2 = *(const f32x4*)(p.w2 + 4 * i);
+                    const f32x4 u1 = EARLY ? e1 : *(const f32x4*)(p.w1 + 4 * i), u2 = EARLY ? e2 : *(const f32x4*)(p.w2 + 4 * i);
 #pragma unroll
                     for (int k = 0; k < 4; ++k) y[c][k] = y[c][k] * r1 * u1[k] + z[c][k] * r2 * u2[k];
                 }
             }
         }
-        if (!p.w) {
+        if (!p.w && !p.nw) {
 #pragma unroll
             for (int c = 0; c < KEEP; ++c) { const int i = tid + c * THREADS; if (i < quads) *(f32x4*)(xr + 4 * i) = y[c]; }
             return;
@@ -327,16 +344,21 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
             }
             return 1.f / sqrtf(block_total(s) * inv_n + eps);
         };
-        const float r = normed(y, p.eps);
+        if (p.w) {
+            const float r = normed(y, p.eps);
 #pragma unroll
-        for (int c = 0; c < KEEP; ++c) {
-            const int i = tid + c * THREADS;
-            if (i < quads) {
-                const f32x4 w = *(const f32x4*)(p.w + 4 * i), b = p.b ? *(const f32x4*)(p.b + 4 * i) : zero;
+            for (int c = 0; c < KEEP; ++c) {
+                const int i = tid + c * THREADS;
+                if (i < quads) {
+                    const f32x4 w = EARLY ? ew : *(const f32x4*)(p.w + 4 * i), b = EARLY ? eb : (p.b ? *(const f32x4*)(p.b + 4 * i) : zero);
 #pragma unroll
-                for (int k = 0; k < 4; ++k) xs[c][k] += y[c][k] * r * w[k] + b[k];
-                *(f32x4*)(xr + 4 * i) = xs[c];
+                    for (int k = 0; k < 4; ++k) xs[c][k] += y[c][k] * r * w[k] + b[k];
+                    *(f32x4*)(xr + 4 * i) = xs[c];
+                }
             }
+        } else {
+#pragma unroll
+            for (int c = 0; c < KEEP; ++c) xs[c] = y[c];
         }
         if (!p.nw) return;
         const float rn = normed(xs, p.next_eps);
@@ -344,7 +366,7 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
         for (int c = 0; c < KEEP; ++c) {
             const int i = tid + c * THREADS;
             if (i < quads) {
-                const f32x4 w = *(const f32x4*)(p.nw + 4 * i), b = p.nb ? *(const f32x4*)(p.nb + 4 * i) : zero;
+                const f32x4 w = EARLY ? enw : *(const f32x4*)(p.nw + 4 * i), b = EARLY ? enb : (p.nb ? *(const f32x4*)(p.nb + 4 * i) : zero);
                 Out4 o;
 #pragma unroll
                 for (int k = 0; k < 4; ++k) o.v[k] = from_f32<TN>(xs[c][k] * rn * w[k] + b[k]);
@@ -361,7 +383,7 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
         r2 = p.pair_scale / sqrtf(block_total(s1) * inv_n + p.pair_eps);
     }
     auto y = [&](int i) { return a2r ? ar[i] * r1 * p.w1[i] + a2r[i] * r2 * p.w2[i] : ar[i]; };
-    if (!p.w) {
+    if (!p.w && !p.nw) {
         for (int i = tid; i < width; i += THREADS) xr[i] = y(i);
         return;
     }
@@ -370,7 +392,11 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
     float mean = block_total(s) * inv_n;
     s = 0.f;
     for (int i = tid; i < width; i += THREADS) { const float v = y(i) - mean; s += v * v; }
-    float r = 1.f / sqrtf(block_total(s) * inv_n + p.eps);
+    float r = 1.f / sqrtf(block_total(s) * inv_n + (p.w ? p.eps : p.next_eps));
+    if (!p.w) {
+        for (int i = tid; i < width; i += THREADS) nr[i] = from_f32<TN>((y(i) - mean) * r * p.nw[i] + (p.nb ? p.nb[i] : 0.f));
+        return;
+    }
     s = 0.f;
     for (int i = tid; i < width; i += THREADS) {
         const float v = xr[i] + (y(i) - mean) * r * p.w[i] + (p.b ? p.b[i] : 0.f);
@@ -385,17 +411,7 @@ __global__ __launch_bounds__(THREADS) void layernorm_add_kernel(LnAdd p, int wid
     for (int i = tid; i < width; i += THREADS) nr[i] = from_f32<TN>((xr[i] - mean) * r * p.nw[i] + (p.nb ? p.nb[i] : 0.f));
 }
 
-extern "C" int li_layernorm_add(float* x, const float* a, const float* a2, const float* w1, const float* w2, float pair_eps,
-                                float pair_scale, const float* w, const float* b, float eps, const float* nw, const float* nb,
-                                float next_eps, void* next, int next_dt, int n_rows, int width, hipStream_t stream) {
-    if (n_rows <= 0) return LI_OK;
-    if (width <= 0 || !x || !a || (a2 && (!w1 || !w2)) || (nw && (!next || !w))) return LI_BAD_ARG;
-    if ((uintptr_t)x % 16 || (uintptr_t)a % 16 || (uintptr_t)a2 % 16 || (uintptr_t)w1 % 16 || (uintptr_t)w2 % 16 || (uintptr_t)w % 16 ||
-        (uintptr_t)b % 16 || (uintptr_t)nw % 16 || (uintptr_t)nb % 16 || (uintptr_t)next % 16)
-        return LI_BAD_ARG;
-    if (!nw) next_dt = DT_F32;
-    const LnAdd p{x, a, a2, w1, w2, pair_eps, pair_scale, w, b, eps, nw, nb, next_eps, next};
-    // few rows (a decode step): as many threads a row as there are pieces of four, so that a row waits for memory once
+static int launch_layernorm_add(const LnAdd& p, int next_dt, int n_rows, int width, hipStream_t stream) {
 #define GO1(TN, TH, K) layernorm_add_kernel<TN, TH, K><<<n_rows, TH, 0, stream>>>(p, width)
 #define GO(TN)                                                                                                   \
     do {                                                                                                         \
@@ -407,6 +423,24 @@ extern "C" int li_layernorm_add(float* x, const float* a, const float* a2, const
 #undef GO1
     LI_CHECK_LAUNCH();
     return LI_OK;
+}
+
+static int layernorm_in_registers(const float* x, const float* w, const float* b, const int* rows, void* out, int out_dt, int n_rows,
+                                  int d, float eps, hipStream_t stream) {
+    const LnAdd p{nullptr, x, nullptr, nullptr, nullptr, 0.f, 1.f, nullptr, nullptr, 0.f, w, b, eps, out, rows};
+    return launch_layernorm_add(p, out_dt, n_rows, d, stream);
+}
+
+extern "C" int li_layernorm_add(float* x, const float* a, const float* a2, const float* w1, const float* w2, float pair_eps,
+                                float pair_scale, const float* w, const float* b, float eps, const float* nw, const float* nb,
+                                float next_eps, void* next, int next_dt, int n_rows, int width, hipStream_t stream) {
+    if (n_rows <= 0) return LI_OK;
+    if (width <= 0 || !x || !a || (a2 && (!w1 || !w2)) || (nw && (!next || !w))) return LI_BAD_ARG;
+    if ((uintptr_t)x % 16 || (uintptr_t)a % 16 || (uintptr_t)a2 % 16 || (uintptr_t)w1 % 16 || (uintptr_t)w2 % 16 || (uintptr_t)w % 16 ||
+        (uintptr_t)b % 16 || (uintptr_t)nw % 16 || (uintptr_t)nb % 16 || (uintptr_t)next % 16)
+        return LI_BAD_ARG;
+    const LnAdd p{x, a, a2, w1, w2, pair_eps, pair_scale, w, b, eps, nw, nb, next_eps, next, nullptr};
+    return launch_layernorm_add(p, nw ? next_dt : DT_F32, n_rows, width, stream);
 }
 
 // out = y1 * s1 (+ y2 * s2) added into x: the same sum for an arrangement without the norm behind it.
@@ -444,21 +478,25 @@ extern "C" int li_cast(const float* x, void* out, int out_dt, int64_t n, hipStre
     return LI_OK;
 }
 
-// out[t][i] = rows[t][col0 + i] in another type: some columns of float32 rows as rows of their own.
+// out[t][i] = rows[t][col0 + i] in another type, `tanh_of`: its tanh: some columns of float32 rows as rows of their own.
 template <class TO>
-__global__ void cast_columns_kernel(const float* __restrict__ rows, int stride, int col0, TO* __restrict__ out, int64_t total, int n) {
+__global__ void cast_columns_kernel(const float* __restrict__ rows, int stride, int col0, TO* __restrict__ out, int64_t total, int n,
+                                    int tanh_of) {
     const int64_t e = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-    if (e < total) out[e] = from_f32<TO>(rows[e / n * stride + col0 + e % n]);
+    if (e >= total) return;
+    const float v = rows[e / n * stride + col0 + e % n];
+    out[e] = from_f32<TO>(tanh_of ? tanhf(v) : v);
 }
 
-extern "C" int li_cast_columns(const float* rows, int stride, int col0, void* out, int out_dt, int n_rows, int n, hipStream_t stream) {
+extern "C" int li_cast_columns(const float* rows, int stride, int col0, void* out, int out_dt, int n_rows, int n, int tanh_of,
+                               hipStream_t stream) {
     if (n_rows <= 0 || n <= 0) return LI_OK;
     if (col0 < 0 || col0 + n > stride) return LI_BAD_ARG;
     const int64_t total = (int64_t)n_rows * n;
     dim3 grid((unsigned)((total + 255) / 256)), block(256);
-    if (out_dt == DT_F32) cast_columns_kernel<float><<<grid, block, 0, stream>>>(rows, stride, col0, (float*)out, total, n);
-    else if (out_dt == DT_F16) cast_columns_kernel<f16><<<grid, block, 0, stream>>>(rows, stride, col0, (f16*)out, total, n);
-    else if (out_dt == DT_BF16) cast_columns_kernel<bf16><<<grid, block, 0, stream>>>(rows, stride, col0, (bf16*)out, total, n);
+    if (out_dt == DT_F32) cast_columns_kernel<float><<<grid, block, 0, stream>>>(rows, stride, col0, (float*)out, total, n, tanh_of);
+    else if (out_dt == DT_F16) cast_columns_kernel<f16><<<grid, block, 0, stream>>>(rows, stride, col0, (f16*)out, total, n, tanh_of);
+    else if (out_dt == DT_BF16) cast_columns_kernel<bf16><<<grid, block, 0, stream>>>(rows, stride, col0, (bf16*)out, total, n, tanh_of);
     else return LI_BAD_ARG;
     LI_CHECK_LAUNCH();
     return LI_OK;
@@ -489,7 +527,7 @@ __global__ void token_shift_kernel(const float* __restrict__ x, const float* __r
     if ((d & 3) == 0) {                                  // four channels a thread at a time
         struct alignas(4 * sizeof(TO)) Out4 { TO v[4]; };
         const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-        for (int i = 4 * threadIdx.x; i < d; i += 4 * blockDim.x) {
+        for (int i = 4 * (blockIdx.y * blockDim.x + threadIdx.x); i < d; i += 4 * blockDim.x * gridDim.y) {
             const f32x4 h = *(const f32x4*)(xr + i), p = prev ? *(const f32x4*)(prev + i) : zero;
             for (int m = 0; m < n_mix; ++m) {
                 const f32x4 w = *(const f32x4*)(mu + (int64_t)m * d + i);
@@ -502,7 +540,7 @@ __global__ void token_shift_kernel(const float* __restrict__ x, const float* __r
         }
         return;
     }
-    for (int i = threadIdx.x; i < d; i += blockDim.x) {
+    for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < d; i += blockDim.x * gridDim.y) {
         const float h = xr[i], p = prev ? prev[i] : 0.f;
         for (int m = 0; m < n_mix; ++m) o[m * apart + i] = from_f32<TO>(h + (p - h) * mu[(int64_t)m * d + i]);
         if (single) st[i] = h;
@@ -525,14 +563,15 @@ extern "C" int li_token_shift(const float* x, const float* mu, float* state, con
     if (d <= 0 || n_mix < 1) return LI_BAD_ARG;
     // a few rows (a decode step): as many threads a row as it has elements to four, so that a thread's loads are few
     const int wide = min(1024, (d / 4 + 63) / 64 * 64);
-    dim3 grid(n_tokens), block(n_tokens < 256 && wide > 64 ? wide : (d >= 1024 ? 256 : 64));
+    dim3 block(n_tokens < 256 && wide > 64 ? wide : (d >= 1024 ? 256 : 64)), grid(n_tokens);
+    if (n_tokens < 256 && n_mix > 1) { block = dim3(128); grid = dim3(n_tokens, (d + 511) / 512); }
     if (out_dt == DT_F32) token_shift_kernel<float><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (float*)out, d, single, n_mix);
     else if (out_dt == DT_F16) token_shift_kernel<f16><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (f16*)out, d, single, n_mix);
     else if (out_dt == DT_BF16) token_shift_kernel<bf16><<<grid, block, 0, stream>>>(x, mu, state, pos, tok_slot, (bf16*)out, d, single, n_mix);
     else return LI_BAD_ARG;
     LI_CHECK_LAUNCH();
     if (single) return LI_OK;
-    token_shift_save_kernel<<<grid, block, 0, stream>>>(x, state, tok_slot, d, n_tokens);
+    token_shift_save_kernel<<<n_tokens, block, 0, stream>>>(x, state, tok_slot, d, n_tokens);
     LI_CHECK_LAUNCH();
     return LI_OK;
 }

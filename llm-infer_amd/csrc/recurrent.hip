@@ -64,7 +64,7 @@ struct DeltaPrep {
     const float* proj;
     int stride, col0, b_col, a_col;
     const float* w;              // [channels, taps]
-    const float* hist;           // [slots, taps - 1, channels]
+    float* hist;                 // [slots, taps - 1, channels]
     const int* pos;
     const int* tok_slot;
     const float* A_log;
@@ -73,6 +73,7 @@ struct DeltaPrep {
     float* gates;
     float* aux;
     int n, taps, H, G, d, dv, tile;
+    int single;                  // every sequence brings one token: the history is brought up to date here
 };
 
 // Up to NV channels a lane, c0 + 64 v + lane, from token to token.
@@ -94,7 +95,7 @@ struct ConvLanes {
     // silu of the convolution at token t, 0 beyond `count`
     __device__ __forceinline__ void at(const DeltaPrep& p, int channels, int c0, int lane, int count, int t, int slot, bool fresh, int inside,
                                        float (&out)[NV]) {
-        const float* h = p.hist + (int64_t)slot * (p.taps - 1) * channels;
+        float* h = p.hist + (int64_t)slot * (p.taps - 1) * channels;
 #pragma unroll
         for (int v = 0; v < NV; ++v) {
             out[v] = 0.f;
@@ -106,7 +107,11 @@ struct ConvLanes {
                     if (fresh) win[v].start(x, p.stride, inside, p.pos[t], h, channels, c);
                     else win[v].next(*x);
                     acc = win[v].sum(w[v], 0.f);
-                } else acc = conv_at(x, p.stride, inside, p.pos[t], h, channels, c, p.w, p.taps, 0.f);
+                    if (p.single) win[v].keep(h, channels, c);
+                } else {
+                    acc = conv_at(x, p.stride, inside, p.pos[t], h, channels, c, p.w, p.taps, 0.f);
+                    if (p.single) conv_keep(*x, h, channels, c, p.taps);
+                }
                 out[v] = rc_silu(acc);
             }
         }
@@ -128,7 +133,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrep p) {
         for (int t = t0; t < t1; ++t) {
             const int slot = p.tok_slot[t];
             const bool fresh = slot != last;
-            const int inside = fresh || !TAPS ? conv_inside(p.tok_slot, t, slot, p.taps) : 0;
+            const int inside = !p.single && (fresh || !TAPS) ? conv_inside(p.tok_slot, t, slot, p.taps) : 0;
             last = slot;
             float q[NV], k[NV], sq = 0.f, sk = 0.f;
             cq.at(p, channels, u * d, lane, d, t, slot, fresh, inside, q);
@@ -170,7 +175,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrep p) {
         for (int t = t0; t < t1; ++t) {
             const int slot = p.tok_slot[t];
             const bool fresh = slot != last;
-            const int inside = fresh || !TAPS ? conv_inside(p.tok_slot, t, slot, p.taps) : 0;
+            const int inside = !p.single && (fresh || !TAPS) ? conv_inside(p.tok_slot, t, slot, p.taps) : 0;
             last = slot;
             float v[1];
             cv.at(p, channels, c0, lane, count, t, slot, fresh, inside, v);
@@ -192,20 +197,45 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaPrep p) {
     }
 }
 
-// Token by token: a workgroup of 4 waves per (sequence, head, 64 columns of S); a lane keeps one column's NR rows of
-// its wave's share in registers.  Both read-outs come from the state before the token, a = S^T k and c = S^T q:
-// u = beta (v - g a),  o = g c + u (k . q),  S <- g S + k u^T; the waves' shares of a and c meet in LDS.
-#define SCAN_WAVES 4
+// What stands behind a recurrence: every head's o divided by its root mean square over dv, times a weight (`w_shared`: dv
+// numbers for all heads, else H dv) and the silu of a gate (float32 rows), in type `dt`.  w null: o as it is, float32.
+struct HeadOut {
+    const float* w;
+    int w_shared;
+    const float* gate;
+    int64_t gate_stride;
+    float eps;
+    void* out;
+    int dt;
+};
+// element `i` of head h of token t (the heads' elements side by side, n = H dv of them), ss the head's sum of squares
+__device__ __forceinline__ void store_head(const HeadOut& ho, int64_t t, int n, int h, int dv, int i, float o, float ss) {
+    const int64_t at = t * n + h * dv + i;
+    if (!ho.w) { ((float*)ho.out)[at] = o; return; }
+    const float z = ho.gate[t * ho.gate_stride + h * dv + i];
+    const float v = o / sqrtf(ss / (float)dv + ho.eps) * ho.w[ho.w_shared ? i : h * dv + i] * rc_silu(z);
+    if (ho.dt == DT_F32) ((float*)ho.out)[at] = v;
+    else if (ho.dt == DT_F16) ((f16*)ho.out)[at] = (f16)v;
+    else ((bf16*)ho.out)[at] = (bf16)v;
+}
 
-template <int NR>
-__global__ __launch_bounds__(64 * SCAN_WAVES) void delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict__ gates,
-                                                                     const float* __restrict__ kq, float* __restrict__ state,
-                                                                     Steps st, float* __restrict__ y, int H, int G, int d, int dv) {
+// Token by token: a workgroup per (sequence, head), and per 64 columns of S where nothing stands behind the recurrence; 4 waves
+// to 64 columns, a lane keeps one column's NR rows of its wave's share in registers.  Both read-outs come from the state
+// before the token, a = S^T k and c = S^T q: u = beta (v - g a),  o = g c + u (k . q),  S <- g S + k u^T; the waves'
+// shares of a and c meet in LDS.
+#define SCAN_WAVES 4
+#define SCAN_COLS 2              // at most this many blocks of 64 columns a workgroup
+
+template <int NR, int CB>
+__global__ __launch_bounds__(64 * SCAN_WAVES * CB) void delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict__ gates,
+                                                                          const float* __restrict__ kq, float* __restrict__ state,
+                                                                          Steps st, HeadOut ho, int H, int G, int d, int dv) {
     constexpr int DP = NR * SCAN_WAVES;                  // rows of S, padded
     __shared__ __attribute__((aligned(16))) float sk[3][DP], sq[3][DP];
-    __shared__ float part[2][SCAN_WAVES][2][64];
-    const int seq = blockIdx.x, h = blockIdx.y, e = h / (H / G), tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int col = blockIdx.z * 64 + lane, C = 2 * G * d + H * dv, r0 = wave * NR;
+    __shared__ float part[2][CB][SCAN_WAVES][2][64], sq_sum[2][CB];
+    const int seq = blockIdx.x, h = blockIdx.y, e = h / (H / G), tid = threadIdx.x, lane = tid & 63;
+    const int wave = (tid >> 6) % SCAN_WAVES, cb = (tid >> 6) / SCAN_WAVES;
+    const int col = (blockIdx.z * CB + cb) * 64 + lane, C = 2 * G * d + H * dv, r0 = wave * NR;
     const int q0 = st.seq_qstart ? st.seq_qstart[seq] : seq, n = st.seq_qlen ? st.seq_qlen[seq] : 1;
     if (n <= 0) return;
     const bool live = col < dv;
@@ -215,7 +245,7 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void delta_scan_kernel(const float
     for (int r = 0; r < NR; ++r) s[r] = (live && r0 + r < d) ? S[(int64_t)(r0 + r) * dv] : 0.f;
     auto stage = [&](int t) {
         const float* row = qkv + (int64_t)(q0 + t) * C;
-        for (int i = tid; i < DP; i += 64 * SCAN_WAVES) {
+        for (int i = tid; i < DP; i += 64 * SCAN_WAVES * CB) {
             sq[t % 3][i] = i < d ? row[e * d + i] : 0.f;
             sk[t % 3][i] = i < d ? row[(G + e) * d + i] : 0.f;
         }
@@ -230,15 +260,26 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void delta_scan_kernel(const float
         float a = 0.f, c = 0.f;
 #pragma unroll
         for (int r = 0; r < NR; ++r) { a += s[r] * k[r]; c += s[r] * q[r]; }
-        part[t & 1][wave][0][lane] = a;
-        part[t & 1][wave][1][lane] = c;
+        part[t & 1][cb][wave][0][lane] = a;
+        part[t & 1][cb][wave][1][lane] = c;
         if (t + 1 < n) stage(t + 1);
         __syncthreads();
         a = c = 0.f;
 #pragma unroll
-        for (int w = 0; w < SCAN_WAVES; ++w) { a += part[t & 1][w][0][lane]; c += part[t & 1][w][1][lane]; }
-        const float u = beta * (v - g * a);
-        if (wave == 0 && live) y[tok * H * dv + h * dv + col] = g * c + u * dot;
+        for (int w = 0; w < SCAN_WAVES; ++w) { a += part[t & 1][cb][w][0][lane]; c += part[t & 1][cb][w][1][lane]; }
+        const float u = beta * (v - g * a), o = g * c + u * dot;
+        float ss = 0.f;
+        if (ho.w) {
+            if (wave == 0) ss = wave_sum(live ? o * o : 0.f);
+            if (CB > 1) {
+                if (wave == 0 && lane == 0) sq_sum[t & 1][cb] = ss;
+                __syncthreads();
+                ss = 0.f;
+#pragma unroll
+                for (int b = 0; b < CB; ++b) ss += sq_sum[t & 1][b];
+            }
+        }
+        if (wave == 0 && live) store_head(ho, tok, H * dv, h, dv, col, o, ss);
 #pragma unroll
         for (int r = 0; r < NR; ++r) s[r] = g * s[r] + k[r] * u;
     }
@@ -248,17 +289,18 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void delta_scan_kernel(const float
     }
 }
 
-// half 0: rows float32, aux [T, G]; half 1: rows bfloat16, aux [T, G, 2] (see delta_prep_kernel).
+// half 0: rows float32, aux [T, G]; half 1: rows bfloat16, aux [T, G, 2] (see delta_prep_kernel).  single: every
+// sequence brings one token, and the history is brought up to date on the way (else the caller does that afterwards).
 extern "C" int li_delta_prep(const float* proj, int stride, int col0, int b_col, int a_col, const float* conv_w, int taps,
-                             const float* hist, const int* pos, const int* tok_slot, const float* A_log, const float* dt_bias,
-                             void* rows, float* gates, float* aux, int half, int n, int H, int G, int d, int dv, hipStream_t stream) {
+                             float* hist, const int* pos, const int* tok_slot, const float* A_log, const float* dt_bias,
+                             void* rows, float* gates, float* aux, int half, int single, int n, int H, int G, int d, int dv, hipStream_t stream) {
     if (n <= 0) return LI_OK;
     if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || taps < 1 || taps > CONV_MAX_TAPS || !hist) return LI_BAD_ARG;
     if (d > 64 * DELTA_MAXV) return LI_UNSUPPORTED;
     const int channels = 2 * G * d + H * dv;
     if (col0 < 0 || col0 + channels > stride || b_col < 0 || b_col + H > stride || a_col < 0 || a_col + H > stride) return LI_BAD_ARG;
     const DeltaPrep p{proj, stride, col0, b_col, a_col, conv_w, hist, pos, tok_slot, A_log, dt_bias, rows, gates, aux, n, taps, H, G, d, dv,
-                      n >= 256 && taps == 4 ? 8 : 1};
+                      !single && n >= 256 && taps == 4 ? 8 : 1, single};
     const int units = G + (H * dv + 63) / 64 + 1;
     dim3 grid((n + p.tile - 1) / p.tile, (units + 3) / 4);
 #define GO1(TAPS, HALF) do { if (d <= 64) delta_prep_kernel<TAPS, HALF, 1><<<grid, 256, 0, stream>>>(p); \
@@ -271,17 +313,23 @@ extern "C" int li_delta_prep(const float* proj, int stride, int col0, int b_col,
     return LI_OK;
 }
 
+// norm_w null: out float32 [T, H dv] is o as it is.
 extern "C" int li_delta_scan(const float* qkv, const float* gates, const float* kq, float* state, const int* seq_slot,
-                             const int* seq_qstart, const int* seq_qlen, float* y, int n_seqs, int H, int G, int d, int dv,
+                             const int* seq_qstart, const int* seq_qlen, const float* norm_w, int w_shared, const float* gate,
+                             int64_t gate_stride, float eps, void* out, int out_dt, int n_seqs, int H, int G, int d, int dv,
                              hipStream_t stream) {
     if (n_seqs <= 0) return LI_OK;
-    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0) return LI_BAD_ARG;
-    if (d > 64 * DELTA_MAXV) return LI_UNSUPPORTED;
+    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || (norm_w && !gate) || (!norm_w && out_dt != DT_F32)) return LI_BAD_ARG;
+    if (d > 64 * DELTA_MAXV || (norm_w && dv > 64 * SCAN_COLS)) return LI_UNSUPPORTED;
     Steps st{nullptr, nullptr, seq_slot, seq_qstart, seq_qlen};
-    dim3 grid(n_seqs, H, (dv + 63) / 64), block(64 * SCAN_WAVES);
-#define GO(NR) delta_scan_kernel<NR><<<grid, block, 0, stream>>>(qkv, gates, kq, state, st, y, H, G, d, dv)
+    const HeadOut ho{norm_w, w_shared, gate, gate_stride, eps, out, out_dt};
+    const int blocks = (dv + 63) / 64, cb = norm_w ? blocks : 1;
+#define GO1(NR, CB) delta_scan_kernel<NR, CB><<<dim3(n_seqs, H, (blocks + CB - 1) / CB), 64 * SCAN_WAVES * CB, 0, stream>>>(qkv, gates, kq, \
+                                                                                                    state, st, ho, H, G, d, dv)
+#define GO(NR) do { if (cb == 1) GO1(NR, 1); else GO1(NR, 2); } while (0)
     if (d <= 16) GO(4); else if (d <= 32) GO(8); else if (d <= 64) GO(16); else if (d <= 128) GO(32); else GO(64);
 #undef GO
+#undef GO1
     LI_CHECK_LAUNCH();
     return LI_OK;
 }
@@ -452,20 +500,21 @@ extern "C" int li_sel_scan(const void* x, int dt, const float* raw, const float*
 // Time mixing with a decay for every key channel and a bonus for the current token.  Per sequence and head, S [d, d]
 // float32 (rows: key channels), w = exp(-exp(raw)) per key channel:
 //   o = (S + diag(u) k v^T)^T r;   S <- diag(w) S + k v^T
-// r, k, v [T, H d] in type T, raw [T, H d] float32 (its bias included), u [H, d].
-// A workgroup of 4 waves per (sequence, head, 64 columns); a lane keeps its column's NR rows of its wave's share in
-// registers, the waves' shares of o meet in LDS.
+// r, k, v in type T, head h's d elements at columns h d of rows `stride` apart; raw [T, H d] float32 (its bias included), u [H, d].
+// A workgroup per (sequence, head), and per 64 columns of S where nothing stands behind the recurrence (HeadOut); 4 waves to
+// 64 columns, a lane keeps its column's NR rows of its wave's share in registers, the waves' shares of o meet in LDS.
 // ---------------------------------------------------------------------------
-template <class T, int NR>
-__global__ __launch_bounds__(64 * SCAN_WAVES) void wkv_scan_kernel(const T* __restrict__ r_, const T* __restrict__ k_,
-                                                                   const T* __restrict__ v_, const float* __restrict__ raw,
-                                                                   const float* __restrict__ bonus, float* __restrict__ state,
-                                                                   Steps st, float* __restrict__ y, int H, int d) {
+template <class T, int NR, int CB>
+__global__ __launch_bounds__(64 * SCAN_WAVES * CB) void wkv_scan_kernel(const T* __restrict__ r_, const T* __restrict__ k_,
+                                                                        const T* __restrict__ v_, int stride,
+                                                                        const float* __restrict__ raw, const float* __restrict__ bonus,
+                                                                        float* __restrict__ state, Steps st, HeadOut ho, int H, int d) {
     constexpr int DP = NR * SCAN_WAVES;
     __shared__ __attribute__((aligned(16))) float sr[3][DP], sk[3][DP], sw[3][DP];
-    __shared__ float part[2][SCAN_WAVES][64], ruk[3][SCAN_WAVES];
-    const int seq = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const int col = blockIdx.z * 64 + lane, r0 = wave * NR;
+    __shared__ float part[2][CB][SCAN_WAVES][64], ruk[3][SCAN_WAVES * CB], sq_sum[2][CB];
+    const int seq = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63;
+    const int wave = (tid >> 6) % SCAN_WAVES, cb = (tid >> 6) / SCAN_WAVES, r0 = wave * NR;
+    const int col = (blockIdx.z * CB + cb) * 64 + lane;
     const int q0 = st.seq_qstart ? st.seq_qstart[seq] : seq, n = st.seq_qlen ? st.seq_qlen[seq] : 1;
     if (n <= 0) return;
     const bool live = col < d;
@@ -476,22 +525,22 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void wkv_scan_kernel(const T* __re
     static_assert(DP <= 64 * SCAN_WAVES, "a thread a key channel");
     const float ub = tid < d ? bonus[h * d + tid] : 0.f;
     auto stage = [&](int t) {
-        const int64_t at = (int64_t)(q0 + t) * H * d + h * d;
+        const int64_t at = (int64_t)(q0 + t) * stride + h * d;
         float rr = 0.f, kk = 0.f, w = 0.f;
         if (tid < d) {
             rr = to_f32(r_[at + tid]);
             kk = to_f32(k_[at + tid]);
-            w = expf(-expf(raw[at + tid]));
+            w = expf(-expf(raw[(int64_t)(q0 + t) * H * d + h * d + tid]));
         }
         if (tid < DP) { sr[t % 3][tid] = rr; sk[t % 3][tid] = kk; sw[t % 3][tid] = w; }
         const float b = wave_sum(rr * ub * kk);
-        if (lane == 0) ruk[t % 3][wave] = b;
+        if (lane == 0) ruk[t % 3][tid >> 6] = b;
     };
     stage(0);
     __syncthreads();
     for (int t = 0; t < n; ++t) {
         const int64_t tok = q0 + t;
-        const float v = live ? to_f32(v_[tok * H * d + h * d + col]) : 0.f;
+        const float v = live ? to_f32(v_[tok * stride + h * d + col]) : 0.f;
         const float *k = sk[t % 3] + r0, *rr = sr[t % 3] + r0, *w = sw[t % 3] + r0;
         float a = 0.f;
 #pragma unroll
@@ -499,15 +548,27 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void wkv_scan_kernel(const T* __re
             a += s[r] * rr[r];
             s[r] = w[r] * s[r] + k[r] * v;
         }
-        part[t & 1][wave][lane] = a;
+        part[t & 1][cb][wave][lane] = a;
         if (t + 1 < n) stage(t + 1);
         __syncthreads();
-        if (wave == 0 && live) {
-            float o = 0.f, b = 0.f;
+        float o = 0.f, ss = 0.f;
+        if (wave == 0) {
+            float b = 0.f;
 #pragma unroll
-            for (int i = 0; i < SCAN_WAVES; ++i) { o += part[t & 1][i][lane]; b += ruk[t % 3][i]; }
-            y[tok * H * d + h * d + col] = o + b * v;
+            for (int i = 0; i < SCAN_WAVES; ++i) o += part[t & 1][cb][i][lane];
+#pragma unroll
+            for (int i = 0; i < SCAN_WAVES * CB; ++i) b += ruk[t % 3][i];
+            o += b * v;
+            if (ho.w) ss = wave_sum(live ? o * o : 0.f);
         }
+        if (CB > 1 && ho.w) {
+            if (wave == 0 && lane == 0) sq_sum[t & 1][cb] = ss;
+            __syncthreads();
+            ss = 0.f;
+#pragma unroll
+            for (int i = 0; i < CB; ++i) ss += sq_sum[t & 1][i];
+        }
+        if (wave == 0 && live) store_head(ho, tok, H * d, h, d, col, o, ss);
     }
     if (live) {
 #pragma unroll
@@ -515,16 +576,21 @@ __global__ __launch_bounds__(64 * SCAN_WAVES) void wkv_scan_kernel(const T* __re
     }
 }
 
-extern "C" int li_wkv_scan(const void* r, const void* k, const void* v, int dt, const float* raw, const float* bonus, float* state,
-                           const int* seq_slot, const int* seq_qstart, const int* seq_qlen, float* y, int n_seqs, int H, int d,
-                           hipStream_t stream) {
+// norm_w null: out float32 [T, H d] is o as it is.
+extern "C" int li_wkv_scan(const void* r, const void* k, const void* v, int dt, int stride, const float* raw, const float* bonus,
+                           float* state, const int* seq_slot, const int* seq_qstart, const int* seq_qlen, const float* norm_w,
+                           int w_shared, const float* gate, int64_t gate_stride, float eps, void* out, int out_dt, int n_seqs, int H,
+                           int d, hipStream_t stream) {
     if (n_seqs <= 0) return LI_OK;
-    if (H <= 0 || d <= 0) return LI_BAD_ARG;
-    if (d > 256) return LI_UNSUPPORTED;
+    if (H <= 0 || d <= 0 || stride < H * d || (norm_w && !gate) || (!norm_w && out_dt != DT_F32)) return LI_BAD_ARG;
+    if (d > 256 || (norm_w && d > 64 * SCAN_COLS)) return LI_UNSUPPORTED;
     Steps st{nullptr, nullptr, seq_slot, seq_qstart, seq_qlen};
-#define GO1(T, NR) wkv_scan_kernel<T, NR><<<dim3(n_seqs, H, (d + 63) / 64), 64 * SCAN_WAVES, 0, stream>>>((const T*)r, (const T*)k, \
-        (const T*)v, raw, bonus, state, st, y, H, d)
-#define GO(T) do { if (d <= 16) GO1(T, 4); else if (d <= 32) GO1(T, 8); else if (d <= 64) GO1(T, 16); else if (d <= 128) GO1(T, 32); else GO1(T, 64); } while (0)
+    const HeadOut ho{norm_w, w_shared, gate, gate_stride, eps, out, out_dt};
+    const int blocks = (d + 63) / 64, cb = norm_w ? blocks : 1;
+#define GO1(T, NR, CB) wkv_scan_kernel<T, NR, CB><<<dim3(n_seqs, H, (blocks + CB - 1) / CB), 64 * SCAN_WAVES * CB, 0, stream>>>( \
+        (const T*)r, (const T*)k, (const T*)v, stride, raw, bonus, state, st, ho, H, d)
+#define GO(T) do { if (d <= 16) GO1(T, 4, 1); else if (d <= 32) GO1(T, 8, 1); else if (d <= 64) GO1(T, 16, 1);                 \
+                   else if (d <= 128 && cb == 2) GO1(T, 32, 2); else if (d <= 128) GO1(T, 32, 1); else GO1(T, 64, 1); } while (0)
     if (dt == DT_F32) GO(float); else if (dt == DT_BF16) GO(bf16); else return LI_BAD_ARG;
 #undef GO
 #undef GO1

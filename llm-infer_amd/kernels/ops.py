@@ -438,6 +438,20 @@ def linear(x: torch.Tensor, w, mode: int = EPI_STORE, out: torch.Tensor | None =
     return out
 
 
+def linear_groups(x: torch.Tensor, w, group_rows: int) -> torch.Tensor:
+    """Several products of few rows as one launch: ``x`` [groups, m <= 32, K] against a tiled weight whose rows from g *
+    ``group_rows`` on (a multiple of 32; the last group: all that are left) read x[g].  Returns float32 [m, N]."""
+    _dev(x, w)
+    _need(is_tiled(w) and x.dim() == 3 and x.dtype == w.dtype and x.shape[2] == w.logical[1], "linear_groups: x [groups, m, K], a tiled weight of its type")
+    g, m, k = x.shape
+    n = w.logical[0]
+    _need(1 <= m <= 32 and group_rows % 32 == 0 and (g - 1) * group_rows < n, "linear_groups: up to 32 rows, groups of multiples of 32 rows of W")
+    out = torch.empty((m, n), dtype=torch.float32, device=x.device)
+    _check(core().li_gemv_tiled_groups(_ptr(x), _ptr(w), DT[x.dtype], _ptr(out), DT[out.dtype], m, n, k, g, group_rows, _stream()),
+           "gemv_tiled_groups")
+    return out
+
+
 def _finish_norm(lazy: "LazyNorm", x: torch.Tensor) -> _RowScale:
     """What the product that reads an unfinished norm needs of it.  In float16 its kernel also leaves the scales
     for the product that adds into these rows next."""
@@ -982,13 +996,13 @@ def cast(x: torch.Tensor, dtype) -> torch.Tensor:
     return out
 
 
-def cast_columns(rows, col0: int, n: int, dtype) -> torch.Tensor:
-    """Columns col0 .. col0 + n of float32 rows as rows of their own in ``dtype``."""
+def cast_columns(rows, col0: int, n: int, dtype, tanh: bool = False) -> torch.Tensor:
+    """Columns col0 .. col0 + n of float32 rows (``tanh``: their tanh) as rows of their own in ``dtype``."""
     _dev(rows)
     _f32_rows(rows, "cast_columns rows")
     _need(dtype in DT and n >= 1 and 0 <= col0 and col0 + n <= rows.shape[1], "cast_columns: columns within the rows")
     out = torch.empty((rows.shape[0], n), dtype=dtype, device=rows.device)
-    _check(mixers().li_cast_columns(_ptr(rows), rows.shape[1], col0, _ptr(out), DT[dtype], rows.shape[0], n, _stream()), "cast_columns")
+    _check(mixers().li_cast_columns(_ptr(rows), rows.shape[1], col0, _ptr(out), DT[dtype], rows.shape[0], n, int(bool(tanh)), _stream()), "cast_columns")
     return out
 
 
@@ -2021,25 +2035,46 @@ def delta_prepare(proj, col0, b_col, a_col, conv_w, history, a_log, dt_bias, ctx
     aux = torch.empty((t, kv_heads, 2) if chunked else (t, kv_heads), dtype=torch.float32, device=dev)
     _check(recurrent().li_delta_prep(_ptr(proj), proj.shape[1], col0, b_col, a_col, _ptr(conv_w), taps, _ptr(history), _ptr(ctx.pos),
                                      _ptr(ctx.tok_slot), _ptr(a_log), _ptr(dt_bias), _ptr(qkv), _ptr(gates), _ptr(aux), int(bool(chunked)),
-                                     t, heads, kv_heads, d, dv, _stream()), "delta_prep")
-    if taps > 1:
+                                     int(t == ctx.n_seqs), t, heads, kv_heads, d, dv, _stream()), "delta_prep")
+    if taps > 1 and t != ctx.n_seqs:                # (a step of one token a sequence has done it on the way)
         conv_history(proj, col0, channels, taps, history, ctx)
     return qkv, gates, aux
 
 
-def delta_scan(qkv, gates, kq, state, ctx, heads, kv_heads, d, dv) -> torch.Tensor:
+SCAN_HEAD_LIMIT = 128         # values up to this wide have their head's norm and gate taken by the kernel of the recurrence
+
+
+def _head_out(head_out, t, heads, dv, dev):
+    """(the output's tensor, what the C interface takes of the norm and gate behind a recurrence)."""
+    if head_out is None:
+        out = torch.empty((t, heads * dv), dtype=torch.float32, device=dev)
+        return out, (None, 0, None, c_int64(0), c_float(0.0), _ptr(out), DT[out.dtype])
+    weight, gate_rows, gate_col, eps, out_dtype = head_out
+    _dev(weight, gate_rows)
+    n = heads * dv
+    _need(dv <= SCAN_HEAD_LIMIT and weight.dtype == torch.float32 and weight.dim() == 1 and weight.numel() in (n, dv), "head norm weight: float32 [heads * dv] or [dv]")
+    _f32_rows(gate_rows, "head norm gate")
+    _need(gate_rows.shape[0] == t and gate_col >= 0 and gate_col + n <= gate_rows.shape[1], "head norm: gate columns beyond the rows")
+    out = torch.empty((t, n), dtype=out_dtype, device=dev)
+    return out, (_ptr(weight), int(weight.numel() == dv), c_void_p(gate_rows.data_ptr() + 4 * gate_col), c_int64(gate_rows.shape[1]),
+                 c_float(eps), _ptr(out), DT[out_dtype])
+
+
+def delta_scan(qkv, gates, kq, state, ctx, heads, kv_heads, d, dv, head_out=None) -> torch.Tensor:
     """The gated delta rule token by token, S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, on what
-    ``delta_prepare`` left; ``state`` float32 [slots, heads, d, dv] is read and left up to date.  Returns float32 [T, heads * dv]."""
+    ``delta_prepare`` left; ``state`` float32 [slots, heads, d, dv] is read and left up to date.  Returns float32 [T, heads *
+    dv].  ``head_out`` (weight, gate_rows, gate_col, eps, dtype; dv up to SCAN_HEAD_LIMIT): what ``gated_head_norm`` makes of that
+    with the gate's silu, in the same kernel."""
     _dev(qkv, gates, kq, state)
     t = qkv.shape[0]
     _need(qkv.dtype == torch.float32 and qkv.shape == (t, 2 * kv_heads * d + heads * dv) and gates.shape == (t, heads, 2)
           and kq.shape == (t, kv_heads), "delta rule: what delta_prepare returns")
     _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, d, dv), "delta state: float32 [slots, heads, d, dv]")
     seq_slot, qstart, qlen = _seq_arrays(ctx, t)
-    y = torch.empty((t, heads * dv), dtype=torch.float32, device=qkv.device)
-    _check(recurrent().li_delta_scan(_ptr(qkv), _ptr(gates), _ptr(kq), _ptr(state), _ptr(seq_slot), _ptr(qstart), _ptr(qlen),
-                                     _ptr(y), ctx.n_seqs, heads, kv_heads, d, dv, _stream()), "delta_scan")
-    return y
+    out, ho = _head_out(head_out, t, heads, dv, qkv.device)
+    _check(recurrent().li_delta_scan(_ptr(qkv), _ptr(gates), _ptr(kq), _ptr(state), _ptr(seq_slot), _ptr(qstart), _ptr(qlen), *ho,
+                                     ctx.n_seqs, heads, kv_heads, d, dv, _stream()), "delta_scan")
+    return out
 
 
 def _scratch(n_elems: int, dtype, device):
@@ -2101,34 +2136,36 @@ def selective_scan(x, raw, dt_bias, bc, b_col, c_col, z_rows, z_col, a2, d_skip,
 
 
 def _wkv_check(r, k, v, raw, bonus, state, heads, d):
-    _dev(r, k, v, raw, bonus, state)
-    t = r.shape[0]
-    for x in (r, k, v, raw):
-        _need(x.shape == (t, heads * d) and x.dtype == (torch.float32 if x is raw else r.dtype), "wkv: rows [T, heads * d] of one type, float32 decays")
+    """r, k, v: rows [T, heads * d] of one type, contiguous or columns of rows of one width; returns (T, their stride)."""
+    t, n = r.shape[0], heads * d
+    _dev(raw, bonus, state)
+    for x in (r, k, v):
+        _need(x.is_cuda and x.shape == (t, n) and x.dtype == r.dtype and x.stride(1) == 1 and x.stride(0) == r.stride(0), "wkv: rows [T, heads * d] of one type")
+    _need(raw.shape == (t, n) and raw.dtype == torch.float32, "wkv: float32 decays")
     _need(1 <= d <= 256 and bonus.dtype == torch.float32 and bonus.shape == (heads, d), "wkv: heads up to 256 wide, float32 bonus [heads, d]")
     _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, d, d), "wkv state: float32 [slots, heads, d, d]")
-    return t
+    return t, (r.stride(0) if t > 1 else max(n, r.stride(0)))
 
 
-def wkv_scan(r, k, v, raw, bonus, state, ctx, heads, d) -> torch.Tensor:
+def wkv_scan(r, k, v, raw, bonus, state, ctx, heads, d, head_out=None) -> torch.Tensor:
     """Time mixing with a decay for every key channel, token by token: w = exp(-exp(raw)), o = (S + diag(bonus) k v^T)^T r,
-    S <- diag(w) S + k v^T per head.  r, k, v [T, heads * d] of one type (float32 or bfloat16), ``raw`` float32 of that
-    shape, ``bonus`` float32 [heads, d]; ``state`` float32 [slots, heads, d, d] is read and left up to date.  Returns float32
-    [T, heads * d]."""
-    t = _wkv_check(r, k, v, raw, bonus, state, heads, d)
+    S <- diag(w) S + k v^T per head.  r, k, v [T, heads * d] of one type (float32 or bfloat16; columns of wider rows will do),
+    ``raw`` float32 of that shape, ``bonus`` float32 [heads, d]; ``state`` float32 [slots, heads, d, d] is read and left up
+    to date.  Returns float32 [T, heads * d]; ``head_out`` as for ``delta_scan``."""
+    t, stride = _wkv_check(r, k, v, raw, bonus, state, heads, d)
     _need(r.dtype in (torch.float32, torch.bfloat16), "wkv: float32 or bfloat16 rows")
     seq_slot, qstart, qlen = _seq_arrays(ctx, t)
-    y = torch.empty((t, heads * d), dtype=torch.float32, device=r.device)
-    _check(recurrent().li_wkv_scan(_ptr(r), _ptr(k), _ptr(v), DT[r.dtype], _ptr(raw), _ptr(bonus), _ptr(state), _ptr(seq_slot),
-                                   _ptr(qstart), _ptr(qlen), _ptr(y), ctx.n_seqs, heads, d, _stream()), "wkv_scan")
-    return y
+    out, ho = _head_out(head_out, t, heads, d, r.device)
+    _check(recurrent().li_wkv_scan(_ptr(r), _ptr(k), _ptr(v), DT[r.dtype], stride, _ptr(raw), _ptr(bonus), _ptr(state), _ptr(seq_slot),
+                                   _ptr(qstart), _ptr(qlen), *ho, ctx.n_seqs, heads, d, _stream()), "wkv_scan")
+    return out
 
 
 def wkv_chunks(r, k, v, raw, bonus, state, ctx, heads, d) -> torch.Tensor:
     """What ``wkv_scan`` computes, for the prompts of a 16-bit model: bfloat16 rows, 32 tokens at a time on the matrix
     cores."""
-    t = _wkv_check(r, k, v, raw, bonus, state, heads, d)
-    _need(r.dtype == torch.bfloat16, "wkv in chunks: bfloat16 rows")
+    t, stride = _wkv_check(r, k, v, raw, bonus, state, heads, d)
+    _need(r.dtype == torch.bfloat16 and stride == heads * d, "wkv in chunks: contiguous bfloat16 rows")
     seq_slot, qstart, qlen = _seq_arrays(ctx, t)
     _need(qstart is not None, "wkv in chunks: per-sequence starts and lengths")
     chunks, dev, lib = decay_chunks(ctx), r.device, recurrent()

@@ -102,6 +102,8 @@ class GatedDelta(Part):
         chunked = _in_chunks(self, ctx)
         rows = ops.delta_prepare(proj, col0, col0 + self.b_col, col0 + self.a_col, self.conv, views[1].state, self.a_log,
                                  self.dt_bias, ctx, H, G, d, dv, chunked)
+        if not chunked and dv <= ops.SCAN_HEAD_LIMIT:      # the norm and gate behind it in the same kernel
+            return ops.delta_scan(*rows, views[0].state, ctx, H, G, d, dv, (self.norm, proj, col0 + self.g_col, self.norm_eps, self.dtype))
         o = (ops.delta_chunks if chunked else ops.delta_scan)(*rows, views[0].state, ctx, H, G, d, dv)
         return ops.gated_head_norm(o, self.norm, proj, col0 + self.g_col, H, self.norm_eps, self.dtype, gate_silu=True)
 
@@ -226,7 +228,15 @@ class TimeMixing(Part):
             raise ValueError(f"{self.prefix}: the decay's two matrices have ranks {tensors[n['w1']].shape[0]} and {tensors[n['w2']].shape[1]}")
         self.decay_rank = tensors[n["w1"]].shape[0]
         self.mu = torch.stack([tensors[n["mu"].format(s)].as_subclass(torch.Tensor).float() for s in self.MIXES]).contiguous()
-        self.w = {s: ops.prepare_weight(tensors[n[s]]) for s in ("r", "k", "v", "g", "w1", "w2")}
+        rows, keys = self.n_heads * self.head_dim, ("r", "k", "v", "g", "w1")
+        self.w_all = None
+        if rows % 32 == 0 and ops.can_tile(tensors[n["r"]]) and len({tensors[n[s]].dtype for s in keys}) == 1:
+            # one matrix, cut where the mixes change: a decode step's five products are one launch over it
+            self.w_all = ops.prepare_weight(torch.cat([tensors[n[s]] for s in keys], 0).contiguous())
+            self.w = {s: self.w_all.rows_from(i * rows, rows if s != "w1" else self.decay_rank) for i, s in enumerate(keys)}
+        else:
+            self.w = {s: ops.prepare_weight(tensors[n[s]]) for s in keys}
+        self.w["w2"] = ops.prepare_weight(tensors[n["w2"]])
         self.w0 = ops.glu_params(tensors[n["w0"]].as_subclass(torch.Tensor).float().contiguous())
         self.bonus, self.norm, self.wo = tensors[n["u"]], tensors[n["norm"]], ops.prepare_weight(tensors[n["o"]])
 
@@ -237,17 +247,26 @@ class TimeMixing(Part):
         _own_state(owns_cache, "time mixing")
         if h.dtype != torch.float32:
             raise ValueError("time mixing reads float32 rows")
-        mix = dict(zip(self.MIXES, ops.token_shift(h, self.mu, views[1].state, ctx.pos, ctx.tok_slot, self.dtype,
-                                                   single=ctx.n_tokens == ctx.n_seqs)))
-        # (bfloat16 whichever 16-bit type the matrices have: the recurrence's chunks take it as it is)
-        kept = torch.float32 if self.dtype == torch.float32 else torch.bfloat16
-        r, k, v = (ops.linear(mix[s], self.w[s], out_dtype=kept) for s in "rkv")
-        gate = ops.linear(mix["g"], self.w["g"], out_dtype=torch.float32)
-        low = ops.linear(mix["w"], self.w["w1"], ops.EPI_BIAS, out_dtype=self.dtype, params=ops.glu_params(act="tanh"))
+        H, d = self.n_heads, self.head_dim
+        c, m = H * d, h.shape[0]
+        mixes = ops.token_shift(h, self.mu, views[1].state, ctx.pos, ctx.tok_slot, self.dtype, single=ctx.n_tokens == ctx.n_seqs)
+        if self.w_all is not None and ctx.is_decode and m <= 16:
+            gate = ops.linear_groups(mixes, self.w_all, c)                     # r | k | v | g | w1, float32
+            r, k, v = (gate[:, i * c:(i + 1) * c] for i in range(3))
+            gate_col, low = 3 * c, ops.cast_columns(gate, 4 * c, self.decay_rank, self.dtype, tanh=True)
+        else:
+            mix = dict(zip(self.MIXES, mixes))
+            # (bfloat16 whichever 16-bit type the matrices have: the recurrence's chunks take it as it is)
+            kept = torch.float32 if self.dtype == torch.float32 else torch.bfloat16
+            r, k, v = (ops.linear(mix[s], self.w[s], out_dtype=kept) for s in "rkv")
+            gate, gate_col = ops.linear(mix["g"], self.w["g"], out_dtype=torch.float32), 0
+            low = ops.linear(mix["w"], self.w["w1"], ops.EPI_BIAS, out_dtype=self.dtype, params=ops.glu_params(act="tanh"))
         raw = ops.linear(low, self.w["w2"], ops.EPI_BIAS, out_dtype=torch.float32, params=self.w0)
-        o = (ops.wkv_chunks if _in_chunks(self, ctx) else ops.wkv_scan)(r, k, v, raw, self.bonus, views[0].state, ctx, self.n_heads,
-                                                                        self.head_dim)
-        return ops.gated_head_norm(o, self.norm, gate, 0, self.n_heads, self.norm_eps, self.dtype, gate_silu=True)
+        chunked = _in_chunks(self, ctx)
+        if not chunked and d <= ops.SCAN_HEAD_LIMIT:       # the norm and gate behind it in the same kernel
+            return ops.wkv_scan(r, k, v, raw, self.bonus, views[0].state, ctx, H, d, (self.norm, gate, gate_col, self.norm_eps, self.dtype))
+        o = (ops.wkv_chunks if chunked else ops.wkv_scan)(r, k, v, raw, self.bonus, views[0].state, ctx, H, d)
+        return ops.gated_head_norm(o, self.norm, gate, gate_col, H, self.norm_eps, self.dtype, gate_silu=True)
 
     def forward_into(self, h, out, ctx, views, owns_cache=True):
         ops.linear(self._rows(h, ctx, views, owns_cache), self.wo, out=out)

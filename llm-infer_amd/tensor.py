@@ -103,12 +103,18 @@ class Tensor(torch.Tensor):
 
     def prefix(self, rows: int) -> "Tensor":
         """The matrix of the first ``rows`` rows, sharing the storage (tiled: a multiple of 16 rows)."""
+        return self.rows_from(0, rows)
+
+    def rows_from(self, first: int, rows: int) -> "Tensor":
+        """The matrix of ``rows`` rows from ``first`` on, sharing the storage (tiled: cut at multiples of 16 rows, but for the
+        matrix's own end)."""
         n, k = self.logical if self.layout == "tiled" else self.shape
         if self.layout == "tiled":
-            if rows % 16 != 0 or not 0 < rows <= n:
+            if first % 16 or (rows % 16 and first + rows != n) or not 0 < rows <= n - first:
                 raise ValueError("a tiled weight is cut at multiples of 16 rows")
-            return Tensor.wrap(self.as_subclass(torch.Tensor)[: rows * k], "tiled", (rows, k), self.owner, self.keeps or self)
-        return Tensor.wrap(self.plain()[:rows], owner=self.owner, keeps=self.keeps or self)
+            end = (first + rows + 15) // 16 * 16
+            return Tensor.wrap(self.as_subclass(torch.Tensor)[first * k: end * k], "tiled", (rows, k), self.owner, self.keeps or self)
+        return Tensor.wrap(self.plain()[first:first + rows], owner=self.owner, keeps=self.keeps or self)
 
     def describe(self) -> str:
         shape = list(self.logical)
