@@ -500,13 +500,13 @@ extern "C" int li_sel_scan(const void* x, int dt, const float* raw, const float*
 // Time mixing with a decay for every key channel and a bonus for the current token.  Per sequence and head, S [d, d]
 // float32 (rows: key channels), w = exp(-exp(raw)) per key channel:
 //   o = (S + diag(u) k v^T)^T r;   S <- diag(w) S + k v^T
-// r, k, v in type T, head h's d elements at columns h d of rows `stride` apart; raw [T, H d] float32 (its bias included), u [H, d].
+// r, k, v float32, head h's d elements at columns h d of rows `stride` apart; raw [T, H d] float32 (its bias included), u [H, d].
 // A workgroup per (sequence, head), and per 64 columns of S where nothing stands behind the recurrence (HeadOut); 4 waves to
 // 64 columns, a lane keeps its column's NR rows of its wave's share in registers, the waves' shares of o meet in LDS.
 // ---------------------------------------------------------------------------
-template <class T, int NR, int CB>
-__global__ __launch_bounds__(64 * SCAN_WAVES * CB) void wkv_scan_kernel(const T* __restrict__ r_, const T* __restrict__ k_,
-                                                                        const T* __restrict__ v_, int stride,
+template <int NR, int CB>
+__global__ __launch_bounds__(64 * SCAN_WAVES * CB) void wkv_scan_kernel(const float* __restrict__ r_, const float* __restrict__ k_,
+                                                                        const float* __restrict__ v_, int stride,
                                                                         const float* __restrict__ raw, const float* __restrict__ bonus,
                                                                         float* __restrict__ state, Steps st, HeadOut ho, int H, int d) {
     constexpr int DP = NR * SCAN_WAVES;
@@ -528,8 +528,8 @@ __global__ __launch_bounds__(64 * SCAN_WAVES * CB) void wkv_scan_kernel(const T*
         const int64_t at = (int64_t)(q0 + t) * stride + h * d;
         float rr = 0.f, kk = 0.f, w = 0.f;
         if (tid < d) {
-            rr = to_f32(r_[at + tid]);
-            kk = to_f32(k_[at + tid]);
+            rr = r_[at + tid];
+            kk = k_[at + tid];
             w = expf(-expf(raw[(int64_t)(q0 + t) * H * d + h * d + tid]));
         }
         if (tid < DP) { sr[t % 3][tid] = rr; sk[t % 3][tid] = kk; sw[t % 3][tid] = w; }
@@ -540,7 +540,7 @@ __global__ __launch_bounds__(64 * SCAN_WAVES * CB) void wkv_scan_kernel(const T*
     __syncthreads();
     for (int t = 0; t < n; ++t) {
         const int64_t tok = q0 + t;
-        const float v = live ? to_f32(v_[tok * stride + h * d + col]) : 0.f;
+        const float v = live ? v_[tok * stride + h * d + col] : 0.f;
         const float *k = sk[t % 3] + r0, *rr = sr[t % 3] + r0, *w = sw[t % 3] + r0;
         float a = 0.f;
 #pragma unroll
@@ -577,7 +577,7 @@ __global__ __launch_bounds__(64 * SCAN_WAVES * CB) void wkv_scan_kernel(const T*
 }
 
 // norm_w null: out float32 [T, H d] is o as it is.
-extern "C" int li_wkv_scan(const void* r, const void* k, const void* v, int dt, int stride, const float* raw, const float* bonus,
+extern "C" int li_wkv_scan(const float* r, const float* k, const float* v, int stride, const float* raw, const float* bonus,
                            float* state, const int* seq_slot, const int* seq_qstart, const int* seq_qlen, const float* norm_w,
                            int w_shared, const float* gate, int64_t gate_stride, float eps, void* out, int out_dt, int n_seqs, int H,
                            int d, hipStream_t stream) {
@@ -587,13 +587,11 @@ extern "C" int li_wkv_scan(const void* r, const void* k, const void* v, int dt, 
     Steps st{nullptr, nullptr, seq_slot, seq_qstart, seq_qlen};
     const HeadOut ho{norm_w, w_shared, gate, gate_stride, eps, out, out_dt};
     const int blocks = (d + 63) / 64, cb = norm_w ? blocks : 1;
-#define GO1(T, NR, CB) wkv_scan_kernel<T, NR, CB><<<dim3(n_seqs, H, (blocks + CB - 1) / CB), 64 * SCAN_WAVES * CB, 0, stream>>>( \
-        (const T*)r, (const T*)k, (const T*)v, stride, raw, bonus, state, st, ho, H, d)
-#define GO(T) do { if (d <= 16) GO1(T, 4, 1); else if (d <= 32) GO1(T, 8, 1); else if (d <= 64) GO1(T, 16, 1);                 \
-                   else if (d <= 128 && cb == 2) GO1(T, 32, 2); else if (d <= 128) GO1(T, 32, 1); else GO1(T, 64, 1); } while (0)
-    if (dt == DT_F32) GO(float); else if (dt == DT_BF16) GO(bf16); else return LI_BAD_ARG;
+#define GO(NR, CB) wkv_scan_kernel<NR, CB><<<dim3(n_seqs, H, (blocks + CB - 1) / CB), 64 * SCAN_WAVES * CB, 0, stream>>>( \
+        r, k, v, stride, raw, bonus, state, st, ho, H, d)
+    if (d <= 16) GO(4, 1); else if (d <= 32) GO(8, 1); else if (d <= 64) GO(16, 1);
+    else if (d <= 128 && cb == 2) GO(32, 2); else if (d <= 128) GO(32, 1); else GO(64, 1);
 #undef GO
-#undef GO1
     LI_CHECK_LAUNCH();
     return LI_OK;
 }

@@ -5,8 +5,8 @@
 // chunks in order with the state in registers, 32 of its rows a wave.
 //
 // The state, decays, gates and unit norms are float32.  A float32 operand of a product enters the matrix cores as the
-// sum of NP bfloat16 numbers, its rounding and the roundings of what is left (three hold all 24 bits of it); q, k and v
-// come in bfloat16, which is exact.  Every product accumulates in float32.
+// sum of NP bfloat16 numbers, its rounding and the roundings of what is left (three hold all 24 bits of it); the delta
+// rule's q, k and v and the other's v come in bfloat16, which is exact.  Every product accumulates in float32.
 //
 // Accumulators of the 16x16x32 instruction: lane l holds column l % 16 and rows 4 (l / 16) + r, r < 4.  Operand A: row
 // l % 16, inner indices 8 (l / 16) + e, e < 8; operand B the same with columns.  Where an operand comes out of two
@@ -419,9 +419,9 @@ extern "C" int li_delta_chunks(const void* rows, const float* norms, const float
 // pair, the block below them as a product of r e^(b_(t-1) - b_15) and k e^(b_15 - b_s) on the float32 matrix cores;
 // `mats` [chunk, head, A]; `packs` [chunk, head, R | K^T] (r e^(b_(t-1)) and k e^(b_n - b_s) as operands, split, each [blocks
 // of 32 channels][NP][2][64][8]); `coef` [chunk, head, 32 blocks]: e^(b_n).
-// r, k, v bfloat16 [T, H d]; raw float32 [T, H d], log w = -exp(raw).
+// r, k float32, v bfloat16 [T, H d]; raw float32 [T, H d], log w = -exp(raw).
 // ---------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void wkv_chunk_kernel(const bf16* __restrict__ r_, const bf16* __restrict__ k_,
+__global__ __launch_bounds__(256) void wkv_chunk_kernel(const float* __restrict__ r_, const float* __restrict__ k_,
                                                         const float* __restrict__ raw, const float* __restrict__ bonus, Chunks cs,
                                                         bf16* __restrict__ mats, float* __restrict__ coef, bf16* __restrict__ packs,
                                                         int H, int d) {
@@ -440,8 +440,8 @@ __global__ __launch_bounds__(256) void wkv_chunk_kernel(const bf16* __restrict__
         const int t = u / DP, c = u - t * DP;
         const bool ok = t < n && c < d;
         const int64_t i = at + (int64_t)(ok ? t : 0) * C + (ok ? c : 0);
-        sr[t * LD + c] = ok ? (float)r_[i] : 0.f;
-        sk[t * LD + c] = ok ? (float)k_[i] : 0.f;
+        sr[t * LD + c] = ok ? r_[i] : 0.f;
+        sk[t * LD + c] = ok ? k_[i] : 0.f;
         sb[(t + 1) * LD + c] = ok ? fmaxf(-expf(raw[i]), LOG_DECAY_MIN) : 0.f;
     }
     for (int c = tid; c < DP; c += 256) sb[c] = 0.f;
@@ -633,7 +633,7 @@ extern "C" int li_wkv_chunk_elems(int d, int which) {
     return which == 0 ? MAT_ELEMS : (which == 1 ? 2 * DB * NP * 2 * 64 * 8 : 32 * DB);
 }
 
-extern "C" int li_wkv_chunks(const void* r, const void* k, const void* v, const float* raw, const float* bonus, float* state,
+extern "C" int li_wkv_chunks(const float* r, const float* k, const void* v, const float* raw, const float* bonus, float* state,
                              const int* seq_slot, const int* seq_qstart, const int* seq_qlen, const int* chunk_seq,
                              const int* chunk_t0, const int* seq_chunk0, int n_chunks, void* mats, float* coef, void* packs, float* y,
                              int n_seqs, int H, int d, hipStream_t stream) {
@@ -645,7 +645,7 @@ extern "C" int li_wkv_chunks(const void* r, const void* k, const void* v, const 
     const size_t lds1 = (size_t)((3 * CH + 1) * (32 * DB + 4) + CH * LDM) * sizeof(float);
     if (lds1 > 48 * 1024 && hipFuncSetAttribute((const void*)wkv_chunk_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1) != hipSuccess)
         return LI_HIP_ERROR;
-    wkv_chunk_kernel<<<dim3(n_chunks, H), 256, lds1, stream>>>((const bf16*)r, (const bf16*)k, raw, bonus, cs, (bf16*)mats, coef,
+    wkv_chunk_kernel<<<dim3(n_chunks, H), 256, lds1, stream>>>(r, k, raw, bonus, cs, (bf16*)mats, coef,
                                                                (bf16*)packs, H, d);
     LI_CHECK_LAUNCH();
     const size_t lds2 = DB > 1 ? (size_t)2 * DB * 128 * 16 : 0;

@@ -2136,11 +2136,11 @@ def selective_scan(x, raw, dt_bias, bc, b_col, c_col, z_rows, z_col, a2, d_skip,
 
 
 def _wkv_check(r, k, v, raw, bonus, state, heads, d):
-    """r, k, v: rows [T, heads * d] of one type, contiguous or columns of rows of one width; returns (T, their stride)."""
+    """r, k, v: rows [T, heads * d], contiguous or columns of rows of one width; returns (T, their stride)."""
     t, n = r.shape[0], heads * d
     _dev(raw, bonus, state)
     for x in (r, k, v):
-        _need(x.is_cuda and x.shape == (t, n) and x.dtype == r.dtype and x.stride(1) == 1 and x.stride(0) == r.stride(0), "wkv: rows [T, heads * d] of one type")
+        _need(x.is_cuda and x.shape == (t, n) and x.stride(1) == 1 and x.stride(0) == r.stride(0), "wkv: rows [T, heads * d] of one width")
     _need(raw.shape == (t, n) and raw.dtype == torch.float32, "wkv: float32 decays")
     _need(1 <= d <= 256 and bonus.dtype == torch.float32 and bonus.shape == (heads, d), "wkv: heads up to 256 wide, float32 bonus [heads, d]")
     _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, d, d), "wkv state: float32 [slots, heads, d, d]")
@@ -2149,23 +2149,24 @@ def _wkv_check(r, k, v, raw, bonus, state, heads, d):
 
 def wkv_scan(r, k, v, raw, bonus, state, ctx, heads, d, head_out=None) -> torch.Tensor:
     """Time mixing with a decay for every key channel, token by token: w = exp(-exp(raw)), o = (S + diag(bonus) k v^T)^T r,
-    S <- diag(w) S + k v^T per head.  r, k, v [T, heads * d] of one type (float32 or bfloat16; columns of wider rows will do),
+    S <- diag(w) S + k v^T per head.  r, k, v float32 [T, heads * d] (columns of wider rows will do),
     ``raw`` float32 of that shape, ``bonus`` float32 [heads, d]; ``state`` float32 [slots, heads, d, d] is read and left up
     to date.  Returns float32 [T, heads * d]; ``head_out`` as for ``delta_scan``."""
     t, stride = _wkv_check(r, k, v, raw, bonus, state, heads, d)
-    _need(r.dtype in (torch.float32, torch.bfloat16), "wkv: float32 or bfloat16 rows")
+    _need(r.dtype == k.dtype == v.dtype == torch.float32, "wkv: float32 rows")
     seq_slot, qstart, qlen = _seq_arrays(ctx, t)
     out, ho = _head_out(head_out, t, heads, d, r.device)
-    _check(recurrent().li_wkv_scan(_ptr(r), _ptr(k), _ptr(v), DT[r.dtype], stride, _ptr(raw), _ptr(bonus), _ptr(state), _ptr(seq_slot),
+    _check(recurrent().li_wkv_scan(_ptr(r), _ptr(k), _ptr(v), stride, _ptr(raw), _ptr(bonus), _ptr(state), _ptr(seq_slot),
                                    _ptr(qstart), _ptr(qlen), *ho, ctx.n_seqs, heads, d, _stream()), "wkv_scan")
     return out
 
 
 def wkv_chunks(r, k, v, raw, bonus, state, ctx, heads, d) -> torch.Tensor:
-    """What ``wkv_scan`` computes, for the prompts of a 16-bit model: bfloat16 rows, 32 tokens at a time on the matrix
-    cores."""
+    """What ``wkv_scan`` computes, for the prompts of a 16-bit model: 32 tokens at a time on the matrix cores; r and k float32,
+    v bfloat16."""
     t, stride = _wkv_check(r, k, v, raw, bonus, state, heads, d)
-    _need(r.dtype == torch.bfloat16 and stride == heads * d, "wkv in chunks: contiguous bfloat16 rows")
+    _need(r.dtype == k.dtype == torch.float32 and v.dtype == torch.bfloat16 and (stride == heads * d or t == 1),
+          "wkv in chunks: contiguous rows, r and k float32, v bfloat16")
     seq_slot, qstart, qlen = _seq_arrays(ctx, t)
     _need(qstart is not None, "wkv in chunks: per-sequence starts and lengths")
     chunks, dev, lib = decay_chunks(ctx), r.device, recurrent()

@@ -195,7 +195,7 @@ class TimeMixing(Part):
     Every head's o is divided by its root mean square (``norm_eps``); the heads side by side are multiplied by a weight
     [n_heads d] and by silu(W_g mix_g), and projected.  S (float32 [n_heads, d, d]) and the previous token's input are
     state of every sequence.  The part reads its rows in float32 (``reads_float32``); decays and the recurrence are float32
-    whatever the matrices' type.  The prompts of a 16-bit model run 32 tokens at a time on the matrix cores, with r, k and v in
+    whatever the matrices' type.  The prompts of a 16-bit model run 32 tokens at a time on the matrix cores, with v in
     bfloat16.  ``names``: local tensor names."""
 
     NAMES = {"mu": "mu_{}", "r": "r_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "g": "g_proj.weight", "w1": "w1", "w2": "w2",
@@ -248,7 +248,7 @@ class TimeMixing(Part):
         if h.dtype != torch.float32:
             raise ValueError("time mixing reads float32 rows")
         H, d = self.n_heads, self.head_dim
-        c, m = H * d, h.shape[0]
+        c, m, chunked = H * d, h.shape[0], _in_chunks(self, ctx)
         mixes = ops.token_shift(h, self.mu, views[1].state, ctx.pos, ctx.tok_slot, self.dtype, single=ctx.n_tokens == ctx.n_seqs)
         if self.w_all is not None and ctx.is_decode and m <= 16:
             gate = ops.linear_groups(mixes, self.w_all, c)                     # r | k | v | g | w1, float32
@@ -256,13 +256,11 @@ class TimeMixing(Part):
             gate_col, low = 3 * c, ops.cast_columns(gate, 4 * c, self.decay_rank, self.dtype, tanh=True)
         else:
             mix = dict(zip(self.MIXES, mixes))
-            # (bfloat16 whichever 16-bit type the matrices have: the recurrence's chunks take it as it is)
-            kept = torch.float32 if self.dtype == torch.float32 else torch.bfloat16
-            r, k, v = (ops.linear(mix[s], self.w[s], out_dtype=kept) for s in "rkv")
+            # (values in bfloat16, whichever 16-bit type the matrices have, where the recurrence runs in chunks)
+            r, k, v = (ops.linear(mix[s], self.w[s], out_dtype=torch.bfloat16 if chunked and s == "v" else torch.float32) for s in "rkv")
             gate, gate_col = ops.linear(mix["g"], self.w["g"], out_dtype=torch.float32), 0
             low = ops.linear(mix["w"], self.w["w1"], ops.EPI_BIAS, out_dtype=self.dtype, params=ops.glu_params(act="tanh"))
         raw = ops.linear(low, self.w["w2"], ops.EPI_BIAS, out_dtype=torch.float32, params=self.w0)
-        chunked = _in_chunks(self, ctx)
         if not chunked and d <= ops.SCAN_HEAD_LIMIT:       # the norm and gate behind it in the same kernel
             return ops.wkv_scan(r, k, v, raw, self.bonus, views[0].state, ctx, H, d, (self.norm, gate, gate_col, self.norm_eps, self.dtype))
         o = (ops.wkv_chunks if chunked else ops.wkv_scan)(r, k, v, raw, self.bonus, views[0].state, ctx, H, d)

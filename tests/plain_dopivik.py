@@ -1,8 +1,8 @@
 """A plain implementation of the Dopivik decoder: whole sequences, no cache, one function per mechanism, token by token
 where there is a recurrence, torch on the CPU in the precision of the tensors it is given (float32 or float64).  It
 shares no code with the engine.  ``round_to`` (a 16-bit type) rounds the activations where a 16-bit engine stores them
-(the rows that enter a product, q, k and v of the attention, the convolved rows, the mixers' outputs before their last
-product) and nothing else: the difference to the unrounded run says how much of a 16-bit engine's error is that
+(the rows that enter a product, q, k and v of the attention, the convolved rows, the values of time mixing, the
+mixers' outputs before their last product) and nothing else: the difference to the unrounded run says how much of a 16-bit engine's error is that
 rounding alone.
 
 Notation: x is the residual stream [T, width]; LN(v) = (v - mean) / sqrt(var + eps) * w + b; N(v) = v / sqrt(mean(v^2) + eps).
@@ -186,6 +186,7 @@ def wkv(h, W, m, eps, round_to=None):
     before = torch.cat([torch.zeros_like(h[:1]), h[:-1]], 0)
     mix = {s: rounded(h + (before - h) * W["mu." + s], round_to) for s in "rkvgw"}
     r, k, v = ((mix[s] @ W[s].T).view(T, H, d) for s in "rkv")
+    v = rounded(v, round_to)
     gate = silu(mix["g"] @ W["g"].T)
     w = torch.exp(-torch.exp(rounded(torch.tanh(mix["w"] @ W["w1"].T), round_to) @ W["w2"].T + W["w0"])).view(T, H, d)
     o, _ = wkv_rule(r, k, v, w, W["u"])
