@@ -85,6 +85,21 @@ __device__ __forceinline__ void pack32(const float* m, int ld, bf16* out, int fi
     }
 }
 
+// A chunk's values as operands, a block of 16 columns each: column 16 b + l % 16, tokens rows32(l, e); out [blocks][64][8].
+// `v` points at the head's first element of the chunk's first token, rows C apart; a token or column that is not there: 0.
+__device__ __forceinline__ void pack_values(const bf16* v, int64_t C, int n, int dv, bf16* out, int first, int step) {
+    for (int u = first; u < (dv + 15) / 16 * 64; u += step) {
+        const int lane = u & 63, col = 16 * (u >> 6) + (lane & 15);
+        bf16x8 p;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const int t = rows32(lane, e);
+            p[e] = t < n && col < dv ? v[t * C + col] : (bf16)0.f;
+        }
+        *(bf16x8*)(out + (int64_t)u * 8) = p;
+    }
+}
+
 // ---------------------------------------------------------------------------
 // The gated delta rule.  In a chunk with the state S before it, b_i the sum of log g up to token i and U the written
 // values,
@@ -92,7 +107,7 @@ __device__ __forceinline__ void pack32(const float* m, int ld, bf16* out, int fi
 //   O = diag(e^b) Q S + A U,   A_ij = e^(b_i - b_j) q_i . k_j  for j <= i
 //   S <- e^(b_n) S + K^T diag(e^(b_n - b)) U
 // delta_chunk_kernel, a wave per (chunk, head): W = (I + L)^-1 diag(beta) by forward substitution, a column a lane; W and A
-// to `mats` [chunk, head, W | A]; the coefficients of the rows to `coef` [chunk, head, 4, 32] (e^b_i / |k_i|, e^b_i
+// to `mats` [chunk, head, W | A | V] (V: pack_values); the coefficients of the rows to `coef` [chunk, head, 4, 32] (e^b_i / |k_i|, e^b_i
 // d^(-1/2) / |q_i|, e^(b_n - b_i) / |k_i|, and e^(b_n)); and, once a key head, the chunk's keys and queries as operands to
 // `packs` [chunk, key head, K | Q | K^T], each [blocks of 32 key dimensions][2][64][8].
 // rows: bfloat16 [T, 2 G d + H dv], q | k | v behind convolution and silu; norms [T, G, 2]: d^(-1/2) / |q|, 1 / |k|;
@@ -100,6 +115,8 @@ __device__ __forceinline__ void pack32(const float* m, int ld, bf16* out, int fi
 // ---------------------------------------------------------------------------
 #define LDM 36                  // floats from row to row of a 32 x 32 matrix in LDS
 #define MAT_ELEMS (NP * 2 * 64 * 8)
+// elements of `count` 32 x 32 operands and the values behind them
+__host__ __device__ __forceinline__ int mat_elems(int count, int dv) { return count * MAT_ELEMS + (dv + 15) / 16 * 64 * 8; }
 
 __global__ __launch_bounds__(64) void delta_chunk_kernel(const bf16* __restrict__ rows, const float* __restrict__ norms,
                                                          const float* __restrict__ gates, Chunks cs, bf16* __restrict__ mats,
@@ -198,9 +215,10 @@ __global__ __launch_bounds__(64) void delta_chunk_kernel(const bf16* __restrict_
         for (int i = 0; i < CH; ++i) sL[i * LDM + col] = w[i] * beta;
     }
     __syncthreads();
-    bf16* m = mats + ((int64_t)chunk * H + h) * 2 * MAT_ELEMS;
+    bf16* m = mats + ((int64_t)chunk * H + h) * mat_elems(2, dv);
     pack32(sL, LDM, m, lane, 64);
     pack32(sA, LDM, m + MAT_ELEMS, lane, 64);
+    pack_values(rows + t0 * C + 2 * G * d + h * dv, C, n, dv, m + 2 * MAT_ELEMS, lane, 64);
     if (h % (H / G) == 0) {
         const int64_t per = (int64_t)DB * 2 * 64 * 8;
         bf16* pk = packs + ((int64_t)chunk * G + e) * 3 * per;
@@ -229,14 +247,13 @@ __global__ __launch_bounds__(64) void delta_chunk_kernel(const bf16* __restrict_
 template <int NO>
 struct DeltaFrags {
     bf16x8 k[2], q[2], kt[2], w[NP][2], a[NP][NO];
-    bf16 v[8];
+    bf16x8 v;
     f32x4 ck[2], cq[NO], ce[2];
     float gn;
 };
 
 template <int NO>
-__global__ __launch_bounds__(NO == 2 ? 64 : 512) void delta_walk_kernel(const bf16* __restrict__ rows, const bf16* __restrict__ mats,
-                                                         const float* __restrict__ coef, const bf16* __restrict__ packs,
+__global__ __launch_bounds__(NO == 2 ? 64 : 512) void delta_walk_kernel(const bf16* __restrict__ mats, const float* __restrict__ coef, const bf16* __restrict__ packs,
                                                          float* __restrict__ state, Chunks cs, float* __restrict__ y, int H, int G,
                                                          int d, int dv) {
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -260,13 +277,13 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void delta_walk_kernel(const bf
         }
     const int o_tile = NO == 2 ? 0 : min(wave, 1);       // the first tile of the output
     const bool writes = wave < 2;
-    const unsigned at = lane * 8, vat = (unsigned)rq * C + cc;
+    const unsigned at = lane * 8;
+    unsigned none = 0;                             // in a vector register: a scalar load of gn would hold up every wait for LDS
+    asm volatile("" : "+v"(none));
     auto fetch = [&](int c, DeltaFrags<NO>& f) {
         const bf16* pk = packs + ((first + c) * G + e) * 3 * per + (int64_t)(2 * wave) * 512;
-        const bf16* mt = mats + ((first + c) * H + h) * 2 * MAT_ELEMS;
+        const bf16* mt = mats + ((first + c) * H + h) * mat_elems(2, dv);
         const float* cf = coef + ((first + c) * H + h) * 4 * CH;
-        const bf16* vb = rows + (q0 + (int64_t)c * CH) * C + 2 * G * d + h * dv;
-        const int left = n - c * CH;
 #pragma unroll
         for (int m = 0; m < 2; ++m) {
             f.k[m] = load_at<bf16x8>(pk + m * 512, at);
@@ -275,19 +292,27 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void delta_walk_kernel(const bf
             f.ck[m] = load_at<f32x4>(cf + 16 * m, rq);
             f.ce[m] = load_at<f32x4>(cf + 2 * CH + 16 * m, rq);
 #pragma unroll
-            for (int i = 0; i < NP; ++i) {
-                f.w[i][m] = load_at<bf16x8>(mt + (i * 2 + m) * 512, at);
-                if (m < NO && writes) f.a[i][m < NO ? m : 0] = load_at<bf16x8>(mt + MAT_ELEMS + (i * 2 + o_tile + m) * 512, at);
-            }
-            if (m < NO) f.cq[m < NO ? m : 0] = load_at<f32x4>(cf + CH + 16 * (o_tile + m), rq);
+            for (int i = 0; i < NP; ++i) f.w[i][m] = load_at<bf16x8>(mt + (i * 2 + m) * 512, at);
+        }
+#pragma unroll
+        for (int m = 0; m < NO; ++m) {
+            f.cq[m] = load_at<f32x4>(cf + CH + 16 * (o_tile + m), rq);
+#pragma unroll
+            for (int i = 0; i < NP; ++i) f.a[i][m] = load_at<bf16x8>(mt + MAT_ELEMS + (i * 2 + o_tile + m) * 512, at);
+        }
+        f.v = load_at<bf16x8>(mt + 2 * MAT_ELEMS + blockIdx.z * 512, at);
+        f.gn = load_at<float>(cf + 3 * CH, none);
+    };
+    f32x4 out[NO];                                 // the last chunk's output: written a chunk later, so that no load waits behind it
+    auto put = [&](int c) {
+        if (!writes || !live || c < 0) return;
+#pragma unroll
+        for (int m = 0; m < NO; ++m)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                // (a token that is not there: some other's value, which W multiplies by 0)
-                if (left >= CH) f.v[4 * m + r] = load_at<bf16>(vb + (int64_t)(16 * m + r) * C, vat);
-                else f.v[4 * m + r] = vb[(int64_t)min(16 * m + rq + r, left - 1) * C + cc];
+                const int t = c * CH + 16 * (o_tile + m) + rq + r;
+                if (t < n) y[(q0 + t) * H * dv + h * dv + col] = out[m][r];
             }
-        }
-        f.gn = cf[3 * CH];
     };
     auto body = [&](int c, const DeltaFrags<NO>& f) {
         const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
@@ -298,6 +323,7 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void delta_walk_kernel(const bf
         f32x4 pk[2], pq[2];
 #pragma unroll
         for (int m = 0; m < 2; ++m) { pk[m] = mul_es(f.k[m], sp, zero); pq[m] = mul_es(f.q[m], sp, zero); }
+        put(c - 1);
         if (nw > 1) {
             f32x4* buf = part + (c & 1) * nw * 256;
 #pragma unroll
@@ -350,24 +376,26 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void delta_walk_kernel(const bf
 #pragma unroll
                 for (int r = 0; r < 4; ++r) o[r] = f.cq[m][r] * pq[m][r];
                 const bf16x8 a[NP] = {f.a[0][m], f.a[1][m], f.a[2][m]};
-                o = mul_ss(a, up, o);
-#pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    const int t = c * CH + 16 * (o_tile + m) + rq + r;
-                    if (t < n && live) y[(q0 + t) * H * dv + h * dv + col] = o[r];
-                }
+                out[m] = mul_ss(a, up, o);
             }
         }
     };
+#pragma unroll
+    for (int m = 0; m < 2; ++m) asm volatile("" : "+v"(s[m]));         // the state has come: no wait for it in the loop
     DeltaFrags<NO> fa, fb;                         // the chunk at work and the next one, in turn
     fetch(0, fa);
+    // (every turn fetches, the last ones the last chunk again: a branch around the loads would make the wait before their use
+    // one for all loads of both ways, the next chunk's among them)
     for (int c = 0; c < n_chunks; c += 2) {
-        if (c + 1 < n_chunks) fetch(c + 1, fb);
+        fetch(min(c + 1, n_chunks - 1), fb);
+        __builtin_amdgcn_sched_barrier(0);         // the loads first
         body(c, fa);
         if (c + 1 >= n_chunks) break;
-        if (c + 2 < n_chunks) fetch(c + 2, fa);
+        fetch(min(c + 2, n_chunks - 1), fa);
+        __builtin_amdgcn_sched_barrier(0);
         body(c + 1, fb);
     }
+    put(n_chunks - 1);
     if (live) {
 #pragma unroll
         for (int m = 0; m < 2; ++m)
@@ -380,9 +408,9 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void delta_walk_kernel(const bf
 }
 
 // Elements of scratch memory that a (chunk, head) and a (chunk, key head) take, in that order: mats and packs.
-extern "C" int li_delta_chunk_elems(int d, int which) { return which == 0 ? 2 * MAT_ELEMS : 3 * ((d + 31) / 32) * 2 * 64 * 8; }
+extern "C" int li_delta_chunk_elems(int d, int dv, int which) { return which == 0 ? mat_elems(2, dv) : 3 * ((d + 31) / 32) * 2 * 64 * 8; }
 
-// mats bfloat16 [chunks, H, li_delta_chunk_elems(d, 0)], packs bfloat16 [chunks, G, li_delta_chunk_elems(d, 1)], coef float32
+// mats bfloat16 [chunks, H, li_delta_chunk_elems(d, dv, 0)], packs bfloat16 [chunks, G, li_delta_chunk_elems(d, dv, 1)], coef float32
 // [chunks, H, 4, 32]: scratch memory.
 extern "C" int li_delta_chunks(const void* rows, const float* norms, const float* gates, float* state, const int* seq_slot,
                                const int* seq_qstart, const int* seq_qlen, const int* chunk_seq, const int* chunk_t0,
@@ -402,7 +430,7 @@ extern "C" int li_delta_chunks(const void* rows, const float* norms, const float
     if (lds2 > 48 * 1024 && hipFuncSetAttribute((const void*)delta_walk_kernel<1>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds2) != hipSuccess)
         return LI_HIP_ERROR;
     dim3 grid(n_seqs, H, (dv + 15) / 16), block(64 * DB);
-#define GO(NO) delta_walk_kernel<NO><<<grid, block, lds2, stream>>>((const bf16*)rows, (const bf16*)mats, coef, (const bf16*)packs, state, \
+#define GO(NO) delta_walk_kernel<NO><<<grid, block, lds2, stream>>>((const bf16*)mats, coef, (const bf16*)packs, state, \
                                                                     cs, y, H, G, d, dv)
     if (DB == 1) GO(2); else GO(1);
 #undef GO
@@ -417,11 +445,12 @@ extern "C" int li_delta_chunks(const void* rows, const float* norms, const float
 //   A_tt = sum over c of r_t u k_t;     S <- diag(e^(b_n)) S + sum over s of (k_s e^(b_n - b_s)) v_s^T
 // Every exponent is at most 0 (a logarithm is taken as no less than LOG_DECAY_MIN).  wkv_chunk_kernel, four waves per (chunk, head): A's two blocks of 16 tokens on the diagonal pair by
 // pair, the block below them as a product of r e^(b_(t-1) - b_15) and k e^(b_15 - b_s) on the float32 matrix cores;
-// `mats` [chunk, head, A]; `packs` [chunk, head, R | K^T] (r e^(b_(t-1)) and k e^(b_n - b_s) as operands, split, each [blocks
+// `mats` [chunk, head, A | V]; `packs` [chunk, head, R | K^T] (r e^(b_(t-1)) and k e^(b_n - b_s) as operands, split, each [blocks
 // of 32 channels][NP][2][64][8]); `coef` [chunk, head, 32 blocks]: e^(b_n).
 // r, k float32, v bfloat16 [T, H d]; raw float32 [T, H d], log w = -exp(raw).
 // ---------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void wkv_chunk_kernel(const float* __restrict__ r_, const float* __restrict__ k_,
+                                                        const bf16* __restrict__ v_,
                                                         const float* __restrict__ raw, const float* __restrict__ bonus, Chunks cs,
                                                         bf16* __restrict__ mats, float* __restrict__ coef, bf16* __restrict__ packs,
                                                         int H, int d) {
@@ -514,7 +543,9 @@ __global__ __launch_bounds__(256) void wkv_chunk_kernel(const float* __restrict_
         for (int i = 0; i < NP; ++i) *(bf16x8*)(pk + kind * per + (((int64_t)blk * NP + i) * 2 + tile) * 512 + lane * 8) = p[i];
     }
     __syncthreads();
-    pack32(sA, LDM, mats + ((int64_t)chunk * H + h) * MAT_ELEMS, tid, 256);
+    bf16* m = mats + ((int64_t)chunk * H + h) * mat_elems(1, d);
+    pack32(sA, LDM, m, tid, 256);
+    pack_values(v_ + at, C, n, d, m + MAT_ELEMS, tid, 256);
 }
 
 template <int NO>
@@ -524,8 +555,7 @@ struct WkvFrags {
 };
 
 template <int NO>
-__global__ __launch_bounds__(NO == 2 ? 64 : 512) void wkv_walk_kernel(const bf16* __restrict__ v_, const bf16* __restrict__ mats,
-                                                       const float* __restrict__ coef, const bf16* __restrict__ packs,
+__global__ __launch_bounds__(NO == 2 ? 64 : 512) void wkv_walk_kernel(const bf16* __restrict__ mats, const float* __restrict__ coef, const bf16* __restrict__ packs,
                                                        float* __restrict__ state, Chunks cs, float* __restrict__ y, int H, int d) {
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     f32x4* part = (f32x4*)smem;                    // [2][waves][2][64]
@@ -548,13 +578,11 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void wkv_walk_kernel(const bf16
         }
     const int o_tile = NO == 2 ? 0 : min(wave, 1);       // the first tile of the output
     const bool writes = wave < 2;
-    const unsigned at = lane * 8, vat = (unsigned)rq * C + cc;
+    const unsigned at = lane * 8;
     auto fetch = [&](int c, WkvFrags<NO>& f) {
         const bf16* pk = packs + ((first + c) * H + h) * 2 * per + (int64_t)wave * NP * 2 * 512;
-        const bf16* mt = mats + ((first + c) * H + h) * MAT_ELEMS;
+        const bf16* mt = mats + ((first + c) * H + h) * mat_elems(1, d);
         const float* cf = coef + ((first + c) * H + h) * 32 * DB + 32 * wave;
-        const bf16* vb = v_ + (q0 + (int64_t)c * CH) * C + h * d;
-        const int left = n - c * CH;
 #pragma unroll
         for (int m = 0; m < 2; ++m) {
             f.dec[m] = load_at<f32x4>(cf + 16 * m, rq);
@@ -562,15 +590,24 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void wkv_walk_kernel(const bf16
             for (int i = 0; i < NP; ++i) {
                 f.r[i][m] = load_at<bf16x8>(pk + (i * 2 + m) * 512, at);
                 f.kt[i][m] = load_at<bf16x8>(pk + per + (i * 2 + m) * 512, at);
-                if (m < NO && writes) f.a[i][m < NO ? m : 0] = load_at<bf16x8>(mt + (i * 2 + o_tile + m) * 512, at);
             }
         }
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {              // token rows32(lane, e); (one that is not there has k = 0 and r = 0)
-            const int row = (e & 3) + 16 * (e >> 2);
-            if (left >= CH) f.v[e] = load_at<bf16>(vb + (int64_t)row * C, vat);
-            else f.v[e] = vb[(int64_t)min(row + rq, left - 1) * C + cc];
-        }
+        for (int m = 0; m < NO; ++m)
+#pragma unroll
+            for (int i = 0; i < NP; ++i) f.a[i][m] = load_at<bf16x8>(mt + (i * 2 + o_tile + m) * 512, at);
+        f.v = load_at<bf16x8>(mt + MAT_ELEMS + blockIdx.z * 512, at);
+    };
+    f32x4 out[NO];                                 // the last chunk's output: written a chunk later, so that no load waits behind it
+    auto put = [&](int c) {
+        if (!writes || !live || c < 0) return;
+#pragma unroll
+        for (int m = 0; m < NO; ++m)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int t = c * CH + 16 * (o_tile + m) + rq + r;
+                if (t < n) y[(q0 + t) * C + h * d + col] = out[m][r];
+            }
     };
     auto body = [&](int c, const WkvFrags<NO>& f) {
         const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
@@ -587,6 +624,7 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void wkv_walk_kernel(const bf16
             for (int i = 0; i < 4; ++i) s[m][i] *= f.dec[m][i];
             s[m] = mul_se(kt, f.v, s[m]);
         }
+        put(c - 1);
         if (nw > 1) {
             f32x4* buf = part + (c & 1) * nw * 128;
 #pragma unroll
@@ -599,23 +637,25 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void wkv_walk_kernel(const bf16
         for (int m = 0; m < NO; ++m) {
             if (!writes) continue;
             const bf16x8 a[NP] = {f.a[0][m], f.a[1][m], f.a[2][m]};
-            o[m] = mul_se(a, f.v, o[m]);
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int t = c * CH + 16 * (o_tile + m) + rq + r;
-                if (t < n && live) y[(q0 + t) * C + h * d + col] = o[m][r];
-            }
+            out[m] = mul_se(a, f.v, o[m]);
         }
     };
+#pragma unroll
+    for (int m = 0; m < 2; ++m) asm volatile("" : "+v"(s[m]));         // the state has come: no wait for it in the loop
     WkvFrags<NO> fa, fb;                           // the chunk at work and the next one, in turn
     fetch(0, fa);
+    // (every turn fetches, the last ones the last chunk again: a branch around the loads would make the wait before their use
+    // one for all loads of both ways, the next chunk's among them)
     for (int c = 0; c < n_chunks; c += 2) {
-        if (c + 1 < n_chunks) fetch(c + 1, fb);
+        fetch(min(c + 1, n_chunks - 1), fb);
+        __builtin_amdgcn_sched_barrier(0);         // the loads first
         body(c, fa);
         if (c + 1 >= n_chunks) break;
-        if (c + 2 < n_chunks) fetch(c + 2, fa);
+        fetch(min(c + 2, n_chunks - 1), fa);
+        __builtin_amdgcn_sched_barrier(0);
         body(c + 1, fb);
     }
+    put(n_chunks - 1);
     if (live) {
 #pragma unroll
         for (int m = 0; m < 2; ++m)
@@ -630,7 +670,7 @@ __global__ __launch_bounds__(NO == 2 ? 64 : 512) void wkv_walk_kernel(const bf16
 // Elements of scratch memory of a (chunk, head): mats (0), packs (1), coef (2, float32).
 extern "C" int li_wkv_chunk_elems(int d, int which) {
     const int DB = (d + 31) / 32;
-    return which == 0 ? MAT_ELEMS : (which == 1 ? 2 * DB * NP * 2 * 64 * 8 : 32 * DB);
+    return which == 0 ? mat_elems(1, d) : (which == 1 ? 2 * DB * NP * 2 * 64 * 8 : 32 * DB);
 }
 
 extern "C" int li_wkv_chunks(const float* r, const float* k, const void* v, const float* raw, const float* bonus, float* state,
@@ -645,12 +685,12 @@ extern "C" int li_wkv_chunks(const float* r, const float* k, const void* v, cons
     const size_t lds1 = (size_t)((3 * CH + 1) * (32 * DB + 4) + CH * LDM) * sizeof(float);
     if (lds1 > 48 * 1024 && hipFuncSetAttribute((const void*)wkv_chunk_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds1) != hipSuccess)
         return LI_HIP_ERROR;
-    wkv_chunk_kernel<<<dim3(n_chunks, H), 256, lds1, stream>>>(r, k, raw, bonus, cs, (bf16*)mats, coef,
+    wkv_chunk_kernel<<<dim3(n_chunks, H), 256, lds1, stream>>>(r, k, (const bf16*)v, raw, bonus, cs, (bf16*)mats, coef,
                                                                (bf16*)packs, H, d);
     LI_CHECK_LAUNCH();
     const size_t lds2 = DB > 1 ? (size_t)2 * DB * 128 * 16 : 0;
     dim3 grid(n_seqs, H, (d + 15) / 16), block(64 * DB);
-#define GO(NO) wkv_walk_kernel<NO><<<grid, block, lds2, stream>>>((const bf16*)v, (const bf16*)mats, coef, (const bf16*)packs, state, cs, y, H, d)
+#define GO(NO) wkv_walk_kernel<NO><<<grid, block, lds2, stream>>>((const bf16*)mats, coef, (const bf16*)packs, state, cs, y, H, d)
     if (DB == 1) GO(2); else GO(1);
 #undef GO
     LI_CHECK_LAUNCH();

@@ -2093,8 +2093,8 @@ def delta_chunks(rows, gates, norms, state, ctx, heads, kv_heads, d, dv) -> torc
     _need(qstart is not None, "delta rule in chunks: per-sequence starts and lengths")
     chunks, dev, lib = decay_chunks(ctx), rows.device, recurrent()
     n = chunks["n_chunks"]
-    mats = _scratch(n * heads * lib.li_delta_chunk_elems(d, 0), torch.bfloat16, dev)
-    packs = _scratch(n * kv_heads * lib.li_delta_chunk_elems(d, 1), torch.bfloat16, dev)
+    mats = _scratch(n * heads * lib.li_delta_chunk_elems(d, dv, 0), torch.bfloat16, dev)
+    packs = _scratch(n * kv_heads * lib.li_delta_chunk_elems(d, dv, 1), torch.bfloat16, dev)
     coef = torch.empty((n, heads, 4, DECAY_CHUNK), dtype=torch.float32, device=dev)
     y = torch.empty((t, heads * dv), dtype=torch.float32, device=dev)
     _check(lib.li_delta_chunks(_ptr(rows), _ptr(norms), _ptr(gates), _ptr(state), _ptr(seq_slot), _ptr(qstart), _ptr(qlen),
