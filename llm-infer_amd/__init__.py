@@ -3,7 +3,8 @@
     engine = llm_infer_amd.load("model_dir", max_tokens=65536)
     new_tokens = engine.generate([[1, 2, 3], [4, 5]], max_new_tokens=16, temperature=0.0)
 """
-from .config import ConfigError, DopivikConfig, DupolornConfig, FavizenConfig, LlamaConfig, ManiraxConfig, RisonexConfig
+from .config import (ConfigError, DopivikConfig, DupolornConfig, FavizenConfig, LlamaConfig, ManiraxConfig, PusisunConfig,
+                     RisonexConfig)
 from .tensor import Tensor
 from .registry import (config_from_dict, config_from_folder, register_architecture, register_block,
                        register_embedding, register_feed_forward, register_head, register_mixer,
@@ -17,6 +18,7 @@ register_architecture("Risonex", RisonexConfig)
 register_architecture("Dupolorn", DupolornConfig)
 register_architecture("Favizen", FavizenConfig)
 register_architecture("Dopivik", DopivikConfig)
+register_architecture("Pusisun", PusisunConfig)
 
 
 def load(folder: str, dtype: str | None = None, max_tokens: int = 8192, n_slots=None, kv_round=None):

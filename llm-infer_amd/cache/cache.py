@@ -7,7 +7,7 @@ pool ``[pages, layers of the group, K part + V part]`` and one page table
 ``[slots, pages per sequence]``; inside a page keys and values lie in the order in
 which the attention kernels feed the matrix cores.  Pages are zeroed when handed
 out, so nothing of an earlier sequence can be read.  A group with a window gives
-pages back once all their tokens have left the window.
+pages back once all their tokens have left the window (except those that hold first tokens which it keeps).
 
 One row more than there are slots lies behind every per-slot table (page tables, lengths, sampling state,
 state groups): the scratch slot, ``Cache.scratch_slot``, which is never handed out.  Its page-table entries
@@ -95,7 +95,8 @@ class KVGroup:
         return view
 
     def first_needed_page(self, length: int) -> int:
-        """First page that a token at position ``length`` (the next one) still reads."""
+        """First page that a token at position ``length`` (the next one) still reads, first tokens that are kept
+        (``keep_first``) aside: their pages were handed out when those tokens came and stay."""
         first = 0
         if self.spec.window is not None:
             first = max(0, length - self.spec.window + 1)
@@ -130,7 +131,7 @@ class KVGroup:
             return
         first = self.first_needed_page(length)
         have = self.pages_of[slot]
-        gone = [p for p in have if p < first]
+        gone = [p for p in have if p < first and p * PAGE >= self.spec.keep_first]
         if gone:
             self.pool.free([have.pop(p) for p in gone])
             for p in gone:

@@ -5,6 +5,7 @@ from .risonex import RisonexConfig
 from .dupolorn import DupolornConfig
 from .favizen import FavizenConfig
 from .dopivik import DopivikConfig
+from .pusisun import PusisunConfig
 
 __all__ = ["PartSpec", "SubLayerSpec", "LayerSpec", "ScheduleEntry", "ModelSpec", "ConfigError", "LlamaConfig", "ManiraxConfig", "RisonexConfig",
-           "DupolornConfig", "FavizenConfig", "DopivikConfig"]
+           "DupolornConfig", "FavizenConfig", "DopivikConfig", "PusisunConfig"]

@@ -45,9 +45,11 @@ struct CachePtrs {
 // exp(sink[h]), a score with no key and no value that is not scaled; `slopes` [H]: the score of the key at position j
 // loses slopes[h] * (p - j); `gate`: head h's output is multiplied by sigmoid(gate[token][gate_col + h]) (float32 rows of
 // gate_stride numbers), with `gate_elem` its element d by sigmoid(gate[token][gate_col + h * HD + d]); `softcap` c: a
-// scaled score s becomes c tanh(s / c) before anything else.
+// scaled score s becomes c tanh(s / c) before anything else; `keep`: the keys before position `keep` are read whatever
+// window and block say (the pages between them and the others are not visited).
 struct AttnExtras {
     int block;
+    int keep;
     const float* sink;
     const float* slopes;
     const float* gate;
@@ -95,7 +97,8 @@ struct WaveAttn {
     // `per` (not 0): every score loses per for every position between the row (at position hi) and its key; `cap` (not 0):
     // the soft cap of the unscaled scores (soft_cap).
     __device__ __forceinline__ void scores(const v8 (&kf)[2 * KS], f32x16 (&s)[2], int t0, int lo, int hi,
-                                           float scale2, bool masked = true, float per = 0.f, float cap = 0.f, float cap_per = 0.f) {
+                                           float scale2, bool masked = true, float per = 0.f, float cap = 0.f, float cap_per = 0.f,
+                                           int keep = 0) {
 #pragma unroll
         for (int b = 0; b < 2; ++b) {
 #pragma unroll
@@ -119,13 +122,13 @@ struct WaveAttn {
                     s[b][r] = fmaf(-per, (float)(hi - t), s[b][r]);
                 }
         }
-        softmax_step(s, t0, lo, hi, scale2, masked);
+        softmax_step(s, t0, lo, hi, scale2, masked, keep);
     }
 
-    // scale2 > 0.  A page whose keys all lie inside lo..hi for every lane of the wave (the
+    // scale2 > 0.  A page whose keys all lie inside lo..hi (or before `keep`) for every lane of the wave (the
     // caller knows: `masked` false) skips the comparisons.
     __device__ __forceinline__ void softmax_step(f32x16 (&s)[2], int t0, int lo, int hi, float scale2,
-                                                 bool masked = true) {
+                                                 bool masked = true, int keep = 0) {
         const int lane = threadIdx.x & 63;
         float mx = -INFINITY;
         if (masked) {
@@ -134,7 +137,7 @@ struct WaveAttn {
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     const int t = t0 + 32 * b + 8 * (r >> 2) + 4 * (lane >> 5) + (r & 3);
-                    const float v = (t >= lo && t <= hi) ? s[b][r] : -INFINITY;
+                    const float v = ((t >= lo || t < keep) && t <= hi) ? s[b][r] : -INFINITY;
                     s[b][r] = v;
                     mx = fmaxf(mx, v);
                 }
@@ -292,14 +295,14 @@ struct PrefillWave {
         l = l * alpha + psum;
     }
 
-    __device__ __forceinline__ void mask(f32x16 (&n)[2], int t0, int lo, int hi) const {
+    __device__ __forceinline__ void mask(f32x16 (&n)[2], int t0, int lo, int hi, int keep) const {
         const int lane = threadIdx.x & 63;
 #pragma unroll
         for (int b = 0; b < 2; ++b)
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 const int t = t0 + 32 * b + 8 * (r >> 2) + 4 * (lane >> 5) + (r & 3);
-                n[b][r] = (t >= lo && t <= hi) ? n[b][r] : -INFINITY;
+                n[b][r] = ((t >= lo || t < keep) && t <= hi) ? n[b][r] : -INFINITY;
             }
     }
 
@@ -425,9 +428,13 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
     }
     lo_max = __builtin_amdgcn_readfirstlane(lo_max);
     hi_min = __builtin_amdgcn_readfirstlane(hi_min);
-    const int p_lo = first_key(base + q0) / PAGE;
+    // The pages are walked as numbers p_lo .. p_hi: p_win .. p_hi are pages of those numbers, and the n_keep numbers before
+    // p_win stand for the pages 0 .. n_keep - 1, whose first keys are kept (page_of)
+    const int p_win = first_key(base + q0) / PAGE;
+    const int n_keep = min((ex.keep + PAGE - 1) / PAGE, p_win), p_lo = p_win - n_keep;
     const int p_hi = (base + min(q0 + TT - 1, qlen - 1)) / PAGE;
-    const int wp_lo = first_key(base + first) / PAGE;
+    const int wp_lo = n_keep ? p_lo : first_key(base + first) / PAGE;
+    auto page_of = [&](int p) { return p < p_win ? p - p_lo : p; };
     const int wp_hi = wave_live ? (base + min(first + 31, qlen - 1)) / PAGE : -1;
     const int* table = c.page_table + (int64_t)seq_slot[seq] * c.max_pages;
     const T* kbase = (const T*)c.k + (int64_t)kvh * k_head_elems(HD);
@@ -455,16 +462,18 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
     // barrier), and nobody reads the keys of page p or the values of page p-1 any more, whose
     // buffers the loads for two steps on now fill.  The page table's entry for a step is read a
     // step before, so that it has arrived with that step's wait.
-    int entry_v = table[p_lo], entry_k = table[min(p_lo + 1, p_hi)];      // of pages p+1 and p+2
+    int entry_v = table[page_of(p_lo)], entry_k = table[page_of(min(p_lo + 1, p_hi))];      // of pages p+1 and p+2
     auto step = [&](int p) {
         __builtin_amdgcn_s_waitcnt(0x0F70);                      // vmcnt(0)
         __syncthreads();
         if (p + 2 <= p_hi) bring(kbase + at_page(entry_k), kbuf(p + 2), KL);
         if (p + 1 <= p_hi) bring(vbase + at_page(entry_v), vbuf(p + 1), VL);
         entry_v = entry_k;
-        entry_k = table[min(p + 3, p_hi)];
+        entry_k = table[page_of(min(p + 3, p_hi))];
     };
-    auto is_masked = [&](int p) { return p * PAGE < lo_max || p * PAGE + PAGE - 1 > hi_min; };
+    auto is_masked = [&](int page) {
+        return (page * PAGE < lo_max && page * PAGE + PAGE > ex.keep) || page * PAGE + PAGE - 1 > hi_min;
+    };
 
     bring(kbase + at_page(entry_v), kbuf(p_lo), KL);
     int p = p_lo - 1;
@@ -476,8 +485,9 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
         step(p);                                                 // p = own_lo - 1: the first page's scores
         a.template scores<false>(kaddr(p + 1), sa, sa, pf, scale2);
         if (cap != 0.f) a.cap(sa, cap, cap_per);
-        if (per != 0.f) a.bias(sa, (p + 1) * PAGE, pos, per);
-        if (is_masked(p + 1)) a.mask(sa, (p + 1) * PAGE, lo, pos);
+        const int page0 = page_of(p + 1);
+        if (per != 0.f) a.bias(sa, page0 * PAGE, pos, per);
+        if (is_masked(page0)) a.mask(sa, page0 * PAGE, lo, pos, ex.keep);
         {
             float mx = -INFINITY;
 #pragma unroll
@@ -489,8 +499,9 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
             step(p);
             a.template scores<true>(kaddr(p + 1), nxt, cur, pf, scale2);
             if (cap != 0.f) a.cap(nxt, cap, cap_per);
-            if (per != 0.f) a.bias(nxt, (p + 1) * PAGE, pos, per);
-            if (is_masked(p + 1)) a.mask(nxt, (p + 1) * PAGE, lo, pos);
+            const int page = page_of(p + 1);
+            if (per != 0.f) a.bias(nxt, page * PAGE, pos, per);
+            if (is_masked(page)) a.mask(nxt, page * PAGE, lo, pos, ex.keep);
             a.rescale();
             a.template mix<true>(vaddr(p), pf, nxt, scale2);
             ++p;
@@ -574,7 +585,10 @@ __global__ __launch_bounds__(64 * W) void attn_decode_kernel(
     if (ex.block > 0) lo = max(lo, pos - pos % ex.block);
     const float bias_per = (ex.slopes && live) ? ex.slopes[h] / scale : 0.f;    // in the units of the unscaled scores
     const float cap = ex.softcap / scale, cap_per = ex.softcap > 0.f ? 2.f * LOG2E / ex.softcap * scale : 0.f;
-    const int p_first = lo / PAGE, p_end = pos / PAGE + 1;
+    // (pages as numbers, the kept ones' right before the window's: see attn_prefill_kernel)
+    const int p_win = lo / PAGE, n_keep = min((ex.keep + PAGE - 1) / PAGE, p_win);
+    const int p_first = p_win - n_keep, p_end = pos / PAGE + 1;
+    auto page_of = [&](int p) { return p < p_win ? p - p_first : p; };
     const int per = (p_end - p_first + S - 1) / S;
     const int p0 = p_first + split * per, p1 = min(p_end, p0 + per);
     const int* table = c.page_table + (int64_t)seq_slot[b] * c.max_pages;
@@ -585,12 +599,13 @@ __global__ __launch_bounds__(64 * W) void attn_decode_kernel(
     f32x16 s[2];
     const T* kbase = (const T*)c.k + (int64_t)kvh * k_head_elems(HD);
     const T* vbase = (const T*)c.v + (int64_t)kvh * v_head_elems(HD);
-    if (p0 < p1) a.load_k(kbase + (int64_t)table[p0] * c.page_stride, kf);
+    if (p0 < p1) a.load_k(kbase + (int64_t)table[page_of(p0)] * c.page_stride, kf);
     for (int p = p0; p < p1; ++p) {
-        a.load_v(vbase + (int64_t)table[p] * c.page_stride, vf);
-        a.scores(kf, s, p * PAGE, lo, live ? pos : -1, scale2, p * PAGE < lo || p * PAGE + PAGE - 1 > pos, bias_per, cap,
-                 cap_per);
-        if (p + 1 < p1) a.load_k(kbase + (int64_t)table[p + 1] * c.page_stride, kf);
+        const int page = page_of(p), t0 = page * PAGE;
+        a.load_v(vbase + (int64_t)table[page] * c.page_stride, vf);
+        a.scores(kf, s, t0, lo, live ? pos : -1, scale2, (t0 < lo && t0 + PAGE > ex.keep) || t0 + PAGE - 1 > pos, bias_per, cap,
+                 cap_per, ex.keep);
+        if (p + 1 < p1) a.load_k(kbase + (int64_t)table[page_of(p + 1)] * c.page_stride, kf);
         a.mix(vf, s);
     }
     float total = a.total();
@@ -775,14 +790,14 @@ extern "C" int li_attn_prefill(const void* q, void* out, int dt, const void* k, 
                                int n_tiles, const int* seq_slot, const int* seq_qstart, const int* seq_qlen,
                                const int* seq_ctx, int H, int K, float scale, int window, int key_block, const float* sink,
                                const float* slopes, const float* gate, int gate_stride, int gate_col, int gate_elem, float softcap,
-                               hipStream_t stream) {
+                               int keep, hipStream_t stream) {
     if (check_heads(H, K)) return LI_BAD_ARG;
-    if (key_block < 0 || !(scale > 0.f) || !(softcap >= 0.f) ||
+    if (key_block < 0 || keep < 0 || !(scale > 0.f) || !(softcap >= 0.f) ||
         (gate && (gate_col < 0 || gate_col + (gate_elem ? H * HD : H) > gate_stride)))
         return LI_BAD_ARG;
     if (n_tiles <= 0) return LI_OK;
     CachePtrs c{k, v, page_stride, page_table, max_pages};
-    const AttnExtras ex{key_block, sink, slopes, gate, gate_stride, gate_col, gate_elem, softcap};
+    const AttnExtras ex{key_block, keep, sink, slopes, gate, gate_stride, gate_col, gate_elem, softcap};
     const int G = H / K;
     const int gw = G % 4 == 0 ? 4 : (G % 2 == 0 ? 2 : 1);        // query heads of a KV head per workgroup
     dim3 grid(n_tiles * gw, K * (G / gw)), block(256);
@@ -836,12 +851,12 @@ extern "C" int li_attn_decode(const void* q, void* out, int dt, const void* k, c
                               const int* page_table, int max_pages, const int* seq_slot, const int* seq_ctx,
                               int n_seqs, int H, int K, float scale, int window, int splits, float* part_o,
                               float* part_ml, int key_block, const float* sink, const float* slopes, const float* gate,
-                              int gate_stride, int gate_col, int gate_elem, float softcap, hipStream_t stream) {
+                              int gate_stride, int gate_col, int gate_elem, float softcap, int keep, hipStream_t stream) {
     if (check_heads(H, K) || splits < 1 || splits > 64) return LI_BAD_ARG;
-    if (key_block < 0 || !(scale > 0.f) || !(softcap >= 0.f) ||
+    if (key_block < 0 || keep < 0 || !(scale > 0.f) || !(softcap >= 0.f) ||
         (gate && (gate_col < 0 || gate_col + (gate_elem ? H * HD : H) > gate_stride)))
         return LI_BAD_ARG;
-    const AttnExtras ex{key_block, sink, slopes, gate, gate_stride, gate_col, gate_elem, softcap};
+    const AttnExtras ex{key_block, keep, sink, slopes, gate, gate_stride, gate_col, gate_elem, softcap};
     const int w = waves_per_group(splits), parts = splits / w;
     if (parts > 64 || (parts > 1 && (!part_o || !part_ml))) return LI_BAD_ARG;
     if (dt != DT_F16 && dt != DT_BF16) return LI_BAD_ARG;

@@ -15,7 +15,8 @@
 // the score of the key at position j loses slopes[head] * (p - j), the sink nothing.  `gate` not null: a head's output
 // is multiplied by the sigmoid of gate[token][gate_col + head] (float32 rows of gate_stride numbers), with `gate_elem`
 // every element of it by the sigmoid of gate[token][gate_col + head * dv + element].  softcap c > 0: a scaled score s
-// becomes c tanh(s / c) before anything else.
+// becomes c tanh(s / c) before anything else.  `keep`: the keys before position `keep` are seen whatever block and window
+// say; the 32 keys at a time between them and the others are not walked.
 #include "common.h"
 
 #ifndef MAP_DIM
@@ -43,7 +44,7 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
     const int* __restrict__ tok_slot, const int* __restrict__ tile_t0, const int* __restrict__ tile_n, int H, int G,
     int dv, float scale, int block, int window, float lambda, float out_eps, float out_scale, int split,
     const float* __restrict__ sink, float* __restrict__ shares_out, const float* __restrict__ slopes,
-    const float* __restrict__ gate, int gate_stride, int gate_col, int gate_elem, float softcap) {
+    const float* __restrict__ gate, int gate_stride, int gate_col, int gate_elem, float softcap, int keep) {
     typedef typename Vec<T>::v8 v8;
     constexpr int D16 = MAP_DIM / 16, KW = MAPS * MAP_DIM, DVB = VALUE_DIM / 32;
     extern __shared__ float lds[];
@@ -122,9 +123,14 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
 #pragma unroll
             for (int u = 0; u < 2; ++u) vn[b][u] = *(const v8*)(vh + ((int64_t)(b * (PAGE / 16) + tb * 2 + u) * 64 + lane) * 8);
     };
-    const int kt_last = p_last / 32, kt_first = lo_tile / 32 + kwave;
-    if (kt_first <= kt_last) fetch(kt_first);
-    for (int kt = kt_first; kt <= kt_last; kt += kstep) {
+    // The walk counts tiles of 32 keys: the numbers from w_win on are tiles of those numbers, the n_keep numbers before it
+    // stand for the tiles 0 .. n_keep - 1, whose keys are kept
+    const int w_win = lo_tile / 32, n_keep = min((keep + 31) / 32, w_win), w_lo = w_win - n_keep;
+    auto tile_of = [&](int w) { return w < w_win ? w - w_lo : w; };
+    const int kt_last = p_last / 32, w_first = w_lo + kwave;
+    if (w_first <= kt_last) fetch(tile_of(w_first));
+    for (int w = w_first; w <= kt_last; w += kstep) {
+        const int kt = tile_of(w);
         v8 kf[MAPS][D16], vf[DVB][2];
 #pragma unroll
         for (int a = 0; a < MAPS; ++a)
@@ -134,7 +140,7 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
         for (int b = 0; b < DVB; ++b)
 #pragma unroll
             for (int u = 0; u < 2; ++u) vf[b][u] = vn[b][u];
-        if (kt + kstep <= kt_last) fetch(kt + kstep);
+        if (w + kstep <= kt_last) fetch(tile_of(w + kstep));
         v8 phi[MAPS][2], plo[MAPS][2];
 #pragma unroll
         for (int a = 0; a < MAPS; ++a) {
@@ -153,7 +159,7 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
                 for (int r = 0; r < 16; ++r) acc[r] = soft_cap(acc[r], softcap * back, per);
             }
             float tmax = -INFINITY;
-            if (whole_tile && kt * 32 >= lo_last && kt * 32 + 31 <= p0) {
+            if (whole_tile && (kt * 32 >= lo_last || kt * 32 + 32 <= keep) && kt * 32 + 31 <= p0) {
                 if (slopes) {
 #pragma unroll
                     for (int r = 0; r < 16; ++r) {
@@ -169,7 +175,7 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     const int key = kt * 32 + 8 * (r >> 2) + 4 * half + (r & 3);
-                    const bool seen = has_query && key >= lo_q && key <= pq;
+                    const bool seen = has_query && (key >= lo_q || key < keep) && key <= pq;
                     acc[r] = seen ? acc[r] * scale2 - slope2 * (float)(pq - key) : -INFINITY;
                     tmax = fmaxf(tmax, acc[r]);
                 }
@@ -380,12 +386,12 @@ extern "C" int li_diffattn(const void* q, void* out, int dt, const void* k_pages
                            const int* tile_n, int n_tiles, int H, int G, int maps, int dv, float scale, int block, int window,
                            float lambda, float out_eps, float out_scale, const float* sink, int key_shares, float* part,
                            const float* slopes, const float* gate, int gate_stride, int gate_col, int gate_elem, float softcap,
-                           hipStream_t stream) {
+                           int keep, hipStream_t stream) {
     if (n_tiles <= 0) return LI_OK;
     if (gate && (gate_col < 0 || gate_col + (gate_elem ? H * dv : H) > gate_stride)) return LI_BAD_ARG;
     if (!gate) gate_elem = 0;
     if (softcap < 0.f || (softcap > 0.f && !(scale > 0.f))) return LI_BAD_ARG;
-    if (H <= 0 || G <= 0 || H % G || dv <= 0 || dv > VALUE_DIM || block < 0 || window < 0) return LI_BAD_ARG;
+    if (H <= 0 || G <= 0 || H % G || dv <= 0 || dv > VALUE_DIM || block < 0 || window < 0 || keep < 0) return LI_BAD_ARG;
     if (maps < 1 || maps > 2 || (dt != DT_F16 && dt != DT_BF16)) return LI_UNSUPPORTED;
     if ((tile_t0 == nullptr) != (tile_n == nullptr)) return LI_BAD_ARG;
     MapPages pg{k_pages, v_pages, page_stride, page_table, max_pages};
@@ -410,7 +416,7 @@ extern "C" int li_diffattn(const void* q, void* out, int dt, const void* k_pages
             return LI_HIP_ERROR;                                                                                                     \
         kfn<<<grid, threads, lds, stream>>>((const T*)q, (T*)out, pg, pos, tok_slot, tile_t0, tile_n, H, G, dv, scale, block, window, \
                                             lambda, out_eps, out_scale, split, sink, part, slopes, gate, gate_stride, gate_col,      \
-                                            gate_elem, softcap);                                                                     \
+                                            gate_elem, softcap, keep);                                                               \
         if (shares > 1)                                                                                                              \
             diff_attn_merge_kernel<T, M><<<n_tiles * H, 64, 0, stream>>>(part, (T*)out, H, shares, dv, lambda, out_eps, out_scale, sink, \
                                                                       gate, gate_stride, gate_col, gate_elem);                       \

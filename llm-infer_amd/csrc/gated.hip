@@ -57,6 +57,9 @@ extern "C" int li_scale_values(float* x, int64_t n, float s, hipStream_t stream)
 // channel (column c of the rows is channel c; the last tap is the token's own), y_t = sum_j w[c][j] u_(t - taps + 1 + j):
 // inputs before the first token that a sequence brings to this step come from `hist` [slots, taps - 1, channels] (the
 // last inputs of the steps before, oldest first; before position 0 they are zero), which this kernel only reads.
+// `q_norm` (float32 [H d]) and `k_norm` ([G d]) not null (not with a convolution): a token's q columns, and its k columns,
+// are divided by the root mean square of all of them together (`norm_eps` inside the root) and multiplied by these weights
+// before the rotation.  `magnitude` multiplies sine and cosine.
 // ---------------------------------------------------------------------------
 struct StorePages {
     void* k;
@@ -73,12 +76,28 @@ __global__ void rot_store_kernel(const float* __restrict__ rows, int stride, int
                                  const float* __restrict__ inv_freq, int rot, const int* __restrict__ pos,
                                  const int* __restrict__ tok_slot, T* __restrict__ q_out, StorePages pg, int H, int G,
                                  int d, int dv, const float* __restrict__ conv_w, int taps, const float* __restrict__ hist,
-                                 int channels) {
+                                 int channels, const float* __restrict__ q_norm, const float* __restrict__ k_norm,
+                                 float norm_eps, float magnitude) {
+    __shared__ float scratch[16];
     __shared__ float cs[2 * ROT_MAX_PAIRS];               // cos and sin of the token's angles, one pair of them a pair of dimensions
     const int t = blockIdx.x, p = pos[t], DP = round_up(d, 16), half = rot >> 1;
-    for (int j = threadIdx.x; j < half; j += blockDim.x) sincosf((float)p * inv_freq[j], &cs[2 * j + 1], &cs[2 * j]);
+    for (int j = threadIdx.x; j < half; j += blockDim.x) {
+        float sn, cn;
+        sincosf((float)p * inv_freq[j], &sn, &cn);
+        cs[2 * j] = cn * magnitude; cs[2 * j + 1] = sn * magnitude;
+    }
     if (half) __syncthreads();
     const float* row = rows + (int64_t)t * stride;
+    float q_rms = 1.f, k_rms = 1.f;                       // 1 / the root mean square of the token's q and k columns
+    if (q_norm) {
+        auto rms_of = [&](const float* u, int n) {
+            float ss = 0.f;
+            for (int i = threadIdx.x; i < n; i += blockDim.x) ss += u[i] * u[i];
+            return 1.f / sqrtf(block_sum(ss, scratch) / (float)n + norm_eps);
+        };
+        q_rms = rms_of(row + q_col, H * d);
+        if (G > 0) k_rms = rms_of(row + k_col, G * d);
+    }
     const int slot = tok_slot[t];
     // how many tokens before this one its sequence has in this step (at most taps - 1 matter)
     int inside = 0;
@@ -111,11 +130,14 @@ __global__ void rot_store_kernel(const float* __restrict__ rows, int stride, int
             const int src = is_q ? q_col + u * d : k_col + (u - H) * d;
             float val = 0.f;
             if (i < d) {
-                val = value(src + i);
+                const float* nw = !q_norm ? nullptr : (is_q ? q_norm + u * d : k_norm + (u - H) * d);
+                const float rms = is_q ? q_rms : k_rms;
+                auto normed = [&](int c) { return nw ? value(src + c) * rms * nw[c] : value(src + c); };
+                val = normed(i);
                 if (i < rot) {
                     const int j = i < half ? i : i - half;
                     const float c_ = cs[2 * j], s_ = cs[2 * j + 1];
-                    val = i < half ? val * c_ - value(src + i + half) * s_ : val * c_ + value(src + i - half) * s_;
+                    val = i < half ? val * c_ - normed(i + half) * s_ : val * c_ + normed(i - half) * s_;
                 }
             }
             if (is_q) q_out[((int64_t)t * H + u) * DP + i] = from_f32<T>(val);
@@ -131,12 +153,13 @@ extern "C" int li_rot_store(const float* rows, int stride, int q_col, int k_col,
                             const int* pos, const int* tok_slot, void* q_out, void* k_pages, void* v_pages,
                             int64_t page_stride, const int* page_table, int max_pages, int dt, int n, int H, int G_store,
                             int d, int dv, const float* conv_w, int taps, const float* hist, int channels,
-                            hipStream_t stream) {
+                            const float* q_norm, const float* k_norm, float norm_eps, float magnitude, hipStream_t stream) {
     if (n <= 0) return LI_OK;
     if (H <= 0 || G_store < 0 || d <= 0 || dv <= 0 || rot < 0 || rot > d || (rot & 1) || (rot && !inv_freq)) return LI_BAD_ARG;
     if (rot > 2 * ROT_MAX_PAIRS) return LI_UNSUPPORTED;
     if (q_col < 0 || q_col + H * d > stride) return LI_BAD_ARG;
     if (G_store && (k_col < 0 || v_col < 0 || k_col + G_store * d > stride || v_col + G_store * dv > stride)) return LI_BAD_ARG;
+    if (q_norm && (conv_w || (G_store && !k_norm))) return LI_BAD_ARG;
     if (conv_w) {
         // every column that is read is a channel of the convolution
         const int last = G_store ? (k_col + G_store * d > v_col + G_store * dv ? k_col + G_store * d : v_col + G_store * dv) : 0;
@@ -147,7 +170,8 @@ extern "C" int li_rot_store(const float* rows, int stride, int q_col, int k_col,
     const int total = (H + G_store) * round_up(d, 16) + G_store * dv;
     dim3 grid(n, n >= 512 ? 1 : (total + 255) / 256);
     DISPATCH_T(dt, (rot_store_kernel<T><<<grid, 256, 0, stream>>>(rows, stride, q_col, k_col, v_col, inv_freq, rot, pos, tok_slot,
-                                                              (T*)q_out, pg, H, G_store, d, dv, conv_w, taps, hist, channels)));
+                                                              (T*)q_out, pg, H, G_store, d, dv, conv_w, taps, hist, channels, q_norm,
+                                                              k_norm, norm_eps, magnitude)));
     LI_CHECK_LAUNCH();
     return LI_OK;
 }
@@ -156,6 +180,8 @@ extern "C" int li_rot_store(const float* rows, int stride, int q_col, int k_col,
 // x[t] += (y[t] + b) / sqrt(mean((y[t] + b)^2) + eps) * w: the norm on a sub-layer's output and the residual sum in
 // one pass over the row (b may be null).  `next_w` not null: the norm that reads the finished row next is taken too,
 // next[t] = x[t] / sqrt(mean(x[t]^2) + next_eps) * next_w in type TN, while the row is still in registers.
+// `add_vec` not null: the finished row also gains the vector add_vec (one for all rows) and, `add_rows` not null, its row of
+// add_rows, before that next norm (what a stretch of layers that runs several times takes in ahead of a pass).
 // One workgroup a row; the row stays in registers up to 8,192 elements (a multiple of 4), else it is read again.
 // ---------------------------------------------------------------------------
 #define RA_THREADS 256
@@ -166,7 +192,8 @@ extern "C" int li_rot_store(const float* rows, int stride, int q_col, int k_col,
 template <class TN, bool EARLY>
 __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_kernel(float* __restrict__ x, const float* __restrict__ y,
                                                                  const float* __restrict__ b, const float* __restrict__ w,
-                                                                 float eps, int width, const float* __restrict__ next_w,
+                                                                 float eps, int width, const float* __restrict__ add_rows,
+                                                                 const float* __restrict__ add_vec, const float* __restrict__ next_w,
                                                                  float next_eps, TN* __restrict__ next) {
     __shared__ float scratch[16];
     const int64_t row = blockIdx.x;
@@ -203,6 +230,14 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_kernel(float* __restri
                 f32x4 o = xs[c];
                 o[0] += keep[c][0] * r * ws[c][0]; o[1] += keep[c][1] * r * ws[c][1];
                 o[2] += keep[c][2] * r * ws[c][2]; o[3] += keep[c][3] * r * ws[c][3];
+                if (add_vec) {
+                    if (add_rows) {
+                        const f32x4 e = *(const f32x4*)(add_rows + row * width + 4 * i);
+                        o[0] += e[0]; o[1] += e[1]; o[2] += e[2]; o[3] += e[3];
+                    }
+                    const f32x4 e = *(const f32x4*)(add_vec + 4 * i);
+                    o[0] += e[0]; o[1] += e[1]; o[2] += e[2]; o[3] += e[3];
+                }
                 *(f32x4*)(xr + 4 * i) = o;
                 keep[c] = o;
                 s2 += o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
@@ -224,7 +259,11 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_kernel(float* __restri
     for (int i = threadIdx.x; i < width; i += RA_THREADS) { const float v = yr[i] + (b ? b[i] : 0.f); ss += v * v; }
     const float r = 1.f / sqrtf(block_sum(ss, scratch) / (float)width + eps);
     for (int i = threadIdx.x; i < width; i += RA_THREADS) {
-        const float o = xr[i] + (yr[i] + (b ? b[i] : 0.f)) * r * w[i];
+        float o = xr[i] + (yr[i] + (b ? b[i] : 0.f)) * r * w[i];
+        if (add_vec) {
+            if (add_rows) o += add_rows[row * width + i];
+            o += add_vec[i];
+        }
         xr[i] = o;
         s2 += o * o;
     }
@@ -234,14 +273,38 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_kernel(float* __restri
 }
 
 extern "C" int li_rmsnorm_add(float* x, const float* y, const float* b, const float* w, float eps, int n_rows, int width,
-                              const float* next_w, float next_eps, void* next, int next_dt, hipStream_t stream) {
+                              const float* add_rows, const float* add_vec, const float* next_w, float next_eps, void* next,
+                              int next_dt, hipStream_t stream) {
     if (n_rows <= 0) return LI_OK;
-    if (width <= 0 || !x || !y || !w || (next_w && !next)) return LI_BAD_ARG;
+    if (width <= 0 || !x || !y || !w || (next_w && !next) || (add_rows && !add_vec)) return LI_BAD_ARG;
     if (!next_w) next_dt = DT_F32;
     if (n_rows <= 64)
-        DISPATCH_T(next_dt, (rmsnorm_add_kernel<T, true><<<n_rows, RA_THREADS, 0, stream>>>(x, y, b, w, eps, width, next_w, next_eps, (T*)next)));
+        DISPATCH_T(next_dt, (rmsnorm_add_kernel<T, true><<<n_rows, RA_THREADS, 0, stream>>>(x, y, b, w, eps, width, add_rows, add_vec, next_w,
+                                                                                       next_eps, (T*)next)));
     else
-        DISPATCH_T(next_dt, (rmsnorm_add_kernel<T, false><<<n_rows, RA_THREADS, 0, stream>>>(x, y, b, w, eps, width, next_w, next_eps, (T*)next)));
+        DISPATCH_T(next_dt, (rmsnorm_add_kernel<T, false><<<n_rows, RA_THREADS, 0, stream>>>(x, y, b, w, eps, width, add_rows, add_vec, next_w,
+                                                                                       next_eps, (T*)next)));
+    LI_CHECK_LAUNCH();
+    return LI_OK;
+}
+
+// out[t] = x[t] (+ rows[t]) + vec: one vector for all rows, and (rows not null) a row of another tensor.
+__global__ void add_rows_kernel(const float* __restrict__ x, const float* __restrict__ rows, const float* __restrict__ vec,
+                                float* __restrict__ out, int width) {
+    const int64_t at = (int64_t)blockIdx.x * width;
+    for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < width; i += gridDim.y * blockDim.x) {
+        float v = x[at + i];
+        if (rows) v += rows[at + i];
+        out[at + i] = v + vec[i];
+    }
+}
+
+extern "C" int li_add_rows(const float* x, const float* rows, const float* vec, float* out, int n_rows, int width,
+                           hipStream_t stream) {
+    if (n_rows <= 0 || width <= 0) return LI_OK;
+    if (!x || !vec || !out) return LI_BAD_ARG;
+    dim3 grid(n_rows, n_rows >= 1024 ? 1 : (width + 1023) / 1024);
+    add_rows_kernel<<<grid, 256, 0, stream>>>(x, rows, vec, out, width);
     LI_CHECK_LAUNCH();
     return LI_OK;
 }

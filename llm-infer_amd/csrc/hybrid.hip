@@ -182,7 +182,7 @@ __global__ __launch_bounds__(64 * DA_WAVES) void diff_attn_kernel(
     const T* __restrict__ q, T* __restrict__ out, MapPages pg, const int* __restrict__ pos,
     const int* __restrict__ tok_slot, int H, int G, int d, int dv, float scale, int block, int window, float lambda,
     float out_eps, float out_scale, const float* __restrict__ sink, const float* __restrict__ slopes,
-    const float* __restrict__ gate, int gate_stride, int gate_col, int gate_elem, float softcap) {
+    const float* __restrict__ gate, int gate_stride, int gate_col, int gate_elem, float softcap, int keep) {
     extern __shared__ float lds[];
     const int DP = round_up(d, 16), KW = MAPS * DP;
     float* sq = lds;                                   // [KW]
@@ -205,12 +205,15 @@ __global__ __launch_bounds__(64 * DA_WAVES) void diff_attn_kernel(
 #pragma unroll
         for (int c = 0; c < DA_MAXV; ++c) o[a][c] = 0.f;
     }
-    const int n_tiles = (p - lo) / 64 + 1;
+    // the kept keys before lo first (n_keep of them, in tiles of 64), then lo .. p
+    const int n_keep = min(keep, lo), k_tiles = (n_keep + 63) / 64;
+    const int n_tiles = k_tiles + (p - lo) / 64 + 1;
     for (int tile = wave; tile < n_tiles; tile += DA_WAVES) {
-        const int j = lo + tile * 64 + lane;           // this lane's key
+        const int j0 = tile < k_tiles ? tile * 64 : lo + (tile - k_tiles) * 64, j_end = tile < k_tiles ? n_keep - 1 : p;
+        const int j = j0 + lane;                       // this lane's key
         float s[MAPS];
         const T* kh = nullptr;
-        if (j <= p) kh = (const T*)pg.k + (int64_t)table[j / PAGE] * pg.page_stride + g * k_head_elems(KW);
+        if (j <= j_end) kh = (const T*)pg.k + (int64_t)table[j / PAGE] * pg.page_stride + g * k_head_elems(KW);
 #pragma unroll
         for (int a = 0; a < MAPS; ++a) {
             float acc = 0.f;
@@ -230,9 +233,9 @@ __global__ __launch_bounds__(64 * DA_WAVES) void diff_attn_kernel(
 #pragma unroll
             for (int c = 0; c < DA_MAXV; ++c) o[a][c] *= f;
         }
-        const int n_keys = min(64, p - (lo + tile * 64) + 1);
+        const int n_keys = min(64, j_end - j0 + 1);
         for (int kk = 0; kk < n_keys; ++kk) {
-            const int jj = lo + tile * 64 + kk;
+            const int jj = j0 + kk;
             const T* vh = (const T*)pg.v + (int64_t)table[jj / PAGE] * pg.page_stride + g * v_head_elems(dv);
             float w[MAPS];
 #pragma unroll
@@ -307,9 +310,9 @@ extern "C" int li_diff_attn(const void* q, void* out, int dt, void* k_pages, voi
                             const int* page_table, int max_pages, const int* pos, const int* tok_slot, int n, int H, int G,
                             int maps, int d, int dv, float scale, int block, int window, float lambda, float out_eps,
                             float out_scale, const float* sink, const float* slopes, const float* gate, int gate_stride,
-                            int gate_col, int gate_elem, float softcap, hipStream_t stream) {
+                            int gate_col, int gate_elem, float softcap, int keep, hipStream_t stream) {
     if (n <= 0) return LI_OK;
-    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || block < 0 || window < 0 || softcap < 0.f) return LI_BAD_ARG;
+    if (H <= 0 || G <= 0 || H % G || d <= 0 || dv <= 0 || block < 0 || window < 0 || keep < 0 || softcap < 0.f) return LI_BAD_ARG;
     if (gate && (gate_col < 0 || gate_col + (gate_elem ? H * dv : H) > gate_stride)) return LI_BAD_ARG;
     if (maps < 1 || maps > 2 || dv > 64 * DA_MAXV) return LI_UNSUPPORTED;
     MapPages pg{k_pages, v_pages, page_stride, page_table, max_pages};
@@ -318,7 +321,7 @@ extern "C" int li_diff_attn(const void* q, void* out, int dt, void* k_pages, voi
     if (lds > 60000) return LI_UNSUPPORTED;
 #define GO(M) diff_attn_kernel<T, M><<<grid, blk, lds, stream>>>((const T*)q, (T*)out, pg, pos, tok_slot, H, G, d, dv, scale, \
                                                                  block, window, lambda, out_eps, out_scale, sink, slopes, gate, \
-                                                                 gate_stride, gate_col, gate_elem, softcap)
+                                                                 gate_stride, gate_col, gate_elem, softcap, keep)
     DISPATCH_T(dt, { if (maps == 1) GO(1); else GO(2); });
 #undef GO
     LI_CHECK_LAUNCH();
@@ -641,12 +644,12 @@ extern "C" int li_gated_group_norm(const float* y, const float* zrows, int z_str
 }
 
 // ---------------------------------------------------------------------------
-// out[t][j] = w[j] . h[t] in float32 for a few rows of a float32 matrix w [n, width] (a router's): one
+// out[t][j] = w[j] . h[t] (+ bias[j]) in float32 for a few rows of a float32 matrix w [n, width] (a router's): one
 // workgroup per (token, output), its threads stride the width; every sum has one fixed order whatever the batch.
 // ---------------------------------------------------------------------------
 template <class T, int TOK>
 __global__ __launch_bounds__(256) void small_logits_kernel(const T* __restrict__ h, const float* __restrict__ w,
-                                                           float* __restrict__ out, int n_rows, int width, int n) {
+                                                           float* __restrict__ out, const float* __restrict__ bias, int n_rows, int width, int n) {
     __shared__ float scratch[16];
     const int t0 = blockIdx.x * TOK, j = blockIdx.y, tid = threadIdx.x;
     const float* wj = w + (int64_t)j * width;
@@ -673,20 +676,20 @@ __global__ __launch_bounds__(256) void small_logits_kernel(const T* __restrict__
 #pragma unroll
         for (int u = 0; u < 16; ++u) acc += part[k][u];
         acc = block_sum(acc, scratch);                     // the waves' sums in wave order
-        if (tid == 0 && t0 + k < n_rows) out[(int64_t)(t0 + k) * n + j] = acc;
+        if (tid == 0 && t0 + k < n_rows) out[(int64_t)(t0 + k) * n + j] = bias ? acc + bias[j] : acc;
     }
 }
 
-extern "C" int li_small_logits(const void* h, int dt, const float* w, float* out, int n_rows, int width, int n,
+extern "C" int li_small_logits(const void* h, int dt, const float* w, float* out, const float* bias, int n_rows, int width, int n,
                                hipStream_t stream) {
     if (n_rows <= 0 || n <= 0) return LI_OK;
     if (width <= 0 || n > 65535) return LI_BAD_ARG;
     if (n_rows >= 256) {                                   // many tokens: four a workgroup share every weight fetched
         dim3 grid((n_rows + 3) / 4, n);
-        DISPATCH_T(dt, (small_logits_kernel<T, 4><<<grid, 256, 0, stream>>>((const T*)h, w, out, n_rows, width, n)));
+        DISPATCH_T(dt, (small_logits_kernel<T, 4><<<grid, 256, 0, stream>>>((const T*)h, w, out, bias, n_rows, width, n)));
     } else {
         dim3 grid(n_rows, n);
-        DISPATCH_T(dt, (small_logits_kernel<T, 1><<<grid, 256, 0, stream>>>((const T*)h, w, out, n_rows, width, n)));
+        DISPATCH_T(dt, (small_logits_kernel<T, 1><<<grid, 256, 0, stream>>>((const T*)h, w, out, bias, n_rows, width, n)));
     }
     LI_CHECK_LAUNCH();
     return LI_OK;

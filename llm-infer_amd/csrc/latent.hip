@@ -128,12 +128,16 @@ extern "C" int li_softcap(float* x, int64_t n, float cap, hipStream_t stream) {
 // out of the sum a head's output is W_uv (sum of weights * c): one key [c | k_rot] and one value c for all heads.
 // The pages hold them in the matrix instruction's operand order (common.h), keys KW = r + rd rounded up to 16 wide
 // with zeros behind, values r wide.
-// latent_store_kernel, per token, from the float32 rows of the input product (q heads [d | rd] from column q_col,
-// then [latent r | rotated part rd] from column kv_col): c = the latent divided by its root mean square over r,
-// times a weight; the rotated parts turned by the token's position (pairs (2i, 2i + 1) of the first `rot` of the
-// rd dimensions, angle p * freq[i]; the rest pass); key and value into the page of the token's position; every
-// head's rotated query part (and the zeros behind it) into q_out [T, H, KW] from column r on.  The first r columns
-// of q_out are the product per head's (head_linear_kernel).
+// latent_store_kernel, per token, does up to three things (each is left out where its tensor is null):
+//   * from `kv_rows` (float32, [latent r | rotated part rd] from column kv_col): c = the latent divided by its root mean
+//     square over r, times a weight; the rotated part turned by the token's position; key and value into the page of the
+//     token's position;
+//   * from `kv_rows` too: qr columns from column cq_col, the latent that queries go through, divided by their root mean
+//     square and multiplied by a weight, into cq_out [T, qr];
+//   * from `q_rows` (float32, heads [d | rd] from column q_col): every head's rotated query part (and the zeros behind it)
+//     into q_out [T, H, KW] from column r on.  The first r columns of q_out are the product per head's (head_linear_kernel).
+// Turned are the first `rot` of the rd dimensions, in pairs (2i, 2i + 1) or, `half_pairs`, (i, i + rot / 2), by the angle
+// p * freq[i]; sine and cosine are multiplied by `magnitude`; the other dimensions pass.
 // ---------------------------------------------------------------------------
 struct MapPages {
     void* k;
@@ -143,61 +147,96 @@ struct MapPages {
     int max_pages;
 };
 
-__device__ __forceinline__ float rotated(const float* __restrict__ x, int j, int rot, float p,
-                                         const float* __restrict__ freq) {
+#define LATENT_MAX_PAIRS 256
+
+// Dimension j of x behind the rotation; cs: cosine and sine of every pair.
+__device__ __forceinline__ float rotated(const float* __restrict__ x, int j, int rot, int half_pairs,
+                                         const float* __restrict__ cs) {
     if (j >= rot) return x[j];
-    const int pair = j >> 1;
-    const float a = p * freq[pair], c = cosf(a), s = sinf(a);
-    const float u = x[2 * pair], v = x[2 * pair + 1];
-    return (j & 1) ? v * c + u * s : u * c - v * s;
+    const int half = rot >> 1;
+    const int pair = half_pairs ? (j < half ? j : j - half) : j >> 1;
+    const bool second = half_pairs ? j >= half : j & 1;
+    const float u = half_pairs ? x[pair] : x[2 * pair], v = half_pairs ? x[pair + half] : x[2 * pair + 1];
+    const float c = cs[2 * pair], s = cs[2 * pair + 1];
+    return second ? v * c + u * s : u * c - v * s;
 }
 
 template <class T>
-__global__ void latent_store_kernel(const float* __restrict__ proj, int stride, int q_col, int kv_col,
-                                    const float* __restrict__ norm_w, float eps, const float* __restrict__ freq, int rot,
+__global__ void latent_store_kernel(const float* __restrict__ q_rows, int q_stride, int q_col, const float* __restrict__ kv_rows,
+                                    int kv_stride, int kv_col, const float* __restrict__ norm_w, float eps,
+                                    const float* __restrict__ freq, int rot, int half_pairs, float magnitude,
                                     const int* __restrict__ pos, const int* __restrict__ tok_slot, T* __restrict__ q_out,
-                                    MapPages pg, int H, int d, int rd, int r, int KW) {
+                                    MapPages pg, int H, int d, int rd, int r, int KW, int cq_col, int qr,
+                                    const float* __restrict__ cq_w, T* __restrict__ cq_out) {
     __shared__ float scratch[16];
+    __shared__ float cs[2 * LATENT_MAX_PAIRS];
     const int t = blockIdx.x, p = pos[t];
-    const float* row = proj + (int64_t)t * stride;
-    const float* lat = row + kv_col;
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < r; i += blockDim.x) ss += lat[i] * lat[i];
-    const float rr = 1.f / sqrtf(block_sum(ss, scratch) / (float)r + eps);
-    const int page = pg.page_table[(int64_t)tok_slot[t] * pg.max_pages + p / PAGE], off = p % PAGE;
-    T* kp = (T*)pg.k + (int64_t)page * pg.page_stride;
-    T* vp = (T*)pg.v + (int64_t)page * pg.page_stride;
-    const float fp = (float)p;
-    // (few tokens: the grid's second dimension shares a token's key and heads among several workgroups)
-    for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < KW; i += gridDim.y * blockDim.x) {
-        float v = 0.f;
-        if (i < r) {
-            v = lat[i] * rr * norm_w[i];
-            vp[v_offset(off, i, r)] = from_f32<T>(v);
-        } else if (i < r + rd) {
-            v = rotated(lat + r, i - r, rot, fp, freq);
-        }
-        kp[k_offset(off, i, KW)] = from_f32<T>(v);
+    for (int j = threadIdx.x; j < rot >> 1; j += blockDim.x) {
+        float sn, cn;
+        sincosf((float)p * freq[j], &sn, &cn);
+        cs[2 * j] = cn * magnitude; cs[2 * j + 1] = sn * magnitude;
     }
-    const int tail = KW - r;
-    for (int idx = blockIdx.y * blockDim.x + threadIdx.x; idx < H * tail; idx += gridDim.y * blockDim.x) {
-        const int h = idx / tail, j = idx - h * tail;
-        const float v = j < rd ? rotated(row + q_col + (int64_t)h * (d + rd) + d, j, rot, fp, freq) : 0.f;
-        q_out[((int64_t)t * H + h) * KW + r + j] = from_f32<T>(v);
+    __syncthreads();
+    // (few tokens: the grid's second dimension shares a token's work among several workgroups)
+    const int first = blockIdx.y * blockDim.x + threadIdx.x, step = gridDim.y * blockDim.x;
+    auto rms_of = [&](const float* u, int n) {
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < n; i += blockDim.x) ss += u[i] * u[i];
+        return 1.f / sqrtf(block_sum(ss, scratch) / (float)n + eps);
+    };
+    if (kv_rows) {
+        const float* lat = kv_rows + (int64_t)t * kv_stride + kv_col;
+        const float rr = rms_of(lat, r);
+        const int page = pg.page_table[(int64_t)tok_slot[t] * pg.max_pages + p / PAGE], off = p % PAGE;
+        T* kp = (T*)pg.k + (int64_t)page * pg.page_stride;
+        T* vp = (T*)pg.v + (int64_t)page * pg.page_stride;
+        for (int i = first; i < KW; i += step) {
+            float v = 0.f;
+            if (i < r) {
+                v = lat[i] * rr * norm_w[i];
+                vp[v_offset(off, i, r)] = from_f32<T>(v);
+            } else if (i < r + rd) {
+                v = rotated(lat + r, i - r, rot, half_pairs, cs);
+            }
+            kp[k_offset(off, i, KW)] = from_f32<T>(v);
+        }
+        if (cq_w) {
+            const float* c = kv_rows + (int64_t)t * kv_stride + cq_col;
+            const float rq = rms_of(c, qr);
+            for (int i = first; i < qr; i += step) cq_out[(int64_t)t * qr + i] = from_f32<T>(c[i] * rq * cq_w[i]);
+        }
+    }
+    if (q_rows) {
+        const float* row = q_rows + (int64_t)t * q_stride + q_col;
+        const int tail = KW - r;
+        for (int idx = first; idx < H * tail; idx += step) {
+            const int h = idx / tail, j = idx - h * tail;
+            const float v = j < rd ? rotated(row + (int64_t)h * (d + rd) + d, j, rot, half_pairs, cs) : 0.f;
+            q_out[((int64_t)t * H + h) * KW + r + j] = from_f32<T>(v);
+        }
     }
 }
 
-extern "C" int li_latent_store(const float* proj, int stride, int q_col, int kv_col, const float* norm_w, float eps,
-                               const float* freq, int rot, const int* pos, const int* tok_slot, void* q_out, void* k_pages,
-                               void* v_pages, int64_t page_stride, const int* page_table, int max_pages, int dt, int n,
-                               int H, int d, int rd, int r, hipStream_t stream) {
+extern "C" int li_latent_store(const float* q_rows, int q_stride, int q_col, const float* kv_rows, int kv_stride, int kv_col,
+                               const float* norm_w, float eps, const float* freq, int rot, int half_pairs, float magnitude,
+                               const int* pos, const int* tok_slot, void* q_out, void* k_pages, void* v_pages,
+                               int64_t page_stride, const int* page_table, int max_pages, int dt, int n, int H, int d, int rd,
+                               int r, int cq_col, int qr, const float* cq_w, void* cq_out, hipStream_t stream) {
     if (n <= 0) return LI_OK;
-    if (H <= 0 || d < 0 || rd < 0 || r <= 0 || rot < 0 || rot > rd || rot % 2) return LI_BAD_ARG;
+    if (H <= 0 || d < 0 || rd < 0 || r <= 0 || rot < 0 || rot > rd || rot % 2 || (rot && !freq)) return LI_BAD_ARG;
+    if (rot > 2 * LATENT_MAX_PAIRS) return LI_UNSUPPORTED;
+    if ((kv_rows && (kv_col < 0 || kv_col + r + rd > kv_stride || !norm_w)) ||
+        (q_rows && (q_col < 0 || q_col + H * (d + rd) > q_stride || !q_out)) ||
+        (cq_w && (!kv_rows || !cq_out || qr <= 0 || cq_col < 0 || cq_col + qr > kv_stride)))
+        return LI_BAD_ARG;
     MapPages pg{k_pages, v_pages, page_stride, page_table, max_pages};
     const int KW = round_up(r + rd, 16);
-    dim3 grid(n, n >= 256 ? 1 : min(16, (max(KW, H * (KW - r)) + 255) / 256));
-    DISPATCH_T(dt, (latent_store_kernel<T><<<grid, 256, 0, stream>>>(proj, stride, q_col, kv_col, norm_w, eps, freq, rot, pos,
-                                                                  tok_slot, (T*)q_out, pg, H, d, rd, r, KW)));
+    const int most = max(kv_rows ? max(KW, cq_w ? qr : 0) : 0, q_rows ? H * (KW - r) : 0);
+    dim3 grid(n, n >= 256 ? 1 : max(1, min(16, (most + 255) / 256)));
+    DISPATCH_T(dt, (latent_store_kernel<T><<<grid, 256, 0, stream>>>(q_rows, q_stride, q_col, kv_rows, kv_stride, kv_col, norm_w,
+                                                                  eps, freq, rot, half_pairs, magnitude, pos, tok_slot,
+                                                                  (T*)q_out, pg, H, d, rd, r, KW, cq_col, qr, cq_w,
+                                                                  (T*)cq_out)));
     LI_CHECK_LAUNCH();
     return LI_OK;
 }

@@ -170,9 +170,13 @@ class DecoderModel(Part):
             history[0].copy_(x0)
             history[1].copy_(x0)
             x, n_hist = history[1], 1
+        entered = False              # the layer before has taken what this entry's ``before`` part adds along
         for i, e in enumerate(self.schedule):
-            if self._before[i] is not None:
-                x = self.stream_parts[self._before[i]].forward(x, x0, ctx)       # a new tensor: x0 stays as it is
+            if entered:
+                entered = False
+            elif self._before[i] is not None:
+                part = self.stream_parts[self._before[i]]                        # (a new tensor: x0 stays as it is)
+                x = part.forward(x, x0, ctx, e.pass_no) if getattr(part, "takes_pass", False) else part.forward(x, x0, ctx)
             elif x is x0 and self.stream_parts and history is None:
                 x = ops.copy_rows(x0)            # the layers add in place, and a later part reads the embedding's output
             # one view for a mixer, or the list of its views for one that asks several things of the cache
@@ -183,7 +187,13 @@ class DecoderModel(Part):
                 # the norm that reads the residual stream after this layer: the next layer's first
                 nxt = self.layers[self.schedule[i + 1].layer] if i + 1 < len(self.schedule) else None
                 first = getattr(nxt, "first_norm", None)
-                layer.forward(x, ctx, views, e.cache_from is None, next_norm=first() if first else None)
+                extra = {}
+                if getattr(layer, "takes_also", False) and nxt is not None and self._before[i + 1] is not None and self._after[i] is None:
+                    # a part ahead of the next entry that only adds to the stream: in this layer's last pass over the rows
+                    part = self.stream_parts[self._before[i + 1]]
+                    if hasattr(part, "addends"):
+                        extra["also"], entered = part.addends(x0, self.schedule[i + 1].pass_no), True
+                layer.forward(x, ctx, views, e.cache_from is None, next_norm=first() if first else None, **extra)
             else:
                 layer.forward(x, ctx, views, e.cache_from is None)
             if self._after[i] is not None:

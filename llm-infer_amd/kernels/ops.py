@@ -701,14 +701,15 @@ def prefill_meta(ctx) -> dict:
 
 
 def attention_prefill(q, kv, meta, n_heads, n_kv_heads, head_dim, scale, window, block=None, sink=None, slopes=None,
-                      gate=None, gate_col: int = 0, softcap: float | None = None, gate_elem: bool = False) -> torch.Tensor:
+                      gate=None, gate_col: int = 0, softcap: float | None = None, gate_elem: bool = False, keep_first: int = 0) -> torch.Tensor:
     """16-bit attention for a step with whole prompts.  ``kv``: (k_pages, v_pages, page_stride,
     page_table); ``meta``: dict of int32 device arrays tile_seq, tile_q0, seq_slot, seq_qstart,
     seq_qlen, seq_ctx and the int n_tiles.  ``block`` b: a token at position p reads no key before p - p % b;
     ``sink`` (float32 [H]): every head's sum of weights also counts exp(sink[h]); ``slopes`` (float32 [H]): the
     score of the key at position j loses slopes[h] * (p - j); ``gate`` (float32 rows [T, >= gate_col + H]): head
     h's output is multiplied by sigmoid(gate[t][gate_col + h]), with ``gate_elem`` its element d by
-    sigmoid(gate[t][gate_col + h * hd + d]); ``softcap`` c: a scaled score s becomes c tanh(s / c) before anything else."""
+    sigmoid(gate[t][gate_col + h * hd + d]); ``softcap`` c: a scaled score s becomes c tanh(s / c) before anything else;
+    ``keep_first``: the keys before that position are read whatever window and block say."""
     k_pages, v_pages, page_stride, page_table = kv
     _dev(q, k_pages, v_pages, page_table, sink, slopes, gate)
     for name, vec in (("sink", sink), ("slopes", slopes)):
@@ -726,14 +727,15 @@ def attention_prefill(q, kv, meta, n_heads, n_kv_heads, head_dim, scale, window,
         _ptr(meta["seq_qstart"]), _ptr(meta["seq_qlen"]), _ptr(meta["seq_ctx"]), n_heads, n_kv_heads,
         c_float(scale), int(window or 0), int(block or 0), _ptr(sink), _ptr(slopes), _ptr(gate),
         gate.stride(0) if gate is not None else 0, int(gate_col), int(bool(gate_elem and gate is not None)),
-        c_float(softcap or 0.0), _stream()), "attn_prefill")
+        c_float(softcap or 0.0), int(keep_first), _stream()), "attn_prefill")
     return out
 
 
 def attention_decode(q, kv, seq_slot, seq_ctx, n_seqs, n_heads, n_kv_heads, head_dim, scale, window,
-                     splits: int = 1, block=None, sink=None, slopes=None, gate=None, gate_col: int = 0, softcap: float | None = None, gate_elem: bool = False) -> torch.Tensor:
+                     splits: int = 1, block=None, sink=None, slopes=None, gate=None, gate_col: int = 0, softcap: float | None = None, gate_elem: bool = False,
+                     keep_first: int = 0) -> torch.Tensor:
     """16-bit attention for one new token per sequence; q [B, H, hd].  ``block``, ``sink``, ``slopes``, ``gate``,
-    ``gate_elem``, ``softcap``: as for ``attention_prefill``."""
+    ``gate_elem``, ``softcap``, ``keep_first``: as for ``attention_prefill``."""
     k_pages, v_pages, page_stride, page_table = kv
     _dev(q, k_pages, v_pages, page_table, seq_slot, seq_ctx, sink, slopes, gate)
     for name, vec in (("sink", sink), ("slopes", slopes)):
@@ -759,7 +761,7 @@ def attention_decode(q, kv, seq_slot, seq_ctx, n_seqs, n_heads, n_kv_heads, head
         page_table.shape[1], _ptr(seq_slot), _ptr(seq_ctx), n_seqs, n_heads, n_kv_heads, c_float(scale),
         int(window or 0), splits, _ptr(part_o), _ptr(part_ml), int(block or 0), _ptr(sink), _ptr(slopes), _ptr(gate),
         gate.stride(0) if gate is not None else 0, int(gate_col), int(bool(gate_elem and gate is not None)),
-        c_float(softcap or 0.0), _stream()), "attn_decode")
+        c_float(softcap or 0.0), int(keep_first), _stream()), "attn_decode")
     return out
 
 
@@ -1341,7 +1343,7 @@ def _diffattn_lib(map_dim: int, value_dim: int):
     return lib
 
 
-def diff_tile_pairs(qlens, lens_before, block, window) -> tuple:
+def diff_tile_pairs(qlens, lens_before, block, window, keep_first: int = 0) -> tuple:
     """The work items of the matrix-core differential attention for sequences that bring ``qlens`` tokens behind
     ``lens_before``: tiles of up to DIFF_TILE consecutive tokens of one sequence, paired so that a tile that sees many
     keys shares a wave with one that sees few.  Returns (first rows, row counts), two entries an item (a missing
@@ -1354,7 +1356,8 @@ def diff_tile_pairs(qlens, lens_before, block, window) -> tuple:
             start = first - first % block if block else 0
             if window:
                 start = max(start, first - window + 1)
-            tiles.append((last // 32 - start // 32 + 1, at + lo, n))         # (steps of 32 keys, first row, rows)
+            kept = min((keep_first + 31) // 32, start // 32)
+            tiles.append((last // 32 - start // 32 + 1 + kept, at + lo, n))  # (steps of 32 keys, first row, rows)
         at += q
     tiles.sort(key=lambda t: (-t[0], t[1]))
     t0, n = [], []
@@ -1365,23 +1368,23 @@ def diff_tile_pairs(qlens, lens_before, block, window) -> tuple:
     return t0, n
 
 
-def diff_tiles(ctx, block=None, window=None):
+def diff_tiles(ctx, block=None, window=None, keep_first: int = 0):
     """The work items of the matrix-core differential attention for a step (``diff_tile_pairs``) as int32 device
-    arrays and their number; made once per step for each (block, window) and shared.  None for a step in which every
+    arrays and their number; made once per step for each (block, window, keep_first) and shared.  None for a step in which every
     sequence brings one token (every token is then an item of its own)."""
     if ctx.n_tokens == ctx.n_seqs or getattr(ctx, "host_qlens", None) is None:
         return None
 
     def make():
-        t0, n = diff_tile_pairs(ctx.host_qlens, ctx.host_lens_before, int(block or 0), int(window or 0))
+        t0, n = diff_tile_pairs(ctx.host_qlens, ctx.host_lens_before, int(block or 0), int(window or 0), int(keep_first))
         both = torch.tensor([t0, n], dtype=torch.int32).to(ctx.device)
         return both[0], both[1], len(t0) // 2
-    return ctx.shared(("diff_attention_tiles", DIFF_TILE, int(block or 0), int(window or 0)), make)
+    return ctx.shared(("diff_attention_tiles", DIFF_TILE, int(block or 0), int(window or 0), int(keep_first)), make)
 
 
 def diff_attention(q, kv, pos, tok_slot, n_heads, n_kv_heads, maps, d, dv, scale, block, window, lam, out_eps, out_scale,
                    out_dtype, tiles=None, sink=None, key_shares: int = 1, slopes=None, gate=None, gate_col: int = 0,
-                   softcap: float | None = None, gate_elem: bool = False) -> torch.Tensor:
+                   softcap: float | None = None, gate_elem: bool = False, keep_first: int = 0) -> torch.Tensor:
     """Attention of ``maps`` softmax maps (1 or 2) over the same values: o = a_1 - lam a_2, then (``out_eps`` not
     None) o divided by its root mean square over dv, times ``out_scale``.  A token at position p sees the keys
     from p - p % block on (``block`` 0: from 0; ``window`` w: at most the last w).  q [T, H, maps * DP] as
@@ -1394,7 +1397,8 @@ def diff_attention(q, kv, pos, tok_slot, n_heads, n_kv_heads, maps, d, dv, scale
     ``slopes`` (float32 [H]): the score of the key at position j loses slopes[head] * (p - j); the sink loses nothing.
     ``gate`` (float32 rows [T, >= gate_col + H]): head h's output is multiplied by sigmoid(gate[t][gate_col + h]),
     with ``gate_elem`` its element i by sigmoid(gate[t][gate_col + h * dv + i]).  ``softcap`` c: a scaled score s becomes
-    c tanh(s / c) before anything else."""
+    c tanh(s / c) before anything else.  ``keep_first``: the keys before that position are seen whatever block and window
+    say."""
     _dev(q, pos, tok_slot, sink, slopes, gate)
     _need(sink is None or (sink.dtype == torch.float32 and sink.numel() == n_heads), "sink: float32 [H]")
     _need(slopes is None or (slopes.dtype == torch.float32 and slopes.numel() == n_heads and slopes.is_contiguous()), "slopes: float32 [H]")
@@ -1403,7 +1407,7 @@ def diff_attention(q, kv, pos, tok_slot, n_heads, n_kv_heads, maps, d, dv, scale
           "gate: float32 rows with a column for every head (or every element of every head)")
     _need(softcap is None or softcap > 0, "softcap: positive")
     extra = (_ptr(slopes), _ptr(gate), gate.stride(0) if gate is not None else 0, int(gate_col),
-             int(bool(gate_elem and gate is not None)), c_float(softcap or 0.0))
+             int(bool(gate_elem and gate is not None)), c_float(softcap or 0.0), int(keep_first))
     t = q.shape[0]
     dp = padded_map_dim(d)
     _need(maps in (1, 2) and dv <= 512 and n_heads % n_kv_heads == 0, "diff_attention: one or two maps, values up to 512 wide")
@@ -1442,13 +1446,15 @@ def diff_attention_fits(d: int, dv: int) -> bool:
     return padded_map_dim(d) <= 256 and (dv + 31) // 32 * 32 <= 256
 
 
-def small_logits(h, w) -> torch.Tensor:
-    """h W^T in float32 for a float32 matrix of a few rows (a router's): every sum in one fixed order."""
-    _dev(h, w)
+def small_logits(h, w, bias=None) -> torch.Tensor:
+    """h W^T (+ bias) in float32 for a float32 matrix of a few rows (a router's): every sum in one fixed order."""
+    _dev(h, w, bias)
+    _need(bias is None or (bias.dtype == torch.float32 and bias.shape == (w.shape[0],) and bias.is_contiguous()),
+          "small_logits: a float32 bias for every row")
     _need(h.dim() == 2 and h.dtype in DT and w.dtype == torch.float32 and w.dim() == 2 and w.shape[1] == h.shape[1],
           "small_logits: h [T, width], a float32 matrix [n, width]")
     out = torch.empty((h.shape[0], w.shape[0]), dtype=torch.float32, device=h.device)
-    _check(hybrid().li_small_logits(_ptr(h), DT[h.dtype], _ptr(w), _ptr(out), h.shape[0], h.shape[1], w.shape[0], _stream()),
+    _check(hybrid().li_small_logits(_ptr(h), DT[h.dtype], _ptr(w), _ptr(out), _ptr(bias), h.shape[0], h.shape[1], w.shape[0], _stream()),
            "small_logits")
     return out
 
@@ -1711,30 +1717,78 @@ def conv_add(rows, weight, history, ctx, out_dtype) -> torch.Tensor:
     return out
 
 
-def latent_store(proj, q_col, kv_col, norm_weight, eps, inv_freq, rot, pos, tok_slot, kv, n_heads, d, rd, r) -> torch.Tensor:
-    """From the float32 rows of latent attention's input product (from column ``q_col`` every head's [d unrotated | rd
-    rotated] query dimensions, from ``kv_col`` [latent r | rotated key part rd]): the latent divided by its root mean
-    square, times ``norm_weight`` [r]; the rotated parts turned by position (the first ``rot`` of their rd dimensions
-    in pairs (2i, 2i + 1), angle pos * inv_freq[i]); the key [latent | rotated part] (zeros up to the next multiple
-    of 16) and the value (the latent) into the pages.  Returns q [T, H, KW] in the cache's type with every head's
-    rotated part from column r on; the first r columns are left for ``head_linear``."""
-    _dev(proj, norm_weight, inv_freq, pos, tok_slot)
-    _f32_rows(proj, "latent_store rows")
-    t = proj.shape[0]
-    kw = padded_map_dim(r + rd)
-    _need(q_col >= 0 and kv_col >= 0 and max(q_col + n_heads * (d + rd), kv_col + r + rd) <= proj.shape[1], "latent_store: columns beyond the rows")
+def latent_store(kv_rows, kv_col, norm_weight, eps, position, pos, tok_slot, kv, d, rd, r, cq=None) -> torch.Tensor | None:
+    """From the float32 rows of latent attention's input product (from column ``kv_col`` [latent r | rotated key part
+    rd]): the latent divided by its root mean square, times ``norm_weight`` [r]; the rotated part turned by position; the
+    key [latent | rotated part] (zeros up to the next multiple of 16) and the value (the latent) into the pages.
+    ``position``: (inv_freq, rot, half_pairs, magnitude): the first ``rot`` of the rd dimensions are turned in pairs
+    (2i, 2i + 1) or, ``half_pairs``, (i, i + rot / 2) by the angle pos * inv_freq[i], sine and cosine times ``magnitude``.
+    ``cq`` (column, weight float32 [q_rank]): those columns of the rows, divided by their root mean square and multiplied
+    by the weight, are returned as [T, q_rank] in the cache's type (the latent that queries go through)."""
+    _dev(kv_rows, norm_weight, pos, tok_slot)
+    _f32_rows(kv_rows, "latent_store rows")
+    t = kv_rows.shape[0]
+    _need(kv_col >= 0 and kv_col + r + rd <= kv_rows.shape[1], "latent_store: columns beyond the rows")
     _need(norm_weight.dtype == torch.float32 and norm_weight.shape == (r,), "latent norm weight: float32 [r]")
-    _need(0 <= rot <= rd and rot % 2 == 0, "latent_store: an even number of rotated dimensions within rd")
-    if rot:
-        _need(inv_freq is not None and inv_freq.dtype == torch.float32 and inv_freq.numel() >= rot // 2, "inv_freq: float32 [rot / 2]")
     _i32(pos, t, "positions")
     _i32(tok_slot, t, "slots")
+    k_pages, v_pages, page_stride, page_table = _map_pages_check(kv, 1, padded_map_dim(r + rd), r)
+    cq_col, cq_w = cq if cq is not None else (0, None)
+    out = None
+    if cq_w is not None:
+        _dev(cq_w)
+        _need(cq_w.dtype == torch.float32 and cq_w.dim() == 1 and 0 <= cq_col and cq_col + cq_w.numel() <= kv_rows.shape[1],
+              "latent_store: the query latent's columns and float32 weight")
+        out = torch.empty((t, cq_w.numel()), dtype=k_pages.dtype, device=kv_rows.device)
+    _check(hybrid().li_latent_store(None, 0, 0, _ptr(kv_rows), kv_rows.shape[1], kv_col, _ptr(norm_weight), c_float(eps),
+                                    *_rotation(position, rd), _ptr(pos), _ptr(tok_slot), None, _ptr(k_pages), _ptr(v_pages),
+                                    c_int64(page_stride), _ptr(page_table), page_table.shape[1], DT[k_pages.dtype], t, 1, d, rd, r,
+                                    cq_col, 0 if cq_w is None else cq_w.numel(), _ptr(cq_w), _ptr(out), _stream()), "latent_store")
+    return out
+
+
+def _rotation(position, rd):
+    inv_freq, rot, half_pairs, magnitude = position
+    _dev(inv_freq)
+    _need(0 <= rot <= rd and rot % 2 == 0, "latent attention: an even number of rotated dimensions within rd")
+    if rot:
+        _need(inv_freq is not None and inv_freq.dtype == torch.float32 and inv_freq.numel() >= rot // 2, "inv_freq: float32 [rot / 2]")
+    return _ptr(inv_freq), rot, int(bool(half_pairs)), c_float(magnitude)
+
+
+def latent_queries(q_rows, q_col, position, pos, n_heads, d, rd, r, dtype) -> torch.Tensor:
+    """From float32 rows (from column ``q_col`` every head's [d unrotated | rd rotated] query dimensions): q [T, H, KW] of
+    ``dtype``, KW = r + rd rounded up to 16, with every head's rotated part turned by position (``position`` as for
+    ``latent_store``) from column r on and zeros behind it; the first r columns are left for ``head_linear``."""
+    _dev(q_rows, pos)
+    _f32_rows(q_rows, "latent_queries rows")
+    t = q_rows.shape[0]
+    _need(q_col >= 0 and q_col + n_heads * (d + rd) <= q_rows.shape[1], "latent_queries: columns beyond the rows")
+    _need(dtype in DT, "latent_queries: q's type")
+    _i32(pos, t, "positions")
+    q = torch.empty((t, n_heads, padded_map_dim(r + rd)), dtype=dtype, device=q_rows.device)
+    _check(hybrid().li_latent_store(_ptr(q_rows), q_rows.shape[1], q_col, None, 0, 0, None, c_float(0.0), *_rotation(position, rd),
+                                    _ptr(pos), None, _ptr(q), None, None, c_int64(0), None, 0, DT[dtype], t, n_heads, d, rd, r,
+                                    0, 0, None, None, _stream()), "latent_queries")
+    return q
+
+
+def latent_store_queries(rows, q_col, kv_col, norm_weight, eps, position, pos, tok_slot, kv, n_heads, d, rd, r) -> torch.Tensor:
+    """``latent_store`` and ``latent_queries`` in one launch, for queries that lie in the same rows."""
+    _dev(rows, norm_weight, pos, tok_slot)
+    _f32_rows(rows, "latent_store rows")
+    t = rows.shape[0]
+    _need(q_col >= 0 and kv_col >= 0 and max(q_col + n_heads * (d + rd), kv_col + r + rd) <= rows.shape[1], "latent_store: columns beyond the rows")
+    _need(norm_weight.dtype == torch.float32 and norm_weight.shape == (r,), "latent norm weight: float32 [r]")
+    _i32(pos, t, "positions")
+    _i32(tok_slot, t, "slots")
+    kw = padded_map_dim(r + rd)
     k_pages, v_pages, page_stride, page_table = _map_pages_check(kv, 1, kw, r)
-    q = torch.empty((t, n_heads, kw), dtype=k_pages.dtype, device=proj.device)
-    _check(hybrid().li_latent_store(_ptr(proj), proj.shape[1], q_col, kv_col, _ptr(norm_weight), c_float(eps), _ptr(inv_freq), rot,
-                                    _ptr(pos), _ptr(tok_slot), _ptr(q), _ptr(k_pages), _ptr(v_pages), c_int64(page_stride),
-                                    _ptr(page_table), page_table.shape[1], DT[k_pages.dtype], t, n_heads, d, rd, r, _stream()),
-           "latent_store")
+    q = torch.empty((t, n_heads, kw), dtype=k_pages.dtype, device=rows.device)
+    _check(hybrid().li_latent_store(_ptr(rows), rows.shape[1], q_col, _ptr(rows), rows.shape[1], kv_col, _ptr(norm_weight), c_float(eps),
+                                    *_rotation(position, rd), _ptr(pos), _ptr(tok_slot), _ptr(q), _ptr(k_pages), _ptr(v_pages),
+                                    c_int64(page_stride), _ptr(page_table), page_table.shape[1], DT[k_pages.dtype], t, n_heads, d, rd,
+                                    r, 0, 0, None, None, _stream()), "latent_store")
     return q
 
 
@@ -1895,7 +1949,7 @@ def conv_history(rows, col0, channels, taps, history, ctx) -> None:
 
 
 def rot_store(rows, q_col, k_col, v_col, inv_freq, rot, pos, tok_slot, kv, n_heads, n_kv_store, d, dv, q_dtype=None,
-              conv=None) -> torch.Tensor:
+              conv=None, norm=None, magnitude: float = 1.0) -> torch.Tensor:
     """From float32 rows with a token's q heads [H, d] from column ``q_col``, k heads [G, d] from ``k_col`` and values
     [G, dv] from ``v_col`` (it may equal ``k_col``: the values are the keys before their rotation): q and k turned by
     position in their first ``rot`` dimensions, dimension i paired with i + rot / 2, angle pos * inv_freq[i]; k and v
@@ -1903,8 +1957,10 @@ def rot_store(rows, q_col, k_col, v_col, inv_freq, rot, pos, tok_slot, kv, n_hea
     is stored (``kv`` may be None, ``q_dtype`` says q's type).  ``conv`` (weight float32 [channels, taps], history float32
     [slots, taps - 1, channels]): column c of the rows is channel c of a causal convolution over time that everything
     read passes first (the last tap is the token's own; inputs before the step's first token of a sequence come from
-    the history, which is only read: ``conv_history`` brings it up to date afterwards).  Returns q [T, H, DP] in the
-    cache's type."""
+    the history, which is only read: ``conv_history`` brings it up to date afterwards).  ``norm`` (q weight float32 [H d],
+    k weight [G d], eps; not with a convolution): all q columns of a token together, and all its k columns, are divided
+    by their root mean square and multiplied by these weights before the rotation.  ``magnitude`` multiplies sine and cosine.
+    Returns q [T, H, DP] in the cache's type."""
     _dev(rows, inv_freq, pos, tok_slot)
     _f32_rows(rows, "rot_store rows")
     t = rows.shape[0]
@@ -1934,24 +1990,40 @@ def rot_store(rows, q_col, k_col, v_col, inv_freq, rot, pos, tok_slot, kv, n_hea
               "rot_store: conv weight float32 [channels, taps <= 16] for the first columns of the rows")
         _need(hist.dtype == torch.float32 and hist.dim() == 3 and tuple(hist.shape[1:]) == (max(taps - 1, 1), channels),
               "rot_store: conv history float32 [slots, taps - 1, channels]")
+    q_norm = k_norm = None
+    norm_eps = 0.0
+    if norm is not None:
+        q_norm, k_norm, norm_eps = norm
+        _dev(q_norm, k_norm)
+        _need(conv is None, "rot_store: a norm of q and k and a convolution are not built together")
+        for w, n in ((q_norm, n_heads * d), (k_norm, n_kv_store * d)):
+            _need(n == 0 or (w is not None and w.dtype == torch.float32 and w.shape == (n,) and w.is_contiguous()),
+                  "rot_store: q and k norm weights float32 [heads * d]")
     q = torch.empty((t, n_heads, dp), dtype=q_dtype, device=rows.device)
     _check(hybrid().li_rot_store(_ptr(rows), rows.shape[1], q_col, k_col, v_col, _ptr(inv_freq), rot, _ptr(pos), _ptr(tok_slot),
                                  _ptr(q), _ptr(k_pages), _ptr(v_pages), c_int64(page_stride), _ptr(page_table), max_pages,
                                  DT[q_dtype], t, n_heads, n_kv_store, d, dv, _ptr(conv_w), taps, _ptr(hist), channels,
-                                 _stream()), "rot_store")
+                                 _ptr(q_norm), _ptr(k_norm), c_float(norm_eps), c_float(magnitude), _stream()), "rot_store")
     return q
 
 
-def rmsnorm_add(x, y, weight, eps: float, bias=None, next_norm=None) -> torch.Tensor:
+def rmsnorm_add(x, y, weight, eps: float, bias=None, next_norm=None, also=None) -> torch.Tensor:
     """x += (y + bias) / sqrt(mean((y + bias)^2) + eps) * weight, row by row, in place (all float32).  ``next_norm``
     (weight float32 [width], eps, dtype): the RMS norm that reads the finished rows next is taken in the same pass and
-    left for it (``prepared_rmsnorm`` finds it as long as nothing else writes into ``x``)."""
+    left for it (``prepared_rmsnorm`` finds it as long as nothing else writes into ``x``).  ``also`` (rows of x's shape or
+    None, vector float32 [width]): the finished rows gain them before that norm is taken."""
     _dev(x, y, weight, bias)
+    add_rows, add_vec = also if also is not None else (None, None)
+    _dev(add_rows, add_vec)
     _f32_rows(x, "rmsnorm_add x")
     _f32_rows(y, "rmsnorm_add y")
     width = x.shape[1]
     _need(y.shape == x.shape and weight.dtype == torch.float32 and weight.shape == (width,), "rmsnorm_add: rows of one shape, a float32 weight")
     _need(bias is None or (bias.dtype == torch.float32 and bias.shape == (width,)), "rmsnorm_add: a float32 bias")
+    if also is not None:
+        _need(add_vec.dtype == torch.float32 and add_vec.shape == (width,) and add_vec.is_contiguous(), "rmsnorm_add: a float32 vector to add")
+        _need(add_rows is None or (add_rows.dtype == torch.float32 and add_rows.shape == x.shape and add_rows.is_contiguous()
+                                   and add_rows.data_ptr() != x.data_ptr()), "rmsnorm_add: float32 rows of x's shape to add")
     _drop_row_stats(x)
     nw = normed = None
     n_eps, n_dt = 0.0, torch.float32
@@ -1960,11 +2032,23 @@ def rmsnorm_add(x, y, weight, eps: float, bias=None, next_norm=None) -> torch.Te
         _dev(nw)
         _need(nw.dtype == torch.float32 and nw.shape == (width,) and n_dt in DT, "rmsnorm_add: the next norm's float32 weight and type")
         normed = torch.empty(x.shape, dtype=n_dt, device=x.device)
-    _check(hybrid().li_rmsnorm_add(_ptr(x), _ptr(y), _ptr(bias), _ptr(weight), c_float(eps), x.shape[0], width, _ptr(nw),
-                                   c_float(n_eps), _ptr(normed), DT[n_dt], _stream()), "rmsnorm_add")
+    _check(hybrid().li_rmsnorm_add(_ptr(x), _ptr(y), _ptr(bias), _ptr(weight), c_float(eps), x.shape[0], width,
+                                   _ptr(add_rows), _ptr(add_vec), _ptr(nw), c_float(n_eps), _ptr(normed), DT[n_dt], _stream()),
+           "rmsnorm_add")
     if normed is not None:
         x._li_normed = (normed, nw, float(n_eps), x._version)
     return x
+
+
+def add_rows(x, rows, vec) -> torch.Tensor:
+    """x (+ rows) + vec as a new float32 tensor (``vec`` [width] is added to every row)."""
+    _dev(x, rows, vec)
+    _f32_rows(x, "add_rows x")
+    _need(rows is None or (rows.dtype == torch.float32 and rows.shape == x.shape and rows.is_contiguous()), "add_rows: rows of one shape")
+    _need(vec.dtype == torch.float32 and vec.shape == (x.shape[1],) and vec.is_contiguous(), "add_rows: a float32 vector")
+    out = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    _check(hybrid().li_add_rows(_ptr(x), _ptr(rows), _ptr(vec), _ptr(out), x.shape[0], x.shape[1], _stream()), "add_rows")
+    return out
 
 
 def table_route(token_ids, table, n_experts: int, gate_logits=None, has_gate: int = 0) -> torch.Tensor:

@@ -141,9 +141,12 @@ class SandwichBlock(Block):
                 raise ValueError("a sandwich block has one norm before each part and one with a weight after it")
             if getattr(s.part, "reads_float32", False):
                 s.norm.dtype = torch.float32
+        # the last pass over the rows can add more to them (``also`` of forward)
+        self.takes_also = getattr(self.sublayers[-1].post_norm, "adds_also", False)
 
-    def forward(self, x, ctx, cache_views, owns_cache=True, next_norm=None):
-        """``next_norm``: the norm that reads ``x`` after this layer, if the caller knows it."""
+    def forward(self, x, ctx, cache_views, owns_cache=True, next_norm=None, also=None):
+        """``next_norm``: the norm that reads ``x`` after this layer, if the caller knows it.  ``also`` (rows or None, a
+        vector): added to ``x`` behind this layer, before that norm."""
         views = iter(cache_views)
         ops.expect_norm(x, None)                 # no product adds into x itself: no norm rides along
         for i, s in enumerate(self.sublayers):
@@ -159,7 +162,10 @@ class SandwichBlock(Block):
             else:
                 y = torch.zeros_like(x)
                 _run_part(s, h, ctx, view, y, owns_cache)
-            s.post_norm.add_into(x, y, bias, after)
+            if also is not None and i + 1 == len(self.sublayers):
+                s.post_norm.add_into(x, y, bias, after, also)
+            else:
+                s.post_norm.add_into(x, y, bias, after)
 
 
 @register_block("post_norm")

@@ -169,7 +169,8 @@ class RoutedExperts(Part):
 
     The router has n_experts + ``n_identity`` outputs; its logits and everything after them are float32:
     s = softmax(W_router h); the ``top`` outputs with the largest s + correction are chosen (``correction``: a
-    tensor with one number an output, used for the choice only); their weights are s / (sum of the chosen s +
+    tensor with one number an output, used for the choice only; ``router_bias``: a tensor with one number an output that is
+    part of its logit); their weights are s / (sum of the chosen s +
     1e-20) * ``route_scale``.  The last ``n_identity`` outputs have no matrices: chosen, they add weight * h.
     ``shared_ff`` > 0: one more expert of that width runs for every token; ``shared_gate``: it is weighted by
     sigmoid(w_sg . h).
@@ -188,11 +189,12 @@ class RoutedExperts(Part):
     # through every expert and 3.46 sorted by expert (40 launches a layer and a wait for the counts against 3 launches),
     # 1,024 tokens 4.90 and 4.86, 2,048 tokens 8.58 and 7.50
     GROUPED_FROM = 256
+    writes_rows = True          # forward_into overwrites the rows it is handed
 
     def __init__(self, *, hidden_size, n_experts, expert_ff, top, n_identity=0, route_scale=1.0, correction=True,
                  shared_ff=0, shared_gate=True, gated=True, activation="silu", scores="softmax", renormalize=True,
                  weight_on="output", routing="router", vocab_size=0, limit=None, shared_limit=None, alpha=1.702,
-                 up_shift=1.0, names=None, prefix, dtype, device):
+                 up_shift=1.0, router_bias=False, names=None, prefix, dtype, device):
         if not 1 <= top <= n_experts + n_identity:
             raise ValueError(f"routed experts: top {top} of {n_experts + n_identity} outputs")
         if scores not in ("softmax", "sigmoid") or weight_on not in ("output", "input"):
@@ -206,6 +208,9 @@ class RoutedExperts(Part):
         self.clamped = bool(gated) and activation == "clamped_swish"
         if self.clamped and not (limit is not None and float(limit) > 0):
             raise ValueError("routed experts: the clamped activation needs a positive limit")
+        if router_bias and routing == "table":
+            raise ValueError("routed experts: a table has no logits to bias")
+        self.router_bias = bool(router_bias)
         self.table_routing, self.vocab_size = routing == "table", int(vocab_size)
         self.takes_ctx = self.table_routing           # the token ids come with the step
         self.limit, self.alpha, self.up_shift = float(limit or 0.0), float(alpha), float(up_shift)
@@ -217,10 +222,10 @@ class RoutedExperts(Part):
         self.hidden_size, self.n_experts, self.expert_ff, self.top = hidden_size, n_experts, expert_ff, top
         self.n_identity, self.route_scale, self.correction = n_identity, float(route_scale), bool(correction)
         self.shared_ff, self.shared_gate = int(shared_ff or 0), bool(shared_gate) and bool(shared_ff)
-        self.names = {"router": "router.weight", "correction": "router.correction", "expert": "e{}.", "shared": "shared.",
+        self.names = {"router": "router.weight", "router_bias": "router.bias", "correction": "router.correction", "expert": "e{}.", "shared": "shared.",
                       "gate": "gate", "up": "up", "down": "down", "shared_gate": "shared.sg", "table": "table", **(names or {})}
         self.prefix, self.dtype, self.device = prefix, dtype, device
-        self.w_router = self.w_gate_up = self.w_down = self.bias = None
+        self.w_router = self.w_gate_up = self.w_down = self.bias = self.b_router = None
 
     def _experts(self):
         n = self.names
@@ -233,6 +238,8 @@ class RoutedExperts(Part):
             out = {n["table"]: ParamSpec((self.vocab_size, self.top), "int", f"distinct:{self.n_experts}")}
         else:
             out = {n["router"]: ParamSpec((self.n_experts + self.n_identity, d), "vector", "wide")}
+        if self.router_bias:
+            out[n["router_bias"]] = ParamSpec((self.n_experts + self.n_identity,), "vector", "small")
         if self.correction:
             out[n["correction"]] = ParamSpec((self.n_experts + self.n_identity,), "vector", "small")
         for p, f in self._experts():
@@ -268,6 +275,9 @@ class RoutedExperts(Part):
         rows = ([] if self.table_routing else [tensors[n["router"]].float()]) + \
             ([tensors[n["shared_gate"]].float().view(1, d)] if self.shared_gate else [])
         self.w_router = torch.cat(rows, 0).contiguous() if rows else None     # float32: the logits are summed in float32
+        if self.router_bias:
+            b = tensors[n["router_bias"]].as_subclass(torch.Tensor).float()
+            self.b_router = torch.cat([b, torch.zeros((int(self.shared_gate),), dtype=torch.float32, device=b.device)]).contiguous()
         self.table = tensors[n["table"]] if self.table_routing else None
         self.bias = tensors[n["correction"]] if self.correction else None
 
@@ -327,18 +337,19 @@ class RoutedExperts(Part):
                 raise ValueError("routed experts: a table chooses by token id and needs the step")
             gate = ops.small_logits(h, self.w_router) if self.shared_gate else None
             return ops.table_route(ctx.token_ids, self.table, self.n_experts, gate, has_gate)
-        logits = ops.small_logits(h, self.w_router)
+        logits = ops.small_logits(h, self.w_router, self.b_router)
         return ops.moe_route(logits, self.bias, h, residual, self.n_experts + self.n_identity, self.n_experts, self.top,
                              has_gate, self.route_scale, self.sigmoid_scores, self.renormalize)
 
-    def forward(self, h, residual, ctx=None):
-        weights = self._weights(h, residual, ctx)
-        if (self.per_expert is not None and self.n_experts and h.shape[0] * self.top >= self.GROUPED_FROM * self.n_experts
-                and not torch.cuda.is_current_stream_capturing()):
-            return self._grouped(h, residual, weights)
+    def _is_grouped(self, h) -> bool:
+        """True where every expert runs its own two products on its own tokens' rows."""
+        return (self.per_expert is not None and self.n_experts > 0 and h.shape[0] * self.top >= self.GROUPED_FROM * self.n_experts
+                and not torch.cuda.is_current_stream_capturing())
+
+    def _dense_hidden(self, h, weights):
+        """The hidden rows of all experts side by side, every expert's block with the token's weight for it."""
         if not self.gated:
-            t = self._hidden(h, self.w_gate_up, weights, None, None, self.n_experts, self.expert_ff, self.shared_ff)
-            return ops.linear(t, self.w_down, ops.EPI_ADD, out=residual)
+            return self._hidden(h, self.w_gate_up, weights, None, None, self.n_experts, self.expert_ff, self.shared_ff)
         if self.clamped:
             # the shared expert's outputs, behind the others', take its own limit
             t = ops.linear(h, self.w_gate_up, ops.EPI_CLAMPGLU, out_dtype=self.dtype,
@@ -346,5 +357,19 @@ class RoutedExperts(Part):
                                                  self.n_experts * self.expert_ff))
         else:
             t = ops.linear(h, self.w_gate_up, ops.EPI_SWIGLU, out_dtype=self.dtype)
-        ops.scale_blocks(t, weights, self.n_experts, self.expert_ff, self.shared_ff)
-        ops.linear(t, self.w_down, ops.EPI_ADD, out=residual)
+        return ops.scale_blocks(t, weights, self.n_experts, self.expert_ff, self.shared_ff)
+
+    def forward(self, h, residual, ctx=None):
+        weights = self._weights(h, residual, ctx)
+        if self._is_grouped(h):
+            return self._grouped(h, residual, weights)
+        ops.linear(self._dense_hidden(h, weights), self.w_down, ops.EPI_ADD, out=residual)
+
+    def forward_into(self, h, out, ctx=None, view=None, owns_cache=True):
+        """The result written over the float32 rows ``out``."""
+        if self.n_identity or self._is_grouped(h):
+            out.zero_()                          # the outputs that pass a token on, or the experts one by one, add into it
+            self.forward(h, out, ctx)
+        else:
+            ops.linear(self._dense_hidden(h, self._weights(h, out, ctx)), self.w_down, out=out)
+        return None

@@ -10,7 +10,8 @@ from .base import Part
 
 _NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "g": "g_proj.weight",
           "sink": "sink", "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias",
-          "q_conv": "q_conv.weight", "k_conv": "k_conv.weight", "v_conv": "v_conv.weight"}
+          "q_conv": "q_conv.weight", "k_conv": "k_conv.weight", "v_conv": "v_conv.weight", "q_norm": "q_norm.weight",
+          "k_norm": "k_norm.weight"}
 
 
 @register_mixer("gated_attention")
@@ -32,6 +33,10 @@ class GatedAttention(Part):
     * the layer's position part (``rope_half``): q and k are turned in their first ``rotary_dim`` dimensions, i paired
       with i + rotary_dim / 2; values never are.
     * ``bias``: q, k and v have biases, added in the projection.
+    * ``qk_norm_eps``: q and k as projected are each divided by the root mean square of all their rows together (all heads
+      at once; this eps inside the root) and multiplied by a weight for every row, before any rotation.
+    * ``keep_first`` n: with a window or blocks, the keys of the first n positions stay visible to every later token, at
+      their true positions (their pages are never given back).
     * ``conv_taps`` n > 0: a causal convolution over time, channel by channel, directly behind the projection of q, k
       and v (weights [channels, n], the last column the current token's; zeros before a sequence's first token).  The
       last n - 1 projected rows of every sequence are state of the cache.
@@ -55,7 +60,7 @@ class GatedAttention(Part):
 
     def __init__(self, *, hidden_size, n_heads, n_kv_heads, head_dim, v_head_dim=None, scale, window=None, block=None,
                  sink=True, gate=True, softcap=None, values="own", bias=False, conv_taps=0, slope_exponent=None, reads_kv=False,
-                 keep_window="own", keep_block="own", names=None, position=None, prefix, dtype, device):
+                 keep_window="own", keep_block="own", keep_first=0, qk_norm_eps=None, names=None, position=None, prefix, dtype, device):
         if n_heads % n_kv_heads != 0:
             raise ValueError("n_heads must be a multiple of n_kv_heads")
         if values not in ("own", "keys"):
@@ -80,6 +85,13 @@ class GatedAttention(Part):
             raise ValueError("gated attention: gate True (one number a head), 'elements' or False")
         if softcap is not None and not float(softcap) > 0:
             raise ValueError("gated attention: a positive soft cap")
+        if int(keep_first) < 0:
+            raise ValueError("gated attention: keep_first is a number of positions")
+        if qk_norm_eps is not None and (conv_taps or values == "keys"):
+            raise ValueError("gated attention: a norm of q and k is built without convolutions and with values of their own")
+        # (without a window or blocks every key is seen anyway)
+        self.keep_first = int(keep_first) if self.window is not None or self.block is not None else 0
+        self.qk_norm_eps = None if qk_norm_eps is None else float(qk_norm_eps)
         self.sink, self.gate, self.values_are_keys, self.bias = bool(sink), bool(gate), values == "keys", bool(bias)
         self.gate_elem, self.softcap = gate == "elements", None if softcap is None else float(softcap)
         self.gate_rows = (n_heads * v_head_dim if self.gate_elem else n_heads) if self.gate else 0
@@ -99,7 +111,7 @@ class GatedAttention(Part):
         self.gate_col = self.channels
         if self.conv_taps:
             self.keeps_when_reading = (0,)       # the convolution's history is the layer's own whatever keys it reads
-        self.w_in = self.wo = self.b_in = self.conv = self.sinks = self.slopes = None
+        self.w_in = self.wo = self.b_in = self.conv = self.sinks = self.slopes = self.qk_norm = None
 
     def _kv_names(self):
         return [] if self.reads_kv else (["k"] if self.values_are_keys else ["k", "v"])
@@ -112,6 +124,8 @@ class GatedAttention(Part):
             out[n[key]] = ParamSpec((rows[key], w))
             if self.bias:
                 out[n[key + "_bias"]] = ParamSpec((rows[key],), "vector", "small")
+            if self.qk_norm_eps is not None and key != "v":
+                out[n[key + "_norm"]] = ParamSpec((rows[key],), "vector", "ones")
             if self.conv_taps:
                 out[n[key + "_conv"]] = ParamSpec((rows[key], self.conv_taps), "vector", "wide")
         if self.sink:
@@ -133,6 +147,8 @@ class GatedAttention(Part):
             self.b_in = ops.glu_params(torch.cat([b, pad]).contiguous())
         if self.conv_taps:
             self.conv = torch.cat([plain(tensors[n[k + "_conv"]]).float() for k in keys], 0).contiguous()
+        if self.qk_norm_eps is not None:
+            self.qk_norm = (tensors[n["q_norm"]], None if self.reads_kv else tensors[n["k_norm"]], self.qk_norm_eps)
         self.sinks = tensors[n["sink"]] if self.sink else None
         if self.slope_exponent is not None:
             H = self.n_heads
@@ -140,7 +156,8 @@ class GatedAttention(Part):
                 .to(torch.float32).to(self.wo.device)
 
     def cache_specs(self):
-        kv = KVSpec(self.n_kv_heads, ops.padded_map_dim(self.head_dim), self.keep_window, self.v_head_dim, self.keep_block, "maps")
+        kv = KVSpec(self.n_kv_heads, ops.padded_map_dim(self.head_dim), self.keep_window, self.v_head_dim, self.keep_block, "maps",
+                    self.keep_first)
         if self.conv_taps:
             return [StateSpec((max(self.conv_taps - 1, 1), self.channels), "float32"), kv]
         return [kv]
@@ -162,7 +179,7 @@ class GatedAttention(Part):
         shares = max(1, ctx.decode_splits(self.n_kv_heads, self.n_heads) // 4)
         for span in (self.block, self.window):
             if span:
-                shares = min(shares, max(1, span // 128))
+                shares = min(shares, max(1, (span + self.keep_first) // 128))
         return shares
 
     def _splits(self, ctx) -> int:
@@ -171,7 +188,7 @@ class GatedAttention(Part):
         splits = ctx.decode_splits(self.n_kv_heads, self.n_heads)
         for span in (self.block, self.window):
             if span:
-                splits = min(splits, max(1, span // 128))
+                splits = min(splits, max(1, (span + self.keep_first) // 128))
         return 1 << (splits.bit_length() - 1)
 
     def attend(self, h, ctx, views, owns_cache, proj=None, col0=0):
@@ -191,7 +208,8 @@ class GatedAttention(Part):
         # the convolution rides in the kernel that turns and stores; the history is brought up to date behind it
         conv = (self.conv, views[0].state) if self.conv_taps else None
         q = ops.rot_store(proj, col0 + self.q_col, col0 + self.k_col, col0 + self.v_col, getattr(self.position, "inv_freq", None) if self.rot else None,
-                          self.rot, ctx.pos, ctx.tok_slot, kv, H, 0 if self.reads_kv else G, d, dv, kv[0].dtype, conv)
+                          self.rot, ctx.pos, ctx.tok_slot, kv, H, 0 if self.reads_kv else G, d, dv, kv[0].dtype, conv,
+                          self.qk_norm, float(getattr(self.position, "magnitude", 1.0)))
         if self.conv_taps > 1:
             ops.conv_history(proj, 0, self.channels, self.conv_taps, views[0].state, ctx)
         if self.dtype != torch.float32 and d == dv and d % 16 == 0 and d <= 256:
@@ -201,17 +219,18 @@ class GatedAttention(Part):
             gate, gate_col = proj if self.gate else None, col0 + self.gate_col
             if ctx.is_decode:
                 a = ops.attention_decode(q, kv, ctx.seq_slot, ctx.seq_ctx, ctx.n_seqs, H, G, d, self.scale, self.window,
-                                         self._splits(ctx), self.block, self.sinks, self.slopes, gate, gate_col, self.softcap, self.gate_elem)
+                                         self._splits(ctx), self.block, self.sinks, self.slopes, gate, gate_col, self.softcap, self.gate_elem,
+                                         self.keep_first)
             else:
                 a = ops.attention_prefill(q, kv, ops.prefill_meta(ctx), H, G, d, self.scale, self.window, self.block, self.sinks,
-                                          self.slopes, gate, gate_col, self.softcap, self.gate_elem)
+                                          self.slopes, gate, gate_col, self.softcap, self.gate_elem, self.keep_first)
             return a.view(a.shape[0], H * dv)
         sixteen = self.dtype != torch.float32 and ops.diff_attention_fits(d, dv)
         return ops.diff_attention(q, kv, ctx.pos, ctx.tok_slot, H, G, 1, d, dv, self.scale, self.block, self.window, 0.0, None, 1.0,
-                                  self.dtype, ops.diff_tiles(ctx, self.block, self.window) if sixteen else None, sink=self.sinks,
+                                  self.dtype, ops.diff_tiles(ctx, self.block, self.window, self.keep_first) if sixteen else None, sink=self.sinks,
                                   key_shares=self._key_shares(ctx) if sixteen else 1, slopes=self.slopes,
                                   gate=proj if self.gate else None, gate_col=col0 + self.gate_col, softcap=self.softcap,
-                                  gate_elem=self.gate_elem)
+                                  gate_elem=self.gate_elem, keep_first=self.keep_first)
 
     def forward(self, h, ctx, views, residual, owns_cache=True):
         ops.linear(self.attend(h, ctx, views, owns_cache), self.wo, ops.EPI_ADD, out=residual)

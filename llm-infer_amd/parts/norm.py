@@ -14,6 +14,7 @@ class RMSNorm(Part):
     """out = x / sqrt(mean(x^2) + eps) * weight, in float32; the weight is kept in float32
     (include/kernels_cpu.hpp:43-54, src/model/block.cpp:81-83)."""
     can_be_lazy = True          # forward takes ``lazy``
+    adds_also = True            # add_into takes ``also``
 
     def __init__(self, *, size: int, eps: float, name: str = "weight", one_plus: bool = False, scalar: bool = False,
                  prefix: str, dtype, device):
@@ -50,13 +51,13 @@ class RMSNorm(Part):
                 return ready
         return ops.rmsnorm(x, self.weight, self.eps, self.dtype, rows)
 
-    def add_into(self, x, y, bias=None, next_norm=None) -> None:
+    def add_into(self, x, y, bias=None, next_norm=None, also=None) -> None:
         """x += this norm of (y + bias), in one pass that also takes the norm that reads ``x`` next where that is one of
-        this kind."""
+        this kind.  ``also`` (rows or None, a vector): added to ``x`` as well, before that norm."""
         nxt = None
         if isinstance(next_norm, RMSNorm) and next_norm.weight is not None:
             nxt = (next_norm.weight, next_norm.eps, next_norm.dtype)
-        ops.rmsnorm_add(x, y.rows() if isinstance(y, ops.NormedPair) else y, self.weight, self.eps, bias, nxt)
+        ops.rmsnorm_add(x, y.rows() if isinstance(y, ops.NormedPair) else y, self.weight, self.eps, bias, nxt, also)
 
 
 @register_norm("layernorm")

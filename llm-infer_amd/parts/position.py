@@ -17,7 +17,11 @@ class RotaryPosition(Part):
     "high", "original"} stretches by wavelength instead: with l = 2 pi / f, a frequency whose l is shorter than
     original / high stays, one whose l is longer than original / low becomes f / factor, and between the two
     s = (original / l - low) / (high - low) blends them, (1 - s) f / factor + s f; the frequencies are then made in
-    float64 and rounded once.
+    float64 and rounded once.  ``yarn`` {"factor", "original", "fast", "slow"} stretches by dimension: with D(t) = rotary_dim
+    ln(original / (2 pi t)) / (2 ln theta), the pairs up to max(floor(D(fast)), 0) keep their frequency, those from
+    min(ceil(D(slow)), rotary_dim - 1) on are divided by factor, a linear ramp between the two blends, and sine and cosine
+    are multiplied by ``magnitude`` = 0.1 ln(factor) + 1 (1 without ``yarn``); only mixers whose own kernels turn their
+    dimensions take a magnitude.
 
     The kernels rotate adjacent pairs only.  A half-paired model runs on them unchanged because a
     score is a sum over the dimensions of a head and does not care about their order: the mixer asks
@@ -35,7 +39,10 @@ class RotaryPosition(Part):
     """
 
     def __init__(self, *, theta: float, rotary_dim: int, head_dim: int, pairing: str = "adjacent",
-                 scaling_factor: float = 1.0, wavelength_scaling: dict | None = None, prefix: str = "", dtype, device):
+                 scaling_factor: float = 1.0, wavelength_scaling: dict | None = None, yarn: dict | None = None,
+                 prefix: str = "", dtype, device):
+        if yarn is not None and wavelength_scaling is not None:
+            raise ValueError("rotation: one way of stretching the frequencies")
         self.rotary_dim, self.head_dim, self.pairing, self.theta = rotary_dim, head_dim, pairing, float(theta)
         self.scaling_factor = float(scaling_factor)
         self.prefix = prefix
@@ -44,6 +51,9 @@ class RotaryPosition(Part):
         inv = 1.0 / torch.pow(torch.tensor(float(theta), dtype=torch.float32), i / float(rotary_dim))
         if wavelength_scaling is not None:
             inv = scaled_by_wavelength(float(theta), rotary_dim, wavelength_scaling)
+        self.magnitude = 1.0
+        if yarn is not None:
+            inv, self.magnitude = scaled_by_ramp(float(theta), rotary_dim, yarn)
         if self.scaling_factor != 1.0:
             # linear scaling: every frequency divided by the factor, i.e. positions counted in its units
             inv = inv / self.scaling_factor
@@ -61,7 +71,12 @@ class RotaryPosition(Part):
             order[2 * j], order[2 * j + 1] = j, j + half
         return order
 
+    def _plain_turn(self):
+        if self.magnitude != 1.0:
+            raise ValueError("rotation with a magnitude: not built for mixers that turn q and k in their product")
+
     def rotate_store(self, qkv, ctx, kv_view, n_heads, n_kv_heads, head_dim):
+        self._plain_turn()
         k = v = table = stride = None
         if n_kv_heads > 0:
             k, v, table, stride = kv_view.k, kv_view.v, kv_view.page_table, kv_view.page_stride
@@ -72,6 +87,7 @@ class RotaryPosition(Part):
     def project_rotate_store(self, h, w, ctx, kv_view, n_heads, n_kv_heads, head_dim):
         """q, k, v = h W^T, rotated and stored (the rows of W's q and k heads in ``head_row_order``); with
         16-bit storage the rotation and the cache write happen in the product's epilogue."""
+        self._plain_turn()
         return _project(self, h, w, ctx, kv_view, n_heads, n_kv_heads, head_dim, self.inv_freq, self.rotary_dim,
                         True, self._table(ctx))
 
@@ -111,6 +127,26 @@ def scaled_by_wavelength(theta: float, rotary_dim: int, scaling: dict) -> torch.
             f = (1.0 - s) * f / factor + s * f
         out.append(f)
     return torch.tensor(out, dtype=torch.float64).to(torch.float32)
+
+
+def scaled_by_ramp(theta: float, rotary_dim: int, scaling: dict) -> tuple:
+    """(theta^(-2i / rotary_dim) for every pair i, stretched along a ramp of the pairs, and the factor of sine and cosine;
+    see ``RotaryPosition``); float64 throughout, the frequencies rounded to float32 at the end."""
+    import math
+    factor, original, fast, slow = (float(scaling[k]) for k in ("factor", "original", "fast", "slow"))
+    if not (factor > 0 and original > 0 and fast > 0 and slow > 0 and theta > 0 and theta != 1.0):
+        raise ValueError("yarn: factor, original, fast and slow positive, a base other than 1")
+
+    def pair_that_turns(times):                  # ``times`` times over the original positions, as a fraction of a pair
+        return rotary_dim * math.log(original / (2.0 * math.pi * times)) / (2.0 * math.log(theta))
+    begin = max(math.floor(pair_that_turns(fast)), 0)
+    end = min(math.ceil(pair_that_turns(slow)), rotary_dim - 1)
+    out = []
+    for i in range(rotary_dim // 2):
+        f = theta ** (-2.0 * i / rotary_dim)
+        ramp = min(max((i - begin) / max(end - begin, 0.001), 0.0), 1.0)
+        out.append(f / factor * ramp + f * (1.0 - ramp))
+    return torch.tensor(out, dtype=torch.float64).to(torch.float32), 0.1 * math.log(factor) + 1.0
 
 
 def _project(part, h, w, ctx, kv_view, n_heads, n_kv_heads, head_dim, inv_freq, rotary_dim, fusable, table=None):

@@ -30,6 +30,37 @@ class Reinject(Part):
         return ops.linear(ops.concat_cast(x, x0, self.dtype), self.weight, out_dtype=torch.float32)
 
 
+@register_stream("pass_entry")
+class PassEntry(Part):
+    """Ahead of pass t of a stretch of layers that runs ``times`` times: x <- x + step[t], and for t > 0 the embedding's
+    output x0 is added too.  ``name``: local name of the vectors' tensor [times, hidden], kept in float32.  A layer that
+    ends with a pass over the finished rows may take the sum along (``addends``)."""
+
+    takes_pass = True           # forward is handed the number of the pass
+
+    def __init__(self, *, hidden_size, times, name="step", prefix, dtype, device):
+        if times < 1:
+            raise ValueError("a repeated stretch of layers: at least one pass")
+        self.hidden_size, self.times, self.name = hidden_size, int(times), name
+        self.prefix, self.dtype, self.device = prefix, dtype, device
+        self.steps = None
+
+    def params(self):
+        return {self.name: ParamSpec((self.times, self.hidden_size), "vector", "small")}
+
+    def bind(self, tensors):
+        t = tensors[self.name].as_subclass(torch.Tensor)
+        self.steps = [t[i].contiguous() for i in range(self.times)]
+
+    def addends(self, x0, pass_no: int):
+        """What is added to the stream: (rows or None, vector)."""
+        return (x0 if pass_no > 0 else None), self.steps[pass_no]
+
+    def forward(self, x, x0, ctx, pass_no: int):
+        """A new float32 tensor; ``x`` and ``x0`` stay as they are."""
+        return ops.add_rows(x, *self.addends(x0, pass_no))
+
+
 @register_stream("depth_average")
 class DepthAverage(Part):
     """x <- sum over j < n_terms of w[j] X_j: a weighted average over depth of the residual stream's values so far,
