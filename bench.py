@@ -62,7 +62,7 @@ def main() -> int:
                     help="leave out the long contexts, batch 128 and the generation run that the default run adds to points")
     ap.add_argument("--generate", type=int, default=0,
                     help="also generate for this many 128-token prompts with budgets drawn from 16..512 tokens")
-    ap.add_argument("--compare", default="", choices=["", "manirax", "risonex", "dupolorn", "favizen", "dopivik"],
+    ap.add_argument("--compare", default="", choices=["", "manirax", "risonex", "dupolorn", "favizen", "dopivik", "pusisun"],
                     help="instead of the default workload: prefill and decode throughput of this design at a few "
                          "layer sizes beside the Llama decoder at equal sizes (random weights, a few layers each)")
     ap.add_argument("--sizes", default="", help="with --compare: the layer sizes to run, comma separated (default: all)")
@@ -216,6 +216,23 @@ def compare_configs(design: str, size: dict, layers: int, context: int) -> dict:
         stack = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": size["ff"]}} for i in range(layers)]
         other = {"architecture": "Dopivik", "embedding": {"scale": 1.0}, "layers": stack, "norm": {"eps": 1e-5},
                  "vocab": size["vocab"], "width": w, "max_positions": context}
+        return {"llama": llama, design: other}
+    if design == "pusisun":
+        # the Llama decoder's heads: latent attention (hd unrotated and hd / 2 rotated query dimensions a head behind a latent
+        # of 3/8 of the width, values a head wide, a latent of 3 hd / 2 for keys and values, stretched frequencies) in every
+        # other layer; in the others attention with biases, a norm over all of q and of k, a sink, a bias by distance and a
+        # window of 1,024 positions beside the first 16; sixteen experts of a quarter of the feed-forward's width, four of
+        # them chosen (as many multiplications a token as the Llama decoder's feed-forward).  The second layer runs twice, so
+        # that as many layers run as the Llama decoder has
+        lat = {"heads": H, "dim": hd, "rot_dim": hd // 2, "vdim": hd, "kv_rank": 3 * hd // 2, "q_rank": 3 * w // 8,
+               "scale": (3 * hd // 2) ** -0.5, "rot": {"base": 10000.0, "dims": hd // 2,
+                                                       "scaling": {"factor": 40.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+        att = {"heads": H, "kv_heads": G, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": 1024, "keep_first": 16}}
+        routed = {"kind": "moe", "expert": {"ff": size["ff"] // 4}, "router": {"experts": 16, "top": 4}}
+        stack = [{"type": "attention" if i % 2 else "latent_attention", "mixer": att if i % 2 else lat, "mlp": routed}
+                 for i in range(max(2, layers - 1))]
+        other = {"architecture": "Pusisun", "embedding": {"scale": 1.0}, "layers": stack, "loop": {"start": 1, "stop": 2, "times": 2},
+                 "norm": {"eps": 1e-5}, "vocab": size["vocab"], "width": w, "max_positions": context}
         return {"llama": llama, design: other}
     assert design == "manirax"
     # the attention of the same heads beside a linear attention of half as many heads with states of hd x hd

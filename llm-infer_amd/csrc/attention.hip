@@ -433,7 +433,7 @@ __global__ __launch_bounds__(256, HD <= 128 ? 2 : 1) void attn_prefill_kernel(
     const int p_win = first_key(base + q0) / PAGE;
     const int n_keep = min((ex.keep + PAGE - 1) / PAGE, p_win), p_lo = p_win - n_keep;
     const int p_hi = (base + min(q0 + TT - 1, qlen - 1)) / PAGE;
-    const int wp_lo = n_keep ? p_lo : first_key(base + first) / PAGE;
+    const int wp_lo = ex.keep > 0 ? p_lo : first_key(base + first) / PAGE;      // (a wave behind the first may begin beyond kept keys)
     auto page_of = [&](int p) { return p < p_win ? p - p_lo : p; };
     const int wp_hi = wave_live ? (base + min(first + 31, qlen - 1)) / PAGE : -1;
     const int* table = c.page_table + (int64_t)seq_slot[seq] * c.max_pages;

@@ -325,54 +325,49 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
 
 // The states of the workgroups that shared a token's keys (`part` [token, head, shares, map, 2 + VALUE_DIM]: maximum in
 // units of log 2, sum, output) added up in the order of the shares, then the sink, the difference of the maps and the
-// norm as above: one wave per (token, head).
+// norm as above: one workgroup per (token, head), a thread an output element, 16 shares' loads in flight at a time.
+#define MERGE_THREADS ((VALUE_DIM + 63) / 64 * 64)
+
 template <class T, int MAPS>
-__global__ __launch_bounds__(64) void diff_attn_merge_kernel(const float* __restrict__ part, T* __restrict__ out, int H,
-                                                             int S, int dv, float lambda, float out_eps, float out_scale,
-                                                             const float* __restrict__ sink, const float* __restrict__ gate,
-                                                             int gate_stride, int gate_col, int gate_elem) {
-    constexpr int W = 2 + VALUE_DIM, NV = (VALUE_DIM + 63) / 64;
+__global__ __launch_bounds__(MERGE_THREADS) void diff_attn_merge_kernel(const float* __restrict__ part, T* __restrict__ out, int H,
+                                                                        int S, int dv, float lambda, float out_eps, float out_scale,
+                                                                        const float* __restrict__ sink, const float* __restrict__ gate,
+                                                                        int gate_stride, int gate_col, int gate_elem) {
+    constexpr int W = 2 + VALUE_DIM;
+    __shared__ float scratch[16];
     const int64_t unit = blockIdx.x;
-    const int h = (int)(unit % H), lane = threadIdx.x;
-    float val[MAPS][NV];
+    const int h = (int)(unit % H), lane = threadIdx.x & 63, i = threadIdx.x;
+    float val[MAPS];
 #pragma unroll
     for (int a = 0; a < MAPS; ++a) {
         const float* p = part + (unit * S * MAPS + a) * W;
-        // lane s fetches share s's maximum and sum (S is at most 64), so no load waits for another
+        // lane s of every wave fetches share s's maximum and sum (S is at most 64), so no load waits for another
         const float ms = lane < S ? p[(int64_t)lane * MAPS * W] : -INFINITY, ls = lane < S ? p[(int64_t)lane * MAPS * W + 1] : 0.f;
+        float first[16];                                   // the first 16 shares' outputs are on their way meanwhile
+#pragma unroll
+        for (int u = 0; u < 16; ++u) first[u] = u < S && i < VALUE_DIM ? p[(int64_t)u * MAPS * W + 2 + i] : 0.f;
         const float s2 = sink ? sink[h] * 1.4426950408889634f : -INFINITY;
         const float M = fmaxf(wave_max(ms), s2);
         const float fs = ms == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(ms - M);
         const float L = wave_sum(ls * fs) + (sink ? __builtin_amdgcn_exp2f(s2 - M) : 0.f);
-        float O[NV];
+        float O = 0.f;
+        for (int s0 = 0; s0 < S; s0 += 16) {
+            float t[16];
 #pragma unroll
-        for (int v = 0; v < NV; ++v) O[v] = 0.f;
-#pragma unroll 4
-        for (int s = 0; s < S; ++s) {
-            const float f = __shfl(fs, s, WAVE);
-            const float* q = p + (int64_t)s * MAPS * W + 2;
+            for (int u = 0; u < 16; ++u) t[u] = s0 == 0 ? first[u] : (s0 + u < S && i < VALUE_DIM ? p[(int64_t)(s0 + u) * MAPS * W + 2 + i] : 0.f);
 #pragma unroll
-            for (int v = 0; v < NV; ++v) if (v * 64 + lane < VALUE_DIM) O[v] += q[v * 64 + lane] * f;
+            for (int u = 0; u < 16; ++u) O += t[u] * __shfl(fs, min(s0 + u, 63), WAVE);
         }
-#pragma unroll
-        for (int v = 0; v < NV; ++v) val[a][v] = O[v] / L;
+        val[a] = O / L;
     }
-    float ss = 0.f, res[NV];
-#pragma unroll
-    for (int v = 0; v < NV; ++v) {
-        float x = val[0][v];
-        if (MAPS == 2) x -= lambda * val[MAPS - 1][v];
-        res[v] = v * 64 + lane < dv ? x : 0.f;
-        ss += res[v] * res[v];
-    }
-    ss = wave_sum(ss);
-    float rr = out_eps >= 0.f ? out_scale / sqrtf(ss / (float)dv + out_eps) : out_scale;
+    float x = val[0];
+    if (MAPS == 2) x -= lambda * val[MAPS - 1];
+    if (i >= dv) x = 0.f;
+    float rr = out_scale;
+    if (out_eps >= 0.f) rr = out_scale / sqrtf(block_sum(x * x, scratch) / (float)dv + out_eps);
     const float* grow = gate ? gate + (unit / H) * gate_stride + gate_col : nullptr;
     if (gate && !gate_elem) rr *= 1.f / (1.f + expf(-grow[h]));
-#pragma unroll
-    for (int v = 0; v < NV; ++v)
-        if (v * 64 + lane < dv)
-            out[unit * dv + v * 64 + lane] = from_f32<T>(res[v] * rr * (gate_elem ? 1.f / (1.f + expf(-grow[h * dv + v * 64 + lane])) : 1.f));
+    if (i < dv) out[unit * dv + i] = from_f32<T>(x * rr * (gate_elem ? 1.f / (1.f + expf(-grow[h * dv + i])) : 1.f));
 }
 
 extern "C" int li_diffattn_map_dim() { return MAP_DIM; }
@@ -418,7 +413,7 @@ extern "C" int li_diffattn(const void* q, void* out, int dt, const void* k_pages
                                             lambda, out_eps, out_scale, split, sink, part, slopes, gate, gate_stride, gate_col,      \
                                             gate_elem, softcap, keep);                                                               \
         if (shares > 1)                                                                                                              \
-            diff_attn_merge_kernel<T, M><<<n_tiles * H, 64, 0, stream>>>(part, (T*)out, H, shares, dv, lambda, out_eps, out_scale, sink, \
+            diff_attn_merge_kernel<T, M><<<n_tiles * H, MERGE_THREADS, 0, stream>>>(part, (T*)out, H, shares, dv, lambda, out_eps, out_scale, sink, \
                                                                       gate, gate_stride, gate_col, gate_elem);                       \
     } while (0)
 #define GO(T, M) do { if (hc) GO1(T, M, false, true); else if (split) GO1(T, M, false, false); else GO1(T, M, true, false); } while (0)

@@ -149,6 +149,93 @@ __global__ void rot_store_kernel(const float* __restrict__ rows, int stride, int
     }
 }
 
+// The same, four columns at a time, where nothing is convolved and every part begins and ends at a multiple of four columns
+// (the host sees to it): a token's sums of squares, q, k and v as float32 quads in, q and k as quads out.
+template <class T>
+__global__ __launch_bounds__(256) void rot_store_vec_kernel(const float* __restrict__ rows, int stride, int q_col, int k_col, int v_col,
+                                                            const float* __restrict__ inv_freq, int rot,
+                                                            const int* __restrict__ pos, const int* __restrict__ tok_slot,
+                                                            T* __restrict__ q_out, StorePages pg, int H, int G, int d, int dv,
+                                                            const float* __restrict__ q_norm, const float* __restrict__ k_norm,
+                                                            float norm_eps, float magnitude) {
+    struct alignas(4 * sizeof(T)) Out4 { T v[4]; };
+    __shared__ float scratch[16];
+    __shared__ float cs[2 * ROT_MAX_PAIRS];
+    const int t = blockIdx.x, p = pos[t], DP = round_up(d, 16), half = rot >> 1;
+    const float* row = rows + (int64_t)t * stride;
+    float q_rms = 1.f, k_rms = 1.f;
+    if (q_norm) {
+        auto squares = [&](const float* u, int n) {
+            float ss = 0.f;
+#pragma unroll 4
+            for (int i = 4 * threadIdx.x; i < n; i += 1024) {
+                const f32x4 x = *(const f32x4*)(u + i);
+                ss += x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+            }
+            return ss;
+        };
+        const float sq = squares(row + q_col, H * d), sk = G > 0 ? squares(row + k_col, G * d) : 0.f;
+        q_rms = 1.f / sqrtf(block_sum(sq, scratch) / (float)(H * d) + norm_eps);
+        if (G > 0) k_rms = 1.f / sqrtf(block_sum(sk, scratch) / (float)(G * d) + norm_eps);
+    }
+    for (int j = threadIdx.x; j < half; j += blockDim.x) {
+        float sn, cn;
+        sincosf((float)p * inv_freq[j], &sn, &cn);
+        cs[2 * j] = cn * magnitude; cs[2 * j + 1] = sn * magnitude;
+    }
+    if (half) __syncthreads();
+    T* kp = nullptr;
+    T* vp = nullptr;
+    const int off = p % PAGE;
+    if (G > 0) {
+        const int page = pg.page_table[(int64_t)tok_slot[t] * pg.max_pages + p / PAGE];
+        kp = (T*)pg.k + (int64_t)page * pg.page_stride;
+        vp = (T*)pg.v + (int64_t)page * pg.page_stride;
+    }
+    const int dq = DP >> 2, n_qk = (H + G) * dq, total = n_qk + G * (dv >> 2);
+    for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < total; e += gridDim.y * blockDim.x) {
+        if (e < n_qk) {
+            const int u = e / dq, i = 4 * (e - u * dq);
+            const bool is_q = u < H;
+            const float* src = row + (is_q ? q_col + u * d : k_col + (u - H) * d);
+            const float* nw = !q_norm ? nullptr : (is_q ? q_norm + u * d : k_norm + (u - H) * d);
+            const float rms = is_q ? q_rms : k_rms;
+            auto normed = [&](int c) {
+                f32x4 x = *(const f32x4*)(src + c);
+                if (nw) {
+                    const f32x4 w = *(const f32x4*)(nw + c);
+#pragma unroll
+                    for (int k = 0; k < 4; ++k) x[k] *= rms * w[k];
+                }
+                return x;
+            };
+            f32x4 val = {0.f, 0.f, 0.f, 0.f};
+            if (i < d) {
+                val = normed(i);
+                if (i < rot) {
+                    const int j = i < half ? i : i - half;
+                    const f32x4 other = normed(i < half ? i + half : i - half);
+#pragma unroll
+                    for (int k = 0; k < 4; ++k) {
+                        const float c_ = cs[2 * (j + k)], s_ = cs[2 * (j + k) + 1];
+                        val[k] = i < half ? val[k] * c_ - other[k] * s_ : val[k] * c_ + other[k] * s_;
+                    }
+                }
+            }
+            Out4 o;
+#pragma unroll
+            for (int k = 0; k < 4; ++k) o.v[k] = from_f32<T>(val[k]);
+            if (is_q) *(Out4*)(q_out + ((int64_t)t * H + u) * DP + i) = o;
+            else *(Out4*)(kp + (int64_t)(u - H) * k_head_elems(DP) + k_offset(off, i, DP)) = o;      // (consecutive in the page)
+        } else {
+            const int r = 4 * (e - n_qk), g = r / dv, j = r - g * dv;
+            const f32x4 x = *(const f32x4*)(row + v_col + r);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) vp[(int64_t)g * v_head_elems(dv) + v_offset(off, j + k, dv)] = from_f32<T>(x[k]);
+        }
+    }
+}
+
 extern "C" int li_rot_store(const float* rows, int stride, int q_col, int k_col, int v_col, const float* inv_freq, int rot,
                             const int* pos, const int* tok_slot, void* q_out, void* k_pages, void* v_pages,
                             int64_t page_stride, const int* page_table, int max_pages, int dt, int n, int H, int G_store,
@@ -168,6 +255,15 @@ extern "C" int li_rot_store(const float* rows, int stride, int q_col, int k_col,
     }
     StorePages pg{k_pages, v_pages, page_stride, page_table, max_pages};
     const int total = (H + G_store) * round_up(d, 16) + G_store * dv;
+    if (!conv_w && !((d | dv | rot / 2 | q_col | stride) & 3) && (!G_store || !((k_col | v_col) & 3)) &&
+        !(((uintptr_t)rows | (uintptr_t)q_norm | (uintptr_t)k_norm | (uintptr_t)q_out | (uintptr_t)k_pages) & 15) && !(page_stride & 3)) {
+        dim3 quads(n, n >= 512 ? 1 : (total / 4 + 255) / 256);
+        DISPATCH_T(dt, (rot_store_vec_kernel<T><<<quads, 256, 0, stream>>>(rows, stride, q_col, k_col, v_col, inv_freq, rot, pos, tok_slot,
+                                                                      (T*)q_out, pg, H, G_store, d, dv, q_norm, k_norm, norm_eps,
+                                                                      magnitude)));
+        LI_CHECK_LAUNCH();
+        return LI_OK;
+    }
     dim3 grid(n, n >= 512 ? 1 : (total + 255) / 256);
     DISPATCH_T(dt, (rot_store_kernel<T><<<grid, 256, 0, stream>>>(rows, stride, q_col, k_col, v_col, inv_freq, rot, pos, tok_slot,
                                                               (T*)q_out, pg, H, G_store, d, dv, conv_w, taps, hist, channels, q_norm,
@@ -284,6 +380,109 @@ extern "C" int li_rmsnorm_add(float* x, const float* y, const float* b, const fl
     else
         DISPATCH_T(next_dt, (rmsnorm_add_kernel<T, false><<<n_rows, RA_THREADS, 0, stream>>>(x, y, b, w, eps, width, add_rows, add_vec, next_w,
                                                                                        next_eps, (T*)next)));
+    LI_CHECK_LAUNCH();
+    return LI_OK;
+}
+
+// The same with y the weighted sum of a few rows: y[t] = sum over j < top of weights[t][j] * rows[slot_of[t][j]] (slot_of -1:
+// nothing), in the order of j: what a token's chosen experts have made, summed on the way.  width a multiple of 4, at most
+// 4 NC RA_THREADS.
+template <class TN, int NC>
+__global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_pairs_kernel(float* __restrict__ x, const float* __restrict__ rows,
+                                                                       const int* __restrict__ slot_of,
+                                                                       const float* __restrict__ weights, int top,
+                                                                       const float* __restrict__ w, float eps, int width,
+                                                                       const float* __restrict__ add_rows,
+                                                                       const float* __restrict__ add_vec,
+                                                                       const float* __restrict__ next_w, float next_eps,
+                                                                       TN* __restrict__ next) {
+    struct alignas(4 * sizeof(TN)) Out4 { TN v[4]; };
+    __shared__ float scratch[16];
+    const int64_t row = blockIdx.x;
+    const int quads = width >> 2;
+    float* xr = x + row * width;
+    int at[NC];                                            // this thread's quads (beyond the row: its last one, counted nowhere)
+    bool in[NC];
+    f32x4 y[NC], xs[NC], ws[NC];
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+        in[c] = threadIdx.x + c * RA_THREADS < quads;
+        at[c] = 4 * min((int)threadIdx.x + c * RA_THREADS, quads - 1);
+        y[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+        xs[c] = *(const f32x4*)(xr + at[c]);
+        ws[c] = *(const f32x4*)(w + at[c]);
+    }
+    for (int j0 = 0; j0 < top; j0 += 4) {                  // four rows' loads in flight at a time
+        f32x4 t[4][NC];
+        float f[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int s = j0 + k < top ? slot_of[row * top + j0 + k] : -1;
+            f[k] = s >= 0 ? weights[row * top + j0 + k] : 0.f;
+#pragma unroll
+            for (int c = 0; c < NC; ++c) t[k][c] = s >= 0 ? *(const f32x4*)(rows + (int64_t)s * width + at[c]) : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+#pragma unroll
+            for (int c = 0; c < NC; ++c)
+#pragma unroll
+                for (int q = 0; q < 4; ++q) y[c][q] += f[k] * t[k][c][q];
+    }
+    float ss = 0.f, s2 = 0.f;
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+        if (in[c]) ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
+    const float r = 1.f / sqrtf(block_sum(ss, scratch) / (float)width + eps);
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+        f32x4 o = xs[c];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) o[q] += y[c][q] * r * ws[c][q];
+        if (add_vec) {
+            if (add_rows) {
+                const f32x4 e = *(const f32x4*)(add_rows + row * width + at[c]);
+#pragma unroll
+                for (int q = 0; q < 4; ++q) o[q] += e[q];
+            }
+            const f32x4 e = *(const f32x4*)(add_vec + at[c]);
+#pragma unroll
+            for (int q = 0; q < 4; ++q) o[q] += e[q];
+        }
+        xs[c] = o;
+        if (next_w) ws[c] = *(const f32x4*)(next_w + at[c]);
+        if (in[c]) {
+            *(f32x4*)(xr + at[c]) = o;
+            s2 += o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
+        }
+    }
+    if (!next_w) return;
+    const float r2 = 1.f / sqrtf(block_sum(s2, scratch) / (float)width + next_eps);
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+        if (in[c]) {
+            Out4 v;
+#pragma unroll
+            for (int q = 0; q < 4; ++q) v.v[q] = from_f32<TN>(xs[c][q] * r2 * ws[c][q]);
+            *(Out4*)(next + row * width + at[c]) = v;
+        }
+    }
+}
+
+extern "C" int li_rmsnorm_add_pairs(float* x, const float* rows, const int* slot_of, const float* weights, int top, const float* w,
+                                    float eps, int n_rows, int width, const float* add_rows, const float* add_vec,
+                                    const float* next_w, float next_eps, void* next, int next_dt, hipStream_t stream) {
+    if (n_rows <= 0) return LI_OK;
+    if (width <= 0 || top < 1 || !x || !rows || !slot_of || !weights || !w || (next_w && !next) || (add_rows && !add_vec)) return LI_BAD_ARG;
+    if (width % 4 || width > 4 * 8 * RA_THREADS) return LI_UNSUPPORTED;
+    if (!next_w) next_dt = DT_F32;
+    const int quads = width / 4, nc = quads <= RA_THREADS ? 1 : (quads <= 2 * RA_THREADS ? 2 : (quads <= 4 * RA_THREADS ? 4 : 8));
+#define GO(NC)                                                                                                             \
+    DISPATCH_T(next_dt, (rmsnorm_add_pairs_kernel<T, NC><<<n_rows, RA_THREADS, 0, stream>>>(x, rows, slot_of, weights, top, w, eps, \
+                                                                                         width, add_rows, add_vec, next_w, next_eps, \
+                                                                                         (T*)next)))
+    if (nc == 1) GO(1); else if (nc == 2) GO(2); else if (nc == 4) GO(4); else GO(8);
+#undef GO
     LI_CHECK_LAUNCH();
     return LI_OK;
 }

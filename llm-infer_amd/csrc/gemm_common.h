@@ -377,6 +377,17 @@ static void launch_splitk_add_norm(const float* ws, int splits, const Epilogue& 
 #undef GO
 }
 
+// The rows of a product of several experts (gemm_wreg's pairs mode): pairs sorted by expert, counts[e] of them from
+// offsets[e] on; pair p reads row row_of[p] of X (null: row p) and writes row p; expert e's tiled matrix begins w_stride
+// elements behind expert e - 1's.
+struct PairTiles {
+    const int* counts;
+    const int* offsets;
+    const int* row_of;
+    int n_experts;
+    int64_t w_stride;
+};
+
 static int make_epilogue(Epilogue& e, void* C, int mode, int out_dt, int M, int N, const RopeStore* rs) {
     e.C = C; e.mode = mode; e.out_dt = out_dt; e.M = M; e.N = N;
     e.rs = RopeStore{};

@@ -15,10 +15,14 @@ __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) {
 // before the next group starts.  The workgroups that are resident on an XCD together (32 or 64)
 // then cover a near-square block of tiles and share its rows of X and W through that L2; with
 // the tiles of X simply fastest they would share one tile of W and stream all of X past it.
-__device__ __forceinline__ void tile_of_workgroup(int GM, int& bx, int& by, int& bz) {
-    const int gx = gridDim.x, gy = gridDim.y;
+// gx: the tiles of X (fewer than the grid's where a kernel finds out itself how many there are; the workgroups beyond
+// gx * gridDim.y have none then, bx = -1).
+__device__ __forceinline__ void tile_of_workgroup(int GM, int& bx, int& by, int& bz, int gx) {
+    const int gy = gridDim.y;
     const int total = gx * gy * gridDim.z;
-    const int L = blockIdx.x + gx * (blockIdx.y + gy * blockIdx.z);
+    const int L = blockIdx.x + gridDim.x * (blockIdx.y + gy * blockIdx.z);
+    bx = -1;
+    if (L >= total) return;
     const int xcd = L & 7, per = total >> 3, rem = total & 7;
     const int id = xcd * per + min(xcd, rem) + (L >> 3);
     bz = id / (gx * gy);
@@ -55,7 +59,7 @@ __global__ __launch_bounds__(256) void gemm_big_kernel(const T* __restrict__ X, 
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int wn = wave & 1, wm = wave >> 1;
     int bx, by, bz;
-    tile_of_workgroup(8, bx, by, bz);
+    tile_of_workgroup(8, bx, by, bz, gridDim.x);
     const int m0 = bx * BM, n0 = by * BN;
     const int n_limit = TILED ? ((e.N + 15) & ~15) : e.N;
     const int kb = bz * k_per_split, ke = min(K, kb + k_per_split);   // this workgroup's share of K
@@ -235,10 +239,15 @@ __device__ __forceinline__ void wreg_epilogue(const Epilogue& e, int m, int n, c
     else epilogue4_base(e, m, n, v);
 }
 
+// MODE_PAIRS: the products of several experts as one launch (PairTiles): a tile of X is up to BM consecutive pairs of one
+// expert, read through row_of, and the workgroup's W is that expert's.  How many tiles there are is counted here, from the
+// experts' counts; the grid holds as many as there can be.  Every epilogue of MODE -1, K whole.
+enum { MODE_PAIRS = -2 };
+
 template <class T, int NI, int MODE, int MJ = 8, int A = 2>
 __global__ __launch_bounds__(256) void gemm_wreg_kernel(const T* __restrict__ X, const T* __restrict__ Wt,
                                                         int K, int k_per_split, float* __restrict__ ws, Epilogue e,
-                                                        int wg_blocks, RowScale rsc) {
+                                                        int wg_blocks, RowScale rsc, PairTiles pt) {
     typedef typename Vec<T>::v8 v8;
     // A step is 64 of K: two halves of 32, each one matrix instruction deep.
     // MJ: fragments of X (16 rows each) per wave and half step; every wave takes all the tile's rows of X
@@ -251,12 +260,48 @@ __global__ __launch_bounds__(256) void gemm_wreg_kernel(const T* __restrict__ X,
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int wn = wave;
-    int bx, by, bz;
-    tile_of_workgroup(8, bx, by, bz);
+    int bx, by, bz, m0;
+    if constexpr (MODE == MODE_PAIRS) {
+        int all = 0;
+        for (int e0 = 0; e0 < pt.n_experts; e0 += 64) {
+            int tiles = e0 + lane < pt.n_experts ? (pt.counts[e0 + lane] + BM - 1) / BM : 0;
+#pragma unroll
+            for (int o = 32; o > 0; o >>= 1) tiles += __shfl_xor(tiles, o, WAVE);
+            all += tiles;
+        }
+        tile_of_workgroup(8, bx, by, bz, __builtin_amdgcn_readfirstlane(all));
+        if (bx < 0) return;
+        int expert = 0, before = 0, row0 = 0, rows = 0;
+        for (int e0 = 0; e0 < pt.n_experts; e0 += 64) {
+            const int c = e0 + lane < pt.n_experts ? pt.counts[e0 + lane] : 0, mine = (c + BM - 1) / BM;
+            int incl = mine;                                 // tiles of this expert and those of the 64 before it
+#pragma unroll
+            for (int o = 1; o < 64; o <<= 1) {
+                const int u = __shfl_up(incl, o, WAVE);
+                if (lane >= o) incl += u;
+            }
+            const uint64_t behind = __builtin_amdgcn_ballot_w64(before + incl > bx);
+            if (behind) {
+                const int at = __builtin_ctzll(behind);
+                expert = __builtin_amdgcn_readfirstlane(e0 + at);
+                row0 = (bx - before - __builtin_amdgcn_readfirstlane(__shfl(incl - mine, at, WAVE))) * BM;
+                rows = __builtin_amdgcn_readfirstlane(__shfl(c, at, WAVE));
+                break;
+            }
+            before += __builtin_amdgcn_readfirstlane(__shfl(incl, 63, WAVE));
+        }
+        const int first = __builtin_amdgcn_readfirstlane(pt.offsets[expert]);
+        m0 = first + row0;
+        e.M = first + rows;
+        Wt += expert * pt.w_stride;
+    } else {
+        tile_of_workgroup(8, bx, by, bz, gridDim.x);
+        m0 = bx * BM;
+    }
     // wg_blocks: the blocks of 16 rows of W that a workgroup takes of its 4 NI (fewer: more workgroups, for a
     // product whose full tiles would leave CUs without one); a wave whose block lies beyond them fetches and
     // multiplies the workgroup's last block again and stores nothing of it
-    const int m0 = bx * BM, n0 = by * 16 * wg_blocks;
+    const int n0 = by * 16 * wg_blocks;
     const int n_end = min(e.N, n0 + 16 * wg_blocks);
     const int kb = bz * k_per_split, ke = min(K, kb + k_per_split);
     // a share of K that is 32 more than a multiple of 64 ends with a step of one half
@@ -280,7 +325,8 @@ __global__ __launch_bounds__(256) void gemm_wreg_kernel(const T* __restrict__ X,
 #pragma unroll
     for (int i = 0; i < PER_WAVE; ++i) {
         const int q = wave * PER_WAVE + i, p = lane >> 3;
-        const int row = min(m0 + 8 * q + p, e.M - 1);
+        int row = min(m0 + 8 * q + p, e.M - 1);
+        if constexpr (MODE == MODE_PAIRS) { if (pt.row_of) row = pt.row_of[row]; }
         xoff[i] = ((uint32_t)row * (uint32_t)K + 8 * ((lane & 7) ^ p)) * 2;
     }
     // Loads past the last step of K are not branched around: they fetch the last step again (into a buffer
@@ -666,7 +712,7 @@ extern "C" int li_gemm_wreg(const void* X, const void* Wt, int dt, void* C, int 
             allowed = true;                                                                               \
         }                                                                                                 \
         kfn<<<grid, block, lds, stream>>>((const T*)X, (const T*)Wt, K, k_per_split, ws, e, wg_blocks,     \
-                                          rsc ? *rsc : no_scale);                                         \
+                                          rsc ? *rsc : no_scale, PairTiles{});                            \
     } while (0)
 #define BY_MODE(T, NI, MJ, A)                             \
     do {                                                  \
@@ -698,5 +744,54 @@ extern "C" int li_gemm_wreg(const void* X, const void* Wt, int dt, void* C, int 
         splitk_reduce_kernel<<<(unsigned)((quads + 255) / 256), 256, 0, stream>>>(ws, splits, e);
         LI_CHECK_LAUNCH();
     }
+    return LI_OK;
+}
+
+// The products of several experts as one launch: C[p] = epilogue(W_e X[row_of[p]]) for all n_pairs pairs (PairTiles; mode
+// EPI_STORE or EPI_SWIGLU; N, K of one expert's matrix; x_rows: rows of X).  tile as for li_gemm_wreg; few_rows 1: the tile
+// has 64 pairs (tile 2 only).
+extern "C" int li_gemm_wreg_pairs(const void* X, const void* Wt, int dt, void* C, int out_dt, int mode, int x_rows, int n_pairs,
+                                  int N, int K, int tile, int few_rows, const int* counts, const int* offsets, const int* row_of,
+                                  int n_experts, int64_t w_stride, hipStream_t stream) {
+    int rc = check_common(X, Wt, C, n_pairs, N, K, mode, out_dt);
+    if (rc) return rc;
+    if ((dt != DT_F16 && dt != DT_BF16) || (mode != EPI_STORE && mode != EPI_SWIGLU) || !counts || !offsets || n_experts < 1)
+        return LI_BAD_ARG;
+    if (tile < 0 || tile > 2 || few_rows < 0 || few_rows > 1 || (few_rows && tile != 2) || (!row_of && x_rows < n_pairs)) return LI_BAD_ARG;
+    if (K % 32 != 0 || ((uintptr_t)X & 15) || ((uintptr_t)Wt & 15) || w_stride % 8) return LI_UNSUPPORTED;
+    if ((int64_t)x_rows * K * 2 >= ((int64_t)1 << 32)) return LI_UNSUPPORTED;
+    if (n_pairs == 0) return LI_OK;
+    Epilogue e;
+    rc = make_epilogue(e, C, mode, out_dt, n_pairs, N, nullptr);
+    if (rc) return rc;
+    const int bn = 256 - 64 * tile, bm = few_rows ? 64 : 128, ahead = few_rows ? 4 : 2, wg_blocks = bn / 16;
+    const PairTiles pt{counts, offsets, row_of, n_experts, w_stride};
+    // as many tiles as there can be: whole ones, and one that is not full for every expert that has pairs
+    dim3 grid(n_pairs / bm + min(n_experts, n_pairs), ((N + 15) / 16 + wg_blocks - 1) / wg_blocks), block(256);
+    const size_t stages = (size_t)(ahead + 1) * 2 * (bm / 16) * 1024, strips = (size_t)4 * 2 * 16 * (bn / 4 + 4) * 4;
+    const size_t lds = (stages > strips ? stages : strips) + (size_t)2 * bm * 4 + (256 + 16) * 4;
+    const int k_whole = (K + 31) / 32 * 32;
+#define GO(T, NI, MJ, A)                                                                                  \
+    do {                                                                                                  \
+        auto kfn = gemm_wreg_kernel<T, NI, MODE_PAIRS, MJ, A>;                                            \
+        if (lds > 64 * 1024) {                                                                            \
+            static bool allowed = false;           /* more than 64 KiB of LDS is asked for once */       \
+            if (!allowed && hipFuncSetAttribute((const void*)kfn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
+                return LI_HIP_ERROR;                                                                      \
+            allowed = true;                                                                               \
+        }                                                                                                 \
+        kfn<<<grid, block, lds, stream>>>((const T*)X, (const T*)Wt, K, k_whole, nullptr, e, wg_blocks, RowScale{}, pt); \
+    } while (0)
+#define LAUNCH(T)                                       \
+    do {                                                \
+        if (tile == 0) GO(T, 4, 8, 2);                  \
+        else if (tile == 1) GO(T, 3, 8, 2);             \
+        else if (few_rows) GO(T, 2, 4, 4);              \
+        else GO(T, 2, 8, 2);                            \
+    } while (0)
+    if (dt == DT_F16) LAUNCH(f16); else LAUNCH(bf16);
+#undef LAUNCH
+#undef GO
+    LI_CHECK_LAUNCH();
     return LI_OK;
 }

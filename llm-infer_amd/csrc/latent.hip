@@ -251,6 +251,8 @@ extern "C" int li_latent_store(const float* q_rows, int q_stride, int q_col, con
 // outputs x up to 128 tokens of one head (a fragment of W serves four tiles of 32 tokens), W^T as operand A and the tokens' inputs (rounded to the 16-bit type where they
 // come in float32, as the sum of two such numbers) as operand B of the 32x32x16 matrix instruction, both read straight from memory, 16 bytes a lane
 // where n_in and the rows allow; the four waves of a workgroup take four blocks of outputs for the same tokens.
+// head_linear_few_kernel (up to 32 tokens, everything at multiples of 16 bytes): the same with one tile of tokens and a wave a
+// workgroup, eight steps' operands asked for at once, so that a decode step waits for memory once or twice.
 // ---------------------------------------------------------------------------
 #define HL_TOK 16
 
@@ -367,6 +369,63 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const TI* __restr
     }
 }
 
+#define HLF_STEPS 8
+
+template <class TI, class T>
+__global__ __launch_bounds__(64) void head_linear_few_kernel(const TI* __restrict__ in, int64_t in_st, int in_sh,
+                                                             const T* __restrict__ W, T* __restrict__ out, int64_t out_st,
+                                                             int out_sh, const float* __restrict__ gate, int64_t gate_st,
+                                                             int n_tokens, int n_in, int n_out) {
+    typedef typename Vec<T>::v8 v8;
+    const int lane = threadIdx.x, col = lane & 31, half = lane >> 5, h = blockIdx.x, j0 = blockIdx.y * 32;
+    const bool j_ok = j0 + col < n_out, t_ok = col < n_tokens;
+    const T* wrow = W + ((int64_t)h * n_out + (j_ok ? j0 + col : 0)) * n_in + 8 * half;
+    const TI* xrow = in + (int64_t)(t_ok ? col : 0) * in_st + (int64_t)h * in_sh + 8 * half;
+    f32x16 acc;
+#pragma unroll
+    for (int r = 0; r < 16; ++r) acc[r] = 0.f;
+    for (int k0 = 0; k0 < n_in; k0 += 16 * HLF_STEPS) {
+        v8 a[HLF_STEPS], b[HLF_STEPS];
+        f32x4 lo[HLF_STEPS], hi[HLF_STEPS];
+#pragma unroll
+        for (int u = 0; u < HLF_STEPS; ++u) {
+            const v8 z = {};
+            const int k = k0 + 16 * u;
+            const bool in_k = k + 8 * half + 8 <= n_in;    // (n_in is a multiple of 8)
+            a[u] = in_k && j_ok ? *(const v8*)(wrow + k) : z;
+            if (sizeof(TI) == 4) {
+                const f32x4 zf = {0.f, 0.f, 0.f, 0.f};
+                lo[u] = in_k && t_ok ? *(const f32x4*)((const float*)xrow + k) : zf;
+                hi[u] = in_k && t_ok ? *(const f32x4*)((const float*)xrow + k + 4) : zf;
+            } else b[u] = in_k && t_ok ? *(const v8*)((const T*)xrow + k) : z;
+        }
+#pragma unroll
+        for (int u = 0; u < HLF_STEPS; ++u) {
+            if (sizeof(TI) == 4) {
+                v8 b2;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) {
+                    const float x = e < 4 ? lo[u][e & 3] : hi[u][e & 3];
+                    b[u][e] = from_f32<T>(x);
+                    b2[e] = from_f32<T>(x - to_f32(b[u][e]));
+                }
+                acc = mfma32(a[u], b[u], acc);
+                acc = mfma32(a[u], b2, acc);
+            } else acc = mfma32(a[u], b[u], acc);
+        }
+    }
+    if (!t_ok) return;
+#pragma unroll
+    for (int r = 0; r < 16; ++r) {
+        const int j = j0 + 8 * (r >> 2) + 4 * half + (r & 3);
+        if (j < n_out) {
+            float v = acc[r];
+            if (gate) v *= lt_sigmoid(gate[(int64_t)col * gate_st + (int64_t)h * n_out + j]);
+            out[(int64_t)col * out_st + (int64_t)h * out_sh + j] = from_f32<T>(v);
+        }
+    }
+}
+
 extern "C" int li_head_linear(const void* in, int in_dt, int64_t in_st, int in_sh, const void* W, int w_dt, void* out,
                               int64_t out_st, int out_sh, const float* gate, int64_t gate_st, int n_tokens, int H, int n_in,
                               int n_out, hipStream_t stream) {
@@ -378,6 +437,17 @@ extern "C" int li_head_linear(const void* in, int in_dt, int64_t in_st, int in_s
         const int vec = n_in % 8 == 0 && (uintptr_t)W % 16 == 0 && (uintptr_t)in % 16 == 0 && (in_st * isz) % 16 == 0 &&
                         ((int64_t)in_sh * isz) % 16 == 0;
         dim3 grid((n_tokens + 32 * HLM_TT - 1) / (32 * HLM_TT), H, (n_out + 127) / 128);
+        if (vec && n_tokens <= 32) {
+            dim3 few(H, (n_out + 31) / 32);
+#define GOF(TI, T) head_linear_few_kernel<TI, T><<<few, 64, 0, stream>>>((const TI*)in, in_st, in_sh, (const T*)W, (T*)out, out_st, out_sh, \
+                                                                        gate, gate_st, n_tokens, n_in, n_out)
+            if (in_dt == DT_F32) { if (w_dt == DT_F16) GOF(float, f16); else GOF(float, bf16); }
+            else if (in_dt == w_dt) { if (w_dt == DT_F16) GOF(f16, f16); else GOF(bf16, bf16); }
+            else return LI_BAD_ARG;
+#undef GOF
+            LI_CHECK_LAUNCH();
+            return LI_OK;
+        }
 #define GOM(TI, T) head_linear_mfma_kernel<TI, T><<<grid, 256, 0, stream>>>((const TI*)in, in_st, in_sh, (const T*)W, (T*)out, out_st, \
                                                                            out_sh, gate, gate_st, n_tokens, n_in, n_out, vec)
         if (in_dt == DT_F32) { if (w_dt == DT_F16) GOM(float, f16); else GOM(float, bf16); }

@@ -28,7 +28,7 @@ ATTN_SOURCE = "attention.hip"
 MIXER_SOURCES = ("mixers.hip",)
 # the headers a library's sources include (its stamp covers them)
 HEADERS = {"libli_core.so": ("common.h", "gemm_common.h", "no_alloc.h"), "libli_hybrid.so": ("common.h", "conv.h"),
-           "libli_recurrent.so": ("common.h", "conv.h")}
+           "libli_recurrent.so": ("common.h", "conv.h"), "libli_experts.so": ("common.h", "gemm_common.h")}
 DEFAULT_HEADERS = ("common.h",)
 FLAGS = ["--offload-arch=" + ARCH, "-O3", "-std=c++17", "-fPIC",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unused-command-line-argument"]
@@ -214,6 +214,15 @@ def recurrent_library(force=False):
     return _load("libli_recurrent.so", RECURRENT_SOURCES, (), force)
 
 
+EXPERT_SOURCES = ("experts.hip",)
+
+
+def experts_library(force=False):
+    """Routed experts by pairs of token and expert (csrc/experts.hip: the router, the sorted pairs, the products of few
+    pairs, their sum): a library of its own, as the mixers' is."""
+    return _load("libli_experts.so", EXPERT_SOURCES, (), force)
+
+
 DIFF_ATTN_SOURCE = "diff_attention.hip"
 
 
@@ -256,6 +265,7 @@ def build_all(head_dims=(16, 32, 48, 64, 128), force=True, sigmoid_head_dims=((4
     mixers_library(force=force)
     hybrid_library(force=force)
     recurrent_library(force=force)
+    experts_library(force=force)
     with ThreadPoolExecutor(max_workers=4) as pool:
         list(pool.map(lambda p: _build_library(*_sigmoid_attention_args(*p), force), sigmoid_head_dims))
         list(pool.map(lambda p: _build_library(*_diff_attention_args(*p), force), diff_head_dims))

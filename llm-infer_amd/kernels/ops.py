@@ -2012,13 +2012,20 @@ def rmsnorm_add(x, y, weight, eps: float, bias=None, next_norm=None, also=None) 
     (weight float32 [width], eps, dtype): the RMS norm that reads the finished rows next is taken in the same pass and
     left for it (``prepared_rmsnorm`` finds it as long as nothing else writes into ``x``).  ``also`` (rows of x's shape or
     None, vector float32 [width]): the finished rows gain them before that norm is taken."""
+    width = x.shape[1]
+    pairs = None
+    if isinstance(y, PairSum):
+        if bias is None and width % 4 == 0 and width <= 8192:
+            pairs, y = y, y.rows
+        else:
+            y = y.tensor()
     _dev(x, y, weight, bias)
     add_rows, add_vec = also if also is not None else (None, None)
     _dev(add_rows, add_vec)
     _f32_rows(x, "rmsnorm_add x")
     _f32_rows(y, "rmsnorm_add y")
-    width = x.shape[1]
-    _need(y.shape == x.shape and weight.dtype == torch.float32 and weight.shape == (width,), "rmsnorm_add: rows of one shape, a float32 weight")
+    _need(tuple((y if pairs is None else pairs).shape) == tuple(x.shape) and weight.dtype == torch.float32 and weight.shape == (width,),
+          "rmsnorm_add: rows of one shape, a float32 weight")
     _need(bias is None or (bias.dtype == torch.float32 and bias.shape == (width,)), "rmsnorm_add: a float32 bias")
     if also is not None:
         _need(add_vec.dtype == torch.float32 and add_vec.shape == (width,) and add_vec.is_contiguous(), "rmsnorm_add: a float32 vector to add")
@@ -2032,12 +2039,146 @@ def rmsnorm_add(x, y, weight, eps: float, bias=None, next_norm=None, also=None) 
         _dev(nw)
         _need(nw.dtype == torch.float32 and nw.shape == (width,) and n_dt in DT, "rmsnorm_add: the next norm's float32 weight and type")
         normed = torch.empty(x.shape, dtype=n_dt, device=x.device)
-    _check(hybrid().li_rmsnorm_add(_ptr(x), _ptr(y), _ptr(bias), _ptr(weight), c_float(eps), x.shape[0], width,
-                                   _ptr(add_rows), _ptr(add_vec), _ptr(nw), c_float(n_eps), _ptr(normed), DT[n_dt], _stream()),
-           "rmsnorm_add")
+    if pairs is not None:
+        _check(hybrid().li_rmsnorm_add_pairs(_ptr(x), _ptr(y), _ptr(pairs.slot_of), _ptr(pairs.weights), pairs.slot_of.shape[1], _ptr(weight),
+                                             c_float(eps), x.shape[0], width, _ptr(add_rows), _ptr(add_vec), _ptr(nw), c_float(n_eps),
+                                             _ptr(normed), DT[n_dt], _stream()), "rmsnorm_add_pairs")
+    else:
+        _check(hybrid().li_rmsnorm_add(_ptr(x), _ptr(y), _ptr(bias), _ptr(weight), c_float(eps), x.shape[0], width,
+                                       _ptr(add_rows), _ptr(add_vec), _ptr(nw), c_float(n_eps), _ptr(normed), DT[n_dt], _stream()),
+               "rmsnorm_add")
     if normed is not None:
         x._li_normed = (normed, nw, float(n_eps), x._version)
     return x
+
+
+class PairSum:
+    """Rows that are still a sum: row t is the sum over j of weights[t, j] * rows[slot_of[t, j]] (slot_of -1: nothing), what
+    a token's chosen experts have made.  A pass that adds the rows up anyway takes it as it is (``rmsnorm_add``); everything
+    else asks for ``tensor()`` or ``add_to(out)``."""
+
+    def __init__(self, rows, slot_of, weights):
+        self.rows, self.slot_of, self.weights = rows, slot_of, weights
+        self.shape = (slot_of.shape[0], rows.shape[1])
+
+    def _sum(self, out, add: bool):
+        _dev(self.rows, self.slot_of, self.weights, out)
+        t, top = self.slot_of.shape
+        _need(out.dtype == torch.float32 and tuple(out.shape) == self.shape and out.is_contiguous(), "pair sum: float32 rows")
+        _drop_row_stats(out)
+        _check(experts().li_pair_sum(_ptr(self.rows), _ptr(self.slot_of), _ptr(self.weights), t, top, self.shape[1], _ptr(out), int(add),
+                                     _stream()), "pair_sum")
+        return out
+
+    def tensor(self) -> torch.Tensor:
+        return self._sum(torch.empty(self.shape, dtype=torch.float32, device=self.rows.device), False)
+
+    def add_to(self, out) -> None:
+        self._sum(out, True)
+
+
+_experts = None
+
+
+def experts():
+    global _experts
+    if _experts is None:
+        _experts = build.experts_library()
+    return _experts
+
+
+ROUTER_MAX = 512          # outputs of a router that ``route_pairs`` takes
+
+
+class SortedPairs:
+    """A step's pairs (token, chosen expert) sorted by expert, all on the device: ``weights`` float32 and ``slot_of`` int32
+    [T, top], ``counts`` and ``offsets`` int32 [experts], ``row_of`` int32 [T * top]."""
+
+    def __init__(self, t, top, n_experts, device):
+        self.t, self.top, self.n_experts = t, top, n_experts
+        ints = torch.empty((3 * t * top + 2 * n_experts,), dtype=torch.int32, device=device)
+        self.chosen, self.slot_of = ints[:t * top].view(t, top), ints[t * top:2 * t * top].view(t, top)
+        self.row_of = ints[2 * t * top:3 * t * top]
+        self.counts, self.offsets = ints[3 * t * top:3 * t * top + n_experts], ints[3 * t * top + n_experts:]
+        self.weights = torch.empty((t, top), dtype=torch.float32, device=device)
+
+
+def router_weight(w, dtype):
+    """A router's matrix [n, K] (K a multiple of 32) as ``route_pairs`` takes it: the sum of up to three 16-bit matrices of
+    n rows rounded up to 16, one behind the other and tiled (the rounding of W to ``dtype`` and the roundings of what is
+    left; those that are all zero are left out, so a matrix stored in that type is one)."""
+    w = w.as_subclass(torch.Tensor).float()
+    n, k = w.shape
+    _need(k % 32 == 0, "router_weight: a width that is a multiple of 32")
+    parts, rest = [], w
+    for _ in range(3):
+        part = torch.zeros(((n + 15) // 16 * 16, k), dtype=dtype, device=w.device)
+        part[:n] = rest
+        rest = rest - part[:n].float()
+        parts.append(part)
+        if not bool(rest.any()):
+            break
+    return prepare_weight(torch.cat(parts, 0).contiguous())
+
+
+def route_pairs(h, w_router, bias, n_experts: int, top: int, scale: float = 1.0) -> SortedPairs:
+    """The router of experts that run by pairs: logits h W^T (+ bias) for W as ``router_weight`` leaves it (products of a
+    float32 W, float32 sums), the ``top`` largest of every token chosen, their weights the softmax over them alone times
+    ``scale``; the pairs sorted by expert."""
+    _dev(h, w_router, bias)
+    n, (rows, k) = n_experts, matrix_shape(w_router)
+    parts = rows // ((n + 15) // 16 * 16)
+    _need(is_tiled(w_router) and h.dim() == 2 and h.dtype == w_router.dtype and h.shape[1] == k and h.is_contiguous()
+          and rows == parts * ((n + 15) // 16 * 16) and 1 <= parts <= 3, "route_pairs: 16-bit rows and a matrix of router_weight")
+    _need(h.dtype in (torch.float16, torch.bfloat16) and 1 <= top <= n <= ROUTER_MAX and n + top <= 640, f"route_pairs: up to {ROUTER_MAX} experts, with those chosen 640")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.shape == (n,) and bias.is_contiguous()), "route_pairs: a float32 bias")
+    t = h.shape[0]
+    p = SortedPairs(t, top, n, h.device)
+    lists = (_ptr(p.counts), _ptr(p.offsets), _ptr(p.row_of), _ptr(p.slot_of))
+    small = t <= 16                                        # one workgroup has every token: it sorts the pairs too
+    _check(experts().li_router(_ptr(h), _ptr(w_router), DT[h.dtype], _ptr(bias), parts, t, k, n, top, c_float(scale), _ptr(p.chosen),
+                               _ptr(p.weights), *(lists if small else (None,) * 4), _stream()), "router")
+    if not small:
+        _check(experts().li_sort_pairs(_ptr(p.chosen), t * top, top, n, *lists, _stream()), "sort_pairs")
+    return p
+
+
+@functools.lru_cache(maxsize=1024)
+def _pairs_plan(pairs: int, n_experts: int, n: int, k: int) -> tuple:
+    """(tile, few_rows) of gemm_wreg's pairs mode: tiles of 64 pairs where an expert has no more on average, else the tile
+    of least estimated time, each expert's last tile half full."""
+    if pairs <= 64 * n_experts:
+        return 2, 1
+    return min(((_wreg_cost(t, 1, pairs + 64 * n_experts, n, k), t) for t in (0, 1, 2)))[1], 0
+
+
+def linear_pairs(x, w, p: SortedPairs, mode: int = EPI_STORE, gather: bool = True, out_dtype=None, force: str | None = None) -> torch.Tensor:
+    """Every pair's product with its expert's matrix: ``w`` is the experts' matrices [N, K] stacked in one tiled matrix
+    [E N, K] (N a multiple of 16); row p of the result belongs to pair p and comes of row ``row_of[p]`` of ``x`` (``gather``
+    False: row p).  EPI_STORE, or EPI_SWIGLU over interleaved gate/up rows.  ``force`` "gemv" or "wreg:<tile>:<few rows>"
+    picks a kernel for tests."""
+    _dev(x, w)
+    rows, k = matrix_shape(w)
+    pairs, e = p.t * p.top, p.n_experts
+    n = rows // e
+    _need(is_tiled(w) and rows == n * e and n % 16 == 0 and x.dtype == w.dtype and x.dim() == 2 and x.shape[1] == k and x.is_contiguous(),
+          "linear_pairs: the experts' matrices stacked and tiled, rows of their type")
+    _need(x.shape[0] == (p.t if gather else pairs), "linear_pairs: a row for every token (or for every pair)")
+    _need(mode in (EPI_STORE, EPI_SWIGLU), "linear_pairs: store or silu(gate) * up")
+    out = torch.empty((pairs, n // 2 if mode == EPI_SWIGLU else n), dtype=out_dtype or x.dtype, device=x.device)
+    row_of = _ptr(p.row_of) if gather else None
+    # few pairs an expert: its matrix is streamed once straight into the operands
+    kind = force or ("gemv" if pairs <= 16 * e else "wreg")
+    if kind == "gemv":
+        _check(experts().li_experts_gemv(_ptr(x), _ptr(w), DT[x.dtype], _ptr(out), DT[out.dtype], mode, pairs, n, k, c_int64(n * k), e,
+                                         _ptr(p.counts), _ptr(p.offsets), row_of, _stream()), "experts_gemv")
+        return out
+    tile, few = _pairs_plan(pairs, e, n, k)
+    if ":" in kind:
+        tile, few = (int(v) for v in kind.split(":")[1:3])
+    _check(core().li_gemm_wreg_pairs(_ptr(x), _ptr(w), DT[x.dtype], _ptr(out), DT[out.dtype], mode, x.shape[0], pairs, n, k, tile, few,
+                                     _ptr(p.counts), _ptr(p.offsets), row_of, e, c_int64(n * k), _stream()), "gemm_wreg_pairs")
+    return out
 
 
 def add_rows(x, rows, vec) -> torch.Tensor:

@@ -175,7 +175,14 @@ class RoutedExperts(Part):
     ``shared_ff`` > 0: one more expert of that width runs for every token; ``shared_gate``: it is weighted by
     sigmoid(w_sg . h).
 
-    How it runs.  Few tokens (a decode step, a short prompt, and every step of a float32 model): the experts' gate
+    How it runs.  Gated silu experts of a 16-bit model with a softmax router and nothing beside them (no outputs that pass a
+    token on, no shared expert, no correction, weights over the chosen alone): by pairs of token and chosen expert,
+    whatever the number of tokens (csrc/experts.hip): one kernel for the logits and the choice, the pairs sorted by expert on
+    the device, two products in which every expert multiplies its own pairs' rows and an expert without pairs is not
+    read, and the weighted sum of a token's rows in the pass that adds it to the stream.  Nothing waits for the host, and
+    such a step can be recorded.
+
+    All others.  Few tokens (a decode step, a short prompt, and every step of a float32 model): the experts' gate
     and up matrices are stacked (the shared expert's behind them) into one product whose epilogue applies
     silu(gate) * up; every expert's block of the hidden row is multiplied by the token's weight for that expert,
     zero where it was not chosen; one product against the down matrices side by side then sums the experts.
@@ -189,6 +196,7 @@ class RoutedExperts(Part):
     # through every expert and 3.46 sorted by expert (40 launches a layer and a wait for the counts against 3 launches),
     # 1,024 tokens 4.90 and 4.86, 2,048 tokens 8.58 and 7.50
     GROUPED_FROM = 256
+    makes_rows = False          # by pairs: forward_rows hands over the rows as a sum (set when the weights are bound)
     writes_rows = True          # forward_into overwrites the rows it is handed
 
     def __init__(self, *, hidden_size, n_experts, expert_ff, top, n_identity=0, route_scale=1.0, correction=True,
@@ -237,7 +245,8 @@ class RoutedExperts(Part):
         if self.table_routing:
             out = {n["table"]: ParamSpec((self.vocab_size, self.top), "int", f"distinct:{self.n_experts}")}
         else:
-            out = {n["router"]: ParamSpec((self.n_experts + self.n_identity, d), "vector", "wide")}
+            # (kept in float32; random weights are drawn as numbers of the matrices' type, as a file stores them)
+            out = {n["router"]: ParamSpec((self.n_experts + self.n_identity, d), "vector", "wide_matrix")}
         if self.router_bias:
             out[n["router_bias"]] = ParamSpec((self.n_experts + self.n_identity,), "vector", "small")
         if self.correction:
@@ -252,6 +261,9 @@ class RoutedExperts(Part):
 
     def bind(self, tensors):
         n, d = self.names, self.hidden_size
+        self.paired = self.makes_rows = self._pairs_fit(tensors)
+        if self.paired:
+            return self._bind_pairs(tensors)
         gu, down = [], []
         for p, f in self._experts():
             u = tensors[p + n["up"]]
@@ -280,6 +292,32 @@ class RoutedExperts(Part):
             self.b_router = torch.cat([b, torch.zeros((int(self.shared_gate),), dtype=torch.float32, device=b.device)]).contiguous()
         self.table = tensors[n["table"]] if self.table_routing else None
         self.bias = tensors[n["correction"]] if self.correction else None
+
+    def _pairs_fit(self, tensors) -> bool:
+        """True if the experts can run by pairs: the kind of router and experts the kernels take, and a width that tiles."""
+        if (self.dtype == torch.float32 or not self.gated or self.clamped or self.table_routing or self.n_identity or self.shared_ff
+                or self.correction or self.sigmoid_scores or not self.renormalize or self.on_input
+                or self.n_experts > ops.ROUTER_MAX or self.n_experts + self.top > 640 or self.hidden_size % 32):
+            return False
+        p = self.names["expert"].format(0)
+        # (matrices that are stored wider than the model's type are kept so)
+        return all(tensors[p + self.names[k]].dtype == self.dtype for k in ("gate", "up", "down"))
+
+    def _bind_pairs(self, tensors):
+        n, d, f = self.names, self.hidden_size, self.expert_ff
+        fp = (f + 31) // 32 * 32                # the hidden rows' width, zeros behind an expert's own
+        gate_up = down = None
+        for i, (p, _) in enumerate(self._experts()):
+            g, u, dn = (tensors[p + n[k]].as_subclass(torch.Tensor) for k in ("gate", "up", "down"))
+            if gate_up is None:                 # (stacked as they come: one expert's tensors at a time beside the stack)
+                gate_up = torch.zeros((self.n_experts, fp, 2, d), dtype=self.dtype, device=g.device)
+                down = torch.zeros((self.n_experts, d, fp), dtype=self.dtype, device=g.device)
+            gate_up[i, :f, 0], gate_up[i, :f, 1], down[i, :, :f] = g, u, dn
+        self.w_gate_up = ops.prepare_weight(gate_up.view(self.n_experts * fp * 2, d))
+        self.w_down = ops.prepare_weight(down.view(self.n_experts * d, fp))
+        self.w_router = ops.router_weight(tensors[n["router"]], self.dtype)
+        self.b_router = tensors[n["router_bias"]] if self.router_bias else None
+        self.per_expert = None
 
     @staticmethod
     def _rows(stacked, r0, n, own):
@@ -359,7 +397,15 @@ class RoutedExperts(Part):
             t = ops.linear(h, self.w_gate_up, ops.EPI_SWIGLU, out_dtype=self.dtype)
         return ops.scale_blocks(t, weights, self.n_experts, self.expert_ff, self.shared_ff)
 
+    def forward_rows(self, h, ctx=None, view=None, owns_cache=True):
+        """The result as rows that are still a sum (``ops.PairSum``); by pairs only (``makes_rows``)."""
+        p = ops.route_pairs(h, self.w_router, self.b_router, self.n_experts, self.top, self.route_scale)
+        t = ops.linear_pairs(h, self.w_gate_up, p, ops.EPI_SWIGLU)
+        return ops.PairSum(ops.linear_pairs(t, self.w_down, p, gather=False, out_dtype=torch.float32), p.slot_of, p.weights)
+
     def forward(self, h, residual, ctx=None):
+        if self.paired:
+            return self.forward_rows(h).add_to(residual)
         weights = self._weights(h, residual, ctx)
         if self._is_grouped(h):
             return self._grouped(h, residual, weights)

@@ -30,7 +30,7 @@ class WeightError(ValueError):
 class ParamSpec:
     shape: tuple
     kind: str = "matrix"        # "matrix" | "vector" | "int"
-    init: str = "normal"        # random-weights mode: "normal" N(0, 0.02) | "ones" 1 + N(0, 0.01) | "small" | "half" | "wide" | "mean"
+    init: str = "normal"        # random-weights mode: "normal" N(0, 0.02) | "ones" 1 + N(0, 0.01) | "small" | "half" | "wide" | "wide_matrix" | "mean"
     free: tuple = ()            # axes whose size the checkpoint sets (``shape`` holds what random weights take there)
 
 
