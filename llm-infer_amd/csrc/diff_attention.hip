@@ -108,16 +108,21 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
             for (int r = 0; r < 16; ++r) o[a][b][r] = 0.f;
     }
 
-    // the fragments of the 32 keys after the ones at work are fetched before the work begins
+    // The fragments of the 32 keys after the ones at work: where the registers hold two sets of them (TWO) they are fetched
+    // before the work begins; else a map's keys right behind its scores and the values behind the outputs, each into the
+    // registers that have just been read (two sets of wide keys and values spill, and a spilled register's reload waits for
+    // every load issued before it).
+    constexpr bool TWO = MAPS * MAP_DIM + VALUE_DIM <= 256;
     v8 kn[MAPS][D16], vn[DVB][2];
-    auto fetch = [&](int kt) {
+    auto fetch_k = [&](int kt, int a) {
         const int page = table[kt >> 1], tb = kt & 1;                      // two blocks of 32 keys a page
         const T* kh = (const T*)pg.k + (int64_t)page * pg.page_stride + g * k_head_elems(KW);
+#pragma unroll
+        for (int s = 0; s < D16; ++s) kn[a][s] = *(const v8*)(kh + ((int64_t)(tb * (KW / 16) + a * D16 + s) * 64 + lane) * 8);
+    };
+    auto fetch_v = [&](int kt) {
+        const int page = table[kt >> 1], tb = kt & 1;
         const T* vh = (const T*)pg.v + (int64_t)page * pg.page_stride + g * v_head_elems(VALUE_DIM);
-#pragma unroll
-        for (int a = 0; a < MAPS; ++a)
-#pragma unroll
-            for (int s = 0; s < D16; ++s) kn[a][s] = *(const v8*)(kh + ((int64_t)(tb * (KW / 16) + a * D16 + s) * 64 + lane) * 8);
 #pragma unroll
         for (int b = 0; b < DVB; ++b)
 #pragma unroll
@@ -128,19 +133,31 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
     const int w_win = lo_tile / 32, n_keep = min((keep + 31) / 32, w_win), w_lo = w_win - n_keep;
     auto tile_of = [&](int w) { return w < w_win ? w - w_lo : w; };
     const int kt_last = p_last / 32, w_first = w_lo + kwave;
-    if (w_first <= kt_last) fetch(tile_of(w_first));
+    if (w_first <= kt_last) {
+#pragma unroll
+        for (int a = 0; a < MAPS; ++a) fetch_k(tile_of(w_first), a);
+        fetch_v(tile_of(w_first));
+    }
     for (int w = w_first; w <= kt_last; w += kstep) {
         const int kt = tile_of(w);
+        // (without TWO the last turn fetches its own keys again, which nothing reads: a branch around the loads would wait for all)
+        const int kt_next = tile_of(w + kstep <= kt_last ? w + kstep : w);
         v8 kf[MAPS][D16], vf[DVB][2];
+        if constexpr (TWO) {
 #pragma unroll
-        for (int a = 0; a < MAPS; ++a)
+            for (int a = 0; a < MAPS; ++a)
 #pragma unroll
-            for (int s = 0; s < D16; ++s) kf[a][s] = kn[a][s];
+                for (int s = 0; s < D16; ++s) kf[a][s] = kn[a][s];
 #pragma unroll
-        for (int b = 0; b < DVB; ++b)
+            for (int b = 0; b < DVB; ++b)
 #pragma unroll
-            for (int u = 0; u < 2; ++u) vf[b][u] = vn[b][u];
-        if (w + kstep <= kt_last) fetch(tile_of(w + kstep));
+                for (int u = 0; u < 2; ++u) vf[b][u] = vn[b][u];
+            if (w + kstep <= kt_last) {
+#pragma unroll
+                for (int a = 0; a < MAPS; ++a) fetch_k(kt_next, a);
+                fetch_v(kt_next);
+            }
+        }
         v8 phi[MAPS][2], plo[MAPS][2];
 #pragma unroll
         for (int a = 0; a < MAPS; ++a) {
@@ -149,8 +166,9 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
             for (int r = 0; r < 16; ++r) acc[r] = 0.f;
 #pragma unroll
             for (int s = 0; s < D16; ++s) {
-                acc = mfma32(kf[a][s], qf[a][s], acc);
+                acc = mfma32(TWO ? kf[a][s] : kn[a][s], qf[a][s], acc);
             }
+            if constexpr (!TWO) fetch_k(kt_next, a);
             // scores in units of log 2, so that a weight is one hardware 2^x; 32 keys that every query of a whole tile
             // sees need no mask
             if (softcap > 0.f) {
@@ -216,10 +234,12 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
             for (int u = 0; u < 2; ++u) {
 #pragma unroll
                 for (int a = 0; a < MAPS; ++a) {
-                    o[a][b] = mfma32(vf[b][u], phi[a][u], o[a][b]);
-                    if (SPLIT_W) o[a][b] = mfma32(vf[b][u], plo[a][u], o[a][b]);
+                    const v8 v = TWO ? vf[b][u] : vn[b][u];
+                    o[a][b] = mfma32(v, phi[a][u], o[a][b]);
+                    if (SPLIT_W) o[a][b] = mfma32(v, plo[a][u], o[a][b]);
                 }
             }
+        if constexpr (!TWO) fetch_v(kt_next);
     }
     if (split && nw > 1) {
         // a tile of one token whose keys the waves have shared: wave 0 adds up their states in wave order
@@ -236,6 +256,36 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
             }
         }
         __syncthreads();
+        if (HC && gridDim.z > 1) {
+            // the keys were shared among workgroups too: this one's sums go to `shares_out` [token, head, share, map,
+            // 2 + VALUE_DIM] (every wave a part of the values) and diff_attn_merge_kernel finishes
+            if (has_query) {
+#pragma unroll
+                for (int a = 0; a < MAPS; ++a) {
+                    float* mine = shares_out + ((((int64_t)t0 * H + hq) * gridDim.z + blockIdx.z) * MAPS + a) * W;
+                    float M = -INFINITY, L = 0.f, f[4];
+                    for (int v = 0; v < nw; ++v) M = fmaxf(M, lds[((v * MAPS + a) * 32 + col) * W]);
+#pragma unroll
+                    for (int v = 0; v < 4; ++v) {
+                        const float* theirs = lds + ((v * MAPS + a) * 32 + col) * W;
+                        f[v] = v >= nw || theirs[0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(theirs[0] - M);
+                        if (v < nw) L += theirs[1] * f[v];
+                    }
+                    if (wave == 0 && half == 0) { mine[0] = M; mine[1] = L; }
+                    for (int i = 2 * wave + half; i < VALUE_DIM / 4; i += 2 * nw) {
+                        float sum[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                        for (int v = 0; v < 4; ++v)
+#pragma unroll
+                            for (int q = 0; q < 4; ++q)
+                                if (v < nw) sum[q] += lds[((v * MAPS + a) * 32 + col) * W + 2 + 4 * i + q] * f[v];
+#pragma unroll
+                        for (int q = 0; q < 4; ++q) mine[2 + 4 * i + q] = sum[q];
+                    }
+                }
+            }
+            return;
+        }
         if (wave != 0) return;
         if (HC || col == 0) {
             const int cs = HC ? 32 : 1, c0 = HC ? col : 0;
@@ -261,23 +311,6 @@ __global__ __launch_bounds__(256) void diff_attn_mfma_kernel(
                 m[a] = M; l[a] = L;
             }
         }
-    }
-    if (HC && gridDim.z > 1) {
-        // the keys were shared among workgroups: this one's state goes to `shares_out` [token, head, share, map, 2 + VALUE_DIM]
-        // and diff_attn_merge_kernel finishes
-        constexpr int W = 2 + VALUE_DIM;
-        if (has_query) {
-#pragma unroll
-            for (int a = 0; a < MAPS; ++a) {
-                float* mine = shares_out + ((((int64_t)t0 * H + hq) * gridDim.z + blockIdx.z) * MAPS + a) * W;
-                if (half == 0) { mine[0] = m[a]; mine[1] = l[a]; }
-#pragma unroll
-                for (int b = 0; b < DVB; ++b)
-#pragma unroll
-                    for (int r = 0; r < 16; ++r) mine[2 + b * 32 + 8 * (r >> 2) + 4 * half + (r & 3)] = o[a][b][r];
-            }
-        }
-        return;
     }
     if (sink) {
         // the sink joins every map's sum as one more weight, exp(sink - maximum), with nothing to add to the output

@@ -298,7 +298,7 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_kernel(float* __restri
     TN* nr = next + row * width;
     float ss = 0.f, s2 = 0.f;
     if ((width & 3) == 0 && width <= 4 * RA_KEEP * RA_THREADS) {
-        f32x4 keep[RA_KEEP], xs[RA_KEEP], ws[RA_KEEP];
+        f32x4 keep[RA_KEEP], xs[RA_KEEP], ws[RA_KEEP], nw[RA_KEEP], ad[RA_KEEP];
         const int quads = width >> 2;
 #pragma unroll
         for (int c = 0; c < RA_KEEP; ++c) {
@@ -308,6 +308,14 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_kernel(float* __restri
                 if (EARLY) {
                     xs[c] = *(const f32x4*)(xr + 4 * i);
                     ws[c] = *(const f32x4*)(w + 4 * i);
+                    if (next_w) nw[c] = *(const f32x4*)(next_w + 4 * i);
+                    if (add_vec) {
+                        ad[c] = *(const f32x4*)(add_vec + 4 * i);
+                        if (add_rows) {
+                            const f32x4 e = *(const f32x4*)(add_rows + row * width + 4 * i);
+                            ad[c][0] += e[0]; ad[c][1] += e[1]; ad[c][2] += e[2]; ad[c][3] += e[3];
+                        }
+                    }
                 }
                 if (b) { const f32x4 bb = *(const f32x4*)(b + 4 * i); v[0] += bb[0]; v[1] += bb[1]; v[2] += bb[2]; v[3] += bb[3]; }
                 keep[c] = v;
@@ -327,17 +335,21 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_kernel(float* __restri
                 o[0] += keep[c][0] * r * ws[c][0]; o[1] += keep[c][1] * r * ws[c][1];
                 o[2] += keep[c][2] * r * ws[c][2]; o[3] += keep[c][3] * r * ws[c][3];
                 if (add_vec) {
-                    if (add_rows) {
-                        const f32x4 e = *(const f32x4*)(add_rows + row * width + 4 * i);
-                        o[0] += e[0]; o[1] += e[1]; o[2] += e[2]; o[3] += e[3];
+                    f32x4 e;
+                    if (EARLY) e = ad[c];
+                    else {
+                        e = *(const f32x4*)(add_vec + 4 * i);
+                        if (add_rows) {
+                            const f32x4 e2 = *(const f32x4*)(add_rows + row * width + 4 * i);
+                            e[0] += e2[0]; e[1] += e2[1]; e[2] += e2[2]; e[3] += e2[3];
+                        }
                     }
-                    const f32x4 e = *(const f32x4*)(add_vec + 4 * i);
                     o[0] += e[0]; o[1] += e[1]; o[2] += e[2]; o[3] += e[3];
                 }
                 *(f32x4*)(xr + 4 * i) = o;
                 keep[c] = o;
                 s2 += o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
-                if (next_w) ws[c] = *(const f32x4*)(next_w + 4 * i);
+                if (next_w) ws[c] = EARLY ? nw[c] : *(const f32x4*)(next_w + 4 * i);
             }
         }
         if (!next_w) return;
@@ -387,7 +399,7 @@ extern "C" int li_rmsnorm_add(float* x, const float* y, const float* b, const fl
 // The same with y the weighted sum of a few rows: y[t] = sum over j < top of weights[t][j] * rows[slot_of[t][j]] (slot_of -1:
 // nothing), in the order of j: what a token's chosen experts have made, summed on the way.  width a multiple of 4, at most
 // 4 NC RA_THREADS.
-template <class TN, int NC>
+template <class TN, int NC, bool EARLY>
 __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_pairs_kernel(float* __restrict__ x, const float* __restrict__ rows,
                                                                        const int* __restrict__ slot_of,
                                                                        const float* __restrict__ weights, int top,
@@ -403,7 +415,7 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_pairs_kernel(float* __
     float* xr = x + row * width;
     int at[NC];                                            // this thread's quads (beyond the row: its last one, counted nowhere)
     bool in[NC];
-    f32x4 y[NC], xs[NC], ws[NC];
+    f32x4 y[NC], xs[NC], ws[NC], nw[NC], ad[NC];
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
         in[c] = threadIdx.x + c * RA_THREADS < quads;
@@ -411,6 +423,15 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_pairs_kernel(float* __
         y[c] = f32x4{0.f, 0.f, 0.f, 0.f};
         xs[c] = *(const f32x4*)(xr + at[c]);
         ws[c] = *(const f32x4*)(w + at[c]);
+        if (EARLY && next_w) nw[c] = *(const f32x4*)(next_w + at[c]);
+        if (EARLY && add_vec) {
+            ad[c] = *(const f32x4*)(add_vec + at[c]);
+            if (add_rows) {
+                const f32x4 e = *(const f32x4*)(add_rows + row * width + at[c]);
+#pragma unroll
+                for (int q = 0; q < 4; ++q) ad[c][q] += e[q];
+            }
+        }
     }
     for (int j0 = 0; j0 < top; j0 += 4) {                  // four rows' loads in flight at a time
         f32x4 t[4][NC];
@@ -440,17 +461,21 @@ __global__ __launch_bounds__(RA_THREADS) void rmsnorm_add_pairs_kernel(float* __
 #pragma unroll
         for (int q = 0; q < 4; ++q) o[q] += y[c][q] * r * ws[c][q];
         if (add_vec) {
-            if (add_rows) {
-                const f32x4 e = *(const f32x4*)(add_rows + row * width + at[c]);
+            f32x4 e;
+            if (EARLY) e = ad[c];
+            else {
+                e = *(const f32x4*)(add_vec + at[c]);
+                if (add_rows) {
+                    const f32x4 e2 = *(const f32x4*)(add_rows + row * width + at[c]);
 #pragma unroll
-                for (int q = 0; q < 4; ++q) o[q] += e[q];
+                    for (int q = 0; q < 4; ++q) e[q] += e2[q];
+                }
             }
-            const f32x4 e = *(const f32x4*)(add_vec + at[c]);
 #pragma unroll
             for (int q = 0; q < 4; ++q) o[q] += e[q];
         }
         xs[c] = o;
-        if (next_w) ws[c] = *(const f32x4*)(next_w + at[c]);
+        if (next_w) ws[c] = EARLY ? nw[c] : *(const f32x4*)(next_w + at[c]);
         if (in[c]) {
             *(f32x4*)(xr + at[c]) = o;
             s2 += o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
@@ -477,11 +502,13 @@ extern "C" int li_rmsnorm_add_pairs(float* x, const float* rows, const int* slot
     if (width % 4 || width > 4 * 8 * RA_THREADS) return LI_UNSUPPORTED;
     if (!next_w) next_dt = DT_F32;
     const int quads = width / 4, nc = quads <= RA_THREADS ? 1 : (quads <= 2 * RA_THREADS ? 2 : (quads <= 4 * RA_THREADS ? 4 : 8));
-#define GO(NC)                                                                                                             \
-    DISPATCH_T(next_dt, (rmsnorm_add_pairs_kernel<T, NC><<<n_rows, RA_THREADS, 0, stream>>>(x, rows, slot_of, weights, top, w, eps, \
+#define GO(NC) do { if (n_rows <= 64) GO1(NC, true); else GO1(NC, false); } while (0)
+#define GO1(NC, EARLY)                                                                                                     \
+    DISPATCH_T(next_dt, (rmsnorm_add_pairs_kernel<T, NC, EARLY><<<n_rows, RA_THREADS, 0, stream>>>(x, rows, slot_of, weights, top, w, eps, \
                                                                                          width, add_rows, add_vec, next_w, next_eps, \
                                                                                          (T*)next)))
     if (nc == 1) GO(1); else if (nc == 2) GO(2); else if (nc == 4) GO(4); else GO(8);
+#undef GO1
 #undef GO
     LI_CHECK_LAUNCH();
     return LI_OK;

@@ -369,14 +369,45 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const TI* __restr
     }
 }
 
+// Besides, where `tail` has positions: the workgroups behind those of the product turn the rotated query parts (what
+// latent_store_kernel does of q_rows; 4 tokens a workgroup), into the columns behind the product's.
+struct QueryTail {
+    const float* rows;          // rotated parts: row t, head h at rows + t * stride + h * head_stride, rd of them
+    const float* freq;
+    const int* pos;             // null: no tail
+    int stride, head_stride, rot, half_pairs, rd, col, width;      // the output's columns col .. width - 1 of a head
+    float magnitude;
+};
+
 #define HLF_STEPS 8
+#define HLF_TAIL 4
 
 template <class TI, class T>
 __global__ __launch_bounds__(64) void head_linear_few_kernel(const TI* __restrict__ in, int64_t in_st, int in_sh,
                                                              const T* __restrict__ W, T* __restrict__ out, int64_t out_st,
                                                              int out_sh, const float* __restrict__ gate, int64_t gate_st,
-                                                             int n_tokens, int n_in, int n_out) {
+                                                             int n_tokens, int n_in, int n_out, int out_blocks, QueryTail tail) {
     typedef typename Vec<T>::v8 v8;
+    if ((int)blockIdx.y >= out_blocks) {
+        const int n = tail.width - tail.col, t0 = (blockIdx.y - out_blocks) * HLF_TAIL, half_rot = tail.rot >> 1;
+        for (int e = threadIdx.x; e < HLF_TAIL * n; e += 64) {
+            const int t = t0 + e / n, j = e % n;
+            if (t >= n_tokens) break;
+            const float* x = tail.rows + (int64_t)t * tail.stride + (int64_t)blockIdx.x * tail.head_stride;
+            float v = j < tail.rd ? x[j] : 0.f;
+            if (j < tail.rot) {
+                const int pair = tail.half_pairs ? (j < half_rot ? j : j - half_rot) : j >> 1;
+                const bool second = tail.half_pairs ? j >= half_rot : j & 1;
+                const float other = x[tail.half_pairs ? (second ? pair : pair + half_rot) : (second ? j - 1 : j + 1)];
+                float sn, cn;
+                sincosf((float)tail.pos[t] * tail.freq[pair], &sn, &cn);
+                cn *= tail.magnitude; sn *= tail.magnitude;
+                v = second ? v * cn + other * sn : v * cn - other * sn;
+            }
+            out[(int64_t)t * out_st + (int64_t)blockIdx.x * out_sh + tail.col + j] = from_f32<T>(v);
+        }
+        return;
+    }
     const int lane = threadIdx.x, col = lane & 31, half = lane >> 5, h = blockIdx.x, j0 = blockIdx.y * 32;
     const bool j_ok = j0 + col < n_out, t_ok = col < n_tokens;
     const T* wrow = W + ((int64_t)h * n_out + (j_ok ? j0 + col : 0)) * n_in + 8 * half;
@@ -428,9 +459,13 @@ __global__ __launch_bounds__(64) void head_linear_few_kernel(const TI* __restric
 
 extern "C" int li_head_linear(const void* in, int in_dt, int64_t in_st, int in_sh, const void* W, int w_dt, void* out,
                               int64_t out_st, int out_sh, const float* gate, int64_t gate_st, int n_tokens, int H, int n_in,
-                              int n_out, hipStream_t stream) {
+                              int n_out, const QueryTail* tail, hipStream_t stream) {
     if (n_tokens <= 0) return LI_OK;
     if (H <= 0 || n_in <= 0 || n_out <= 0) return LI_BAD_ARG;
+    const QueryTail no_tail{};
+    if (tail && (!tail->pos || !tail->rows || tail->rot < 0 || tail->rot > tail->rd || (tail->rot & 1) || (tail->rot && !tail->freq) ||
+                 tail->col < n_out || tail->width > out_sh))
+        return LI_BAD_ARG;
     if (w_dt == DT_F16 || w_dt == DT_BF16) {
         // 16 bytes a lane where every fragment begins at a multiple of 16 bytes
         const int isz = in_dt == DT_F32 ? 4 : 2;
@@ -438,9 +473,11 @@ extern "C" int li_head_linear(const void* in, int in_dt, int64_t in_st, int in_s
                         ((int64_t)in_sh * isz) % 16 == 0;
         dim3 grid((n_tokens + 32 * HLM_TT - 1) / (32 * HLM_TT), H, (n_out + 127) / 128);
         if (vec && n_tokens <= 32) {
-            dim3 few(H, (n_out + 31) / 32);
+            const int out_blocks = (n_out + 31) / 32;
+            dim3 few(H, out_blocks + (tail ? (n_tokens + HLF_TAIL - 1) / HLF_TAIL : 0));
 #define GOF(TI, T) head_linear_few_kernel<TI, T><<<few, 64, 0, stream>>>((const TI*)in, in_st, in_sh, (const T*)W, (T*)out, out_st, out_sh, \
-                                                                        gate, gate_st, n_tokens, n_in, n_out)
+                                                                        gate, gate_st, n_tokens, n_in, n_out, out_blocks,      \
+                                                                        tail ? *tail : no_tail)
             if (in_dt == DT_F32) { if (w_dt == DT_F16) GOF(float, f16); else GOF(float, bf16); }
             else if (in_dt == w_dt) { if (w_dt == DT_F16) GOF(f16, f16); else GOF(bf16, bf16); }
             else return LI_BAD_ARG;
@@ -448,6 +485,7 @@ extern "C" int li_head_linear(const void* in, int in_dt, int64_t in_st, int in_s
             LI_CHECK_LAUNCH();
             return LI_OK;
         }
+        if (tail) return LI_UNSUPPORTED;           // (only in the kernel of a few tokens)
 #define GOM(TI, T) head_linear_mfma_kernel<TI, T><<<grid, 256, 0, stream>>>((const TI*)in, in_st, in_sh, (const T*)W, (T*)out, out_st, \
                                                                            out_sh, gate, gate_st, n_tokens, n_in, n_out, vec)
         if (in_dt == DT_F32) { if (w_dt == DT_F16) GOM(float, f16); else GOM(float, bf16); }
@@ -457,6 +495,7 @@ extern "C" int li_head_linear(const void* in, int in_dt, int64_t in_st, int in_s
         LI_CHECK_LAUNCH();
         return LI_OK;
     }
+    if (tail) return LI_UNSUPPORTED;
     const size_t lds = (size_t)HL_TOK * n_in * sizeof(float);
     if (lds > 64000) return LI_UNSUPPORTED;
     dim3 grid((n_tokens + HL_TOK - 1) / HL_TOK, H);

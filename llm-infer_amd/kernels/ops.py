@@ -1792,7 +1792,33 @@ def latent_store_queries(rows, q_col, kv_col, norm_weight, eps, position, pos, t
     return q
 
 
-def head_linear(x, x_col, x_head_stride, w, out, out_col, out_head_stride, gate=None, gate_col=0) -> torch.Tensor:
+class _QueryTail(ctypes.Structure):
+    _fields_ = [("rows", c_void_p), ("freq", c_void_p), ("pos", c_void_p), ("stride", c_int), ("head_stride", c_int), ("rot", c_int),
+                ("half_pairs", c_int), ("rd", c_int), ("col", c_int), ("width", c_int), ("magnitude", c_float)]
+
+
+def absorbed_queries(q_rows, q_col, w_uk, position, pos, n_heads, d, rd, r, dtype) -> torch.Tensor:
+    """Latent attention's queries [T, H, KW] of ``dtype`` from the float32 rows of their product (every head's [d | rd] from
+    ``q_col``): W_uk^T of the unrotated part (``w_uk`` [H, r, d], None with d 0: zeros) in the first r columns, the rotated part turned
+    by position behind it (``position`` as for ``latent_store``).  A few tokens of a 16-bit model take one launch."""
+    t = q_rows.shape[0]
+    kw = padded_map_dim(r + rd)
+    if d and dtype != torch.float32 and t <= 32 and d % 8 == 0 and (d + rd) % 4 == 0 and q_col % 4 == 0 and q_rows.shape[1] % 4 == 0:
+        _i32(pos, t, "positions")
+        freq, rot, half_pairs, magnitude = _rotation(position, rd)
+        q = torch.empty((t, n_heads, kw), dtype=dtype, device=q_rows.device)
+        tail = _QueryTail(q_rows.data_ptr() + 4 * (q_col + d), freq, pos.data_ptr(), q_rows.shape[1], d + rd, rot, half_pairs, rd, r, kw,
+                          magnitude.value) if kw > r else None
+        return head_linear(q_rows, q_col, d + rd, w_uk, q, 0, kw, _tail=tail)
+    q = latent_queries(q_rows, q_col, position, pos, n_heads, d, rd, r, dtype)
+    if d:
+        head_linear(q_rows, q_col, d + rd, w_uk, q, 0, kw)                     # q' into the first r columns of every head
+    else:
+        q[:, :, :r].zero_()
+    return q
+
+
+def head_linear(x, x_col, x_head_stride, w, out, out_col, out_head_stride, gate=None, gate_col=0, _tail=None) -> torch.Tensor:
     """A product per head: out[t, out_col + h * out_head_stride + j] = sum over i of w[h, j, i] * x[t, x_col + h *
     x_head_stride + i], ``w`` [H, n_out, n_in] in the model's type (a 16-bit model runs it on the matrix cores, a float32
     input as the sum of two 16-bit numbers), ``x`` [T, ...] float32 or of that type, ``out``
@@ -1815,7 +1841,8 @@ def head_linear(x, x_col, x_head_stride, w, out, out_col, out_head_stride, gate=
                                    x_head_stride, _ptr(w), DT[w.dtype], c_void_p(o2.data_ptr() + out_col * o2.element_size()),
                                    c_int64(o2.shape[1]), out_head_stride,
                                    c_void_p(gate.data_ptr() + 4 * gate_col) if gate is not None else None,
-                                   c_int64(gate.shape[1] if gate is not None else 0), t, H, n_in, n_out, _stream()), "head_linear")
+                                   c_int64(gate.shape[1] if gate is not None else 0), t, H, n_in, n_out,
+                                   ctypes.byref(_tail) if _tail is not None else None, _stream()), "head_linear")
     return out
 
 
@@ -2145,10 +2172,14 @@ def route_pairs(h, w_router, bias, n_experts: int, top: int, scale: float = 1.0)
 
 @functools.lru_cache(maxsize=1024)
 def _pairs_plan(pairs: int, n_experts: int, n: int, k: int) -> tuple:
-    """(tile, few_rows) of gemm_wreg's pairs mode: tiles of 64 pairs where an expert has no more on average, else the tile
-    of least estimated time, each expert's last tile half full."""
-    if pairs <= 64 * n_experts:
+    """(tile, few_rows) of gemm_wreg's pairs mode: tiles of 64 pairs where an expert has about half of that, else the tile
+    of least estimated time, each expert's last tile half full (measured, 16 experts, up 7,168 x 4,096 and down 4,096 x 3,584:
+    32 pairs an expert 178.6 and 89.6 us with tiles of 64 pairs against 176.9 and 91.7 with the best of 128, 64 pairs 220 and
+    119 against 185 and 99; 512 pairs down 273 us with the widest tile, 293 and 301 with the others)."""
+    if pairs <= 40 * n_experts:
         return 2, 1
+    if pairs >= 256 * n_experts and n >= 4096:
+        return 0, 0
     return min(((_wreg_cost(t, 1, pairs + 64 * n_experts, n, k), t) for t in (0, 1, 2)))[1], 0
 
 
@@ -2167,8 +2198,9 @@ def linear_pairs(x, w, p: SortedPairs, mode: int = EPI_STORE, gather: bool = Tru
     _need(mode in (EPI_STORE, EPI_SWIGLU), "linear_pairs: store or silu(gate) * up")
     out = torch.empty((pairs, n // 2 if mode == EPI_SWIGLU else n), dtype=out_dtype or x.dtype, device=x.device)
     row_of = _ptr(p.row_of) if gather else None
-    # few pairs an expert: its matrix is streamed once straight into the operands
-    kind = force or ("gemv" if pairs <= 16 * e else "wreg")
+    # few pairs an expert: its matrix is streamed once straight into the operands (measured as above: 8 pairs an expert 156.5
+    # and 82.7 us against 169.6 and 84.7, 16 pairs 206 and 114 against 172 and 87)
+    kind = force or ("gemv" if pairs <= 10 * e else "wreg")
     if kind == "gemv":
         _check(experts().li_experts_gemv(_ptr(x), _ptr(w), DT[x.dtype], _ptr(out), DT[out.dtype], mode, pairs, n, k, c_int64(n * k), e,
                                          _ptr(p.counts), _ptr(p.offsets), row_of, _stream()), "experts_gemv")

@@ -104,19 +104,18 @@ class LatentAttention(Part):
         proj = ops.linear(h, self.w_in, out_dtype=torch.float32)
         kv = view.as_tuple()
         if self.q_rank is None:
-            kv_col, q_rows = H * (d + rd), proj
+            kv_col = H * (d + rd)
             q = ops.latent_store_queries(proj, 0, kv_col, self.kv_norm, self.norm_eps, self.turn, ctx.pos, ctx.tok_slot, kv, H, d, rd, r)
+            if d:
+                ops.head_linear(proj, 0, d + rd, self.w_uk, q, 0, q.shape[2])          # q' into the first r columns of every head
+            else:
+                q[:, :, :r].zero_()
         else:
             kv_col = self.q_rank
             cq = ops.latent_store(proj, kv_col, self.kv_norm, self.norm_eps, self.turn, ctx.pos, ctx.tok_slot, kv, d, rd, r,
                                   (0, self.q_norm))
             q_rows = ops.linear(cq, self.w_uq, out_dtype=torch.float32)
-            q = ops.latent_queries(q_rows, 0, self.turn, ctx.pos, H, d, rd, r, cq.dtype)
-        kw = q.shape[2]
-        if d:
-            ops.head_linear(q_rows, 0, d + rd, self.w_uk, q, 0, kw)            # q' into the first r columns of every head
-        else:
-            q[:, :, :r].zero_()
+            q = ops.absorbed_queries(q_rows, 0, self.w_uk, self.turn, ctx.pos, H, d, rd, r, cq.dtype)
         sixteen = self.dtype != torch.float32 and ops.diff_attention_fits(self.key_dim, r)
         a = ops.diff_attention(q, kv, ctx.pos, ctx.tok_slot, H, 1, 1, self.key_dim, r, self.scale, None, self.window, 0.0, None,
                                1.0, self.dtype, ops.diff_tiles(ctx, None, self.window) if sixteen else None, sink=self.sinks,

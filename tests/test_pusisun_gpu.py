@@ -200,6 +200,35 @@ def test_products_per_head_of_a_few_tokens(lib, dtype):
                 assert error(out.cpu(), want) < (0.03 if src.dtype != torch.float32 else 0.02), (n, n_in, n_out)
 
 
+@pytest.mark.parametrize("dtype", ["bfloat16", "float16", "float32"])
+def test_queries_of_a_few_tokens_in_one_launch(lib, dtype):
+    """The query taken into the latents' space beside its rotated part: in the launch of a few tokens and in two."""
+    from llm_infer_amd.kernels import ops
+    g = torch.Generator().manual_seed(10)
+    for H, d, rd, rot, r, half in ((3, 8, 12, 8, 20, True), (2, 24, 4, 4, 33, False), (4, 64, 0, 0, 48, True), (1, 16, 8, 8, 40, True),
+                                   (2, 10, 6, 6, 16, True), (2, 0, 16, 16, 16, True)):
+        freqs = (50.0 ** (-torch.arange(max(rot // 2, 1)) / 3.0)).float().to(DEV)
+        w = torch.randn(H, r, d, generator=g).to(DT[dtype]) if d else None
+        for n in (1, 5, 32, 33):
+            rows_ = torch.randn(n, H * (d + rd) + 4, generator=g)
+            pos = torch.randint(0, 300, (n,), generator=g, dtype=torch.int32)
+            q = ops.absorbed_queries(rows_.to(DEV), 4, None if w is None else w.to(DEV), (freqs if rot else None, rot, half, 1.3), pos.to(DEV), H, d,
+                                     rd, r, DT[dtype]).cpu()
+            part = rows_[:, 4:].view(n, H, d + rd).double()
+            tol = 1e-4 if dtype == "float32" else 0.03
+            if d:
+                assert error(q[:, :, :r], torch.einsum("thd,hrd->thr", part[..., :d], w.double())) < tol, (H, d, n)
+            else:
+                assert float(q[:, :, :r].abs().max()) == 0.0
+            turned = part[..., d:].clone()
+            order = list(range(rot)) if half else list(range(0, rot, 2)) + list(range(1, rot, 2))
+            if rot:
+                turned[..., order] = P.turn(turned[..., order], pos, freqs.double().cpu()[:rot // 2], 1.3)
+            if rd:
+                assert error(q[:, :, r:r + rd], turned) < tol, (H, d, n)
+            assert q.shape[2] == r + rd or float(q[:, :, r + rd:].abs().max()) == 0.0
+
+
 def check_pairs(p, chosen, weights):
     """Sorted pairs against a choice [T, top] (experts ascending) and its weights, exactly."""
     T, top = chosen.shape
