@@ -49,10 +49,10 @@ def test_turning_half_pairs_with_a_magnitude():
     assert torch.allclose(s(9, 4), s(25, 20))
 
 
-@pytest.mark.parametrize("scaling", [(4.0, 512, 32.0, 1.0), (2.0, 40, 3.0, 2.9), (40.0, 100000, 1.0, 0.5), (8.0, 10, 40.0, 20.0)])
+@pytest.mark.parametrize("scaling", [(6.0, 700, 30.0, 1.5), (2.0, 40, 3.0, 2.9), (40.0, 100000, 1.0, 0.5), (8.0, 10, 40.0, 20.0)])
 def test_stretched_frequencies(scaling):
     sc = dict(zip(("factor", "original", "fast", "slow"), scaling))
-    f0, (f, mag) = P.stretched_frequencies(32, 10000.0, None)[0], P.stretched_frequencies(32, 10000.0, sc)
+    f0, (f, mag) = P.stretched_frequencies(40, 20000.0, None)[0], P.stretched_frequencies(40, 20000.0, sc)
     assert math.isclose(mag, 0.1 * math.log(sc["factor"]) + 1.0)
     assert (f <= f0 * (1 + 1e-12)).all() and (f >= f0 / sc["factor"] * (1 - 1e-12)).all()
     ratio = f / f0
@@ -66,7 +66,7 @@ def test_stretched_frequencies(scaling):
     assert torch.allclose(ratio[few], torch.tensor(1.0 / sc["factor"], dtype=D))
     # the library's own table
     from llm_infer_amd.parts.position import scaled_by_ramp
-    own, own_mag = scaled_by_ramp(10000.0, 32, sc)
+    own, own_mag = scaled_by_ramp(20000.0, 40, sc)
     assert torch.allclose(own.double(), f, rtol=1e-6) and math.isclose(own_mag, mag)
 
 
