@@ -421,6 +421,8 @@ MIXERS = [
     M.latent(40, 16, 16, 16, 32, 32, scaling=(16.0, 30, 4.0, 0.5)),               # two tiles of heads
     M.latent(1, 8, 0, 40, 16, 5),                                                 # nothing turned, one head
     M.latent(4, 64, 64, 64, 128, 96, scaling=(40.0, 4096, 32.0, 1.0)),
+    M.latent(3, 16, 20, 16, 300, 40, scaling=(4.0, 60, 8.0, 1.0)),                # a latent beyond what the matrix-core kernel takes
+    M.attention(2, 1, 272, 40, 30, 3),                                            # keys beyond it, with kept tokens
     M.attention(3, 1, 20, 9, 30, 3),                                              # a padded head, values narrower than keys
     M.attention(4, 4, 8, 40, 1, 2),                                               # only the token itself and the first two
     M.attention(16, 2, 64, 64, 70, 65),                                           # one size: the other kernels; more than a page kept
